@@ -1,4 +1,5 @@
-"""ctypes binding of ``libzipage_hip.so`` (the C ABI in ``include/zipage_hip.h``).
+"""ctypes binding of ``libzipage_hip.so`` and ``libzipage_models.so`` (the C ABIs in
+``include/zipage_hip.h`` and ``include/zipage_models.h``).
 
 The product path has no CPU fallback: if the shared object is missing or a symbol cannot
 be resolved, importing a kernel wrapper raises.  ctypes releases the GIL for the duration
@@ -15,6 +16,7 @@ import torch
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libzipage_hip.so")
+MODELS_LIB_PATH = os.path.join(_HERE, "libzipage_models.so")
 
 ZP_BF16, ZP_F16, ZP_F32 = 0, 1, 2
 _DTYPES = {torch.bfloat16: ZP_BF16, torch.float16: ZP_F16, torch.float32: ZP_F32}
@@ -84,36 +86,73 @@ I64_RETURNING = {
 }
 EXPORTS = sorted(list(SIGNATURES) + list(I64_RETURNING) + ["zp_abi_version", "zp_last_error"])
 
+# the model-side library, in the order of include/zipage_models.h
+MODEL_SIGNATURES = {
+    "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, i32, ptr],
+    "zp_residual_norm": [ptr, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32, f32,
+                         i32, ptr],
+    "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
+    "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, f32, i32, ptr],
+    "zp_gather_rows": [ptr, ptr, ptr, i32, i32, i64, ptr],
+    "zp_headwise_linear": [ptr, ptr, ptr, i32, i32, i32, i32, i32, ptr],
+    "zp_latent_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, f32,
+                                 i32, ptr, i64, ptr],
+    "zp_latent_tiles_attention": [ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, i64, i64, i64, f32,
+                                  i32, ptr],
+}
+MODEL_I64_RETURNING = {"zp_latent_rows_workspace": [i32, i32, i32, i32, i32, i32, i32]}
+MODEL_EXPORTS = sorted(list(MODEL_SIGNATURES) + list(MODEL_I64_RETURNING))
+
 _lib = None
+_models = None
 
 
-def load() -> C.CDLL:
-    """Load the shared object once and type every entry point.  Raises if absent."""
-    global _lib
-    if _lib is not None:
-        return _lib
-    if not os.path.exists(LIB_PATH):
+def _open(path: str, signatures: dict, i64_returning: dict) -> C.CDLL:
+    if not os.path.exists(path):
         raise RuntimeError(
-            f"{LIB_PATH} is missing: build it with `python -m zipage_amd.build` "
-            "(there is no CPU fallback for the compression kernels)")
-    lib = C.CDLL(LIB_PATH)
-    for name, args in SIGNATURES.items():
+            f"{path} is missing: build it with `python -m zipage_amd.build` "
+            "(there is no CPU fallback for the HIP kernels)")
+    lib = C.CDLL(path)
+    for name, args in signatures.items():
         fn = getattr(lib, name)
         fn.argtypes, fn.restype = args, i32
-    for name, args in I64_RETURNING.items():
+    for name, args in i64_returning.items():
         fn = getattr(lib, name)
         fn.argtypes, fn.restype = args, i64
     lib.zp_abi_version.argtypes, lib.zp_abi_version.restype = [], i32
     lib.zp_last_error.argtypes, lib.zp_last_error.restype = [], C.c_char_p
-    _lib = lib
     return lib
+
+
+def load() -> C.CDLL:
+    """Load the compression library once and type every entry point.  Raises if absent."""
+    global _lib
+    if _lib is None:
+        _lib = _open(LIB_PATH, SIGNATURES, I64_RETURNING)
+    return _lib
+
+
+def load_models() -> C.CDLL:
+    """The same for the model-side library."""
+    global _models
+    if _models is None:
+        _models = _open(MODELS_LIB_PATH, MODEL_SIGNATURES, MODEL_I64_RETURNING)
+    return _models
+
+
+def _check(lib, name: str, rc: int) -> None:
+    if rc != 0:
+        raise RuntimeError(f"{name} failed ({rc}): {lib.zp_last_error().decode()}")
 
 
 def call(name: str, *args) -> None:
     lib = load()
-    rc = getattr(lib, name)(*args)
-    if rc != 0:
-        raise RuntimeError(f"{name} failed ({rc}): {lib.zp_last_error().decode()}")
+    _check(lib, name, getattr(lib, name)(*args))
+
+
+def call_models(name: str, *args) -> None:
+    lib = load_models()
+    _check(lib, name, getattr(lib, name)(*args))
 
 
 def dtype_tag(t: torch.Tensor) -> int:

@@ -1,7 +1,9 @@
-"""Build libzipage_hip.so (gfx950) in-tree with hipcc.
+"""Build the HIP libraries (gfx950) in-tree with hipcc.
 
-Run as ``python -m zipage_amd.build``.  The library is one shared object with a plain C
-ABI (``include/zipage_hip.h``); it does not link against torch.
+Run as ``python -m zipage_amd.build``.  Two shared objects with a plain C ABI, neither linked
+against torch: ``libzipage_hip.so`` (``include/zipage_hip.h``: the compression path and the kernels
+of the models that use it) and ``libzipage_models.so`` (``include/zipage_models.h``: the kernels of
+the other models), so that a model served without compression compiles only what it runs.
 """
 from __future__ import annotations
 
@@ -13,19 +15,25 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libzipage_hip.so")
+MODELS_LIB = os.path.join(HERE, "libzipage_models.so")
 
 # packed fp32 VALU ops are disabled on purpose (some forms misbehave on this fleet)
-FLAGS = [
-    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",
+BASE_FLAGS = [
+    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC",
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
-    # keep a*b+c as two roundings: the stages restate torch ops that round after each op
-    "-ffp-contract=off",
     "-Wno-unused-command-line-argument",
 ]
+# keep a*b+c as two roundings: the compression stages restate torch ops that round after each op
+FLAGS = BASE_FLAGS + ["-ffp-contract=off"]
+
+MODEL_SOURCES = ("latent.hip", "residual.hip")     # these and the error reporting
+COMMON_SOURCES = ("runtime.hip",)
 
 
-def sources():
-    return sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".hip"))
+def sources(models: bool = False):
+    names = [f for f in os.listdir(CSRC) if f.endswith(".hip")]
+    keep = (lambda f: f in MODEL_SOURCES or f in COMMON_SOURCES) if models else (lambda f: f not in MODEL_SOURCES)
+    return sorted(os.path.join(CSRC, f) for f in names if keep(f))
 
 
 def _run(cmd, verbose):
@@ -40,23 +48,41 @@ def _run(cmd, verbose):
         print(err, file=sys.stderr)
 
 
-def build(verbose: bool = True, jobs: int | None = None) -> str:
-    """Compile every source to an object file (in parallel) and link the shared object."""
+def build(verbose: bool = True, jobs: int | None = None, libs: tuple[str, ...] = (LIB, MODELS_LIB)) -> str:
+    """Compile the sources of ``libs`` to object files (in parallel) and link the shared objects."""
     from concurrent.futures import ThreadPoolExecutor
     hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
     extra = os.environ.get("ZP_EXTRA_HIPCC_FLAGS", "").split()
-    objdir = os.path.join(HERE, "build")
-    os.makedirs(objdir, exist_ok=True)
-    compile_flags = [f for f in FLAGS if f != "-shared"]
-    srcs = sources()
-    objs = [os.path.join(objdir, os.path.basename(s)[:-4] + ".o") for s in srcs]
-    jobs = jobs or min(len(srcs), os.cpu_count() or 1, 16)
+    work, links = [], []
+    for lib in libs:
+        models = lib == MODELS_LIB
+        objdir = os.path.join(HERE, "build", "models" if models else "")
+        os.makedirs(objdir, exist_ok=True)
+        objs = []
+        for src in sources(models):
+            obj = os.path.join(objdir, os.path.basename(src)[:-4] + ".o")
+            work.append([hipcc, *(BASE_FLAGS if models else FLAGS), *extra, "-c", src, "-o", obj])
+            objs.append(obj)
+        links.append((lib, objs))
+    jobs = jobs or min(len(work), os.cpu_count() or 1, 16)
     with ThreadPoolExecutor(max_workers=jobs) as pool:
-        list(pool.map(lambda so: _run([hipcc, *compile_flags, *extra, "-c", so[0], "-o", so[1]], verbose),
-                      zip(srcs, objs)))
-    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB + ".tmp"], verbose)
-    os.replace(LIB + ".tmp", LIB)
-    return LIB
+        list(pool.map(lambda cmd: _run(cmd, verbose), work))
+    for lib, objs in links:
+        _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", lib + ".tmp"], verbose)
+        os.replace(lib + ".tmp", lib)
+    return libs[0]
+
+
+def ensure(lib: str) -> str:
+    """Build ``lib`` if it is not there yet (one process at a time)."""
+    if not os.path.exists(lib):
+        import fcntl
+        os.makedirs(os.path.join(HERE, "build"), exist_ok=True)
+        with open(os.path.join(HERE, "build", ".lock"), "w") as lock:
+            fcntl.flock(lock, fcntl.LOCK_EX)
+            if not os.path.exists(lib):
+                build(verbose=False, libs=(lib,))
+    return lib
 
 
 if __name__ == "__main__":

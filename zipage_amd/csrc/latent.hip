@@ -1,0 +1,833 @@
+// Latent attention: keys and values of all heads are linear images of one cached vector c per token
+// (R elements), so the cache holds c alone.
+//
+//   latent_norm_store   RMS norms of the two low-rank projections of a token; c goes to its slot
+//   headwise            per-head product out[n, h] = W[h] in[n, h]  (q -> W_uk^T q, sum p c -> W_uv sum p c)
+//   latent_rows         attention of single tokens over the paged latents, all heads of a token on
+//                       one read of its context: score = (W_uk^T q) . c, out = sum p c
+//   latent_tiles        attention of runs of prompt tokens over expanded keys and values
+//   latent_plain        float32 form of latent_rows (true fp32 products), any sizes
+//
+// Both bf16 attention kernels keep S^T = K Q^T and O^T = V^T P^T: in that orientation the MFMA
+// result layout of S^T (column = query, four consecutive keys per lane) IS the operand layout of
+// P^T once the 32 keys of a step are numbered (lane group g holds keys 4g..4g+3 and
+// 16+4g..16+4g+3), so the softmax weights never leave their lane: no LDS and no barrier in the key
+// loop, every wave is its own flash loop.  V^T operands are built from row-major 16-byte loads of
+// eight keys x eight columns by v_perm; the column order that results (MFMA t, row m <-> column
+// 8m + t) leaves eight consecutive output columns in each lane.
+#include "models.h"
+#include <math.h>
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef zp_u32x4 u32x4;
+typedef zp_f32x4 f32x4;
+
+__device__ __forceinline__ f32x4 mfma_bf16(const u32x4& a, const u32x4& b, const f32x4& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
+                                                 __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+__device__ __forceinline__ uint32_t pack_bf16(float lo, float hi) {
+  const zp_f32x2 f = {lo, hi};
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, zp_bf16x2));
+}
+// key of operand element i (0..7) held by lane group g, within a step of 32 keys
+__device__ __forceinline__ int step_key(int g, int i) { return i < 4 ? 4 * g + i : 12 + 4 * g + i; }
+
+// Eight rows (keys) of eight bf16 columns -> for column t the four dwords of its eight keys.
+__device__ __forceinline__ u32x4 column_of(const u32x4* rows, int t) {
+  const uint32_t sel = (t & 1) ? 0x07060302u : 0x05040100u;
+  u32x4 o;
+#pragma unroll
+  for (int d = 0; d < 4; ++d)
+    o[d] = __builtin_amdgcn_perm(rows[2 * d + 1][t >> 1], rows[2 * d][t >> 1], sel);
+  return o;
+}
+
+// ------------------------------------------------------------------ norms of the low-rank rows
+struct NormStoreArgs {
+  const void* in;        // (n, q_width + c_width) T
+  const float* wq;       // (q_width,)
+  const float* wc;       // (c_width,)
+  void* q_out;           // (n, q_width) T
+  void* c_out;           // (n, c_width) T or null
+  void* cache;           // (num_slots, c_width) T
+  const int32_t* slots;  // (n,), -1 skips
+  int n, q_width, c_width, q_norm, c_norm;
+  int64_t num_slots;
+  float eps;
+};
+constexpr int kNormPieces = 8;   // 8-element pieces per lane: ranks up to 4096
+
+// One wave per (token, part).
+template <typename T>
+__global__ __launch_bounds__(256) void latent_norm_store_kernel(NormStoreArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int item = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int row = item >> 1;
+  if (row >= a.n) return;
+  const bool is_c = item & 1;
+  const int width = is_c ? a.c_width : a.q_width;
+  const int pieces = width / 8;
+  const int64_t src = (int64_t)row * (a.q_width + a.c_width) + (is_c ? a.q_width : 0);
+  const float* w = is_c ? a.wc : a.wq;
+  float v[kNormPieces][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < kNormPieces; ++k) {
+    const int pc = lane + k * 64;
+    if (pc < pieces) {
+      Vec8<T>::ld(a.in, src + pc * 8, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+    }
+  }
+  ss = wave_sum(ss);
+  const float rs = 1.f / sqrtf(ss / (float)(is_c ? a.c_norm : a.q_norm) + a.eps);
+  int64_t slot = is_c ? a.slots[row] : -1;
+  if (slot >= a.num_slots) slot = -1;
+#pragma unroll
+  for (int k = 0; k < kNormPieces; ++k) {
+    const int pc = lane + k * 64;
+    if (pc < pieces) {
+      float wv[8];
+      Vec8<F32>::ld(w, pc * 8, wv);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] = v[k][i] * rs * wv[i];
+      if (is_c) {
+        if (slot >= 0) Vec8<T>::st(a.cache, slot * width + pc * 8, v[k]);
+        if (a.c_out) Vec8<T>::st(a.c_out, (int64_t)row * width + pc * 8, v[k]);
+      } else {
+        Vec8<T>::st(a.q_out, (int64_t)row * width + pc * 8, v[k]);
+      }
+    }
+  }
+}
+
+// ------------------------------------------------------------------ gather of cached rows
+__global__ __launch_bounds__(256) void gather_rows_kernel(const char* src, const int32_t* rows, char* out,
+                                                          int64_t total, int pieces, int64_t num_rows) {
+  const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (id >= total) return;
+  const int64_t r = id / pieces, pc = id - r * pieces;
+  int64_t s = rows[r];
+  if (s < 0 || s >= num_rows) s = 0;
+  ((u32x4*)out)[id] = ((const u32x4*)src)[s * pieces + pc];
+}
+
+// ------------------------------------------------------------------ per-head product
+struct HeadArgs {
+  const void* in;   // (n, H, K) T
+  const void* w;    // (H, M, K) T
+  void* out;        // (n, H, M) T
+  int n, H, K, M;
+};
+constexpr int kTokTiles = 4;
+
+// A wave owns 16 outputs of one head for up to 64 tokens: W is the row operand, so a lane ends
+// with four consecutive outputs of one token.
+template <typename T>
+__global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
+  const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
+  const int m0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16;
+  const int h = blockIdx.y;
+  const int n0 = blockIdx.z * 16 * kTokTiles;
+  if (m0 >= a.M) return;
+  const int tiles = min(kTokTiles, (a.n - n0 + 15) / 16);
+  f32x4 acc[kTokTiles];
+#pragma unroll
+  for (int t = 0; t < kTokTiles; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int64_t wrow = ((int64_t)h * a.M + m0 + l16) * a.K;
+  int64_t xrow[kTokTiles];
+#pragma unroll
+  for (int t = 0; t < kTokTiles; ++t)
+    xrow[t] = ((int64_t)min(n0 + t * 16 + l16, a.n - 1) * a.H + h) * a.K;
+  if constexpr (T::bytes == 2) {
+    const uint16_t* w = (const uint16_t*)a.w;
+    const uint16_t* x = (const uint16_t*)a.in;
+    for (int k = g * 8; k < a.K; k += 32) {
+      const u32x4 wf = *(const u32x4*)(w + wrow + k);
+#pragma unroll
+      for (int t = 0; t < kTokTiles; ++t)
+        if (t < tiles) acc[t] = mfma_bf16(wf, *(const u32x4*)(x + xrow[t] + k), acc[t]);
+    }
+  } else {
+    const float* w = (const float*)a.w;
+    const float* x = (const float*)a.in;
+    for (int k = g; k < a.K; k += 4) {
+      const float wf = w[wrow + k];
+#pragma unroll
+      for (int t = 0; t < kTokTiles; ++t)
+        if (t < tiles) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf, x[xrow[t] + k], acc[t], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < kTokTiles; ++t) {
+    const int n = n0 + t * 16 + l16;
+    if (t < tiles && n < a.n) {
+      const int64_t at = ((int64_t)n * a.H + h) * a.M + m0 + g * 4;
+      if constexpr (T::bytes == 2) {
+        uint2 o;
+        o.x = pack_bf16(acc[t][0], acc[t][1]);
+        o.y = pack_bf16(acc[t][2], acc[t][3]);
+        *(uint2*)((uint16_t*)a.out + at) = o;
+      } else {
+        *(f32x4*)((float*)a.out + at) = acc[t];
+      }
+    }
+  }
+}
+
+// ------------------------------------------------------------------ single tokens over the pages
+struct RowsArgs {
+  const void* q;          // (n, H, R) T
+  const void* cache;      // (pages, BS, R) T
+  const int32_t* table;   // (B, NB) page ids
+  const int32_t* ctx;     // (n,) tokens of the sequence up to and including this one; 0 = inert
+  const int32_t* seq;     // (n,) row of table, or null: row i
+  void* out;              // (n, H, R) T
+  float* part;            // splits > 1: (n, H, splits, R) fp32, then (n, H, splits, 2) max and sum
+  int n, H, R, BS, bs_shift, B, NB, num_pages;
+  int window;             // a token sees the last `window` tokens including itself; 0 = all
+  int splits;             // key ranges handled by different workgroups
+  int hw;                 // waves of a workgroup on different heads (1, 2, 4); the others split keys
+  int lds_pages;          // page ids held in LDS
+  float scale;
+};
+
+__device__ __forceinline__ int page_of(const RowsArgs& a, int t) {
+  return a.bs_shift >= 0 ? t >> a.bs_shift : t / a.BS;
+}
+
+// NCB column blocks of 128 cover R.  Workgroup: one token, 16 * hw heads, one key range.
+template <int NCB>
+__global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  int* pg = (int*)lds_raw;
+  float* merge = (float*)(lds_raw + ((a.lds_pages * 4 + 15) & ~15));
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int l16 = lane & 15, g = lane >> 4;
+  const int hw = a.hw, kw = 4 / hw, hwi = wave % hw, kwi = wave / hw;
+  const int hgroups = (a.H + 16 * hw - 1) / (16 * hw);
+  int id = blockIdx.x;
+  const int split = id % a.splits;
+  id /= a.splits;
+  const int hg = id % hgroups;
+  const int row = id / hgroups;
+  const int head = (hg * hw + hwi) * 16 + l16;
+  const bool head_ok = head < a.H;
+  const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
+  const int n = min(a.ctx[row], a.NB * a.BS);
+  const int lo = a.window > 0 ? max(0, n - a.window) : 0;
+  const int p0 = page_of(a, lo);
+  constexpr int KS = 4 * NCB;
+  const int nks = a.R / 32;
+
+  if (n > 0) {
+    const int np = page_of(a, n - 1) - p0 + 1;
+    for (int j = tid; j < np && j < a.lds_pages; j += 256) {
+      const int p = a.table[(int64_t)seq * a.NB + p0 + j];
+      pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
+    }
+  }
+  __syncthreads();
+  const uint16_t* cache = (const uint16_t*)a.cache;
+  auto key_row = [&](int t) -> const uint16_t* {
+    t = min(max(t, lo), n - 1);
+    const int p = page_of(a, t);
+    return cache + ((int64_t)pg[p - p0] * a.BS + (t - p * a.BS)) * a.R;
+  };
+
+  u32x4 qf[KS];
+  {
+    const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + (head_ok ? head : 0)) * a.R + g * 8;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+      qf[ks] = (head_ok && ks < nks) ? *(const u32x4*)(q + ks * 32) : u32x4{0u, 0u, 0u, 0u};
+  }
+  f32x4 o[NCB * 8];
+#pragma unroll
+  for (int i = 0; i < NCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  const float sc = a.scale * 1.44269504088896f;
+
+  if (n > 0) {
+    const int b1 = (n - 1) >> 5;
+    for (int b = (lo >> 5) + split * kw + kwi; b <= b1; b += a.splits * kw) {
+      const int k0 = b * 32;
+      f32x4 s[2];
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt) {
+        const uint16_t* kr = key_row(k0 + tt * 16 + l16) + g * 8;
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+          if (ks < nks) acc = mfma_bf16(*(const u32x4*)(kr + ks * 32), qf[ks], acc);
+        s[tt] = acc;
+      }
+      float p[8], mx = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int key = k0 + step_key(g, i);
+        p[i] = (key >= lo && key < n) ? s[i >> 2][i & 3] * sc : -INFINITY;
+        mx = fmaxf(mx, p[i]);
+      }
+      mx = fmaxf(mx, lane_xor16(mx));
+      mx = fmaxf(mx, lane_xor32(mx));
+      const float mn = fmaxf(m, mx);          // finite: every step holds a visible key
+      const float f = __builtin_amdgcn_exp2f(m - mn);
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
+        sum += p[i];
+      }
+      l = l * f + sum;
+      m = mn;
+      if (__any(f != 1.f)) {
+#pragma unroll
+        for (int i = 0; i < NCB * 8; ++i) o[i] *= f;
+      }
+      const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                        pack_bf16(p[6], p[7])};
+      const uint16_t* vr[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) vr[i] = key_row(k0 + step_key(g, i));
+#pragma unroll
+      for (int cb = 0; cb < NCB; ++cb) {
+        const int col = cb * 128 + l16 * 8;
+        const int off = col < a.R ? col : 0;
+        u32x4 v[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = *(const u32x4*)(vr[i] + off);
+#pragma unroll
+        for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v, t), pf, o[cb * 8 + t]);
+      }
+    }
+  }
+  l += lane_xor16(l);
+  l += lane_xor32(l);
+
+  // waves that split the keys of the same heads meet in LDS
+  if (kw > 1) {
+    const int RS = a.R + 4;
+    const int per = 16 * RS + 32;                   // O rows, then max and sum of 16 heads
+    if (kwi > 0) {
+      float* dst = merge + (int64_t)((kwi - 1) * hw + hwi) * per;
+      if (g == 0) { dst[16 * RS + l16] = m; dst[16 * RS + 16 + l16] = l; }
+#pragma unroll
+      for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = cb * 128 + (4 * g + i) * 8;
+          if (col < a.R) {
+            float* d = dst + l16 * RS + col;
+            *(f32x4*)d = f32x4{o[cb * 8][i], o[cb * 8 + 1][i], o[cb * 8 + 2][i], o[cb * 8 + 3][i]};
+            *(f32x4*)(d + 4) = f32x4{o[cb * 8 + 4][i], o[cb * 8 + 5][i], o[cb * 8 + 6][i], o[cb * 8 + 7][i]};
+          }
+        }
+    }
+    __syncthreads();
+    if (kwi > 0) return;
+    for (int k = 1; k < kw; ++k) {
+      const float* src = merge + (int64_t)((k - 1) * hw + hwi) * per;
+      const float m2 = src[16 * RS + l16], l2 = src[16 * RS + 16 + l16];
+      const float mn = fmaxf(m, m2);
+      const float ms = mn == -INFINITY ? 0.f : mn;
+      const float f1 = __builtin_amdgcn_exp2f(m - ms), f2 = __builtin_amdgcn_exp2f(m2 - ms);
+      l = l * f1 + l2 * f2;
+      m = mn;
+#pragma unroll
+      for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = cb * 128 + (4 * g + i) * 8;
+          if (col < a.R) {
+            const float* d = src + l16 * RS + col;
+#pragma unroll
+            for (int t = 0; t < 8; ++t) o[cb * 8 + t][i] = o[cb * 8 + t][i] * f1 + d[t] * f2;
+          }
+        }
+    }
+  }
+  if (!head_ok) return;
+  if (a.splits == 1) {
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    uint16_t* out = (uint16_t*)a.out + ((int64_t)row * a.H + head) * a.R;
+#pragma unroll
+    for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = cb * 128 + (4 * g + i) * 8;
+        if (col < a.R) {
+          float r[8];
+#pragma unroll
+          for (int t = 0; t < 8; ++t) r[t] = o[cb * 8 + t][i] * inv;
+          Vec8<BF16>::st(out, col, r);
+        }
+      }
+  } else {
+    const int64_t at = ((int64_t)row * a.H + head) * a.splits + split;
+    float* out = a.part + at * a.R;
+    float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + at * 2;
+    if (g == 0) { ml[0] = m; ml[1] = l; }
+#pragma unroll
+    for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = cb * 128 + (4 * g + i) * 8;
+        if (col < a.R) {
+          float r[8];
+#pragma unroll
+          for (int t = 0; t < 8; ++t) r[t] = o[cb * 8 + t][i];
+          Vec8<F32>::st(out, col, r);
+        }
+      }
+  }
+}
+
+__global__ __launch_bounds__(64) void latent_rows_combine_kernel(RowsArgs a) {
+  const int64_t item = blockIdx.x;       // (row, head)
+  const float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + item * a.splits * 2;
+  float mx = -INFINITY;
+  for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ml[2 * s]);
+  if (mx == -INFINITY) mx = 0.f;
+  float l = 0.f;
+  for (int s = 0; s < a.splits; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - mx);
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  for (int c = threadIdx.x * 8; c < a.R; c += 512) {
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < a.splits; ++s) {
+      const float f = __builtin_amdgcn_exp2f(ml[2 * s] - mx) * inv;
+      float v[8];
+      Vec8<F32>::ld(a.part, (item * a.splits + s) * a.R + c, v);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc[i] += v[i] * f;
+    }
+    Vec8<BF16>::st(a.out, item * a.R + c, acc);
+  }
+}
+
+// One workgroup per (token, head), plain fp32 arithmetic, any R.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_plain_kernel(RowsArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  float* q = (float*)lds_raw;              // R
+  __shared__ float sc[256];
+  __shared__ float red[4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row = blockIdx.x / a.H;
+  const int64_t qat = (int64_t)blockIdx.x * a.R;
+  const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
+  const int n = min(a.ctx[row], a.NB * a.BS);
+  const int lo = a.window > 0 ? max(0, n - a.window) : 0;
+  for (int c = tid; c < a.R; c += 256) q[c] = Elem<T>::ld(a.q, qat + c);
+  auto key_at = [&](int t) -> int64_t {
+    const int p = page_of(a, t);
+    int page = a.table[(int64_t)seq * a.NB + p];
+    if (page < 0 || page >= a.num_pages) page = 0;
+    return ((int64_t)page * a.BS + (t - p * a.BS)) * a.R;
+  };
+  constexpr int kCols = 16;                // columns per thread: R <= 4096
+  float o[kCols];
+#pragma unroll
+  for (int i = 0; i < kCols; ++i) o[i] = 0.f;
+  float m = -INFINITY, l = 0.f;
+  for (int c0 = lo; c0 < n; c0 += 256) {
+    const int cnt = min(256, n - c0);
+    __syncthreads();                       // q is there; the last chunk's scores are used up
+    for (int j = wave; j < cnt; j += 4) {
+      const int64_t at = key_at(c0 + j);
+      float acc = 0.f;
+      for (int c = lane; c < a.R; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
+      acc = wave_sum(acc);
+      if (lane == 0) sc[j] = acc * a.scale;
+    }
+    __syncthreads();
+    float mx = tid < cnt ? sc[tid] : -INFINITY;
+    mx = wave_max(mx);
+    if (lane == 0) red[wave] = mx;
+    __syncthreads();
+    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    const float mn = fmaxf(m, mx);
+    const float f = expf(m - mn);
+    __syncthreads();
+    const float p = tid < cnt ? expf(sc[tid] - mn) : 0.f;
+    sc[tid] = p;
+    const float s = wave_sum(p);
+    if (lane == 0) red[wave] = s;
+    __syncthreads();
+    l = l * f + red[0] + red[1] + red[2] + red[3];
+    m = mn;
+#pragma unroll
+    for (int i = 0; i < kCols; ++i) o[i] *= f;
+    for (int j = 0; j < cnt; ++j) {
+      const int64_t at = key_at(c0 + j);
+      const float pj = sc[j];
+#pragma unroll
+      for (int i = 0; i < kCols; ++i) {
+        const int c = tid + i * 256;
+        if (c < a.R) o[i] = fmaf(pj, Elem<T>::ld(a.cache, at + c), o[i]);
+      }
+    }
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+  for (int i = 0; i < kCols; ++i) {
+    const int c = tid + i * 256;
+    if (c < a.R) Elem<T>::st(a.out, qat + c, o[i] * inv);
+  }
+}
+
+// ------------------------------------------------------------------ runs of prompt tokens
+struct TilesArgs {
+  const uint16_t* q;      // token rows of q_st elements, head h at h * D
+  const uint16_t* k;      // key rows of kv_st elements, head h at h * D
+  const uint16_t* v;      // value rows of kv_st elements, head h at h * V
+  uint16_t* out;          // token rows of H * V elements
+  const int32_t* tiles;   // (T, 4): first query row, queries, first key row of the run, position
+                          // of the first query counted from that key
+  int T, H, D, V, window;
+  int64_t q_rows, k_rows, q_st, kv_st;
+  float scale;
+};
+
+constexpr int kTileQ = 128;   // queries per workgroup
+
+// A wave owns 16 * kQT queries of one head at a time and walks only the keys those queries see.
+template <int DKS, int VCB, int kQT>
+__global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
+  const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
+  const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
+  // host-made descriptors: rows outside the buffers are not touched
+  if (q0 < 0 || kb < 0 || rel < 0 || q0 + nq > a.q_rows || kb + rel + nq > a.k_rows) return;
+  const int nks = a.D / 32;
+  const float sc = a.scale * 1.44269504088896f;
+  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + h * a.D + g * 8;
+  const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + h * a.V;
+  for (int w0 = wave * 16 * kQT; w0 < nq; w0 += 64 * kQT) {
+    const int hi = rel + min(w0 + 16 * kQT, nq) - 1;            // last key any query here sees
+    const int lo = a.window > 0 ? max(0, rel + w0 - a.window + 1) : 0;
+
+    u32x4 qf[kQT][DKS];
+    int qpos[kQT];
+  #pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      const int qi = min(w0 + t * 16 + l16, nq - 1);
+      qpos[t] = rel + qi;
+      const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + h * a.D + g * 8;
+  #pragma unroll
+      for (int ks = 0; ks < DKS; ++ks)
+        qf[t][ks] = ks < nks ? *(const u32x4*)(q + ks * 32) : u32x4{0u, 0u, 0u, 0u};
+    }
+    f32x4 o[kQT][VCB * 8];
+    float m[kQT], l[kQT];
+  #pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      m[t] = -INFINITY;
+      l[t] = 0.f;
+  #pragma unroll
+      for (int i = 0; i < VCB * 8; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+
+    for (int k0 = lo; k0 <= hi; k0 += 32) {
+      f32x4 s[kQT][2];
+  #pragma unroll
+      for (int tt = 0; tt < 2; ++tt) {
+        const uint16_t* kr = kbase + (int64_t)min(k0 + tt * 16 + l16, hi) * a.kv_st;
+        u32x4 kf[DKS];
+  #pragma unroll
+        for (int ks = 0; ks < DKS; ++ks)
+          if (ks < nks) kf[ks] = *(const u32x4*)(kr + ks * 32);
+  #pragma unroll
+        for (int t = 0; t < kQT; ++t) {
+          f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  #pragma unroll
+          for (int ks = 0; ks < DKS; ++ks)
+            if (ks < nks) acc = mfma_bf16(kf[ks], qf[t][ks], acc);
+          s[t][tt] = acc;
+        }
+      }
+      // every query of the wave sees all 32 keys: no masks
+      const bool inner = k0 + 31 <= rel + w0 &&
+                         (a.window <= 0 || k0 > rel + w0 + 16 * kQT - 1 - a.window);
+      u32x4 pf[kQT];
+  #pragma unroll
+      for (int t = 0; t < kQT; ++t) {
+        float p[8], mx = -INFINITY;
+  #pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          p[i] = s[t][i >> 2][i & 3] * sc;
+          if (!inner) {
+            const int back = qpos[t] - (k0 + step_key(g, i));
+            if (back < 0 || (a.window > 0 && back >= a.window)) p[i] = -INFINITY;
+          }
+          mx = fmaxf(mx, p[i]);
+        }
+        mx = fmaxf(mx, lane_xor16(mx));
+        mx = fmaxf(mx, lane_xor32(mx));
+        const float mn = fmaxf(m[t], mx);
+        const float ms = mn == -INFINITY ? 0.f : mn;   // a query whose window starts later
+        const float f = __builtin_amdgcn_exp2f(m[t] - ms);
+        float sum = 0.f;
+  #pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          p[i] = __builtin_amdgcn_exp2f(p[i] - ms);
+          sum += p[i];
+        }
+        l[t] = l[t] * f + sum;
+        m[t] = mn;
+        if (__any(f != 1.f)) {
+  #pragma unroll
+          for (int i = 0; i < VCB * 8; ++i) o[t][i] *= f;
+        }
+        pf[t] = u32x4{pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                      pack_bf16(p[6], p[7])};
+      }
+  #pragma unroll
+      for (int cb = 0; cb < VCB; ++cb) {
+        const int col = cb * 128 + l16 * 8;
+        const uint16_t* vc = vbase + (col < a.V ? col : 0);
+        u32x4 v[8];
+  #pragma unroll
+        for (int i = 0; i < 8; ++i)
+          v[i] = *(const u32x4*)(vc + (int64_t)min(k0 + step_key(g, i), hi) * a.kv_st);
+  #pragma unroll
+        for (int c = 0; c < 8; ++c) {
+          const u32x4 vf = column_of(v, c);
+  #pragma unroll
+          for (int t = 0; t < kQT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
+        }
+      }
+    }
+  #pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      float lt = l[t];
+      lt += lane_xor16(lt);
+      lt += lane_xor32(lt);
+      const float inv = lt > 0.f ? 1.f / lt : 0.f;
+      const int qi = w0 + t * 16 + l16;
+      if (qi >= nq) continue;
+      uint16_t* out = a.out + ((int64_t)(q0 + qi) * a.H + h) * a.V;
+  #pragma unroll
+      for (int cb = 0; cb < VCB; ++cb)
+  #pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = cb * 128 + (4 * g + i) * 8;
+          if (col < a.V) {
+            float r[8];
+  #pragma unroll
+            for (int c = 0; c < 8; ++c) r[c] = o[t][cb * 8 + c][i] * inv;
+            Vec8<BF16>::st(out, col, r);
+          }
+        }
+    }
+  }
+}
+
+bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
+
+constexpr int kMaxLdsPages = 4096;
+
+int rows_hw(int H) {
+  const int tiles = (H + 15) / 16;
+  return tiles >= 4 ? 4 : (tiles >= 2 ? 2 : 1);
+}
+
+// Key ranges per token: enough workgroups to cover the chip, at least two 32-key steps per wave.
+int rows_splits(int n, int H, int window, int NB, int BS) {
+  const int hw = rows_hw(H), kw = 4 / hw;
+  const int groups = n * ((H + 16 * hw - 1) / (16 * hw));
+  int64_t keys = (int64_t)NB * BS;
+  if (window > 0 && window < keys) keys = window;
+  const int steps = (int)((keys + 31) / 32);
+  int s = 512 / (groups > 0 ? groups : 1);
+  s = s < steps / (2 * kw) ? s : steps / (2 * kw);
+  s = s < 32 ? s : 32;
+  return s < 1 ? 1 : s;
+}
+
+template <int NCB> int launch_latent_rows(RowsArgs a, hipStream_t st) {
+  const int kw = 4 / a.hw;
+  const size_t merge = kw > 1 ? sizeof(float) * (size_t)(kw - 1) * a.hw * (16 * (a.R + 4) + 32) : 0;
+  const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + merge;
+  if (smem > 64 * 1024 &&
+      hipFuncSetAttribute((const void*)latent_rows_kernel<NCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                          (int)smem) != hipSuccess) {
+    zp_set_error("latent_rows_attention: cannot reserve %zu bytes of LDS", smem);
+    return ZP_EHIP;
+  }
+  const int hgroups = (a.H + 16 * a.hw - 1) / (16 * a.hw);
+  hipLaunchKernelGGL((latent_rows_kernel<NCB>), dim3((unsigned)a.n * hgroups * a.splits), dim3(256), smem, st, a);
+  ZP_LAUNCH_CHECK();
+  if (a.splits > 1) {
+    hipLaunchKernelGGL(latent_rows_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
+    ZP_LAUNCH_CHECK();
+  }
+  return ZP_OK;
+}
+
+}  // namespace
+
+#define ZP_MODEL_DTYPE(name)                                       \
+  if (dtype != ZP_BF16 && dtype != ZP_F32) {                       \
+    zp_set_error(name ": bfloat16 and float32 only");              \
+    return ZP_EUNSUPPORTED;                                        \
+  }
+
+extern "C" int zp_latent_norm_store(const void* in, const float* q_weight, const float* c_weight,
+                                    void* q_out, void* c_out, void* cache, const int32_t* slots,
+                                    int32_t n, int32_t q_width, int32_t c_width, int32_t q_norm,
+                                    int32_t c_norm, int64_t num_slots, float eps, int32_t dtype,
+                                    void* stream) {
+  ZP_REQUIRE(n >= 0 && q_width > 0 && c_width > 0 && q_norm > 0 && q_norm <= q_width && c_norm > 0 &&
+                 c_norm <= c_width, "latent_norm_store: bad dims");
+  ZP_MODEL_DTYPE("latent_norm_store");
+  if (q_width % 8 || c_width % 8 || q_width > 512 * kNormPieces || c_width > 512 * kNormPieces) {
+    zp_set_error("latent_norm_store: ranks %d, %d unsupported (multiples of 8, <= %d)", q_width, c_width,
+                 512 * kNormPieces);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(in && q_weight && c_weight && q_out && cache && slots, "latent_norm_store: null pointer");
+  ZP_REQUIRE(aligned16(in) && aligned16(q_weight) && aligned16(c_weight) && aligned16(q_out) &&
+                 aligned16(c_out) && aligned16(cache), "latent_norm_store: tensors must be 16-byte aligned");
+  NormStoreArgs a = {in, q_weight, c_weight, q_out, c_out, cache, slots, n, q_width, c_width, q_norm,
+                     c_norm, num_slots, eps};
+  const unsigned grid = (unsigned)((2 * (int64_t)n + 3) / 4);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == ZP_BF16) hipLaunchKernelGGL((latent_norm_store_kernel<BF16>), dim3(grid), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((latent_norm_store_kernel<F32>), dim3(grid), dim3(256), 0, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n,
+                              int32_t row_bytes, int64_t num_rows, void* stream) {
+  ZP_REQUIRE(n >= 0 && row_bytes > 0 && row_bytes % 16 == 0 && num_rows > 0, "gather_rows: bad dims");
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(src && rows && out && aligned16(src) && aligned16(out), "gather_rows: null or unaligned pointer");
+  const int pieces = row_bytes / 16;
+  const int64_t total = (int64_t)n * pieces;
+  hipLaunchKernelGGL(gather_rows_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0,
+                     (hipStream_t)stream, (const char*)src, rows, (char*)out, total, pieces, num_rows);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_headwise_linear(const void* in, const void* w, void* out, int32_t n, int32_t H,
+                                  int32_t K, int32_t M, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && K > 0 && M > 0, "headwise_linear: bad dims");
+  ZP_MODEL_DTYPE("headwise_linear");
+  if (K % 32 != 0 || M % 16 != 0 || H > 65535) {
+    zp_set_error("headwise_linear: K %d, M %d unsupported (K multiple of 32, M multiple of 16)", K, M);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(in && w && out && aligned16(in) && aligned16(w) && aligned16(out),
+             "headwise_linear: null or unaligned pointer");
+  HeadArgs a = {in, w, out, n, H, K, M};
+  const dim3 grid((M + 63) / 64, H, (n + 16 * kTokTiles - 1) / (16 * kTokTiles));
+  ZP_REQUIRE(grid.z <= 65535, "headwise_linear: too many tokens");
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == ZP_BF16) hipLaunchKernelGGL((headwise_kernel<BF16>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((headwise_kernel<F32>), grid, dim3(256), 0, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int64_t zp_latent_rows_workspace(int32_t n, int32_t H, int32_t R, int32_t window,
+                                            int32_t NB, int32_t BS, int32_t dtype) {
+  if (n < 0 || H <= 0 || R <= 0 || NB <= 0 || BS <= 0) return -1;
+  if (dtype != ZP_BF16 || R > 512) return 0;
+  const int s = rows_splits(n, H, window, NB, BS);
+  return s == 1 ? 0 : (int64_t)n * H * s * (R + 2) * 4;
+}
+
+extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const int32_t* table,
+                                        const int32_t* context_lens, const int32_t* table_rows,
+                                        void* out, int32_t n, int32_t H, int32_t R, int32_t BS,
+                                        int32_t B, int32_t NB, int32_t num_pages, int32_t window,
+                                        float scale, int32_t dtype, void* workspace,
+                                        int64_t workspace_bytes, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && R > 0 && BS > 0 && B > 0 && NB > 0 && num_pages > 0 && window >= 0,
+             "latent_rows_attention: bad dims");
+  ZP_MODEL_DTYPE("latent_rows_attention");
+  if (R % 32 != 0 || R > 4096) {
+    zp_set_error("latent_rows_attention: latent size %d unsupported (multiple of 32, <= 4096)", R);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(q && cache && table && context_lens && out, "latent_rows_attention: null pointer");
+  ZP_REQUIRE(table_rows || n <= B, "latent_rows_attention: more tokens than table rows");
+  ZP_REQUIRE(aligned16(q) && aligned16(cache) && aligned16(out) && aligned16(workspace),
+             "latent_rows_attention: tensors must be 16-byte aligned");
+  RowsArgs a = {};
+  a.q = q; a.cache = cache; a.table = table; a.ctx = context_lens; a.seq = table_rows; a.out = out;
+  a.part = (float*)workspace; a.n = n; a.H = H; a.R = R; a.BS = BS; a.B = B; a.NB = NB;
+  a.num_pages = num_pages; a.window = window; a.scale = scale; a.bs_shift = -1;
+  if ((BS & (BS - 1)) == 0)
+    for (a.bs_shift = 0; (1 << a.bs_shift) < BS; ++a.bs_shift) {}
+  int64_t pages = NB;
+  if (window > 0 && (window - 1) / BS + 2 < pages) pages = (window - 1) / BS + 2;
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == ZP_F32 || R > 512 || pages > kMaxLdsPages) {
+    const size_t smem = sizeof(float) * R;
+    if (dtype == ZP_BF16)
+      hipLaunchKernelGGL((latent_plain_kernel<BF16>), dim3((unsigned)n * H), dim3(256), smem, st, a);
+    else
+      hipLaunchKernelGGL((latent_plain_kernel<F32>), dim3((unsigned)n * H), dim3(256), smem, st, a);
+    ZP_LAUNCH_CHECK();
+    return ZP_OK;
+  }
+  a.hw = rows_hw(H);
+  a.lds_pages = (int)pages;
+  a.splits = rows_splits(n, H, window, NB, BS);
+  ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_latent_rows_workspace(n, H, R, window, NB, BS, dtype)),
+             "latent_rows_attention: workspace too small");
+  switch ((R + 127) / 128) {
+    case 1: return launch_latent_rows<1>(a, st);
+    case 2: return launch_latent_rows<2>(a, st);
+    case 3: return launch_latent_rows<3>(a, st);
+    default: return launch_latent_rows<4>(a, st);
+  }
+}
+
+extern "C" int zp_latent_tiles_attention(const void* q, const void* k, const void* v, void* out,
+                                         const int32_t* tiles, int32_t T, int32_t H, int32_t D,
+                                         int32_t V, int32_t window, int64_t q_rows, int64_t k_rows,
+                                         int64_t q_stride, int64_t kv_stride, float scale,
+                                         int32_t dtype, void* stream) {
+  ZP_REQUIRE(T >= 0 && H > 0 && D > 0 && V > 0 && window >= 0, "latent_tiles_attention: bad dims");
+  if (dtype != ZP_BF16 || D % 32 != 0 || D > 256 || V % 8 != 0 || V > 256) {
+    zp_set_error("latent_tiles_attention: bfloat16, D %d (multiple of 32, <= 256), V %d (multiple of 8, <= 256)", D, V);
+    return ZP_EUNSUPPORTED;
+  }
+  if (T == 0) return ZP_OK;
+  ZP_REQUIRE(q && k && v && out && tiles, "latent_tiles_attention: null pointer");
+  ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && q_stride % 8 == 0 &&
+                 kv_stride % 8 == 0 && q_stride >= (int64_t)H * D && (int64_t)T * H < (1ll << 31),
+             "latent_tiles_attention: unaligned rows or too many tiles");
+  TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (uint16_t*)out, tiles, T, H, D, V,
+                 window, q_rows, k_rows, q_stride, kv_stride, scale};
+  const dim3 grid((unsigned)T * H);
+  hipStream_t st = (hipStream_t)stream;
+#define ZP_TILES(DK, VC, QT) \
+  hipLaunchKernelGGL((latent_tiles_kernel<DK, VC, QT>), grid, dim3(256), 0, st, a)
+  const int dk = D / 32;
+  if (V <= 128) {
+    if (dk <= 2) ZP_TILES(2, 1, 2);
+    else if (dk <= 4) ZP_TILES(4, 1, 2);
+    else if (dk <= 6) ZP_TILES(6, 1, 2);
+    else ZP_TILES(8, 1, 2);
+  } else {
+    if (dk <= 4) ZP_TILES(4, 2, 1);
+    else ZP_TILES(8, 2, 1);
+  }
+#undef ZP_TILES
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}

@@ -1,0 +1,41 @@
+// Device helpers shared by the model-side kernels that exist in bfloat16 and in float32.
+#pragma once
+#include "common.h"
+#include "../../include/zipage_models.h"
+
+typedef uint32_t zp_u32x4 __attribute__((ext_vector_type(4)));
+typedef float zp_f32x4 __attribute__((ext_vector_type(4)));
+
+// Eight consecutive elements as fp32, 16-byte accesses; `i` is a multiple of 8.
+template <typename T> struct Vec8;
+template <> struct Vec8<BF16> {
+  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) {
+    const zp_u32x4 v = *(const zp_u32x4*)((const uint16_t*)p + i);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      o[2 * k] = __uint_as_float(v[k] << 16);
+      o[2 * k + 1] = __uint_as_float(v[k] & 0xffff0000u);
+    }
+  }
+  __device__ static __forceinline__ void st(void* p, int64_t i, const float* o) {
+    zp_u32x4 v;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const zp_f32x2 f = {o[2 * k], o[2 * k + 1]};
+      v[k] = __builtin_bit_cast(uint32_t, __builtin_convertvector(f, zp_bf16x2));
+    }
+    *(zp_u32x4*)((uint16_t*)p + i) = v;
+  }
+};
+template <> struct Vec8<F32> {
+  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) {
+    const zp_f32x4 a = *(const zp_f32x4*)((const float*)p + i);
+    const zp_f32x4 b = *(const zp_f32x4*)((const float*)p + i + 4);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) { o[k] = a[k]; o[k + 4] = b[k]; }
+  }
+  __device__ static __forceinline__ void st(void* p, int64_t i, const float* o) {
+    *(zp_f32x4*)((float*)p + i) = zp_f32x4{o[0], o[1], o[2], o[3]};
+    *(zp_f32x4*)((float*)p + i + 4) = zp_f32x4{o[4], o[5], o[6], o[7]};
+  }
+};

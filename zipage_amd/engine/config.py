@@ -1,17 +1,23 @@
 """Engine switches (zipage/config.py) without the Hugging Face lookup: the model shape is
-given directly because weights are random-initialised."""
+given directly (or read from a model folder by `registry.read_shape`)."""
 from __future__ import annotations
 
 from dataclasses import dataclass, field
+from typing import Any
+
+import torch
 
 from zipage_amd.compress import CompressConfig
 
-from .qwen3 import QWEN3_8B, Qwen3Shape
+from .qwen3 import QWEN3_8B
+from .registry import arch_for_shape
 
 
 @dataclass
 class EngineConfig:
-    shape: Qwen3Shape = QWEN3_8B
+    shape: Any = QWEN3_8B               # the shape class picks the model (engine/registry.py)
+    model_folder: str | None = None     # weights; None: drawn from the seed
+    dtype: torch.dtype = torch.bfloat16
     max_num_batched_tokens: int = 32768
     max_num_seqs: int = 512
     max_concurrency: int = 256          # query-cache rows = sequences resident at once
@@ -34,3 +40,14 @@ class EngineConfig:
         assert self.max_cache_blocks_per_seq >= 1
         self.compress.budget_blocks = self.max_cache_blocks_per_seq
         self.compress.query_cache_len = self.query_cache_len
+        self.arch = arch_for_shape(self.shape)
+        if getattr(self.shape, "max_positions", None) is not None:    # learned positions end there
+            self.max_model_len = min(self.max_model_len, self.shape.max_positions)
+
+    @property
+    def table_width(self) -> int:
+        """Pages a sequence's table holds in the steady state: the budget and the page being
+        written, or, without compression, the longest sequence."""
+        if self.arch.model.compressible:
+            return self.max_cache_blocks_per_seq + 1
+        return -(-self.max_model_len // self.kvcache_block_size)

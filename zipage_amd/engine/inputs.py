@@ -1,9 +1,11 @@
 """Host-side construction of a step's index tensors (numpy only, no device needed)."""
 from __future__ import annotations
 
+from dataclasses import dataclass, field
+
 import numpy as np
 
-from .sequence import Sequence
+from .sequence import Portion, Sequence
 
 HEADER_ROWS = 5   # query row, position, flat K/V slot, context length, token-log column
 
@@ -89,3 +91,82 @@ def encode_compress_tables(seqs: list[Sequence]) -> list[list[int]]:
     width = max(len(s.block_table) for s in seqs)
     return [s.block_table[:-1] + [-s.block_table[-1] - 2] + [-1] * (width - len(s.block_table))
             for s in seqs]
+
+
+# ---------------------------------------------------------------- steps of portions
+RUN_TILE = 128    # queries per entry of a run plan
+
+
+@dataclass
+class Runs:
+    """The multi-token portions of a step as the run attention reads them, for one window."""
+    tiles: np.ndarray             # (T, 4): first query row, queries, first key row, rel. position
+    key_slots: np.ndarray | None  # cache rows to gather as keys; None: the step's own tokens
+
+
+@dataclass
+class PortionPlan:
+    ids: np.ndarray               # token ids; 0 where the id is still on the device
+    rows: np.ndarray              # query row whose last sampled token is the id, or -1
+    positions: np.ndarray
+    slots: np.ndarray
+    context_lens: np.ndarray      # of the tokens attended one by one; they come first
+    table_rows: np.ndarray
+    tables: np.ndarray            # (sequences, width), -1 where nothing is held
+    first_row: list[int]          # token row where each portion starts, in the order given
+    runs: dict = field(default_factory=dict)
+
+
+def plan_runs(portions: list[Portion], block_size: int, window: int | None) -> Runs:
+    """Key rows and query tiles of `portions`, whose tokens follow one another in the query rows.  A
+    run's keys start `window` - 1 tokens before its first token (at 0 without a window)."""
+    tiles, slots, q, k = [], [], 0, 0
+    own = True
+    for p in portions:
+        k_first = 0 if window is None else max(0, p.start - window + 1)
+        own &= k_first == p.start
+        for off in range(0, p.count, RUN_TILE):
+            tiles.append((q + off, min(RUN_TILE, p.count - off), k, p.start - k_first + off))
+        t = np.arange(k_first, p.start + p.count)
+        table = np.asarray(p.seq.block_table, dtype=np.int64)
+        slots.append(table[t // block_size] * block_size + t % block_size)
+        q += p.count
+        k += len(t)
+    return Runs(np.asarray(tiles, dtype=np.int32),
+                None if own else np.concatenate(slots).astype(np.int32))
+
+
+def plan_portions(portions: list[Portion], block_size: int, windows, run_min: int | None) -> PortionPlan:
+    """All inputs of a step that holds portions of any length.  Portions shorter than `run_min`
+    (None: all) are attended token by token and come first."""
+    short = [i for i, p in enumerate(portions) if run_min is None or p.count < run_min]
+    long = [i for i, p in enumerate(portions) if not (run_min is None or p.count < run_min)]
+    first_row = [0] * len(portions)
+    ids, rows, pos, slots, ctx, trows = [], [], [], [], [], []
+    width = max(len(p.seq.block_table) for p in portions)
+    tables = np.full((len(portions), width), -1, dtype=np.int32)
+    n = 0
+    for i in short + long:
+        p = portions[i]
+        first_row[i] = n
+        n += p.count
+        tables[i, :len(p.seq.block_table)] = p.seq.block_table
+        known = p.seq.token_ids[p.start:p.start + p.count]
+        missing = p.count - len(known)      # a sampled token that never came to the host
+        assert missing == 0 or p.count == 1
+        ids.extend(known + [0] * missing)
+        rows.extend([-1] * len(known) + [p.seq.query_id] * missing)
+        t = np.arange(p.start, p.start + p.count)
+        pos.append(t)
+        slots.append(tables[i][t // block_size].astype(np.int64) * block_size + t % block_size)
+    for i in short:
+        p = portions[i]
+        ctx.append(np.arange(p.start + 1, p.start + p.count + 1))
+        trows.append(np.full(p.count, i))
+    cat = lambda a: np.concatenate(a).astype(np.int32) if a else np.zeros(0, np.int32)
+    plan = PortionPlan(np.asarray(ids, np.int32), np.asarray(rows, np.int32), cat(pos), cat(slots),
+                       cat(ctx), cat(trows), tables, first_row)
+    if long:
+        for w in windows:
+            plan.runs[w] = plan_runs([portions[i] for i in long], block_size, w)
+    return plan

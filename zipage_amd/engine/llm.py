@@ -17,7 +17,7 @@ import torch
 from .config import EngineConfig
 from .model_runner import ModelRunner
 from .scheduler import Scheduler
-from .sequence import SamplingParams, Sequence
+from .sequence import Portion, SamplingParams, Sequence
 
 
 class ZipageEngine:
@@ -34,9 +34,21 @@ class ZipageEngine:
     def add_request(self, token_ids: list[int], params: SamplingParams | None = None) -> Sequence:
         seq = Sequence(token_ids, params or SamplingParams(), self.cfg.kvcache_block_size)
         cfg = self.cfg
-        if not 0 < len(seq) <= min(cfg.max_num_batched_tokens, cfg.max_model_len):
-            raise ValueError(f"prompt of {len(seq)} tokens: need 1..{min(cfg.max_num_batched_tokens, cfg.max_model_len)}")
-        if seq.num_blocks > cfg.num_kvcache_blocks:
+        longest = cfg.max_model_len             # a prompt that runs in portions may exceed a step
+        if not self.runner.model.portions:
+            longest = min(cfg.max_num_batched_tokens, longest)
+        if not 0 < len(seq) <= longest:
+            raise ValueError(f"prompt of {len(seq)} tokens: need 1..{longest}")
+        if self.runner.model.portions:
+            if len(seq) + seq.params.max_tokens > cfg.max_model_len + 1:   # the last token drawn is not run
+                raise ValueError(f"{len(seq)} prompt tokens and {seq.params.max_tokens} more: the model has "
+                                 f"{cfg.max_model_len} positions")
+            if not all(0 <= t < self.runner.model.vocab for t in seq.token_ids):
+                raise ValueError("a token id outside the vocabulary")
+            need = self.scheduler.peak_pages(seq, self.runner.model.lookback)
+            if need > cfg.num_kvcache_blocks:
+                raise ValueError(f"the request needs {need} pages, the pool has {cfg.num_kvcache_blocks}")
+        elif seq.num_blocks > cfg.num_kvcache_blocks:
             raise ValueError(f"prompt needs {seq.num_blocks} pages, the pool has {cfg.num_kvcache_blocks}")
         self.runner.reserve_token_log(seq.params.max_tokens + 1)
         self.scheduler.add(seq)
@@ -58,6 +70,8 @@ class ZipageEngine:
 
     def step(self) -> int:
         """One scheduler round; returns +prefilled tokens or -decoded tokens."""
+        if self.runner.model.portions:
+            return self.portion_step()
         seqs, is_prefill = self.scheduler.schedule()
         if not seqs:
             return 0
@@ -77,8 +91,71 @@ class ZipageEngine:
         self.stats["decode_steps"] += 1
         return -len(seqs)
 
+    def portion_step(self) -> int:
+        """A round of a model whose steps hold portions of prompts beside decoded tokens."""
+        lookback = self.runner.model.lookback
+        portions = self.scheduler.schedule_portions(lookback)
+        if not portions:
+            return 0
+        decoded = sum(p.start >= p.seq.num_prompt_tokens for p in portions)
+        prompt = sum(p.count for p in portions if p.start < p.seq.num_prompt_tokens)
+        if decoded and self.stats["decode_steps"] == 0:
+            self._t_decode0 = perf_counter()
+        tok = self.runner.run_portions(portions)
+        for p in portions:
+            self.scheduler.pool.computed(p.seq, p.start + p.count, lookback)
+        if tok is not None:
+            self._finish_step([p.seq for p in portions if p.ends], tok)
+        self.stats["prefill_tokens"] += prompt
+        self.stats["decode_tokens"] += decoded
+        self.stats["decode_steps"] += decoded > 0
+        return prompt or -decoded
+
+    # ------------------------------------------------------------------ given tokens
+    def open_request(self) -> Sequence:
+        """A sequence whose tokens are all given by `feed`."""
+        if not self.runner.model.portions:
+            raise NotImplementedError("this model's steps hold whole prompts or decoded tokens only")
+        if not self.scheduler.free_rows:
+            raise RuntimeError("no free sequence slot")
+        seq = Sequence([], SamplingParams(), self.cfg.kvcache_block_size)
+        seq.query_id = self.scheduler.free_rows.popleft()
+        return seq
+
+    def feed(self, entries: list[tuple[Sequence, list[int], list[int]]]) -> torch.Tensor | None:
+        """One step over the next tokens of each sequence (all of them one batch): (sequence, tokens,
+        places among them whose logits are wanted).  Returns fp32 logits (wanted, vocab)."""
+        r, pool = self.runner, self.scheduler.pool
+        if len({id(s) for s, _, _ in entries}) != len(entries):
+            raise ValueError("a sequence may appear once in a step")
+        for seq, tokens, want in entries:
+            if not tokens or len(seq) + len(tokens) > self.cfg.max_model_len:
+                raise ValueError(f"{len(tokens)} tokens after {len(seq)}: need 1..{self.cfg.max_model_len - len(seq)}")
+            if not all(0 <= t < r.model.vocab for t in tokens):
+                raise ValueError("a token id outside the vocabulary")
+            if not all(0 <= k < len(tokens) for k in want):
+                raise ValueError("a wanted place outside the portion")
+        portions = []
+        for seq, tokens, _ in entries:
+            seq.token_ids.extend(tokens)
+            seq.num_tokens += len(tokens)
+            seq.num_prompt_tokens = seq.num_tokens
+            pool.grow(seq, seq.num_tokens)
+            portions.append(Portion(seq, seq.num_computed_tokens, len(tokens)))
+        logits = r.run_fed(portions, [w for _, _, w in entries])
+        for p in portions:
+            pool.computed(p.seq, p.start + p.count, r.model.lookback)
+        return logits
+
+    def close_request(self, seq: Sequence):
+        self.scheduler.pool.release(seq)
+        self.scheduler.free_rows.append(seq.query_id)
+        seq.finished = True
+
     def async_step(self) -> int:
         r = self.runner
+        if r.model.portions:                      # nothing to compress
+            return self.portion_step()
         if self._inflight is not None and self._inflight[0].query():
             ev, done = self._inflight
             r.run_stream.wait_event(ev)           # their next decode step reads the new pages
@@ -136,7 +213,7 @@ class ZipageEngine:
             if n > 0:
                 torch.cuda.synchronize(dev)       # prefill is timed on its own
                 self.stats["prefill_s"] += perf_counter() - t0
-            elif self.stats["decode_steps"] == 1 and n < 0:
+            elif self.stats["decode_steps"] == 1 and n < 0 and not self.runner.model.portions:
                 self._t_decode0 = t0
         torch.cuda.synchronize(dev)
         if self.stats["decode_steps"]:

@@ -17,9 +17,11 @@ import torch
 from zipage_amd.compress import StageTimer, compress_layers
 
 from .config import EngineConfig
-from .inputs import encode_compress_tables, pack_decode, packed_words, query_slot_mapping, unpack_views
-from .qwen3 import Qwen3, StepContext
-from .sequence import Sequence
+from .inputs import (Runs, encode_compress_tables, pack_decode, packed_words, plan_portions,
+                     query_slot_mapping, unpack_views)
+from .qwen3 import StepContext
+from .registry import build_model
+from .sequence import Portion, Sequence
 
 
 class _PinnedRing:
@@ -48,10 +50,9 @@ class ModelRunner:
     def __init__(self, cfg: EngineConfig, device="cuda:0"):
         self.cfg, self.device = cfg, torch.device(device)
         torch.cuda.set_device(self.device)
-        s = cfg.shape
         self.block_size = cfg.kvcache_block_size
-        self.table_width = cfg.max_cache_blocks_per_seq + 1
-        self.model = Qwen3(s, self.device, seed=cfg.seed)
+        self.table_width = cfg.table_width
+        self.model = build_model(cfg.shape, self.device, cfg.dtype, cfg.seed, cfg.model_folder)
         self.allocate_kv_cache()
         self.run_stream = torch.cuda.Stream(self.device)
         self.compress_stream = torch.cuda.Stream(self.device)
@@ -68,8 +69,12 @@ class ModelRunner:
 
     # ------------------------------------------------------------------ memory
     def allocate_kv_cache(self):
-        """model_runner.py:219-307, with the page count given by the configuration."""
+        """model_runner.py:219-307, with the page count given by the configuration.  A model that is
+        not compressed keeps its own kind of pages and no window queries."""
         cfg, s = self.cfg, self.cfg.shape
+        if not self.model.compressible:
+            self.model.allocate_caches(cfg.num_kvcache_blocks, self.block_size)
+            return
         dt = self.model.dtype
         self.kv_cache = torch.zeros(2, s.layers, cfg.num_kvcache_blocks, self.block_size, s.kv_heads,
                                     s.head_dim, dtype=dt, device=self.device)
@@ -142,7 +147,7 @@ class ModelRunner:
     def _decode_hidden(self, buf: torch.Tensor, Bp: int, TW: int) -> torch.Tensor:
         """The part of the step a graph replays: embedding to final norm."""
         head, tables, triples = unpack_views(buf, Bp, TW)
-        ctx = StepContext(False, head[2], triples, head[3], tables)
+        ctx = StepContext(False, head[2], triples, head[3], tables, runs={})
         return self.model.forward(self.last_token[head[0].long()], head[1].long(), ctx)
 
     def _decode_tail(self, buf: torch.Tensor, Bp: int, TW: int, hidden: torch.Tensor,
@@ -176,7 +181,15 @@ class ModelRunner:
         """One decode step for `seqs`; returns the device tensor of the sampled ids."""
         B = len(seqs)
         temps = [s.params.temperature for s in seqs]
-        graph = self.cfg.use_graph and not any(temps)
+        with torch.cuda.stream(self.run_stream):
+            buf, Bp, TW, hidden = self._run_decode_hidden(seqs, self.cfg.use_graph and not any(temps))
+            t = torch.tensor(temps + [0.0] * (Bp - B), device=self.device) if any(temps) else None
+            return self._decode_tail(buf, Bp, TW, hidden, t)[:B]
+
+    def _run_decode_hidden(self, seqs: list[Sequence], graph: bool):
+        """The last token of every sequence through the model, on the current stream: the packed
+        inputs, their padded batch and table width, and the hidden rows."""
+        B = len(seqs)
         Bp = self._graph_batch(B)      # eager steps pad the same way, so both paths run the same kernels
         # a prompt longer than the table keeps its pages until its first compression
         TW = max(self.table_width, max(len(s.block_table) for s in seqs))
@@ -184,17 +197,101 @@ class ModelRunner:
         words = packed.shape[0]
         pinned, slot = self.ring.next()
         pinned[:words].numpy()[:] = packed
-        with torch.cuda.stream(self.run_stream):
-            t = torch.tensor(temps + [0.0] * (Bp - B), device=self.device) if any(temps) else None
-            if graph:
-                g, sbuf, hidden = self._graph(Bp, TW)
-                sbuf.copy_(pinned[:words], non_blocking=True)
-                self.ring.sent(slot, self.run_stream)
-                g.replay()
-                return self._decode_tail(sbuf, Bp, TW, hidden)[:B]
-            buf = pinned[:words].to(self.device, non_blocking=True)
+        if graph:
+            g, sbuf, hidden = self._graph(Bp, TW)
+            sbuf.copy_(pinned[:words], non_blocking=True)
             self.ring.sent(slot, self.run_stream)
-            return self._decode_tail(buf, Bp, TW, self._decode_hidden(buf, Bp, TW), t)[:B]
+            g.replay()
+            return sbuf, Bp, TW, hidden
+        buf = pinned[:words].to(self.device, non_blocking=True)
+        self.ring.sent(slot, self.run_stream)
+        return buf, Bp, TW, self._decode_hidden(buf, Bp, TW)
+
+    # ------------------------------------------------------------------ steps of portions
+    def prepare_portions(self, portions: list[Portion]):
+        """One packed buffer for a step of portions: (ids, positions, ctx, first row per portion)."""
+        m = self.model
+        plan = plan_portions(portions, self.block_size, m.windows, m.run_min)
+        parts = [plan.ids, plan.rows, plan.positions, plan.slots, plan.context_lens, plan.table_rows,
+                 plan.tables.reshape(-1)]
+        for r in plan.runs.values():
+            parts += [r.tiles.reshape(-1)] + ([] if r.key_slots is None else [r.key_slots])
+        host = torch.empty(sum(-(-len(a) // 4) * 4 for a in parts), dtype=torch.int32, pin_memory=True)
+        view, spans, at = host.numpy(), [], 0
+        for a in parts:
+            view[at:at + len(a)] = a
+            spans.append((at, at + len(a)))
+            at += -(-len(a) // 4) * 4
+        buf = host.to(self.device, non_blocking=True)
+        d = iter([buf[a:b] for a, b in spans])
+        ids, rows, pos, slots, ctx_lens, table_rows = (next(d) for _ in range(6))
+        tables = next(d).view(plan.tables.shape)
+        runs = {}
+        for w, r in plan.runs.items():
+            tiles = next(d).view(-1, 4)
+            runs[w] = Runs(tiles, None if r.key_slots is None else next(d))
+        ids = ids.long()
+        if (plan.rows >= 0).any():
+            ids = torch.where(rows >= 0, self.last_token[rows.clamp_min(0).long()], ids)
+        ctx = StepContext(False, slots, None, ctx_lens, tables, table_rows=table_rows, runs=runs)
+        return ids, pos, ctx, plan.first_row
+
+    @staticmethod
+    def _is_decode(portions: list[Portion]) -> bool:
+        return all(p.count == 1 and p.ends for p in portions)
+
+    def _hand_over(self, portions: list[Portion]):
+        """A decode step takes its token ids from `last_token`: put those there that were given
+        rather than sampled."""
+        given = [p for p in portions if p.start < p.seq.num_prompt_tokens]
+        if given:
+            t = lambda a: torch.tensor(a, pin_memory=True).to(self.device, non_blocking=True)
+            self.last_token.index_put_((t([p.seq.query_id for p in given]),),
+                                       t([p.seq.token_ids[p.start] for p in given]))
+
+    def _portions_hidden(self, portions: list[Portion], graph: bool):
+        """Hidden rows of a step and the row each portion starts at.  A step of single tokens that are
+        their sequences' last is a decode step and replays its graph."""
+        if self._is_decode(portions):
+            hidden = self._run_decode_hidden([p.seq for p in portions], graph)[3]
+            return hidden, list(range(len(portions)))
+        ids, pos, ctx, first = self.prepare_portions(portions)
+        return self.model.forward(ids, pos, ctx), first
+
+    @torch.inference_mode()
+    def run_portions(self, portions: list[Portion]) -> torch.Tensor | None:
+        """One step; samples the next token of every portion that ends its sequence and returns the
+        ids in that order (None without one)."""
+        if self._is_decode(portions):
+            with torch.cuda.stream(self.run_stream):
+                self._hand_over(portions)
+            return self.run_decode([p.seq for p in portions])
+        with torch.cuda.stream(self.run_stream):
+            hidden, first = self._portions_hidden(portions, False)
+            ends = [(f + p.count - 1, p.seq) for p, f in zip(portions, first) if p.ends]
+            if not ends:
+                return None
+            t = lambda a: torch.tensor(a, pin_memory=True).to(self.device, non_blocking=True)
+            temps = [s.params.temperature for _, s in ends]
+            tok = self._sample(self.model.compute_logits(hidden[t([r for r, _ in ends])]),
+                               t(temps) if any(temps) else None)
+            rows, cols = t([s.query_id for _, s in ends]), t([s.num_completion_tokens for _, s in ends])
+            self.last_token.index_put_((rows,), tok)
+            self.token_log.index_put_((rows, cols), tok.int())
+        return tok
+
+    @torch.inference_mode()
+    def run_fed(self, portions: list[Portion], want: list[list[int]]) -> torch.Tensor | None:
+        """One step whose tokens are all given: the fp32 logits at the wanted places of every
+        portion, in order; nothing is sampled."""
+        with torch.cuda.stream(self.run_stream):
+            if self._is_decode(portions):
+                self._hand_over(portions)
+            hidden, first = self._portions_hidden(portions, self.cfg.use_graph)
+            rows = [f + k for f, w in zip(first, want) for k in w]
+            if not rows:
+                return None
+            return self.model.compute_logits(hidden[torch.tensor(rows, device=self.device)]).float()
 
     # ------------------------------------------------------------------ HIP graph
     def _graph_batch(self, B: int) -> int:

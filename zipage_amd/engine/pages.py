@@ -28,6 +28,7 @@ class PagePool:
         self.page_tokens: list[list[int] | None] = [None] * num_pages
         self.by_hash: dict[int, int] = {}
         self.free: deque[int] = deque(range(num_pages))
+        self.reserved = 0                # pages promised to sequences that run in portions
         self.lock = threading.Lock()     # compression hand-back may run on a worker thread
 
     # ------------------------------------------------------------------ primitives
@@ -107,9 +108,80 @@ class PagePool:
 
     def release(self, seq: Sequence):
         for page in reversed(seq.block_table):
-            self._drop(page)
+            if page >= 0:
+                self._drop(page)
         seq.block_table.clear()
-        seq.num_cached_tokens = 0
+        seq.num_cached_tokens = seq.num_computed_tokens = seq.first_page = 0
+        seq.sealed.clear()
+        self.reserved -= seq.reserved_pages
+        seq.reserved_pages = 0
+
+    # ------------------------------------------------------------------ portions
+    # A sequence that runs in portions takes pages as its tokens arrive and gives leading pages
+    # back once every layer's window has passed them; its table keeps -1 there, so table entry
+    # t // page_size still belongs to token t.
+    def reserve(self, seq: Sequence, pages: int) -> bool:
+        """Promise the most pages the sequence will hold at once: a sequence admitted under this
+        rule never waits for a page."""
+        if self.reserved + pages > self.num_pages:
+            return False
+        self.reserved += pages
+        seq.reserved_pages = pages
+        return True
+
+    def share_prefix(self, seq: Sequence, lookback: int):
+        """Start the sequence behind the full prompt pages that are still cached, holding those of
+        them its next token can see.  At least the last token is left to run."""
+        if not self.enable_prefix_cache:
+            return
+        h, hits = -1, []
+        for i in range((len(seq.token_ids) - 1) // self.page_size):
+            toks = seq.block(i)
+            h = self.chain_hash(toks, h)
+            page = self.by_hash.get(h, -1)
+            if page == -1 or self.page_tokens[page] != toks or self.page_hash[page] != h:
+                break
+            hits.append((page, h, toks))
+        computed = len(hits) * self.page_size
+        first = max(0, computed - lookback + 1) // self.page_size
+        for i, (page, h, toks) in enumerate(hits):
+            seq.sealed.append(h)
+            if i < first:
+                seq.block_table.append(-1)
+                continue
+            if self.refcount[page] > 0:
+                self.refcount[page] += 1
+            else:
+                self._take(page)
+                self.page_hash[page], self.page_tokens[page] = h, toks
+            seq.block_table.append(page)
+        seq.num_computed_tokens, seq.first_page = computed, first
+
+    def grow(self, seq: Sequence, tokens: int):
+        """Pages for the first `tokens` tokens."""
+        while len(seq.block_table) * self.page_size < tokens:
+            if not self.free:
+                raise RuntimeError("the page pool is empty")
+            seq.block_table.append(self._take())
+
+    def computed(self, seq: Sequence, tokens: int, lookback: int):
+        """The first `tokens` tokens are in the cache: full prompt pages become shareable, pages
+        that no later token sees are given back."""
+        seq.num_computed_tokens = tokens
+        if self.enable_prefix_cache:
+            known = min(tokens, len(seq.token_ids))
+            for i in range(len(seq.sealed), known // self.page_size):
+                toks = seq.block(i)
+                h = self.chain_hash(toks, seq.sealed[-1] if seq.sealed else -1)
+                seq.sealed.append(h)
+                page = seq.block_table[i]
+                self.page_hash[page], self.page_tokens[page] = h, toks
+                self.by_hash[h] = page
+        first = max(0, tokens - lookback + 1) // self.page_size
+        for i in range(seq.first_page, min(first, len(seq.block_table))):
+            self._drop(seq.block_table[i])
+            seq.block_table[i] = -1
+        seq.first_page = max(seq.first_page, min(first, len(seq.block_table)))
 
     # ------------------------------------------------------------------ decode growth
     def wants_page(self, seq: Sequence) -> bool:

@@ -30,6 +30,13 @@ class Qwen3Shape:
     rope_theta: float = 1e6
     max_position: int = 40960
 
+    @classmethod
+    def from_config(cls, c: dict) -> "Qwen3Shape":
+        """From a Hugging Face style config.json."""
+        return cls(c["num_hidden_layers"], c["hidden_size"], c["num_attention_heads"], c["num_key_value_heads"],
+                   c["head_dim"], c["intermediate_size"], c["vocab_size"], c.get("rms_norm_eps", 1e-6),
+                   c.get("rope_theta", 1e6), c.get("max_position_embeddings", 40960))
+
 
 QWEN3_8B = Qwen3Shape(36, 4096, 32, 8, 128, 12288, 151936)
 QWEN3_0_6B = Qwen3Shape(28, 1024, 16, 8, 128, 3072, 151936)
@@ -46,11 +53,21 @@ class StepContext:
     block_tables: torch.Tensor | None = None        # (B, NB) int32, decode / cached prefill
     seq_lens_q: list[int] | None = None             # prefill: new tokens per sequence
     seq_lens_k: list[int] | None = None             # prefill: total tokens per sequence
+    # steps of portions: the first context_lens.numel() tokens are attended one by one, token i over
+    # row table_rows[i] of block_tables (None: i); the rest belong to runs, planned per window
+    table_rows: torch.Tensor | None = None          # (singles,) int32
+    runs: dict | None = None                        # window -> inputs.Runs
 
 
 class Qwen3:
+    # what the engine asks a model: its cache may be compressed; a step is whole prompts or decodes
+    compressible = True
+    portions = False
+
     def __init__(self, shape: Qwen3Shape, device, dtype=torch.bfloat16, seed: int = 0,
                  init_std: float = 0.02):
+        if dtype not in (torch.bfloat16, torch.float16):
+            raise ValueError(f"Qwen3's layer kernels are 16-bit, not {dtype}")
         self.shape, self.device, self.dtype = shape, torch.device(device), dtype
         s = shape
         g = torch.Generator(device=self.device).manual_seed(seed)

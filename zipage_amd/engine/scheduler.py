@@ -12,14 +12,14 @@ from collections import deque
 
 from .config import EngineConfig
 from .pages import PagePool
-from .sequence import Sequence
+from .sequence import Portion, Sequence
 
 
 class Scheduler:
     def __init__(self, cfg: EngineConfig):
         self.cfg = cfg
         self.pool = PagePool(cfg.num_kvcache_blocks, cfg.kvcache_block_size,
-                             cfg.max_cache_blocks_per_seq + 1, cfg.enable_prefix_cache)
+                             cfg.table_width, cfg.enable_prefix_cache)
         self.waiting: deque[Sequence] = deque()
         self.running: deque[Sequence] = deque()
         self.free_rows: deque[int] = deque(range(cfg.max_concurrency))
@@ -70,6 +70,44 @@ class Scheduler:
             self.running.extend(reversed(rejoin))
         self.running.extendleft(reversed(kept))
         return batch, False
+
+    # ------------------------------------------------------------------ schedule, in portions
+    def peak_pages(self, seq: Sequence, lookback: int) -> int:
+        """The most pages `seq` holds at once: its whole length, or the window before a step's first
+        token and the step's own tokens."""
+        cfg = self.cfg
+        total = min(seq.num_prompt_tokens + seq.params.max_tokens, cfg.max_model_len)
+        step = min(cfg.max_num_batched_tokens, seq.num_prompt_tokens)
+        size = cfg.kvcache_block_size
+        return min(-(-total // size), (lookback + step - 2) // size + 2)
+
+    def schedule_portions(self, lookback: int) -> list[Portion]:
+        """One batch of decoded tokens and portions of prompts: running sequences first, those that
+        decode before those still in their prompt, then new ones, up to max_num_batched_tokens."""
+        cfg = self.cfg
+        left, batch = cfg.max_num_batched_tokens, []
+
+        def run(seq: Sequence):
+            nonlocal left
+            n = min(seq.num_tokens - seq.num_computed_tokens, left)
+            self.pool.grow(seq, seq.num_computed_tokens + n)
+            batch.append(Portion(seq, seq.num_computed_tokens, n))
+            left -= n
+
+        for seq in sorted(self.running, key=lambda s: s.num_tokens - s.num_computed_tokens > 1):
+            if left == 0 or len(batch) == cfg.max_num_seqs:
+                break
+            run(seq)
+        while self.waiting and self.free_rows and left and len(batch) < cfg.max_num_seqs:
+            seq = self.waiting[0]
+            if not self.pool.reserve(seq, self.peak_pages(seq, lookback)):
+                break
+            self.waiting.popleft()
+            seq.query_id = self.free_rows.popleft()
+            self.pool.share_prefix(seq, lookback)
+            self.running.append(seq)
+            run(seq)
+        return batch
 
     def preempt(self, seq: Sequence):
         assert not seq.compressed and not seq.require_compress

@@ -30,6 +30,10 @@ class Sequence:
         self.num_prompt_tokens = len(self.token_ids)
         self.num_tokens = len(self.token_ids)
         self.num_cached_tokens = 0
+        self.num_computed_tokens = 0               # steps of portions: tokens whose rows are cached
+        self.first_page = 0                        # leading table entries given back (-1)
+        self.reserved_pages = 0
+        self.sealed: list[int] = []                # chain hashes of the finished prompt pages
         self.block_table: list[int] = []
         self.new_block_table: list[int] = []       # target table of a pending compression
         self.block_to_release: list[int] = []
@@ -73,3 +77,16 @@ class Sequence:
         self.num_cached_tokens += 1
         if self.num_completion_tokens == 1:
             self.time_prefilled = time.time()
+
+
+@dataclass
+class Portion:
+    """The part of a sequence one step runs: tokens start .. start + count - 1."""
+    seq: Sequence
+    start: int
+    count: int
+
+    @property
+    def ends(self) -> bool:
+        """Its last token is the sequence's last: the next token can be drawn."""
+        return self.start + self.count == self.seq.num_tokens

@@ -1,0 +1,65 @@
+"""Row steps of decoders with an fp32 residual stream (one HIP launch each).
+
+`x` is the stream (N, width) fp32; what feeds a matrix product has the model's dtype.  Widths are
+padded to a multiple of 8 with zeros, `norm_width` is the length the mean runs over."""
+import torch
+
+from zipage_amd import _lib
+
+
+def _rows(t: torch.Tensor | None, width: int):
+    if t is not None:
+        assert t.is_contiguous() and t.shape[-1] == width
+    return _lib.dev_ptr(t)
+
+
+def embed_norm(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.Tensor,
+               pos: torch.Tensor | None, x: torch.Tensor, norm_weight: torch.Tensor, eps: float,
+               norm_width: int, weight_offset: float = 0.0) -> torch.Tensor:
+    """x = embed[tokens] (+ pos[positions]) into `x`; returns its RMS norm times
+    (weight_offset + norm_weight) in the table's dtype.  tokens (N,) int64, positions (N,) int32."""
+    N, W = x.shape
+    assert tokens.dtype == torch.int64 and positions.dtype == torch.int32
+    assert tokens.is_contiguous() and positions.is_contiguous() and tokens.numel() == positions.numel() == N
+    assert x.dtype == torch.float32 and norm_weight.dtype == torch.float32
+    assert pos is None or pos.dtype == embed.dtype
+    out = torch.empty((N, W), dtype=embed.dtype, device=x.device)
+    _lib.call_models("zp_embed_norm", _lib.dev_ptr(tokens), _lib.dev_ptr(positions), _rows(embed, W),
+                     _rows(pos, W), _rows(x, W), _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width,
+                     embed.shape[0], 0 if pos is None else pos.shape[0], float(eps), float(weight_offset),
+                     _lib.dtype_tag(embed), _lib.stream_ptr(x))
+    return out
+
+
+def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | None, eps: float,
+                  norm_width: int, weight_offset: float = 0.0, out_scale: float = 1.0,
+                  x_out: torch.Tensor | None = None, result: torch.Tensor | None = None,
+                  history: torch.Tensor | None = None, mix: torch.Tensor | None = None):
+    """r = x + y, kept in `result`; with `mix`, r <- mix[-1] r + sum_j mix[j] history[j]; kept in
+    `x_out`; returns rmsnorm(r) * (weight_offset + norm_weight) * out_scale in y's dtype (None
+    without a norm).  history (planes, N, width) fp32, of which the first len(mix) - 1 are read."""
+    N, W = x.shape
+    assert x.dtype == torch.float32 and y.shape == x.shape
+    n_hist, plane = 0, 0
+    if mix is not None:
+        assert mix.dtype == torch.float32 and mix.is_contiguous()
+        n_hist = mix.numel() - 1
+        if n_hist:
+            assert history.dtype == torch.float32 and history.shape[0] >= n_hist and history[0].shape == x.shape
+            plane = history.stride(0)
+            assert history.stride(1) == W and history.stride(2) == 1
+    out = torch.empty((N, W), dtype=y.dtype, device=x.device) if norm_weight is not None else None
+    _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), _lib.dev_ptr(history if n_hist else None),
+                     plane, _lib.dev_ptr(mix), n_hist, _rows(result, W), _rows(x_out, W),
+                     _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width, float(eps),
+                     float(weight_offset), float(out_scale), _lib.dtype_tag(y), _lib.stream_ptr(x))
+    return out
+
+
+def xielu(z: torch.Tensor, alpha_p: float, alpha_n: float) -> torch.Tensor:
+    """z > 0: alpha_p z^2 + z / 2; z <= 0: alpha_n (exp(z) - 1 - z) + z / 2."""
+    assert z.is_contiguous()
+    out = torch.empty_like(z)
+    _lib.call_models("zp_xielu", _lib.dev_ptr(z), _lib.dev_ptr(out), z.numel(), float(alpha_p),
+                     float(alpha_n), _lib.dtype_tag(z), _lib.stream_ptr(z))
+    return out
