@@ -9,8 +9,8 @@ import pytest
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def _declared():
-    text = open(os.path.join(ROOT, "include", "zipage_hip.h")).read()
+def _declared(header="zipage_hip.h"):
+    text = open(os.path.join(ROOT, "include", header)).read()
     text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
     return sorted(set(re.findall(r"\b(zp_[a-z_0-9]+)\s*\(", text)))
 
@@ -32,6 +32,21 @@ def test_library_exports_every_declared_symbol():
     for name in _declared():
         assert hasattr(lib, name), f"{name} declared in the header but not exported"
     assert sorted(_lib.EXPORTS) == _declared()
+
+
+def test_models_library_exports_every_declared_symbol():
+    from zipage_amd import _lib
+    lib = _lib.load_models()
+    names = _declared("zipage_models.h")
+    for name in names:
+        assert hasattr(lib, name), f"{name} declared in the header but not exported"
+    assert sorted(_lib.MODEL_EXPORTS) == names
+    # bad arguments are refused on the host, before any launch
+    assert lib.zp_headwise_linear(None, None, None, 1, 2, 33, 16, 0, None) != 0
+    assert b"multiple of 32" in lib.zp_last_error()
+    assert lib.zp_latent_rows_attention(None, None, None, None, None, None, 1, 1, 32, 16, 1, 1, 1, -1, 1.0, 0,
+                                        None, 0, None) == 1
+    assert lib.zp_embed_norm(None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1e-6, 0.0, 0, None) != 0
 
 
 def test_version_and_error_string():

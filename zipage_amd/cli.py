@@ -66,7 +66,6 @@ def trace(args) -> int:
             entries.append((live[e["id"]], e["tokens"], e["want"]))
         logits = eng.feed(entries) if entries else None
         if logits is not None:
-            eng.runner.run_stream.synchronize()
             path = os.path.join(args.out, f"{step['step']}.f32")
             logits.cpu().numpy().astype("<f4").tofile(path + ".part")
             os.replace(path + ".part", path)

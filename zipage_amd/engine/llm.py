@@ -62,7 +62,10 @@ class ZipageEngine:
         return any(not s.params.ignore_eos for s in seqs)
 
     def _finish_step(self, seqs: list[Sequence], tok: torch.Tensor):
-        ids = tok.tolist() if self._needs_host_tokens(seqs) else None
+        ids = None
+        if self._needs_host_tokens(seqs):
+            self.runner.run_stream.synchronize()   # the copy below is on the caller's stream
+            ids = tok.tolist()
         self.scheduler.postprocess(seqs, ids, advance=True)
         for s in seqs:
             if s.finished:

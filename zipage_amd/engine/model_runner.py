@@ -291,7 +291,11 @@ class ModelRunner:
             rows = [f + k for f, w in zip(first, want) for k in w]
             if not rows:
                 return None
-            return self.model.compute_logits(hidden[torch.tensor(rows, device=self.device)]).float()
+            logits = self.model.compute_logits(hidden[torch.tensor(rows, device=self.device)]).float()
+        caller = torch.cuda.current_stream(self.device)
+        caller.wait_stream(self.run_stream)
+        logits.record_stream(caller)
+        return logits
 
     # ------------------------------------------------------------------ HIP graph
     def _graph_batch(self, B: int) -> int:
