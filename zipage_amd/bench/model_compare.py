@@ -1,0 +1,239 @@
+"""Pedivik beside Qwen3 at equal size: prefill and decode throughput through the engine (random
+weights), and every kernel between the matrix products against its roofline, beside the kernel of
+the other model that does the like work.
+
+Equal size: same width, heads, head dimensions and vocabulary; Pedivik's ungated feed-forward is 1.5
+times as wide as Qwen3's gated one, so both hold the same parameters.  Kernels are timed as replays
+of a graph of many launches over buffers that together exceed the caches.
+"""
+from __future__ import annotations
+
+import time
+
+import torch
+
+HBM = 8.0e12          # bytes/s
+MFMA = 2.5e15         # dense bf16 FLOP/s
+BF16 = torch.bfloat16
+
+SIZES = {
+    # width, heads, kv_heads (Qwen3), head dim, gated ff, layers, vocab, q_rank, kv_rank, window
+    "1k": (1024, 16, 8, 128, 3072, 8, 32768, 512, 256, 1024),
+    "4k": (4096, 32, 8, 128, 12288, 8, 32768, 1536, 512, 1024),
+}
+
+
+def shapes(size: str):
+    from zipage_amd.engine import PedivikLayer, PedivikShape, Qwen3Shape
+    W, H, HK, D, FF, L, V, QR, KR, win = SIZES[size]
+    layer = PedivikLayer(H, D, D, QR, KR, D ** -0.5, win, FF * 3 // 2)
+    return (PedivikShape(V, W, (layer,) * L, 8192, 1e-6, 1.0),
+            Qwen3Shape(L, W, H, HK, D, FF, V, max_position=8192))
+
+
+def throughput(shape, batch: int, prompt: int, out_tokens: int) -> dict:
+    """One generate() call per figure: all prompts in one prefill step, then decode steps."""
+    from zipage_amd.engine import EngineConfig, SamplingParams, ZipageEngine
+    total = prompt + out_tokens
+    per = -(-total // 256) + 1
+    cfg = EngineConfig(shape=shape, max_concurrency=batch, max_num_seqs=batch, num_kvcache_blocks=batch * per + 8,
+                       max_cache_blocks_per_seq=per, max_model_len=total + 1, kvcache_block_size=256,
+                       max_num_batched_tokens=batch * prompt)
+    eng = ZipageEngine(cfg)
+    g = torch.Generator().manual_seed(0)
+    prompts = torch.randint(0, shape.vocab, (batch, prompt), generator=g).tolist()
+    run = lambda n: eng.generate(prompts, SamplingParams(max_tokens=n, ignore_eos=True))
+    eng.runner.reserve_token_log(out_tokens + 1)
+    run(3)                                    # products, graphs and allocator warm up
+    for k in ("prefill_s", "decode_s", "decode_tokens", "decode_steps", "prefill_tokens"):
+        eng.stats[k] = 0
+    run(out_tokens)
+    st = eng.stats
+    # the step alone: replays of the decode graph at the last step's inputs
+    r = eng.runner
+    (g_, _, _), = [v for k, v in r._graphs.items()]
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    with torch.cuda.stream(r.run_stream):
+        for _ in range(20):
+            g_.replay()
+    torch.cuda.synchronize()
+    step = (time.perf_counter() - t0) / 20
+    del eng, r
+    torch.cuda.empty_cache()
+    return {"prefill_tok_per_s": round(st["prefill_tokens"] / st["prefill_s"]),
+            "decode_tok_per_s": round(st["decode_tokens"] / st["decode_s"]),
+            "ms_per_decode_step": round(st["decode_s"] / st["decode_steps"] * 1e3, 3),
+            "ms_layers_of_a_decode_step": round(step * 1e3, 3)}
+
+
+def timed(fn, variants: int, launches: int = 24) -> float:
+    """Seconds per call of fn(i): a graph of `launches` calls over `variants` buffer sets."""
+    s = torch.cuda.Stream()
+    with torch.cuda.stream(s):
+        for i in range(min(variants, 3)):
+            fn(i)
+        s.synchronize()
+        g = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(g, stream=s):
+            for i in range(launches):
+                fn(i % variants)
+        g.replay()
+        best = float("inf")
+        for _ in range(5):
+            a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+            a.record(s)
+            g.replay()
+            b.record(s)
+            b.synchronize()
+            best = min(best, a.elapsed_time(b))
+    del g
+    torch.cuda.empty_cache()
+    return best / launches / 1e3
+
+
+def _sets(nbytes: int) -> int:
+    """Buffer sets that together exceed the 256 MB last-level cache."""
+    return max(2, min(24, -(-(1 << 30) // max(nbytes, 1))))
+
+
+def kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dict]:
+    """Rows of (kernel, like kernel): time, roofline time and the fraction of each."""
+    import torch.nn.functional as F
+    from zipage_amd.engine.inputs import plan_runs
+    from zipage_amd.engine.sequence import Portion, Sequence
+    from zipage_amd.layers import (latent_rows_attention, latent_tiles_attention, paged_decode_attention,
+                                   qk_norm_rope_store, residual_norm, rms_norm, silu_and_mul, xielu)
+    from zipage_amd.layers.latent import headwise_linear, latent_norm_store
+    W, H, HK, D, FF, L, V, QR, KR, win = SIZES[size]
+    dev, BS = torch.device("cuda:0"), 256
+    rnd = lambda *s, dt=BF16: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    rows = []
+
+    def put(name, where, secs, byts, flops=0.0):
+        roof = max(byts / HBM, flops / MFMA)
+        rows.append({"kernel": name, "at": where, "us": round(secs * 1e6, 1),
+                     "bound": "hbm" if byts / HBM >= flops / MFMA else "mfma",
+                     "roofline_us": round(roof * 1e6, 1), "frac": round(roof / secs, 3)})
+
+    for phase, N in (("decode", decode_batch), ("prefill", prompts * prompt)):
+        at = f"{phase}, {N} tokens"
+        big = N * W
+        # norms of the stream
+        k = _sets(big * 14)
+        xs, ys = [rnd(N, W, dt=torch.float32) for _ in range(k)], [rnd(N, W) for _ in range(k)]
+        w32, w16 = torch.zeros(W, device=dev), torch.ones(W, device=dev, dtype=BF16)
+        put("residual_norm (fp32 stream)", at,
+            timed(lambda i: residual_norm(xs[i], ys[i], w32, 1e-6, W, 1.0, x_out=xs[i]), k), big * (4 + 2 + 4 + 2))
+        planes = L // 2 + 1
+        kh = max(1, min(k, (8 << 30) // (planes * big * 4)))
+        hist = [rnd(planes + 1, N, W, dt=torch.float32) for _ in range(kh)]
+        mix = torch.full((planes + 1,), 0.3, device=dev)
+        put(f"residual_norm with depth average over {planes} planes", at,
+            timed(lambda i: residual_norm(xs[i], ys[i], w32, 1e-6, W, 1.0, x_out=xs[i], result=hist[i][planes],
+                                          history=hist[i], mix=mix), kh), big * (4 + 2 + 4 + 4 + 2 + 4 * planes))
+        del hist
+        rs = [rnd(N, W) for _ in range(k)]
+        put("like: add_rms_norm (16-bit stream)", at, timed(lambda i: rms_norm(ys[i], w16, 1e-6, rs[i]), k),
+            big * (2 + 2 + 2 + 2))
+        del xs, ys, rs
+        # activations
+        k = _sets(N * FF * 3 // 2 * 4)
+        zs = [rnd(N, FF * 3 // 2) for _ in range(k)]
+        put("xielu", at, timed(lambda i: xielu(zs[i], 0.8, 1.3), k), N * FF * 3 // 2 * 4)
+        del zs
+        gs = [rnd(N, 2 * FF) for _ in range(k)]
+        put("like: silu_and_mul", at, timed(lambda i: silu_and_mul(gs[i]), k), N * FF * 6)
+        del gs
+        # norms and stores of the attention inputs
+        slots = torch.randperm(N, device=dev).int()
+        k = _sets(N * (QR + KR) * 6)
+        downs = [rnd(N, QR + KR) for _ in range(k)]
+        caches = [rnd(-(-N // BS), BS, KR) for _ in range(k)]
+        wq, wc = torch.ones(QR, device=dev), torch.ones(KR, device=dev)
+        put("latent_norm_store", at, timed(lambda i: latent_norm_store(downs[i], wq, wc, QR, KR, 1e-6, caches[i],
+                                                                        slots), k), N * (QR + KR) * 4)
+        del downs, caches
+        qkv_w = (H + 2 * HK) * D
+        k = _sets(N * qkv_w * 4)
+        qkvs = [rnd(N, qkv_w) for _ in range(k)]
+        kcs = [rnd(-(-N // BS), BS, HK, D) for _ in range(2 * k)]
+        pos = torch.arange(N, device=dev, dtype=torch.int32) % 4096
+        cos, sin = rnd(8192, D // 2, dt=torch.float32), rnd(8192, D // 2, dt=torch.float32)
+        nw = torch.ones(D, device=dev, dtype=BF16)
+        put("like: qk_norm_rope_store", at,
+            timed(lambda i: qk_norm_rope_store(qkvs[i], pos, cos, sin, nw, nw, H, HK, D, 1e-6, kcs[2 * i], kcs[2 * i + 1],
+                                               slots), k), N * qkv_w * 4)
+        del qkvs, kcs
+    # ---- decode attention
+    B, ctx_len = decode_batch, prompt
+    per = -(-ctx_len // BS)
+    at = f"decode, {B} sequences, context {ctx_len}"
+    k = _sets(B * win * KR * 2)
+    caches = [rnd(B * per, BS, KR) for _ in range(k)]
+    tables = torch.randperm(B * per, device=dev).int().view(B, per)
+    ctx = torch.full((B,), ctx_len, device=dev, dtype=torch.int32)
+    q = rnd(B, H, KR)
+    seen = min(win, ctx_len)
+    put(f"latent_rows_attention, window {win}", at,
+        timed(lambda i: latent_rows_attention(q, caches[i], tables, ctx, D ** -0.5, win), k),
+        B * seen * KR * 2 + 2 * B * H * KR * 2, 4.0 * B * H * seen * KR)
+    del caches
+    k = max(2, _sets(2 * B * ctx_len * HK * D * 2))
+    kcs = [rnd(B * per, BS, HK, D) for _ in range(2 * k)]
+    qd = rnd(B, H, D)
+    put("like: paged_decode_attention", at,
+        timed(lambda i: paged_decode_attention(qd, kcs[2 * i], kcs[2 * i + 1], ctx, tables, D ** -0.5), k),
+        2 * B * ctx_len * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * ctx_len * D)
+    del kcs
+    k = _sets(H * KR * D * 2)
+    ws, wv = [rnd(H, KR, D) for _ in range(k)], [rnd(H, D, KR) for _ in range(k)]
+    x1, x2 = rnd(B, H, D), rnd(B, H, KR)
+    byts, fl = H * KR * D * 2 + B * H * (KR + D) * 2, 2.0 * B * H * KR * D
+    put("headwise_linear, q into the latent space", at, timed(lambda i: headwise_linear(x1, ws[i]), k), byts, fl)
+    put("headwise_linear, values out of it", at, timed(lambda i: headwise_linear(x2, wv[i]), k), byts, fl)
+    lin = [rnd(W, H * D) for _ in range(_sets(W * H * D * 2))]
+    xl = rnd(B, H * D)
+    put("like: output projection (library product)", at, timed(lambda i: F.linear(xl, lin[i]), len(lin)),
+        W * H * D * 2 + B * (W + H * D) * 2, 2.0 * B * W * H * D)
+    del ws, wv, lin
+    # ---- prefill attention
+    N = prompts * prompt
+    at = f"prefill, {prompts} x {prompt} tokens"
+    seqs = [Sequence([0] * prompt) for _ in range(prompts)]
+    for s in seqs:
+        s.block_table = list(range(per))
+    tiles = torch.as_tensor(plan_runs([Portion(s, 0, prompt) for s in seqs], BS, win).tiles).to(dev)
+    k = 2
+    qs, kvs = [rnd(N, H * D) for _ in range(k)], [rnd(N, H * 2 * D) for _ in range(k)]
+    out = torch.empty(N, H * D, device=dev, dtype=BF16)
+    pairs = sum(min(i + 1, win) for i in range(prompt)) * prompts
+    put(f"latent_tiles_attention, window {win}", at,
+        timed(lambda i: latent_tiles_attention(qs[i], kvs[i], H, D, D, tiles, D ** -0.5, win, out), k, 6),
+        N * H * D * 2 * 4, 4.0 * pairs * H * D)
+    full = torch.as_tensor(plan_runs([Portion(s, 0, prompt) for s in seqs], BS, None).tiles).to(dev)
+    pairs = prompt * (prompt + 1) / 2 * prompts
+    put("latent_tiles_attention, no window", at,
+        timed(lambda i: latent_tiles_attention(qs[i], kvs[i], H, D, D, full, D ** -0.5, None, out), k, 6),
+        N * H * D * 2 * 4, 4.0 * pairs * H * D)
+    del kvs
+    ks = [rnd(prompts, prompt, HK, D) for _ in range(2 * k)]
+    put("like: scaled_dot_product_attention (library, causal)", at,
+        timed(lambda i: F.scaled_dot_product_attention(
+            qs[i].view(prompts, prompt, H, D).transpose(1, 2), ks[2 * i].transpose(1, 2), ks[2 * i + 1].transpose(1, 2),
+            is_causal=True, enable_gqa=True), k, 6), N * (2 * H + 2 * HK) * D * 2, 4.0 * pairs * H * D)
+    return rows
+
+
+def compare(sizes=("1k", "4k"), out_tokens: int = 64) -> dict:
+    """The whole report.  The headline figure is Pedivik's decode rate at the largest size and batch."""
+    report = {"sizes": {}}
+    for size in sizes:
+        pedivik, qwen = shapes(size)
+        entry = {"pedivik": {}, "qwen3": {}}
+        for batch, prompt in ((1, 2048), (64, 2048), (256, 2048)):
+            for name, shape in (("pedivik", pedivik), ("qwen3", qwen)):
+                entry[name][f"{batch} x {prompt}"] = throughput(shape, batch, prompt, out_tokens)
+        entry["kernels"] = kernels(size, 256, 8, 2048)
+        report["sizes"][size] = entry
+    return report

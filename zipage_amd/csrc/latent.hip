@@ -201,13 +201,27 @@ __device__ __forceinline__ int page_of(const RowsArgs& a, int t) {
 }
 
 // NCB column blocks of 128 cover R.  Workgroup: one token, 16 * hw heads, one key range.
+//
+// A wave takes 32 keys at a time.  They come from memory once, as whole 256-byte row pieces (lane: 8
+// keys x 8 columns), and stay in registers as the value operand; the key operand (lane: one key, 8
+// columns per MFMA) would touch 16 cache lines per 16 lanes if it were read from memory, so the wave
+// passes the block through an LDS stage of its own.  The next block's pieces are requested as the
+// value products free their registers.  No barrier until the waves meet at the end.
+template <int NCB> struct RowsStage {
+  static constexpr int kStride = NCB * 128 + 8;                  // elements: rows 16 bytes apart in the banks
+  static constexpr int kBytes = 32 * kStride * 2;                // per wave
+};
+
 template <int NCB>
-__global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
+__global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
+  typedef RowsStage<NCB> Stage;
   int* pg = (int*)lds_raw;
-  float* merge = (float*)(lds_raw + ((a.lds_pages * 4 + 15) & ~15));
+  char* const shared = lds_raw + ((a.lds_pages * 4 + 15) & ~15);
+  float* merge = (float*)shared;                                 // after the key loop
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int l16 = lane & 15, g = lane >> 4;
+  uint16_t* stage = (uint16_t*)(shared + wave * Stage::kBytes);
   const int hw = a.hw, kw = 4 / hw, hwi = wave % hw, kwi = wave / hw;
   const int hgroups = (a.H + 16 * hw - 1) / (16 * hw);
   int id = blockIdx.x;
@@ -238,13 +252,18 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
     const int p = page_of(a, t);
     return cache + ((int64_t)pg[p - p0] * a.BS + (t - p * a.BS)) * a.R;
   };
+  // R may end inside the last column block: columns past it hold the row's start again, and meet
+  // zeros in q or results that are not written
+  auto col_off = [&](int cb) { const int c = cb * 128 + l16 * 8; return c < a.R ? c : 0; };
 
   u32x4 qf[KS];
   {
     const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + (head_ok ? head : 0)) * a.R + g * 8;
 #pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qf[ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
+#pragma unroll
     for (int ks = 0; ks < KS; ++ks)
-      qf[ks] = (head_ok && ks < nks) ? *(const u32x4*)(q + ks * 32) : u32x4{0u, 0u, 0u, 0u};
+      if (!head_ok || ks >= nks) qf[ks] = u32x4{0u, 0u, 0u, 0u};
   }
   f32x4 o[NCB * 8];
 #pragma unroll
@@ -252,20 +271,35 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
   float m = -INFINITY, l = 0.f;
   const float sc = a.scale * 1.44269504088896f;
 
-  if (n > 0) {
-    const int b1 = (n - 1) >> 5;
-    for (int b = (lo >> 5) + split * kw + kwi; b <= b1; b += a.splits * kw) {
-      const int k0 = b * 32;
-      f32x4 s[2];
+  const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = a.splits * kw;
+  int b = (lo >> 5) + split * kw + kwi;
+  if (b <= b1) {
+    u32x4 v[NCB][8];
+    {
 #pragma unroll
-      for (int tt = 0; tt < 2; ++tt) {
-        const uint16_t* kr = key_row(k0 + tt * 16 + l16) + g * 8;
-        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+      for (int i = 0; i < 8; ++i) {
+        const uint16_t* kr = key_row(b * 32 + step_key(g, i));
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks)
-          if (ks < nks) acc = mfma_bf16(*(const u32x4*)(kr + ks * 32), qf[ks], acc);
-        s[tt] = acc;
+        for (int cb = 0; cb < NCB; ++cb) v[cb][i] = *(const u32x4*)(kr + col_off(cb));
       }
+    }
+    for (; b <= b1; b += step) {
+      const int k0 = b * 32;
+#pragma unroll
+      for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+          *(u32x4*)(stage + step_key(g, i) * Stage::kStride + cb * 128 + l16 * 8) = v[cb][i];
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+      f32x4 s[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+        for (int tt = 0; tt < 2; ++tt)
+          s[tt] = mfma_bf16(*(const u32x4*)(stage + (tt * 16 + l16) * Stage::kStride + ks * 32 + g * 8), qf[ks], s[tt]);
+      __builtin_amdgcn_wave_barrier();        // the next block is staged after these reads
       float p[8], mx = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
@@ -275,7 +309,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
       }
       mx = fmaxf(mx, lane_xor16(mx));
       mx = fmaxf(mx, lane_xor32(mx));
-      const float mn = fmaxf(m, mx);          // finite: every step holds a visible key
+      const float mn = fmaxf(m, mx);          // finite: every block holds a visible key
       const float f = __builtin_amdgcn_exp2f(m - mn);
       float sum = 0.f;
 #pragma unroll
@@ -291,18 +325,16 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
       }
       const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
                         pack_bf16(p[6], p[7])};
-      const uint16_t* vr[8];
+      // past the last block the keys clamp to the last row
+      const uint16_t* kr[8];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) vr[i] = key_row(k0 + step_key(g, i));
+      for (int i = 0; i < 8; ++i) kr[i] = key_row((b + step) * 32 + step_key(g, i));
 #pragma unroll
       for (int cb = 0; cb < NCB; ++cb) {
-        const int col = cb * 128 + l16 * 8;
-        const int off = col < a.R ? col : 0;
-        u32x4 v[8];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] = *(const u32x4*)(vr[i] + off);
+        for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v[cb], t), pf, o[cb * 8 + t]);
 #pragma unroll
-        for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v, t), pf, o[cb * 8 + t]);
+        for (int i = 0; i < 8; ++i) v[cb][i] = *(const u32x4*)(kr[i] + col_off(cb));
       }
     }
   }
@@ -311,6 +343,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(RowsArgs a) {
 
   // waves that split the keys of the same heads meet in LDS
   if (kw > 1) {
+    __syncthreads();                                // the stages are used up
     const int RS = a.R + 4;
     const int per = 16 * RS + 32;                   // O rows, then max and sum of 16 heads
     if (kwi > 0) {
@@ -504,7 +537,8 @@ __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
   const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
   // host-made descriptors: rows outside the buffers are not touched
   if (q0 < 0 || kb < 0 || rel < 0 || q0 + nq > a.q_rows || kb + rel + nq > a.k_rows) return;
-  const int nks = a.D / 32;
+  const int nks = a.D / 32;                 // steps past it: as in the rows kernel
+  auto k_off = [&](int ks) { return ks < nks ? ks * 32 : 0; };
   const float sc = a.scale * 1.44269504088896f;
   const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + h * a.D + g * 8;
   const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + h * a.V;
@@ -521,7 +555,10 @@ __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
       const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + h * a.D + g * 8;
   #pragma unroll
       for (int ks = 0; ks < DKS; ++ks)
-        qf[t][ks] = ks < nks ? *(const u32x4*)(q + ks * 32) : u32x4{0u, 0u, 0u, 0u};
+        {
+          qf[t][ks] = *(const u32x4*)(q + k_off(ks));
+          if (ks >= nks) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
+        }
     }
     f32x4 o[kQT][VCB * 8];
     float m[kQT], l[kQT];
@@ -541,13 +578,13 @@ __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
         u32x4 kf[DKS];
   #pragma unroll
         for (int ks = 0; ks < DKS; ++ks)
-          if (ks < nks) kf[ks] = *(const u32x4*)(kr + ks * 32);
+          kf[ks] = *(const u32x4*)(kr + k_off(ks));
   #pragma unroll
         for (int t = 0; t < kQT; ++t) {
           f32x4 acc = {0.f, 0.f, 0.f, 0.f};
   #pragma unroll
           for (int ks = 0; ks < DKS; ++ks)
-            if (ks < nks) acc = mfma_bf16(kf[ks], qf[t][ks], acc);
+            acc = mfma_bf16(kf[ks], qf[t][ks], acc);
           s[t][tt] = acc;
         }
       }
@@ -638,13 +675,14 @@ int rows_hw(int H) {
 }
 
 // Key ranges per token: enough workgroups to cover the chip, at least two 32-key steps per wave.
-int rows_splits(int n, int H, int window, int NB, int BS) {
+int rows_splits(int n, int H, int R, int window, int NB, int BS) {
   const int hw = rows_hw(H), kw = 4 / hw;
   const int groups = n * ((H + 16 * hw - 1) / (16 * hw));
   int64_t keys = (int64_t)NB * BS;
   if (window > 0 && window < keys) keys = window;
   const int steps = (int)((keys + 31) / 32);
-  int s = 512 / (groups > 0 ? groups : 1);
+  const int resident = R <= 256 ? 2 : 1;       // workgroups per CU
+  int s = 256 * resident / (groups > 0 ? groups : 1);
   s = s < steps / (2 * kw) ? s : steps / (2 * kw);
   s = s < 32 ? s : 32;
   return s < 1 ? 1 : s;
@@ -652,7 +690,8 @@ int rows_splits(int n, int H, int window, int NB, int BS) {
 
 template <int NCB> int launch_latent_rows(RowsArgs a, hipStream_t st) {
   const int kw = 4 / a.hw;
-  const size_t merge = kw > 1 ? sizeof(float) * (size_t)(kw - 1) * a.hw * (16 * (a.R + 4) + 32) : 0;
+  size_t merge = kw > 1 ? sizeof(float) * (size_t)(kw - 1) * a.hw * (16 * (a.R + 4) + 32) : 0;
+  if (merge < 4 * (size_t)RowsStage<NCB>::kBytes) merge = 4 * RowsStage<NCB>::kBytes;
   const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + merge;
   if (smem > 64 * 1024 &&
       hipFuncSetAttribute((const void*)latent_rows_kernel<NCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -743,7 +782,7 @@ extern "C" int64_t zp_latent_rows_workspace(int32_t n, int32_t H, int32_t R, int
                                             int32_t NB, int32_t BS, int32_t dtype) {
   if (n < 0 || H <= 0 || R <= 0 || NB <= 0 || BS <= 0) return -1;
   if (dtype != ZP_BF16 || R > 512) return 0;
-  const int s = rows_splits(n, H, window, NB, BS);
+  const int s = rows_splits(n, H, R, window, NB, BS);
   return s == 1 ? 0 : (int64_t)n * H * s * (R + 2) * 4;
 }
 
@@ -785,7 +824,7 @@ extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const 
   }
   a.hw = rows_hw(H);
   a.lds_pages = (int)pages;
-  a.splits = rows_splits(n, H, window, NB, BS);
+  a.splits = rows_splits(n, H, R, window, NB, BS);
   ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_latent_rows_workspace(n, H, R, window, NB, BS, dtype)),
              "latent_rows_attention: workspace too small");
   switch ((R + 127) / 128) {
