@@ -527,120 +527,164 @@ struct TilesArgs {
 };
 
 constexpr int kTileQ = 128;   // queries per workgroup
+constexpr int kTileK = 64;    // keys per LDS tile
 
-// A wave owns 16 * kQT queries of one head at a time and walks only the keys those queries see.
+// A workgroup owns up to 128 queries of one head; key and value tiles pass through LDS once for all of
+// them (double-buffered, the next tile's loads in flight during the products), a wave owns 16 * kQT
+// queries at a time and skips the 32-key steps none of them sees.
+template <int DKS, int VCB> struct TileStage {
+  static constexpr int kK = DKS * 32 + 8, kV = VCB * 128 + 8;    // row strides: rows 16 bytes apart in the banks
+  static constexpr int kElems = kTileK * (kK + kV);
+  static constexpr int kBytes = 2 * kElems * 2;
+};
+
 template <int DKS, int VCB, int kQT>
 __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  extern __shared__ __align__(16) char lds_raw[];
+  typedef TileStage<DKS, VCB> Stage;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
   const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
   const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
   // host-made descriptors: rows outside the buffers are not touched
   if (q0 < 0 || kb < 0 || rel < 0 || q0 + nq > a.q_rows || kb + rel + nq > a.k_rows) return;
-  const int nks = a.D / 32;                 // steps past it: as in the rows kernel
-  auto k_off = [&](int ks) { return ks < nks ? ks * 32 : 0; };
+  const int nks = a.D / 32;
   const float sc = a.scale * 1.44269504088896f;
-  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + h * a.D + g * 8;
+  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + h * a.D;
   const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + h * a.V;
-  for (int w0 = wave * 16 * kQT; w0 < nq; w0 += 64 * kQT) {
-    const int hi = rel + min(w0 + 16 * kQT, nq) - 1;            // last key any query here sees
+
+  for (int wg0 = 0; wg0 < nq; wg0 += 64 * kQT) {              // uniform in the workgroup
+    const int w0 = wg0 + wave * 16 * kQT;
+    const int last = rel + min(wg0 + 64 * kQT, nq) - 1;       // last key any query of the pass sees
+    const int first = a.window > 0 ? max(0, rel + wg0 - a.window + 1) : 0;
+    const int hi = w0 < nq ? rel + min(w0 + 16 * kQT, nq) - 1 : -1;      // the same for the wave
     const int lo = a.window > 0 ? max(0, rel + w0 - a.window + 1) : 0;
 
     u32x4 qf[kQT][DKS];
     int qpos[kQT];
-  #pragma unroll
+#pragma unroll
     for (int t = 0; t < kQT; ++t) {
       const int qi = min(w0 + t * 16 + l16, nq - 1);
       qpos[t] = rel + qi;
       const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + h * a.D + g * 8;
-  #pragma unroll
-      for (int ks = 0; ks < DKS; ++ks)
-        {
-          qf[t][ks] = *(const u32x4*)(q + k_off(ks));
-          if (ks >= nks) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
-        }
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) {
+        // D may end inside the last steps: they read the row's start, against zeros in q
+        qf[t][ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
+        if (ks >= nks) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
+      }
     }
     f32x4 o[kQT][VCB * 8];
     float m[kQT], l[kQT];
-  #pragma unroll
+#pragma unroll
     for (int t = 0; t < kQT; ++t) {
       m[t] = -INFINITY;
       l[t] = 0.f;
-  #pragma unroll
+#pragma unroll
       for (int i = 0; i < VCB * 8; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
-    for (int k0 = lo; k0 <= hi; k0 += 32) {
-      f32x4 s[kQT][2];
-  #pragma unroll
-      for (int tt = 0; tt < 2; ++tt) {
-        const uint16_t* kr = kbase + (int64_t)min(k0 + tt * 16 + l16, hi) * a.kv_st;
-        u32x4 kf[DKS];
-  #pragma unroll
-        for (int ks = 0; ks < DKS; ++ks)
-          kf[ks] = *(const u32x4*)(kr + k_off(ks));
-  #pragma unroll
-        for (int t = 0; t < kQT; ++t) {
-          f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  #pragma unroll
-          for (int ks = 0; ks < DKS; ++ks)
-            acc = mfma_bf16(kf[ks], qf[t][ks], acc);
-          s[t][tt] = acc;
-        }
+    u32x4 rk[DKS], rv[4 * VCB];                                // this thread's pieces of a tile
+    auto fetch = [&](int k0) {
+#pragma unroll
+      for (int j = 0; j < DKS; ++j) {
+        const int id = tid + 256 * j, r = id / (4 * DKS), c = (id % (4 * DKS)) * 8;
+        rk[j] = *(const u32x4*)(kbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.D ? c : 0));
       }
-      // every query of the wave sees all 32 keys: no masks
-      const bool inner = k0 + 31 <= rel + w0 &&
-                         (a.window <= 0 || k0 > rel + w0 + 16 * kQT - 1 - a.window);
-      u32x4 pf[kQT];
-  #pragma unroll
-      for (int t = 0; t < kQT; ++t) {
-        float p[8], mx = -INFINITY;
-  #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          p[i] = s[t][i >> 2][i & 3] * sc;
-          if (!inner) {
-            const int back = qpos[t] - (k0 + step_key(g, i));
-            if (back < 0 || (a.window > 0 && back >= a.window)) p[i] = -INFINITY;
+#pragma unroll
+      for (int j = 0; j < 4 * VCB; ++j) {
+        const int id = tid + 256 * j, r = id / (16 * VCB), c = (id % (16 * VCB)) * 8;
+        rv[j] = *(const u32x4*)(vbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.V ? c : 0));
+      }
+    };
+    fetch(first);
+    __syncthreads();                                           // a pass before this one still reads its tiles
+    int buf = 0;
+    for (int t0 = first; t0 <= last; t0 += kTileK, buf ^= 1) {
+      uint16_t* const ldsk = (uint16_t*)lds_raw + buf * Stage::kElems;
+      uint16_t* const ldsv = ldsk + kTileK * Stage::kK;
+#pragma unroll
+      for (int j = 0; j < DKS; ++j) {
+        const int id = tid + 256 * j;
+        *(u32x4*)(ldsk + id / (4 * DKS) * Stage::kK + (id % (4 * DKS)) * 8) = rk[j];
+      }
+#pragma unroll
+      for (int j = 0; j < 4 * VCB; ++j) {
+        const int id = tid + 256 * j;
+        *(u32x4*)(ldsv + id / (16 * VCB) * Stage::kV + (id % (16 * VCB)) * 8) = rv[j];
+      }
+      __syncthreads();
+      if (t0 + kTileK <= last) fetch(t0 + kTileK);
+#pragma unroll 1
+      for (int sub = 0; sub < kTileK; sub += 32) {
+        const int k0 = t0 + sub;
+        if (k0 > hi || k0 + 31 < lo) continue;                 // uniform in the wave
+        f32x4 s[kQT][2];
+#pragma unroll
+        for (int tt = 0; tt < 2; ++tt) {
+#pragma unroll
+          for (int t = 0; t < kQT; ++t) s[t][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int ks = 0; ks < DKS; ++ks) {
+            const u32x4 kf = *(const u32x4*)(ldsk + (sub + tt * 16 + l16) * Stage::kK + ks * 32 + g * 8);
+#pragma unroll
+            for (int t = 0; t < kQT; ++t) s[t][tt] = mfma_bf16(kf, qf[t][ks], s[t][tt]);
           }
-          mx = fmaxf(mx, p[i]);
         }
-        mx = fmaxf(mx, lane_xor16(mx));
-        mx = fmaxf(mx, lane_xor32(mx));
-        const float mn = fmaxf(m[t], mx);
-        const float ms = mn == -INFINITY ? 0.f : mn;   // a query whose window starts later
-        const float f = __builtin_amdgcn_exp2f(m[t] - ms);
-        float sum = 0.f;
-  #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          p[i] = __builtin_amdgcn_exp2f(p[i] - ms);
-          sum += p[i];
+        // every query of the wave sees all 32 keys: no masks
+        const bool inner = k0 + 31 <= rel + w0 &&
+                           (a.window <= 0 || k0 > rel + w0 + 16 * kQT - 1 - a.window);
+        u32x4 pf[kQT];
+#pragma unroll
+        for (int t = 0; t < kQT; ++t) {
+          float p[8], mx = -INFINITY;
+#pragma unroll
+          for (int i = 0; i < 8; ++i) p[i] = s[t][i >> 2][i & 3] * sc;
+          if (!inner) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+              const int back = qpos[t] - (k0 + step_key(g, i));
+              if (back < 0 || (a.window > 0 && back >= a.window)) p[i] = -INFINITY;
+            }
+          }
+#pragma unroll
+          for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+          mx = fmaxf(mx, lane_xor16(mx));
+          mx = fmaxf(mx, lane_xor32(mx));
+          const float mn = fmaxf(m[t], mx);
+          const float ms = mn == -INFINITY ? 0.f : mn;          // a query whose window starts later
+          const float f = __builtin_amdgcn_exp2f(m[t] - ms);
+          float sum = 0.f;
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            p[i] = __builtin_amdgcn_exp2f(p[i] - ms);
+            sum += p[i];
+          }
+          l[t] = l[t] * f + sum;
+          m[t] = mn;
+          if (__any(f != 1.f)) {
+#pragma unroll
+            for (int i = 0; i < VCB * 8; ++i) o[t][i] *= f;
+          }
+          pf[t] = u32x4{pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                        pack_bf16(p[6], p[7])};
         }
-        l[t] = l[t] * f + sum;
-        m[t] = mn;
-        if (__any(f != 1.f)) {
-  #pragma unroll
-          for (int i = 0; i < VCB * 8; ++i) o[t][i] *= f;
-        }
-        pf[t] = u32x4{pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
-                      pack_bf16(p[6], p[7])};
-      }
-  #pragma unroll
-      for (int cb = 0; cb < VCB; ++cb) {
-        const int col = cb * 128 + l16 * 8;
-        const uint16_t* vc = vbase + (col < a.V ? col : 0);
-        u32x4 v[8];
-  #pragma unroll
-        for (int i = 0; i < 8; ++i)
-          v[i] = *(const u32x4*)(vc + (int64_t)min(k0 + step_key(g, i), hi) * a.kv_st);
-  #pragma unroll
-        for (int c = 0; c < 8; ++c) {
-          const u32x4 vf = column_of(v, c);
-  #pragma unroll
-          for (int t = 0; t < kQT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
+#pragma unroll
+        for (int cb = 0; cb < VCB; ++cb) {
+          u32x4 v[8];
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            v[i] = *(const u32x4*)(ldsv + (sub + step_key(g, i)) * Stage::kV + cb * 128 + l16 * 8);
+#pragma unroll
+          for (int c = 0; c < 8; ++c) {
+            const u32x4 vf = column_of(v, c);
+#pragma unroll
+            for (int t = 0; t < kQT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
+          }
         }
       }
     }
-  #pragma unroll
+#pragma unroll
     for (int t = 0; t < kQT; ++t) {
       float lt = l[t];
       lt += lane_xor16(lt);
@@ -649,20 +693,33 @@ __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
       const int qi = w0 + t * 16 + l16;
       if (qi >= nq) continue;
       uint16_t* out = a.out + ((int64_t)(q0 + qi) * a.H + h) * a.V;
-  #pragma unroll
+#pragma unroll
       for (int cb = 0; cb < VCB; ++cb)
-  #pragma unroll
+#pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int col = cb * 128 + (4 * g + i) * 8;
           if (col < a.V) {
             float r[8];
-  #pragma unroll
+#pragma unroll
             for (int c = 0; c < 8; ++c) r[c] = o[t][cb * 8 + c][i] * inv;
             Vec8<BF16>::st(out, col, r);
           }
         }
     }
   }
+}
+
+template <int DKS, int VCB, int kQT> int launch_latent_tiles(const TilesArgs& a, hipStream_t st) {
+  constexpr int smem = TileStage<DKS, VCB>::kBytes;
+  if (smem > 64 * 1024 &&
+      hipFuncSetAttribute((const void*)latent_tiles_kernel<DKS, VCB, kQT>,
+                          hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
+    zp_set_error("latent_tiles_attention: cannot reserve %d bytes of LDS", smem);
+    return ZP_EHIP;
+  }
+  hipLaunchKernelGGL((latent_tiles_kernel<DKS, VCB, kQT>), dim3((unsigned)a.T * a.H), dim3(256), smem, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
 }
 
 bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
@@ -852,21 +909,14 @@ extern "C" int zp_latent_tiles_attention(const void* q, const void* k, const voi
              "latent_tiles_attention: unaligned rows or too many tiles");
   TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (uint16_t*)out, tiles, T, H, D, V,
                  window, q_rows, k_rows, q_stride, kv_stride, scale};
-  const dim3 grid((unsigned)T * H);
   hipStream_t st = (hipStream_t)stream;
-#define ZP_TILES(DK, VC, QT) \
-  hipLaunchKernelGGL((latent_tiles_kernel<DK, VC, QT>), grid, dim3(256), 0, st, a)
   const int dk = D / 32;
   if (V <= 128) {
-    if (dk <= 2) ZP_TILES(2, 1, 2);
-    else if (dk <= 4) ZP_TILES(4, 1, 2);
-    else if (dk <= 6) ZP_TILES(6, 1, 2);
-    else ZP_TILES(8, 1, 2);
-  } else {
-    if (dk <= 4) ZP_TILES(4, 2, 1);
-    else ZP_TILES(8, 2, 1);
+    if (dk <= 2) return launch_latent_tiles<2, 1, 2>(a, st);
+    if (dk <= 4) return launch_latent_tiles<4, 1, 2>(a, st);
+    if (dk <= 6) return launch_latent_tiles<6, 1, 2>(a, st);
+    return launch_latent_tiles<8, 1, 2>(a, st);
   }
-#undef ZP_TILES
-  ZP_LAUNCH_CHECK();
-  return ZP_OK;
+  if (dk <= 4) return launch_latent_tiles<4, 2, 1>(a, st);
+  return launch_latent_tiles<8, 2, 1>(a, st);
 }
