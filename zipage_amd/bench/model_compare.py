@@ -32,26 +32,25 @@ def shapes(size: str):
 
 
 def throughput(shape, batch: int, prompt: int, out_tokens: int) -> dict:
-    """One generate() call per figure: all prompts in one prefill step, then decode steps."""
+    """One generate() call per figure: prefill in steps of up to 32768 tokens, then decode steps."""
     from zipage_amd.engine import EngineConfig, SamplingParams, ZipageEngine
     total = prompt + out_tokens
     per = -(-total // 256) + 1
     cfg = EngineConfig(shape=shape, max_concurrency=batch, max_num_seqs=batch, num_kvcache_blocks=batch * per + 8,
                        max_cache_blocks_per_seq=per, max_model_len=total + 1, kvcache_block_size=256,
-                       max_num_batched_tokens=batch * prompt)
+                       max_num_batched_tokens=32768)
     eng = ZipageEngine(cfg)
     g = torch.Generator().manual_seed(0)
     prompts = torch.randint(0, shape.vocab, (batch, prompt), generator=g).tolist()
     run = lambda n: eng.generate(prompts, SamplingParams(max_tokens=n, ignore_eos=True))
-    eng.runner.reserve_token_log(out_tokens + 1)
-    run(3)                                    # products, graphs and allocator warm up
+    run(out_tokens)                           # products, graphs and allocator warm up
     for k in ("prefill_s", "decode_s", "decode_tokens", "decode_steps", "prefill_tokens"):
         eng.stats[k] = 0
     run(out_tokens)
     st = eng.stats
     # the step alone: replays of the decode graph at the last step's inputs
     r = eng.runner
-    (g_, _, _), = [v for k, v in r._graphs.items()]
+    g_ = r._graphs[max(r._graphs)][0]
     torch.cuda.synchronize()
     t0 = time.perf_counter()
     with torch.cuda.stream(r.run_stream):

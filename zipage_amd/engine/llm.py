@@ -25,7 +25,7 @@ class ZipageEngine:
         self.cfg = cfg
         self.runner = ModelRunner(cfg, device)
         self.scheduler = Scheduler(cfg)
-        self.stats = dict(prefill_s=0.0, decode_s=0.0, decode_tokens=0, decode_steps=0,
+        self.stats = dict(prefill_s=0.0, decode_s=0.0, decode_tokens=0, decode_steps=0, mixed_decode_tokens=0,
                           prefill_tokens=0, compress_calls=0, compress_seqs=0)
         self._inflight: tuple[torch.cuda.Event, list[Sequence]] | None = None
         self._pending_fetch: list[tuple[Sequence, torch.Tensor]] = []
@@ -102,16 +102,19 @@ class ZipageEngine:
             return 0
         decoded = sum(p.start >= p.seq.num_prompt_tokens for p in portions)
         prompt = sum(p.count for p in portions if p.start < p.seq.num_prompt_tokens)
-        if decoded and self.stats["decode_steps"] == 0:
-            self._t_decode0 = perf_counter()
+        if decoded and not prompt and self.stats["decode_steps"] == 0:
+            self._t_decode0, self._prefill_s0 = perf_counter(), self.stats["prefill_s"]
         tok = self.runner.run_portions(portions)
         for p in portions:
             self.scheduler.pool.computed(p.seq, p.start + p.count, lookback)
         if tok is not None:
             self._finish_step([p.seq for p in portions if p.ends], tok)
         self.stats["prefill_tokens"] += prompt
-        self.stats["decode_tokens"] += decoded
-        self.stats["decode_steps"] += decoded > 0
+        if prompt:                                # timed as prefill: its decoded tokens count apart
+            self.stats["mixed_decode_tokens"] += decoded
+        else:
+            self.stats["decode_tokens"] += decoded
+            self.stats["decode_steps"] += 1
         return prompt or -decoded
 
     # ------------------------------------------------------------------ given tokens
@@ -217,10 +220,12 @@ class ZipageEngine:
                 torch.cuda.synchronize(dev)       # prefill is timed on its own
                 self.stats["prefill_s"] += perf_counter() - t0
             elif self.stats["decode_steps"] == 1 and n < 0 and not self.runner.model.portions:
-                self._t_decode0 = t0
+                self._t_decode0, self._prefill_s0 = t0, self.stats["prefill_s"]
         torch.cuda.synchronize(dev)
         if self.stats["decode_steps"]:
             self.stats["decode_s"] = perf_counter() - self._t_decode0
+            if self.runner.model.portions:        # prompts that arrived between decode steps
+                self.stats["decode_s"] -= self.stats["prefill_s"] - self._prefill_s0
         self.stats["compress_s"] = self.runner.compress_seconds()
         for seq, host in self._pending_fetch:
             seq.token_ids = seq.token_ids[:seq.num_prompt_tokens] + host.tolist()
