@@ -20,12 +20,12 @@ int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* e
                   int32_t norm_width, int64_t vocab, int64_t max_positions, float eps,
                   float weight_offset, int32_t dtype, void* stream);
 
-/* r = x + y (x fp32, y of dtype), written to `result` when given; with a depth average
+/* r = x + the sum of y's n_y planes (x (n, width) fp32; y (n_y, n, width) of dtype), written to `result` when given; with a depth average
  * r <- mix[n_hist] * r + sum_{j < n_hist} mix[j] * hist[j] (hist: planes of (n, width) fp32,
  * hist_plane elements apart); written to `x_out` when given; with norm_weight also
  * out = rmsnorm(r) * (weight_offset + norm_weight) * out_scale.  mix NULL: no average. */
-int zp_residual_norm(const float* x, const void* y, const float* hist, int64_t hist_plane,
-                     const float* mix, int32_t n_hist, float* result, float* x_out,
+int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* hist,
+                     int64_t hist_plane, const float* mix, int32_t n_hist, float* result, float* x_out,
                      const float* norm_weight, void* out, int32_t n, int32_t width,
                      int32_t norm_width, float eps, float weight_offset, float out_scale,
                      int32_t dtype, void* stream);

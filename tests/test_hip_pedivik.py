@@ -77,6 +77,9 @@ def test_residual_norm(dev, dtype, n, width, norm_width, planes):
         _close(after, want, F32)
         normed = O.rms(want[:, :norm_width], 1e-3) * (offset + w.double()[:norm_width]) * scale
         _close(h[:, :norm_width], normed, dtype)
+    parts = torch.stack([y * 0.25, y * 0.5, y * 0.25])       # planes of partial sums: exact halves
+    residual_norm(x, parts, None, 1e-3, norm_width, x_out=after, history=hist, mix=mix)
+    _close(after, want, F32)
     inplace = x.clone()
     assert residual_norm(inplace, y, None, 1e-3, norm_width, x_out=inplace, history=hist, mix=mix) is None
     _close(inplace, want, F32)
@@ -94,6 +97,31 @@ def test_xielu(dev, dtype):
     eps = {BF16: 2.0 ** -8, F32: 2.0 ** -20}[dtype]
     z = z.double().cpu()          # for z < 0 the two terms cancel near one point: measure against z there
     assert ((got - want).abs() <= eps * torch.where(z < -0.125, z.abs(), want.abs()) + 1e-30).all()
+
+
+@pytest.mark.parametrize("n", [1, 7, 64, 1024, 1030])
+def test_residual_linear_in_parts(dev, n):
+    """A long contraction in parts and whole, against fp64; captured into a graph and replayed."""
+    from zipage_amd.layers.linear import ResidualLinear
+    w, x = _rand(dev, BF16, 96, 8192, seed=1, std=0.02), _rand(dev, BF16, n, 8192, seed=2)
+    lin = ResidualLinear(w)
+    planes = lin.forward(x)
+    assert planes.shape == (4 if n <= 1024 else 1, n, 96)
+    want = x.double().cpu() @ w.double().cpu().T
+    _close(planes.double().sum(0), want, BF16)
+    assert ResidualLinear(w[:, :4000].contiguous()).parts is None and ResidualLinear(w.float()).parts is None
+    s = torch.cuda.Stream()
+    s.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(s):
+        g = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(g, stream=s):
+            held = lin.forward(x)
+        for i in range(4):
+            x.copy_(_rand(dev, BF16, n, 8192, seed=10 + i))
+            eager = lin.forward(x)
+            g.replay()
+            s.synchronize()
+            assert torch.equal(held, eager), i
 
 
 # ------------------------------------------------------------------ latent pieces

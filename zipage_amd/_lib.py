@@ -89,7 +89,7 @@ EXPORTS = sorted(list(SIGNATURES) + list(I64_RETURNING) + ["zp_abi_version", "zp
 # the model-side library, in the order of include/zipage_models.h
 MODEL_SIGNATURES = {
     "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, i32, ptr],
-    "zp_residual_norm": [ptr, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32, f32,
+    "zp_residual_norm": [ptr, ptr, i32, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32, f32,
                          i32, ptr],
     "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
     "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, f32, i32, ptr],

@@ -54,6 +54,7 @@ def generate(args) -> int:
 def trace(args) -> int:
     size = 64
     eng = _engine(args.model, args.dtype, -(-args.max_tokens // size), size, 4)
+    os.makedirs(args.out, exist_ok=True)
     live = {}
     for line in sys.stdin:
         if not line.strip():

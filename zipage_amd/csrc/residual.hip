@@ -18,7 +18,9 @@ struct RowArgs {
   const void* pos;        // (max_positions, width) T or null
   int64_t vocab, max_positions;
   const float* x;         // (n, width) fp32
-  const void* y;          // (n, width) T
+  const void* y;          // n_y planes of (n, width) T
+  int64_t y_plane;
+  int n_y;
   // depth average: result_new = sum_j mix[j] * hist[j] + mix[n_hist] * (x + y)
   const float* hist;      // n_hist planes of (n, width) fp32
   int64_t hist_plane;     // elements between planes
@@ -66,9 +68,11 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
         }
       } else {
         Vec8<F32>::ld(a.x, at, v[k]);
-        Vec8<T>::ld(a.y, at, r);
+        for (int j = 0; j < a.n_y; ++j) {
+          Vec8<T>::ld(a.y, j * a.y_plane + at, r);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) v[k][i] += r[i];
+          for (int i = 0; i < 8; ++i) v[k][i] += r[i];
+        }
       }
       if (a.result) Vec8<F32>::st(a.result, at, v[k]);
       if (!EMBED && a.mix) {
@@ -200,12 +204,12 @@ extern "C" int zp_embed_norm(const int64_t* tokens, const int32_t* positions, co
   return launch_rows<true>(a, n, dtype, (hipStream_t)stream);
 }
 
-extern "C" int zp_residual_norm(const float* x, const void* y, const float* hist,
+extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* hist,
                                 int64_t hist_plane, const float* mix, int32_t n_hist,
                                 float* result, float* x_out, const float* norm_weight, void* out,
                                 int32_t n, int32_t width, int32_t norm_width, float eps,
                                 float weight_offset, float out_scale, int32_t dtype, void* stream) {
-  ZP_REQUIRE(n >= 0 && width > 0 && norm_width > 0 && norm_width <= width && n_hist >= 0,
+  ZP_REQUIRE(n >= 0 && width > 0 && norm_width > 0 && norm_width <= width && n_hist >= 0 && n_y >= 1,
              "residual_norm: bad dims");
   ZP_MODEL_DTYPE("residual_norm");
   ZP_ROW_WIDTH("residual_norm");
@@ -217,7 +221,7 @@ extern "C" int zp_residual_norm(const float* x, const void* y, const float* hist
                  aligned16(x_out) && aligned16(norm_weight) && aligned16(out),
              "residual_norm: tensors must be 16-byte aligned");
   RowArgs a = {};
-  a.x = x; a.y = y; a.hist = hist; a.hist_plane = hist_plane; a.mix = mix; a.n_hist = n_hist;
+  a.x = x; a.y = y; a.n_y = n_y; a.y_plane = (int64_t)n * width; a.hist = hist; a.hist_plane = hist_plane; a.mix = mix; a.n_hist = n_hist;
   a.result = result; a.x_out = x_out; a.w = norm_weight; a.out = out; a.width = width;
   a.norm_width = norm_width; a.eps = eps; a.offset = weight_offset; a.out_scale = out_scale;
   return launch_rows<false>(a, n, dtype, (hipStream_t)stream);

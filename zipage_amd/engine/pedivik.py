@@ -16,6 +16,7 @@ import torch
 import torch.nn.functional as F
 
 from zipage_amd.layers.latent import LatentAttention
+from zipage_amd.layers.linear import ResidualLinear
 from zipage_amd.layers.residual import embed_norm, residual_norm, xielu
 
 
@@ -138,7 +139,7 @@ class Pedivik:
                 ffp = -(-l.ff // 8) * 8
                 p["norm2"] = vec(pre + "norm2")
                 p["up"] = dev(_pad_to(get(pre + "mlp.up", l.ff, s.width), ffp, W))
-                p["down"] = dev(_pad_to(get(pre + "mlp.down", s.width, l.ff), W, ffp))
+                p["down"] = ResidualLinear(dev(_pad_to(get(pre + "mlp.down", s.width, l.ff), W, ffp)))
                 act = get(pre + "mlp.act", 2).double().tolist()
                 softplus = lambda a: math.log1p(math.exp(-abs(a))) + max(a, 0.0)
                 p["act"] = (softplus(act[0]), 0.5 + softplus(act[1]))
@@ -164,7 +165,7 @@ class Pedivik:
             if l.ff is not None:
                 ffp = -(-l.ff // 8) * 8
                 p.update(norm2=zeros(), up=_pad_to(w(l.ff, s.width), ffp, W),
-                         down=_pad_to(w(s.width, l.ff), W, ffp), act=(0.8, 1.3))
+                         down=ResidualLinear(_pad_to(w(s.width, l.ff), W, ffp)), act=(0.8, 1.3))
             self.layers.append(p)
 
     # ------------------------------------------------------------------ cache
@@ -193,7 +194,7 @@ class Pedivik:
             y = mixer.forward(h, self.caches[i], ctx)
             if "up" in p:
                 h = residual_norm(x, y, p["norm2"], s.eps, s.width, weight_offset=1.0, x_out=inner)
-                x, y = inner, F.linear(xielu(F.linear(h, p["up"]), *p["act"]), p["down"])
+                x, y = inner, p["down"].forward(xielu(F.linear(h, p["up"]), *p["act"]))
             h = residual_norm(x, y, norms[i + 1], s.eps, s.width, weight_offset=1.0, out_scale=scales[i + 1],
                               x_out=after, result=history[i + 1], history=history, mix=p["dwa"])
             x = after

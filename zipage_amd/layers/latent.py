@@ -9,6 +9,8 @@ import torch.nn.functional as F
 
 from zipage_amd import _lib
 
+from .linear import ResidualLinear
+
 
 def latent_norm_store(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tensor, q_norm: int,
                       c_norm: int, eps: float, cache: torch.Tensor, slot_mapping: torch.Tensor,
@@ -142,7 +144,7 @@ class LatentAttention:
         self.expand = None
         if dtype == torch.bfloat16 and self.can_expand:
             self.expand = put(torch.cat([uk.flatten(0, 1), uv.flatten(0, 1)]))
-        self.o = put(fit(w["o"].view(W, H, V), self.padded_width, H, self.vdim_p).flatten(1, 2))
+        self.o = ResidualLinear(put(fit(w["o"].view(W, H, V), self.padded_width, H, self.vdim_p).flatten(1, 2)))
 
     def random(self, dtype, device, generator, std: float = 0.02):
         r = lambda *s: torch.empty(*s, dtype=dtype, device=device).normal_(0.0, std, generator=generator)
@@ -157,7 +159,7 @@ class LatentAttention:
     def forward(self, h: torch.Tensor, cache: torch.Tensor, ctx) -> torch.Tensor:
         """h (N, padded width); cache (pages, BS, kv_rank_p) of this layer.  The first
         ctx.context_lens.numel() tokens are attended singly, the rest in the runs of
-        ctx.runs[window]."""
+        ctx.runs[window].  Returns planes of partial sums (see ResidualLinear)."""
         N, H = h.shape[0], self.heads
         singles = ctx.context_lens.numel()
         runs = ctx.runs[self.window] if singles < N else None
@@ -177,4 +179,4 @@ class LatentAttention:
             ol = latent_rows_attention(ql, cache, ctx.block_tables, ctx.context_lens, self.scale, self.window,
                                        ctx.table_rows)
             headwise_linear(ol, self.uv, mixed[:singles])
-        return F.linear(mixed, self.o)
+        return self.o.forward(mixed)

@@ -35,11 +35,12 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
                   norm_width: int, weight_offset: float = 0.0, out_scale: float = 1.0,
                   x_out: torch.Tensor | None = None, result: torch.Tensor | None = None,
                   history: torch.Tensor | None = None, mix: torch.Tensor | None = None):
-    """r = x + y, kept in `result`; with `mix`, r <- mix[-1] r + sum_j mix[j] history[j]; kept in
+    """r = x + y (y also as planes (P, N, width), all of them added), kept in `result`; with `mix`, r <- mix[-1] r + sum_j mix[j] history[j]; kept in
     `x_out`; returns rmsnorm(r) * (weight_offset + norm_weight) * out_scale in y's dtype (None
     without a norm).  history (planes, N, width) fp32, of which the first len(mix) - 1 are read."""
     N, W = x.shape
-    assert x.dtype == torch.float32 and y.shape == x.shape
+    y = y if y.dim() == 3 else y.unsqueeze(0)
+    assert x.dtype == torch.float32 and y.shape[1:] == x.shape
     n_hist, plane = 0, 0
     if mix is not None:
         assert mix.dtype == torch.float32 and mix.is_contiguous()
@@ -49,7 +50,7 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
             plane = history.stride(0)
             assert history.stride(1) == W and history.stride(2) == 1
     out = torch.empty((N, W), dtype=y.dtype, device=x.device) if norm_weight is not None else None
-    _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), _lib.dev_ptr(history if n_hist else None),
+    _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), y.shape[0], _lib.dev_ptr(history if n_hist else None),
                      plane, _lib.dev_ptr(mix), n_hist, _rows(result, W), _rows(x_out, W),
                      _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width, float(eps),
                      float(weight_offset), float(out_scale), _lib.dtype_tag(y), _lib.stream_ptr(x))
