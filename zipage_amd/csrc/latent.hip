@@ -205,218 +205,231 @@ __device__ __forceinline__ int page_of(const RowsArgs& a, int t) {
 // A wave takes 32 keys at a time.  They come from memory once, as whole 256-byte row pieces (lane: 8
 // keys x 8 columns), and stay in registers as the value operand; the key operand (lane: one key, 8
 // columns per MFMA) would touch 16 cache lines per 16 lanes if it were read from memory, so the wave
-// passes the block through an LDS stage of its own.  The next block's pieces are requested as the
-// value products free their registers.  No barrier until the waves meet at the end.
-template <int NCB> struct RowsStage {
+// passes each half of the block through an LDS stage of its own.  The next block's pieces are
+// requested as the value products free their registers.  No barrier until the waves meet at the end.
+template <int NCB> struct RowsLds {
   static constexpr int kStride = NCB * 128 + 8;                  // elements: rows 16 bytes apart in the banks
-  static constexpr int kBytes = 32 * kStride * 2;                // per wave
+  static constexpr int kStage = 16 * kStride * 2;                // bytes per wave: 16 keys
+  static constexpr int kQ = 16 * kStride * 2;                    // bytes per 16 heads
 };
+__host__ __device__ inline int rows_merge_floats(int R) { return 16 * (R + 4) + 32; }   // per wave
 
 template <int NCB>
 __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
-  typedef RowsStage<NCB> Stage;
+  typedef RowsLds<NCB> Lds;
   int* pg = (int*)lds_raw;
   char* const shared = lds_raw + ((a.lds_pages * 4 + 15) & ~15);
-  float* merge = (float*)shared;                                 // after the key loop
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int l16 = lane & 15, g = lane >> 4;
-  uint16_t* stage = (uint16_t*)(shared + wave * Stage::kBytes);
   const int hw = a.hw, kw = 4 / hw, hwi = wave % hw, kwi = wave / hw;
+  uint16_t* const stage = (uint16_t*)(shared + wave * Lds::kStage);
+  uint16_t* const qlds = (uint16_t*)(shared + 4 * Lds::kStage);
   const int hgroups = (a.H + 16 * hw - 1) / (16 * hw);
   int id = blockIdx.x;
   const int split = id % a.splits;
   id /= a.splits;
   const int hg = id % hgroups;
   const int row = id / hgroups;
-  const int head = (hg * hw + hwi) * 16 + l16;
-  const bool head_ok = head < a.H;
+  const int head0 = hg * hw * 16;
   const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
   const int n = min(a.ctx[row], a.NB * a.BS);
   const int lo = a.window > 0 ? max(0, n - a.window) : 0;
-  const int p0 = page_of(a, lo);
+  const int p0 = lo >> a.bs_shift;
   constexpr int KS = 4 * NCB;
-  const int nks = a.R / 32;
 
   if (n > 0) {
-    const int np = page_of(a, n - 1) - p0 + 1;
+    const int np = ((n - 1) >> a.bs_shift) - p0 + 1;
     for (int j = tid; j < np && j < a.lds_pages; j += 256) {
       const int p = a.table[(int64_t)seq * a.NB + p0 + j];
       pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
     }
   }
+  // queries to LDS, zeros past R and past the last head
+  for (int it = tid; it < hw * 16 * NCB * 16; it += 256) {
+    const int hl = it / (NCB * 16), c = (it % (NCB * 16)) * 8;
+    u32x4 v = {0u, 0u, 0u, 0u};
+    if (head0 + hl < a.H && c < a.R)
+      v = *(const u32x4*)((const uint16_t*)a.q + ((int64_t)row * a.H + head0 + hl) * a.R + c);
+    *(u32x4*)(qlds + hl * Lds::kStride + c) = v;
+  }
   __syncthreads();
-  const uint16_t* cache = (const uint16_t*)a.cache;
-  auto key_row = [&](int t) -> const uint16_t* {
-    t = min(max(t, lo), n - 1);
-    const int p = page_of(a, t);
-    return cache + ((int64_t)pg[p - p0] * a.BS + (t - p * a.BS)) * a.R;
-  };
   // R may end inside the last column block: columns past it hold the row's start again, and meet
   // zeros in q or results that are not written
-  auto col_off = [&](int cb) { const int c = cb * 128 + l16 * 8; return c < a.R ? c : 0; };
-
-  u32x4 qf[KS];
-  {
-    const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + (head_ok ? head : 0)) * a.R + g * 8;
+  int col_off[NCB];
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) qf[ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-      if (!head_ok || ks >= nks) qf[ks] = u32x4{0u, 0u, 0u, 0u};
+  for (int cb = 0; cb < NCB; ++cb) {
+    const int c = cb * 128 + l16 * 8;
+    col_off[cb] = (c < a.R ? c : 0) * 2;
   }
   f32x4 o[NCB * 8];
 #pragma unroll
   for (int i = 0; i < NCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
   const float sc = a.scale * 1.44269504088896f;
+  const uint16_t* const qrow = qlds + (hwi * 16 + l16) * Lds::kStride + g * 8;
+  const int mask = a.BS - 1;
+  u32x4 v[NCB][8];
+
+  // Page of the visible keys of block b's half (16 keys lie in one page) and the range its rows are
+  // clamped to: keys outside the visible range repeat a visible row, with weight zero.
+  const char* base[2];
+  int from[2], upto[2];
+  auto locate = [&](int b) {
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      const int h0 = b * 32 + hf * 16;
+      from[hf] = min(max(h0, lo), n - 1);
+      upto[hf] = max(min(h0 + 15, n - 1), from[hf]);
+      if (h0 + 15 < lo) upto[hf] = from[hf] = lo;
+      const int page = __builtin_amdgcn_readfirstlane(pg[(from[hf] >> a.bs_shift) - p0]);
+      base[hf] = (const char*)a.cache + (int64_t)page * a.BS * a.R * 2;
+    }
+  };
+  auto row_off = [&](int b, int i) {                             // bytes into the page
+    const int hf = i >> 2;
+    const int key = min(max(b * 32 + step_key(g, i), from[hf]), upto[hf]);
+    return (uint32_t)((key & mask) * a.R * 2);
+  };
 
   const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = a.splits * kw;
   int b = (lo >> 5) + split * kw + kwi;
   if (b <= b1) {
-    u32x4 v[NCB][8];
-    {
+    locate(b);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const uint16_t* kr = key_row(b * 32 + step_key(g, i));
+    for (int i = 0; i < 8; ++i) {
+      const uint32_t ro = row_off(b, i);
 #pragma unroll
-        for (int cb = 0; cb < NCB; ++cb) v[cb][i] = *(const u32x4*)(kr + col_off(cb));
-      }
+      for (int cb = 0; cb < NCB; ++cb) v[cb][i] = *(const u32x4*)(base[i >> 2] + (ro + col_off[cb]));
     }
-    for (; b <= b1; b += step) {
-      const int k0 = b * 32;
+  }
+  for (; b <= b1; b += step) {
+    const int k0 = b * 32;
+    f32x4 s[2];
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
 #pragma unroll
       for (int cb = 0; cb < NCB; ++cb)
 #pragma unroll
-        for (int i = 0; i < 8; ++i)
-          *(u32x4*)(stage + step_key(g, i) * Stage::kStride + cb * 128 + l16 * 8) = v[cb][i];
+        for (int i = 0; i < 4; ++i)
+          *(u32x4*)(stage + (4 * g + i) * Lds::kStride + cb * 128 + l16 * 8) = v[cb][hf * 4 + i];
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-      f32x4 s[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+      f32x4 even = {0.f, 0.f, 0.f, 0.f}, odd = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks)
+      for (int ks = 0; ks < KS; ks += 2) {
+        even = mfma_bf16(*(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + g * 8),
+                         *(const u32x4*)(qrow + ks * 32), even);
+        odd = mfma_bf16(*(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + 32 + g * 8),
+                        *(const u32x4*)(qrow + ks * 32 + 32), odd);
+      }
+      s[hf] = even + odd;
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+      __builtin_amdgcn_wave_barrier();        // the stage is written again after these reads
+      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    }
+    float p[8], mx = -INFINITY;
 #pragma unroll
-        for (int tt = 0; tt < 2; ++tt)
-          s[tt] = mfma_bf16(*(const u32x4*)(stage + (tt * 16 + l16) * Stage::kStride + ks * 32 + g * 8), qf[ks], s[tt]);
-      __builtin_amdgcn_wave_barrier();        // the next block is staged after these reads
-      float p[8], mx = -INFINITY;
+    for (int i = 0; i < 8; ++i) p[i] = s[i >> 2][i & 3] * sc;
+    if (k0 < lo || k0 + 31 >= n) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const int key = k0 + step_key(g, i);
-        p[i] = (key >= lo && key < n) ? s[i >> 2][i & 3] * sc : -INFINITY;
-        mx = fmaxf(mx, p[i]);
+        if (key < lo || key >= n) p[i] = -INFINITY;
       }
-      mx = fmaxf(mx, lane_xor16(mx));
-      mx = fmaxf(mx, lane_xor32(mx));
-      const float mn = fmaxf(m, mx);          // finite: every block holds a visible key
-      const float f = __builtin_amdgcn_exp2f(m - mn);
-      float sum = 0.f;
+    }
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
-        sum += p[i];
-      }
-      l = l * f + sum;
-      m = mn;
-      if (__any(f != 1.f)) {
+    for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+    mx = fmaxf(mx, lane_xor16(mx));
+    mx = fmaxf(mx, lane_xor32(mx));
+    const float mn = fmaxf(m, mx);            // finite: every block holds a visible key
+    const float f = __builtin_amdgcn_exp2f(m - mn);
+    float sum = 0.f;
 #pragma unroll
-        for (int i = 0; i < NCB * 8; ++i) o[i] *= f;
-      }
-      const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
-                        pack_bf16(p[6], p[7])};
-      // past the last block the keys clamp to the last row
-      const uint16_t* kr[8];
+    for (int i = 0; i < 8; ++i) {
+      p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
+      sum += p[i];
+    }
+    l = l * f + sum;
+    m = mn;
+    if (__any(f != 1.f)) {
 #pragma unroll
-      for (int i = 0; i < 8; ++i) kr[i] = key_row((b + step) * 32 + step_key(g, i));
+      for (int i = 0; i < NCB * 8; ++i) o[i] *= f;
+    }
+    const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                      pack_bf16(p[6], p[7])};
+    const int next = min(b + step, b1);       // after the last block its own rows again, unused
+    locate(next);
+    uint32_t ro[8];
 #pragma unroll
-      for (int cb = 0; cb < NCB; ++cb) {
+    for (int i = 0; i < 8; ++i) ro[i] = row_off(next, i);
 #pragma unroll
-        for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v[cb], t), pf, o[cb * 8 + t]);
+    for (int cb = 0; cb < NCB; ++cb) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) v[cb][i] = *(const u32x4*)(kr[i] + col_off(cb));
-      }
+      for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v[cb], t), pf, o[cb * 8 + t]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[cb][i] = *(const u32x4*)(base[i >> 2] + (ro[i] + col_off[cb]));
     }
   }
   l += lane_xor16(l);
   l += lane_xor32(l);
 
-  // waves that split the keys of the same heads meet in LDS
-  if (kw > 1) {
-    __syncthreads();                                // the stages are used up
-    const int RS = a.R + 4;
-    const int per = 16 * RS + 32;                   // O rows, then max and sum of 16 heads
-    if (kwi > 0) {
-      float* dst = merge + (int64_t)((kwi - 1) * hw + hwi) * per;
-      if (g == 0) { dst[16 * RS + l16] = m; dst[16 * RS + 16 + l16] = l; }
+  // the waves meet in LDS: sums, maxima and partial results per wave, then all threads combine those
+  // that split the keys of a head
+  __syncthreads();                                // stages and queries are used up
+  const int RS = a.R + 4, per = rows_merge_floats(a.R);
+  float* const merge = (float*)shared;
+  {
+    float* const dst = merge + wave * per;
+    if (g == 0) { dst[16 * RS + l16] = m; dst[16 * RS + 16 + l16] = l; }
 #pragma unroll
-      for (int cb = 0; cb < NCB; ++cb)
+    for (int cb = 0; cb < NCB; ++cb)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int col = cb * 128 + (4 * g + i) * 8;
-          if (col < a.R) {
-            float* d = dst + l16 * RS + col;
-            *(f32x4*)d = f32x4{o[cb * 8][i], o[cb * 8 + 1][i], o[cb * 8 + 2][i], o[cb * 8 + 3][i]};
-            *(f32x4*)(d + 4) = f32x4{o[cb * 8 + 4][i], o[cb * 8 + 5][i], o[cb * 8 + 6][i], o[cb * 8 + 7][i]};
-          }
+      for (int i = 0; i < 4; ++i) {
+        const int col = cb * 128 + (4 * g + i) * 8;
+        if (col < a.R) {
+          float* d = dst + l16 * RS + col;
+          *(f32x4*)d = f32x4{o[cb * 8][i], o[cb * 8 + 1][i], o[cb * 8 + 2][i], o[cb * 8 + 3][i]};
+          *(f32x4*)(d + 4) = f32x4{o[cb * 8 + 4][i], o[cb * 8 + 5][i], o[cb * 8 + 6][i], o[cb * 8 + 7][i]};
         }
-    }
-    __syncthreads();
-    if (kwi > 0) return;
-    for (int k = 1; k < kw; ++k) {
-      const float* src = merge + (int64_t)((k - 1) * hw + hwi) * per;
-      const float m2 = src[16 * RS + l16], l2 = src[16 * RS + 16 + l16];
-      const float mn = fmaxf(m, m2);
-      const float ms = mn == -INFINITY ? 0.f : mn;
-      const float f1 = __builtin_amdgcn_exp2f(m - ms), f2 = __builtin_amdgcn_exp2f(m2 - ms);
-      l = l * f1 + l2 * f2;
-      m = mn;
-#pragma unroll
-      for (int cb = 0; cb < NCB; ++cb)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int col = cb * 128 + (4 * g + i) * 8;
-          if (col < a.R) {
-            const float* d = src + l16 * RS + col;
-#pragma unroll
-            for (int t = 0; t < 8; ++t) o[cb * 8 + t][i] = o[cb * 8 + t][i] * f1 + d[t] * f2;
-          }
-        }
-    }
+      }
   }
-  if (!head_ok) return;
-  if (a.splits == 1) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    uint16_t* out = (uint16_t*)a.out + ((int64_t)row * a.H + head) * a.R;
+  __syncthreads();
+  const int pieces = a.R / 8;
+  for (int it = tid; it < hw * 16 * pieces; it += 256) {
+    const int hl = it / pieces, pc = it - hl * pieces, head = head0 + hl;
+    if (head >= a.H) break;
+    const float* src = merge + (hl >> 4) * per;   // wave k * hw + (hl / 16) holds key part k
+    const int at = 16 * RS + (hl & 15);
+    float mx = src[at];
+    for (int k = 1; k < kw; ++k) mx = fmaxf(mx, src[k * hw * per + at]);
+    const float ms = mx == -INFINITY ? 0.f : mx;
+    float sum = 0.f, r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < kw; ++k) {
+      const float* part = src + k * hw * per;
+      const float f = __builtin_amdgcn_exp2f(part[at] - ms);
+      sum += part[at + 16] * f;
+      float x[8];
+      Vec8<F32>::ld(part, (hl & 15) * RS + pc * 8, x);
 #pragma unroll
-    for (int cb = 0; cb < NCB; ++cb)
+      for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
+    }
+    const int64_t item = (int64_t)row * a.H + head;
+    if (a.splits == 1) {
+      const float inv = sum > 0.f ? 1.f / sum : 0.f;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int col = cb * 128 + (4 * g + i) * 8;
-        if (col < a.R) {
-          float r[8];
-#pragma unroll
-          for (int t = 0; t < 8; ++t) r[t] = o[cb * 8 + t][i] * inv;
-          Vec8<BF16>::st(out, col, r);
-        }
+      for (int i = 0; i < 8; ++i) r[i] *= inv;
+      Vec8<BF16>::st(a.out, item * a.R + pc * 8, r);
+    } else {
+      const int64_t slot = item * a.splits + split;
+      Vec8<F32>::st(a.part, slot * a.R + pc * 8, r);
+      if (pc == 0) {
+        float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + slot * 2;
+        ml[0] = mx;
+        ml[1] = sum;
       }
-  } else {
-    const int64_t at = ((int64_t)row * a.H + head) * a.splits + split;
-    float* out = a.part + at * a.R;
-    float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + at * 2;
-    if (g == 0) { ml[0] = m; ml[1] = l; }
-#pragma unroll
-    for (int cb = 0; cb < NCB; ++cb)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int col = cb * 128 + (4 * g + i) * 8;
-        if (col < a.R) {
-          float r[8];
-#pragma unroll
-          for (int t = 0; t < 8; ++t) r[t] = o[cb * 8 + t][i];
-          Vec8<F32>::st(out, col, r);
-        }
-      }
+    }
   }
 }
 
@@ -746,10 +759,9 @@ int rows_splits(int n, int H, int R, int window, int NB, int BS) {
 }
 
 template <int NCB> int launch_latent_rows(RowsArgs a, hipStream_t st) {
-  const int kw = 4 / a.hw;
-  size_t merge = kw > 1 ? sizeof(float) * (size_t)(kw - 1) * a.hw * (16 * (a.R + 4) + 32) : 0;
-  if (merge < 4 * (size_t)RowsStage<NCB>::kBytes) merge = 4 * RowsStage<NCB>::kBytes;
-  const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + merge;
+  const size_t merge = 4 * sizeof(float) * (size_t)rows_merge_floats(a.R);
+  const size_t work = 4 * RowsLds<NCB>::kStage + (size_t)a.hw * RowsLds<NCB>::kQ;
+  const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + (merge > work ? merge : work);
   if (smem > 64 * 1024 &&
       hipFuncSetAttribute((const void*)latent_rows_kernel<NCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
                           (int)smem) != hipSuccess) {
@@ -870,7 +882,7 @@ extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const 
   int64_t pages = NB;
   if (window > 0 && (window - 1) / BS + 2 < pages) pages = (window - 1) / BS + 2;
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == ZP_F32 || R > 512 || pages > kMaxLdsPages) {
+  if (dtype == ZP_F32 || R > 512 || pages > kMaxLdsPages || a.bs_shift < 4) {   // bs_shift -1: not a power of two
     const size_t smem = sizeof(float) * R;
     if (dtype == ZP_BF16)
       hipLaunchKernelGGL((latent_plain_kernel<BF16>), dim3((unsigned)n * H), dim3(256), smem, st, a);
