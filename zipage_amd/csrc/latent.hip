@@ -232,6 +232,14 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
   const int hg = id % hgroups;
   const int row = id / hgroups;
   const int head0 = hg * hw * 16;
+  // queries to LDS, zeros past R and past the last head
+  for (int it = tid; it < hw * 16 * NCB * 16; it += 256) {
+    const int hl = it / (NCB * 16), c = (it % (NCB * 16)) * 8;
+    u32x4 v = {0u, 0u, 0u, 0u};
+    if (head0 + hl < a.H && c < a.R)
+      v = *(const u32x4*)((const uint16_t*)a.q + ((int64_t)row * a.H + head0 + hl) * a.R + c);
+    *(u32x4*)(qlds + hl * Lds::kStride + c) = v;
+  }
   const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
   const int n = min(a.ctx[row], a.NB * a.BS);
   const int lo = a.window > 0 ? max(0, n - a.window) : 0;
@@ -244,14 +252,6 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
       const int p = a.table[(int64_t)seq * a.NB + p0 + j];
       pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
     }
-  }
-  // queries to LDS, zeros past R and past the last head
-  for (int it = tid; it < hw * 16 * NCB * 16; it += 256) {
-    const int hl = it / (NCB * 16), c = (it % (NCB * 16)) * 8;
-    u32x4 v = {0u, 0u, 0u, 0u};
-    if (head0 + hl < a.H && c < a.R)
-      v = *(const u32x4*)((const uint16_t*)a.q + ((int64_t)row * a.H + head0 + hl) * a.R + c);
-    *(u32x4*)(qlds + hl * Lds::kStride + c) = v;
   }
   __syncthreads();
   // R may end inside the last column block: columns past it hold the row's start again, and meet
@@ -396,40 +396,46 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
       }
   }
   __syncthreads();
-  const int pieces = a.R / 8;
-  for (int it = tid; it < hw * 16 * pieces; it += 256) {
-    const int hl = it / pieces, pc = it - hl * pieces, head = head0 + hl;
-    if (head >= a.H) break;
-    const float* src = merge + (hl >> 4) * per;   // wave k * hw + (hl / 16) holds key part k
-    const int at = 16 * RS + (hl & 15);
-    float mx = src[at];
-    for (int k = 1; k < kw; ++k) mx = fmaxf(mx, src[k * hw * per + at]);
+  // per head: the common maximum, each key part's factor (over its maximum's place) and the sum
+  if (tid < hw * 16) {
+    float* const src = merge + (tid >> 4) * per + 16 * RS + (tid & 15);   // wave k * hw + tile: key part k
+    float mx = src[0];
+    for (int k = 1; k < kw; ++k) mx = fmaxf(mx, src[k * hw * per]);
     const float ms = mx == -INFINITY ? 0.f : mx;
-    float sum = 0.f, r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    float sum = 0.f;
+    for (int k = 0; k < kw; ++k) {
+      float* const at = src + k * hw * per;
+      const float f = __builtin_amdgcn_exp2f(at[0] - ms);
+      sum += at[16] * f;
+      at[0] = f;
+    }
+    const float inv = a.splits > 1 ? 1.f : (sum > 0.f ? 1.f / sum : 0.f);
+    for (int k = 0; k < kw; ++k) src[k * hw * per] *= inv;
+    const int head = head0 + tid;
+    if (a.splits > 1 && head < a.H) {
+      float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + (((int64_t)row * a.H + head) * a.splits + split) * 2;
+      ml[0] = mx;
+      ml[1] = sum;
+    }
+  }
+  __syncthreads();
+#pragma unroll 2
+  for (int it = tid; it < hw * 256 * NCB; it += 256) {
+    const int hl = it / (16 * NCB), c = it % (16 * NCB) * 8, head = head0 + hl;
+    if (head >= a.H || c >= a.R) continue;
+    const float* src = merge + (hl >> 4) * per;
+    float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     for (int k = 0; k < kw; ++k) {
       const float* part = src + k * hw * per;
-      const float f = __builtin_amdgcn_exp2f(part[at] - ms);
-      sum += part[at + 16] * f;
+      const float f = part[16 * RS + (hl & 15)];
       float x[8];
-      Vec8<F32>::ld(part, (hl & 15) * RS + pc * 8, x);
+      Vec8<F32>::ld(part, (hl & 15) * RS + c, x);
 #pragma unroll
       for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
     }
     const int64_t item = (int64_t)row * a.H + head;
-    if (a.splits == 1) {
-      const float inv = sum > 0.f ? 1.f / sum : 0.f;
-#pragma unroll
-      for (int i = 0; i < 8; ++i) r[i] *= inv;
-      Vec8<BF16>::st(a.out, item * a.R + pc * 8, r);
-    } else {
-      const int64_t slot = item * a.splits + split;
-      Vec8<F32>::st(a.part, slot * a.R + pc * 8, r);
-      if (pc == 0) {
-        float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + slot * 2;
-        ml[0] = mx;
-        ml[1] = sum;
-      }
-    }
+    if (a.splits == 1) Vec8<BF16>::st(a.out, item * a.R + c, r);
+    else Vec8<F32>::st(a.part, (item * a.splits + split) * a.R + c, r);
   }
 }
 
