@@ -68,6 +68,7 @@ def throughput(shape, batch: int, prompt: int, out_tokens: int) -> dict:
 
 def timed(fn, variants: int, launches: int = 24) -> float:
     """Seconds per call of fn(i): a graph of `launches` calls over `variants` buffer sets."""
+    torch.cuda.synchronize()                  # the inputs were made on another stream
     s = torch.cuda.Stream()
     with torch.cuda.stream(s):
         for i in range(min(variants, 3)):
@@ -165,26 +166,27 @@ def kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dic
                                                slots), k), N * qkv_w * 4)
         del qkvs, kcs
     # ---- decode attention
-    B, ctx_len = decode_batch, prompt
+    ctx_len = prompt
     per = -(-ctx_len // BS)
-    at = f"decode, {B} sequences, context {ctx_len}"
-    k = _sets(B * win * KR * 2)
-    caches = [rnd(B * per, BS, KR) for _ in range(k)]
-    tables = torch.randperm(B * per, device=dev).int().view(B, per)
-    ctx = torch.full((B,), ctx_len, device=dev, dtype=torch.int32)
-    q = rnd(B, H, KR)
-    seen = min(win, ctx_len)
-    put(f"latent_rows_attention, window {win}", at,
-        timed(lambda i: latent_rows_attention(q, caches[i], tables, ctx, D ** -0.5, win), k),
-        B * seen * KR * 2 + 2 * B * H * KR * 2, 4.0 * B * H * seen * KR)
-    del caches
-    k = max(2, _sets(2 * B * ctx_len * HK * D * 2))
-    kcs = [rnd(B * per, BS, HK, D) for _ in range(2 * k)]
-    qd = rnd(B, H, D)
-    put("like: paged_decode_attention", at,
-        timed(lambda i: paged_decode_attention(qd, kcs[2 * i], kcs[2 * i + 1], ctx, tables, D ** -0.5), k),
-        2 * B * ctx_len * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * ctx_len * D)
-    del kcs
+    for B in (64, decode_batch):
+        at = f"decode, {B} sequences, context {ctx_len}"
+        k = _sets(B * win * KR * 2)
+        caches = [rnd(B * per, BS, KR) for _ in range(k)]
+        tables = torch.randperm(B * per, device=dev).int().view(B, per)
+        ctx = torch.full((B,), ctx_len, device=dev, dtype=torch.int32)
+        q = rnd(B, H, KR)
+        seen = min(win, ctx_len)
+        put(f"latent_rows_attention, window {win}", at,
+            timed(lambda i: latent_rows_attention(q, caches[i], tables, ctx, D ** -0.5, win), k),
+            B * seen * KR * 2 + 2 * B * H * KR * 2, 4.0 * B * H * seen * KR)
+        del caches
+        k = max(2, _sets(2 * B * ctx_len * HK * D * 2))
+        kcs = [rnd(B * per, BS, HK, D) for _ in range(2 * k)]
+        qd = rnd(B, H, D)
+        put("like: paged_decode_attention", at,
+            timed(lambda i: paged_decode_attention(qd, kcs[2 * i], kcs[2 * i + 1], ctx, tables, D ** -0.5), k),
+            2 * B * ctx_len * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * ctx_len * D)
+        del kcs
     k = _sets(H * KR * D * 2)
     ws, wv = [rnd(H, KR, D) for _ in range(k)], [rnd(H, D, KR) for _ in range(k)]
     x1, x2 = rnd(B, H, D), rnd(B, H, KR)

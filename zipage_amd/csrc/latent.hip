@@ -200,7 +200,8 @@ __device__ __forceinline__ int page_of(const RowsArgs& a, int t) {
   return a.bs_shift >= 0 ? t >> a.bs_shift : t / a.BS;
 }
 
-// NCB column blocks of 128 cover R.  Workgroup: one token, 16 * hw heads, one key range.
+// NCB column blocks of 128 cover R.  Workgroup: one token, 16 * HT * hw heads, one key range.  A wave
+// computes HT tiles of 16 heads on the same keys: with two, the second tile costs no key or value read.
 //
 // A wave takes 32 keys at a time.  They come from memory once, as whole 256-byte row pieces (lane: 8
 // keys x 8 columns), and stay in registers as the value operand; the key operand (lane: one key, 8
@@ -214,8 +215,8 @@ template <int NCB> struct RowsLds {
 };
 __host__ __device__ inline int rows_merge_floats(int R) { return 16 * (R + 4) + 32; }   // per wave
 
-template <int NCB>
-__global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(RowsArgs a) {
+template <int NCB, int HT>
+__global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
   typedef RowsLds<NCB> Lds;
   int* pg = (int*)lds_raw;
@@ -225,15 +226,15 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
   const int hw = a.hw, kw = 4 / hw, hwi = wave % hw, kwi = wave / hw;
   uint16_t* const stage = (uint16_t*)(shared + wave * Lds::kStage);
   uint16_t* const qlds = (uint16_t*)(shared + 4 * Lds::kStage);
-  const int hgroups = (a.H + 16 * hw - 1) / (16 * hw);
+  const int hgroups = (a.H + 16 * HT * hw - 1) / (16 * HT * hw);
   int id = blockIdx.x;
   const int split = id % a.splits;
   id /= a.splits;
   const int hg = id % hgroups;
   const int row = id / hgroups;
-  const int head0 = hg * hw * 16;
+  const int head0 = hg * hw * HT * 16;
   // queries to LDS, zeros past R and past the last head
-  for (int it = tid; it < hw * 16 * NCB * 16; it += 256) {
+  for (int it = tid; it < hw * HT * 16 * NCB * 16; it += 256) {
     const int hl = it / (NCB * 16), c = (it % (NCB * 16)) * 8;
     u32x4 v = {0u, 0u, 0u, 0u};
     if (head0 + hl < a.H && c < a.R)
@@ -246,12 +247,10 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
   const int p0 = lo >> a.bs_shift;
   constexpr int KS = 4 * NCB;
 
-  if (n > 0) {
-    const int np = ((n - 1) >> a.bs_shift) - p0 + 1;
-    for (int j = tid; j < np && j < a.lds_pages; j += 256) {
-      const int p = a.table[(int64_t)seq * a.NB + p0 + j];
-      pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
-    }
+  // every entry gets a valid page, whatever the context length says: no address rests on it
+  for (int j = tid; j < a.lds_pages; j += 256) {
+    const int p = p0 + j < a.NB ? a.table[(int64_t)seq * a.NB + p0 + j] : 0;
+    pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
   }
   __syncthreads();
   // R may end inside the last column block: columns past it hold the row's start again, and meet
@@ -262,12 +261,17 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
     const int c = cb * 128 + l16 * 8;
     col_off[cb] = (c < a.R ? c : 0) * 2;
   }
-  f32x4 o[NCB * 8];
+  f32x4 o[HT][NCB * 8];
+  float m[HT], l[HT];
 #pragma unroll
-  for (int i = 0; i < NCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  for (int ht = 0; ht < HT; ++ht) {
+    m[ht] = -INFINITY;
+    l[ht] = 0.f;
+#pragma unroll
+    for (int i = 0; i < NCB * 8; ++i) o[ht][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
   const float sc = a.scale * 1.44269504088896f;
-  const uint16_t* const qrow = qlds + (hwi * 16 + l16) * Lds::kStride + g * 8;
+  const uint16_t* const qrow = qlds + (hwi * HT * 16 + l16) * Lds::kStride + g * 8;
   const int mask = a.BS - 1;
   u32x4 v[NCB][8];
 
@@ -305,7 +309,7 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
   }
   for (; b <= b1; b += step) {
     const int k0 = b * 32;
-    f32x4 s[2];
+    f32x4 s[HT][2];
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf) {
 #pragma unroll
@@ -316,49 +320,56 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-      f32x4 even = {0.f, 0.f, 0.f, 0.f}, odd = {0.f, 0.f, 0.f, 0.f};
+      f32x4 part[HT][2];                      // even and odd steps: two chains per head tile
 #pragma unroll
-      for (int ks = 0; ks < KS; ks += 2) {
-        even = mfma_bf16(*(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + g * 8),
-                         *(const u32x4*)(qrow + ks * 32), even);
-        odd = mfma_bf16(*(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + 32 + g * 8),
-                        *(const u32x4*)(qrow + ks * 32 + 32), odd);
+      for (int ht = 0; ht < HT; ++ht) part[ht][0] = part[ht][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const u32x4 kf = *(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + g * 8);
+#pragma unroll
+        for (int ht = 0; ht < HT; ++ht)
+          part[ht][ks & 1] = mfma_bf16(kf, *(const u32x4*)(qrow + ht * 16 * Lds::kStride + ks * 32), part[ht][ks & 1]);
       }
-      s[hf] = even + odd;
+#pragma unroll
+      for (int ht = 0; ht < HT; ++ht) s[ht][hf] = part[ht][0] + part[ht][1];
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
       __builtin_amdgcn_wave_barrier();        // the stage is written again after these reads
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
     }
-    float p[8], mx = -INFINITY;
+    u32x4 pf[HT];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) p[i] = s[i >> 2][i & 3] * sc;
-    if (k0 < lo || k0 + 31 >= n) {
+    for (int ht = 0; ht < HT; ++ht) {
+      float p[8], mx = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) p[i] = s[ht][i >> 2][i & 3] * sc;
+      if (k0 < lo || k0 + 31 >= n) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const int key = k0 + step_key(g, i);
+          if (key < lo || key >= n) p[i] = -INFINITY;
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+      mx = fmaxf(mx, lane_xor16(mx));
+      mx = fmaxf(mx, lane_xor32(mx));
+      const float mn = fmaxf(m[ht], mx);      // finite: every block holds a visible key
+      const float f = __builtin_amdgcn_exp2f(m[ht] - mn);
+      float sum = 0.f;
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        const int key = k0 + step_key(g, i);
-        if (key < lo || key >= n) p[i] = -INFINITY;
+        p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
+        sum += p[i];
       }
-    }
+      l[ht] = l[ht] * f + sum;
+      m[ht] = mn;
+      if (__any(f != 1.f)) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
-    mx = fmaxf(mx, lane_xor16(mx));
-    mx = fmaxf(mx, lane_xor32(mx));
-    const float mn = fmaxf(m, mx);            // finite: every block holds a visible key
-    const float f = __builtin_amdgcn_exp2f(m - mn);
-    float sum = 0.f;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
-      sum += p[i];
+        for (int i = 0; i < NCB * 8; ++i) o[ht][i] *= f;
+      }
+      pf[ht] = u32x4{pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                     pack_bf16(p[6], p[7])};
     }
-    l = l * f + sum;
-    m = mn;
-    if (__any(f != 1.f)) {
-#pragma unroll
-      for (int i = 0; i < NCB * 8; ++i) o[i] *= f;
-    }
-    const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
-                      pack_bf16(p[6], p[7])};
     const int next = min(b + step, b1);       // after the last block its own rows again, unused
     locate(next);
     uint32_t ro[8];
@@ -367,75 +378,84 @@ __global__ __launch_bounds__(256, NCB <= 2 ? 2 : 1) void latent_rows_kernel(Rows
 #pragma unroll
     for (int cb = 0; cb < NCB; ++cb) {
 #pragma unroll
-      for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(v[cb], t), pf, o[cb * 8 + t]);
+      for (int t = 0; t < 8; ++t) {
+        const u32x4 vf = column_of(v[cb], t);
+#pragma unroll
+        for (int ht = 0; ht < HT; ++ht) o[ht][cb * 8 + t] = mfma_bf16(vf, pf[ht], o[ht][cb * 8 + t]);
+      }
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[cb][i] = *(const u32x4*)(base[i >> 2] + (ro[i] + col_off[cb]));
     }
   }
-  l += lane_xor16(l);
-  l += lane_xor32(l);
 
-  // the waves meet in LDS: sums, maxima and partial results per wave, then all threads combine those
-  // that split the keys of a head
-  __syncthreads();                                // stages and queries are used up
+  // the waves meet in LDS, one head tile of each at a time: sums, maxima and partial results per
+  // wave, then all threads combine those that split the keys of a head
   const int RS = a.R + 4, per = rows_merge_floats(a.R);
   float* const merge = (float*)shared;
-  {
-    float* const dst = merge + wave * per;
-    if (g == 0) { dst[16 * RS + l16] = m; dst[16 * RS + 16 + l16] = l; }
 #pragma unroll
-    for (int cb = 0; cb < NCB; ++cb)
+  for (int ht = 0; ht < HT; ++ht) {
+    l[ht] += lane_xor16(l[ht]);
+    l[ht] += lane_xor32(l[ht]);
+    __syncthreads();                              // what the LDS held before is used up
+    {
+      float* const dst = merge + wave * per;
+      if (g == 0) { dst[16 * RS + l16] = m[ht]; dst[16 * RS + 16 + l16] = l[ht]; }
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int col = cb * 128 + (4 * g + i) * 8;
-        if (col < a.R) {
-          float* d = dst + l16 * RS + col;
-          *(f32x4*)d = f32x4{o[cb * 8][i], o[cb * 8 + 1][i], o[cb * 8 + 2][i], o[cb * 8 + 3][i]};
-          *(f32x4*)(d + 4) = f32x4{o[cb * 8 + 4][i], o[cb * 8 + 5][i], o[cb * 8 + 6][i], o[cb * 8 + 7][i]};
+      for (int cb = 0; cb < NCB; ++cb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = cb * 128 + (4 * g + i) * 8;
+          if (col < a.R) {
+            float* d = dst + l16 * RS + col;
+            const f32x4* t = o[ht] + cb * 8;
+            *(f32x4*)d = f32x4{t[0][i], t[1][i], t[2][i], t[3][i]};
+            *(f32x4*)(d + 4) = f32x4{t[4][i], t[5][i], t[6][i], t[7][i]};
+          }
         }
+    }
+    __syncthreads();
+    // per head: the common maximum, each key part's factor (over its maximum's place) and the sum
+    if (tid < hw * 16) {
+      float* const src = merge + (tid >> 4) * per + 16 * RS + (tid & 15);   // wave k * hw + tile: key part k
+      float mx = src[0];
+      for (int k = 1; k < kw; ++k) mx = fmaxf(mx, src[k * hw * per]);
+      const float ms = mx == -INFINITY ? 0.f : mx;
+      float sum = 0.f;
+      for (int k = 0; k < kw; ++k) {
+        float* const at = src + k * hw * per;
+        const float f = __builtin_amdgcn_exp2f(at[0] - ms);
+        sum += at[16] * f;
+        at[0] = f;
       }
-  }
-  __syncthreads();
-  // per head: the common maximum, each key part's factor (over its maximum's place) and the sum
-  if (tid < hw * 16) {
-    float* const src = merge + (tid >> 4) * per + 16 * RS + (tid & 15);   // wave k * hw + tile: key part k
-    float mx = src[0];
-    for (int k = 1; k < kw; ++k) mx = fmaxf(mx, src[k * hw * per]);
-    const float ms = mx == -INFINITY ? 0.f : mx;
-    float sum = 0.f;
-    for (int k = 0; k < kw; ++k) {
-      float* const at = src + k * hw * per;
-      const float f = __builtin_amdgcn_exp2f(at[0] - ms);
-      sum += at[16] * f;
-      at[0] = f;
+      const float inv = a.splits > 1 ? 1.f : (sum > 0.f ? 1.f / sum : 0.f);
+      for (int k = 0; k < kw; ++k) src[k * hw * per] *= inv;
+      const int head = head0 + ((tid >> 4) * HT + ht) * 16 + (tid & 15);
+      if (a.splits > 1 && head < a.H) {
+        float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + (((int64_t)row * a.H + head) * a.splits + split) * 2;
+        ml[0] = mx;
+        ml[1] = sum;
+      }
     }
-    const float inv = a.splits > 1 ? 1.f : (sum > 0.f ? 1.f / sum : 0.f);
-    for (int k = 0; k < kw; ++k) src[k * hw * per] *= inv;
-    const int head = head0 + tid;
-    if (a.splits > 1 && head < a.H) {
-      float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.R + (((int64_t)row * a.H + head) * a.splits + split) * 2;
-      ml[0] = mx;
-      ml[1] = sum;
-    }
-  }
-  __syncthreads();
-#pragma unroll 2
-  for (int it = tid; it < hw * 256 * NCB; it += 256) {
-    const int hl = it / (16 * NCB), c = it % (16 * NCB) * 8, head = head0 + hl;
-    if (head >= a.H || c >= a.R) continue;
-    const float* src = merge + (hl >> 4) * per;
-    float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < kw; ++k) {
-      const float* part = src + k * hw * per;
-      const float f = part[16 * RS + (hl & 15)];
-      float x[8];
-      Vec8<F32>::ld(part, (hl & 15) * RS + c, x);
+    __syncthreads();
+#pragma unroll 1
+    for (int it = tid; it < hw * 256 * NCB; it += 256) {
+      const int hl = it / (16 * NCB), c = it % (16 * NCB) * 8;
+      const int head = head0 + ((hl >> 4) * HT + ht) * 16 + (hl & 15);
+      if (head >= a.H || c >= a.R) continue;
+      const float* src = merge + (hl >> 4) * per;
+      float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k < kw; ++k) {
+        const float* part = src + k * hw * per;
+        const float f = part[16 * RS + (hl & 15)];
+        float x[8];
+        Vec8<F32>::ld(part, (hl & 15) * RS + c, x);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
+        for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
+      }
+      const int64_t item = (int64_t)row * a.H + head;
+      if (a.splits == 1) Vec8<BF16>::st(a.out, item * a.R + c, r);
+      else Vec8<F32>::st(a.part, (item * a.splits + split) * a.R + c, r);
     }
-    const int64_t item = (int64_t)row * a.H + head;
-    if (a.splits == 1) Vec8<BF16>::st(a.out, item * a.R + c, r);
-    else Vec8<F32>::st(a.part, (item * a.splits + split) * a.R + c, r);
   }
 }
 
@@ -566,7 +586,7 @@ __global__ __launch_bounds__(256, 2) void latent_tiles_kernel(TilesArgs a) {
   const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
   const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
   // host-made descriptors: rows outside the buffers are not touched
-  if (q0 < 0 || kb < 0 || rel < 0 || q0 + nq > a.q_rows || kb + rel + nq > a.k_rows) return;
+  if (q0 < 0 || kb < 0 || rel < 0 || (int64_t)q0 + nq > a.q_rows || (int64_t)kb + rel + nq > a.k_rows) return;
   const int nks = a.D / 32;
   const float sc = a.scale * 1.44269504088896f;
   const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + h * a.D;
@@ -745,37 +765,39 @@ bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
 
 constexpr int kMaxLdsPages = 4096;
 
-int rows_hw(int H) {
-  const int tiles = (H + 15) / 16;
+// Head tiles per wave, and waves of a workgroup on different heads.
+int rows_ht(int H, int R) { return H > 16 && R <= 256 ? 2 : 1; }   // registers hold 2 x 256 columns
+int rows_hw(int H, int R) {
+  const int tiles = (H + 16 * rows_ht(H, R) - 1) / (16 * rows_ht(H, R));
   return tiles >= 4 ? 4 : (tiles >= 2 ? 2 : 1);
 }
 
 // Key ranges per token: enough workgroups to cover the chip, at least two 32-key steps per wave.
 int rows_splits(int n, int H, int R, int window, int NB, int BS) {
-  const int hw = rows_hw(H), kw = 4 / hw;
-  const int groups = n * ((H + 16 * hw - 1) / (16 * hw));
+  const int hw = rows_hw(H, R), kw = 4 / hw, per = 16 * rows_ht(H, R) * hw;
+  const int groups = n * ((H + per - 1) / per);
   int64_t keys = (int64_t)NB * BS;
   if (window > 0 && window < keys) keys = window;
   const int steps = (int)((keys + 31) / 32);
-  const int resident = R <= 256 ? 2 : 1;       // workgroups per CU
+  const int resident = (R + 127) / 128 * rows_ht(H, R) <= 2 ? 2 : 1;       // workgroups per CU
   int s = 256 * resident / (groups > 0 ? groups : 1);
   s = s < steps / (2 * kw) ? s : steps / (2 * kw);
   s = s < 32 ? s : 32;
   return s < 1 ? 1 : s;
 }
 
-template <int NCB> int launch_latent_rows(RowsArgs a, hipStream_t st) {
+template <int NCB, int HT> int launch_latent_rows(RowsArgs a, hipStream_t st) {
   const size_t merge = 4 * sizeof(float) * (size_t)rows_merge_floats(a.R);
-  const size_t work = 4 * RowsLds<NCB>::kStage + (size_t)a.hw * RowsLds<NCB>::kQ;
+  const size_t work = 4 * RowsLds<NCB>::kStage + (size_t)a.hw * HT * RowsLds<NCB>::kQ;
   const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + (merge > work ? merge : work);
   if (smem > 64 * 1024 &&
-      hipFuncSetAttribute((const void*)latent_rows_kernel<NCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+      hipFuncSetAttribute((const void*)latent_rows_kernel<NCB, HT>, hipFuncAttributeMaxDynamicSharedMemorySize,
                           (int)smem) != hipSuccess) {
     zp_set_error("latent_rows_attention: cannot reserve %zu bytes of LDS", smem);
     return ZP_EHIP;
   }
-  const int hgroups = (a.H + 16 * a.hw - 1) / (16 * a.hw);
-  hipLaunchKernelGGL((latent_rows_kernel<NCB>), dim3((unsigned)a.n * hgroups * a.splits), dim3(256), smem, st, a);
+  const int hgroups = (a.H + 16 * HT * a.hw - 1) / (16 * HT * a.hw);
+  hipLaunchKernelGGL((latent_rows_kernel<NCB, HT>), dim3((unsigned)a.n * hgroups * a.splits), dim3(256), smem, st, a);
   ZP_LAUNCH_CHECK();
   if (a.splits > 1) {
     hipLaunchKernelGGL(latent_rows_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
@@ -897,16 +919,17 @@ extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const 
     ZP_LAUNCH_CHECK();
     return ZP_OK;
   }
-  a.hw = rows_hw(H);
+  a.hw = rows_hw(H, R);
   a.lds_pages = (int)pages;
   a.splits = rows_splits(n, H, R, window, NB, BS);
   ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_latent_rows_workspace(n, H, R, window, NB, BS, dtype)),
              "latent_rows_attention: workspace too small");
+  const bool two = rows_ht(H, R) == 2;
   switch ((R + 127) / 128) {
-    case 1: return launch_latent_rows<1>(a, st);
-    case 2: return launch_latent_rows<2>(a, st);
-    case 3: return launch_latent_rows<3>(a, st);
-    default: return launch_latent_rows<4>(a, st);
+    case 1: return two ? launch_latent_rows<1, 2>(a, st) : launch_latent_rows<1, 1>(a, st);
+    case 2: return two ? launch_latent_rows<2, 2>(a, st) : launch_latent_rows<2, 1>(a, st);
+    case 3: return launch_latent_rows<3, 1>(a, st);
+    default: return launch_latent_rows<4, 1>(a, st);
   }
 }
 
