@@ -150,7 +150,7 @@ def test_latent_norm_store_and_gather(dev, dtype, q, qp, r, rp):
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=ids)
-@pytest.mark.parametrize("n,H,K,M", [(1, 1, 32, 16), (5, 3, 64, 80), (64, 2, 160, 32), (133, 5, 96, 288)])
+@pytest.mark.parametrize("n,H,K,M", [(1, 1, 32, 16), (5, 3, 64, 80), (64, 2, 160, 32), (133, 5, 96, 288), (300, 37, 64, 160)])
 def test_headwise_linear(dev, dtype, n, H, K, M):
     from zipage_amd.layers.latent import headwise_linear
     x, w = _rand(dev, dtype, n, H, K, seed=1), _rand(dev, dtype, H, M, K, seed=2)

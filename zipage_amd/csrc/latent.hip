@@ -123,18 +123,16 @@ struct HeadArgs {
   void* out;        // (n, H, M) T
   int n, H, K, M;
 };
-constexpr int kTokTiles = 4;
 
-// A wave owns 16 outputs of one head for up to 64 tokens: W is the row operand, so a lane ends
-// with four consecutive outputs of one token.
-template <typename T>
+// A wave owns 16 outputs of one head for 16 * kTokTiles tokens: W is the row operand, so a lane ends
+// with four consecutive outputs of one token.  Token rows past the end repeat the last one.
+template <typename T, int kTokTiles>
 __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
   const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
   const int m0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16;
   const int h = blockIdx.y;
   const int n0 = blockIdx.z * 16 * kTokTiles;
   if (m0 >= a.M) return;
-  const int tiles = min(kTokTiles, (a.n - n0 + 15) / 16);
   f32x4 acc[kTokTiles];
 #pragma unroll
   for (int t = 0; t < kTokTiles; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -146,26 +144,31 @@ __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
   if constexpr (T::bytes == 2) {
     const uint16_t* w = (const uint16_t*)a.w;
     const uint16_t* x = (const uint16_t*)a.in;
-    for (int k = g * 8; k < a.K; k += 32) {
+    const int steps = a.K / 32;
+#pragma unroll 4
+    for (int ks = 0; ks < steps; ++ks) {
+      const int k = ks * 32 + g * 8;
       const u32x4 wf = *(const u32x4*)(w + wrow + k);
 #pragma unroll
-      for (int t = 0; t < kTokTiles; ++t)
-        if (t < tiles) acc[t] = mfma_bf16(wf, *(const u32x4*)(x + xrow[t] + k), acc[t]);
+      for (int t = 0; t < kTokTiles; ++t) acc[t] = mfma_bf16(wf, *(const u32x4*)(x + xrow[t] + k), acc[t]);
     }
   } else {
     const float* w = (const float*)a.w;
     const float* x = (const float*)a.in;
-    for (int k = g; k < a.K; k += 4) {
+    const int steps = a.K / 4;
+#pragma unroll 4
+    for (int ks = 0; ks < steps; ++ks) {
+      const int k = ks * 4 + g;
       const float wf = w[wrow + k];
 #pragma unroll
       for (int t = 0; t < kTokTiles; ++t)
-        if (t < tiles) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf, x[xrow[t] + k], acc[t], 0, 0, 0);
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf, x[xrow[t] + k], acc[t], 0, 0, 0);
     }
   }
 #pragma unroll
   for (int t = 0; t < kTokTiles; ++t) {
     const int n = n0 + t * 16 + l16;
-    if (t < tiles && n < a.n) {
+    if (n < a.n) {
       const int64_t at = ((int64_t)n * a.H + h) * a.M + m0 + g * 4;
       if constexpr (T::bytes == 2) {
         uint2 o;
@@ -866,11 +869,22 @@ extern "C" int zp_headwise_linear(const void* in, const void* w, void* out, int3
   ZP_REQUIRE(in && w && out && aligned16(in) && aligned16(w) && aligned16(out),
              "headwise_linear: null or unaligned pointer");
   HeadArgs a = {in, w, out, n, H, K, M};
-  const dim3 grid((M + 63) / 64, H, (n + 16 * kTokTiles - 1) / (16 * kTokTiles));
+  // as many tokens per wave (W is read once for them) as still leave two workgroups per CU
+  const int64_t columns = (int64_t)((M + 63) / 64) * H;
+  int tt = 4;
+  while (tt > 1 && columns * ((n + 16 * tt - 1) / (16 * tt)) < 512) tt >>= 1;
+  const dim3 grid((M + 63) / 64, H, (n + 16 * tt - 1) / (16 * tt));
   ZP_REQUIRE(grid.z <= 65535, "headwise_linear: too many tokens");
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == ZP_BF16) hipLaunchKernelGGL((headwise_kernel<BF16>), grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((headwise_kernel<F32>), grid, dim3(256), 0, st, a);
+#define ZP_HEADWISE(T)                                                                            \
+  do {                                                                                            \
+    if (tt == 4) hipLaunchKernelGGL((headwise_kernel<T, 4>), grid, dim3(256), 0, st, a);          \
+    else if (tt == 2) hipLaunchKernelGGL((headwise_kernel<T, 2>), grid, dim3(256), 0, st, a);     \
+    else hipLaunchKernelGGL((headwise_kernel<T, 1>), grid, dim3(256), 0, st, a);                  \
+  } while (0)
+  if (dtype == ZP_BF16) ZP_HEADWISE(BF16);
+  else ZP_HEADWISE(F32);
+#undef ZP_HEADWISE
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }
