@@ -100,6 +100,7 @@ def test_xielu(dev, dtype):
 
 
 @pytest.mark.parametrize("n", [1, 7, 64, 1024, 1030])
+@torch.inference_mode()                       # as the engine captures: one process, one kind of graph state
 def test_residual_linear_in_parts(dev, n):
     """A long contraction in parts and whole, against fp64; captured into a graph and replayed."""
     from zipage_amd.layers.linear import ResidualLinear

@@ -66,6 +66,7 @@ def throughput(shape, batch: int, prompt: int, out_tokens: int) -> dict:
             "ms_layers_of_a_decode_step": round(step * 1e3, 3)}
 
 
+@torch.inference_mode()
 def timed(fn, variants: int, launches: int = 24) -> float:
     """Seconds per call of fn(i): a graph of `launches` calls over `variants` buffer sets."""
     torch.cuda.synchronize()                  # the inputs were made on another stream
