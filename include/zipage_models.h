@@ -1,6 +1,8 @@
-/* C ABI of libzipage_models.so: the model-side kernels of decoders that need more than the
- * compression library's layer kernels -- an fp32 residual stream, a depth average, latent
- * attention over pages of latents.  Status codes, dtype tags and conventions are those of
+/* C ABI of the model-side kernels of decoders that need more than the compression library's layer
+ * kernels.  Three shared objects, so that a model compiles only what it runs: libzipage_models.so (an
+ * fp32 residual stream, attention of prompt runs), libzipage_latent.so (latent attention over pages of
+ * latents) and libzipage_hybrid.so (grouped-query attention with sinks, recurrent mixers, mixtures of
+ * experts).  Status codes, dtype tags and conventions are those of
  * zipage_hip.h; every entry point here takes ZP_BF16 or ZP_F32 (true 32-bit products), enqueues on
  * `stream`, allocates nothing and may be captured into a HIP graph. */
 #ifndef ZIPAGE_MODELS_H
@@ -11,21 +13,24 @@
 extern "C" {
 #endif
 
-/* x = embed[tokens] (+ pos[positions] when pos is given), fp32; with norm_weight also
+/* ------------------------------------------------------------------ libzipage_models.so */
+
+/* x = embed[tokens] * embed_scale (+ pos[positions] when pos is given), fp32; with norm_weight also
  * out = x / sqrt(mean(x^2) + eps) * (weight_offset + norm_weight).  Rows are `width` long (multiple
  * of 8, zero padded), the mean runs over norm_width.  embed (vocab, width), pos (max_positions,
  * width) and out are of `dtype`; indices are clamped to the tables. */
 int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* embed, const void* pos,
                   float* x, const float* norm_weight, void* out, int32_t n, int32_t width,
-                  int32_t norm_width, int64_t vocab, int64_t max_positions, float eps,
-                  float weight_offset, int32_t dtype, void* stream);
+                  int32_t norm_width, int64_t vocab, int64_t max_positions,
+                  float embed_scale, float eps, float weight_offset, int32_t dtype, void* stream);
 
-/* r = x + the sum of y's n_y planes (x (n, width) fp32; y (n_y, n, width) of dtype), written to `result` when given; with a depth average
+/* r = x + the sum of y's n_y planes (x (n, width) fp32; y (n_y, n, width) of dtype), where with
+ * y_weight the sum is RMS-normed times y_weight before it is added; written to `result` when given; with a depth average
  * r <- mix[n_hist] * r + sum_{j < n_hist} mix[j] * hist[j] (hist: planes of (n, width) fp32,
  * hist_plane elements apart); written to `x_out` when given; with norm_weight also
  * out = rmsnorm(r) * (weight_offset + norm_weight) * out_scale.  mix NULL: no average. */
-int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* hist,
-                     int64_t hist_plane, const float* mix, int32_t n_hist, float* result, float* x_out,
+int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* y_weight,
+                     const float* hist, int64_t hist_plane, const float* mix, int32_t n_hist, float* result, float* x_out,
                      const float* norm_weight, void* out, int32_t n, int32_t width,
                      int32_t norm_width, float eps, float weight_offset, float out_scale,
                      int32_t dtype, void* stream);
@@ -34,6 +39,29 @@ int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* hi
 int zp_xielu(const void* in, void* out, int64_t count, float alpha_p, float alpha_n, int32_t dtype,
              void* stream);
 
+/* out (fp32) = cap * tanh(in / cap). */
+int zp_softcap(const void* in, float* out, int64_t count, float cap, int32_t dtype, void* stream);
+
+/* out[i] = src[rows[i]], rows of row_bytes (multiple of 16). */
+int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n, int32_t row_bytes,
+                   int64_t num_rows, void* stream);
+
+/* Attention of runs of tokens, bfloat16.  tiles (T, 4) int32, one entry per up to 128 queries of one
+ * sequence: first query row, number of queries, row of the run's first key, position of the first
+ * query counted from that key (key rows of a run are consecutive positions).  Query head h reads key
+ * head h / (H / HK).  A query sees its own position and those before it in the run that lie within
+ * `window` (0: no limit) or, with `chunk`, in its own block of `chunk` positions (the run's first key
+ * starts a block); at most one of the two is set.  sinks (H,) or NULL: a logit per head that joins the
+ * denominator only.  q rows q_stride, k and v rows kv_stride, out rows out_stride elements apart, heads
+ * back to back; out is multiplied by out_scale. */
+int zp_run_attention(const void* q, const void* k, const void* v, void* out, const int32_t* tiles,
+                     const float* sinks, int32_t T, int32_t H, int32_t HK, int32_t D, int32_t V,
+                     int32_t window, int32_t chunk, int64_t q_rows, int64_t k_rows, int64_t q_stride,
+                     int64_t kv_stride, int64_t out_stride, float scale, float out_scale,
+                     int32_t dtype, void* stream);
+
+/* ------------------------------------------------------------------ libzipage_latent.so */
+
 /* in (n, q_width + c_width): the first part RMS-normed times q_weight goes to q_out, the second
  * times c_weight to slot slots[i] of the cache (-1 skips) and to c_out when given.  The means run
  * over q_norm and c_norm elements; widths are multiples of 8, zero padded. */
@@ -41,10 +69,6 @@ int zp_latent_norm_store(const void* in, const float* q_weight, const float* c_w
                          void* c_out, void* cache, const int32_t* slots, int32_t n, int32_t q_width,
                          int32_t c_width, int32_t q_norm, int32_t c_norm, int64_t num_slots, float eps,
                          int32_t dtype, void* stream);
-
-/* out[i] = src[rows[i]], rows of row_bytes (multiple of 16). */
-int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n, int32_t row_bytes,
-                   int64_t num_rows, void* stream);
 
 /* out[n, h, :] = w[h] (M, K) in[n, h, :]; K a multiple of 32, M of 16. */
 int zp_headwise_linear(const void* in, const void* w, void* out, int32_t n, int32_t H, int32_t K,
@@ -63,16 +87,109 @@ int zp_latent_rows_attention(const void* q, const void* cache, const int32_t* ta
                              int32_t num_pages, int32_t window, float scale, int32_t dtype,
                              void* workspace, int64_t workspace_bytes, void* stream);
 
-/* Attention of runs of tokens over expanded keys and values, bfloat16.  tiles (T, 4) int32, one
- * entry per up to 128 queries of one sequence: first query row, number of queries, row of the
- * run's first key, position of the first query counted from that key (key rows of a run are
- * consecutive positions).  A query sees its own position and the window - 1 before it (window 0:
- * all before it in the run).  q rows q_stride, k and v rows kv_stride elements apart; out (rows,
- * H, V). */
-int zp_latent_tiles_attention(const void* q, const void* k, const void* v, void* out,
-                              const int32_t* tiles, int32_t T, int32_t H, int32_t D, int32_t V,
-                              int32_t window, int64_t q_rows, int64_t k_rows, int64_t q_stride,
-                              int64_t kv_stride, float scale, int32_t dtype, void* stream);
+/* ------------------------------------------------------------------ libzipage_hybrid.so */
+
+/* Rows `in` (in_stride elements apart) hold q (H heads of D), k (HK of D), v (HK of V).  The first `rot`
+ * dimensions of q's and k's heads turn by positions[i] * freqs[.], dimension j with j + rot / 2.  q goes
+ * to q_out, [k | v] to slot slots[i] of the cache (-1 skips) and to kv_out when given. */
+int zp_rotary_store(const void* in, const int32_t* positions, const float* freqs, void* q_out,
+                    void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H, int32_t HK,
+                    int32_t D, int32_t V, int32_t rot, int64_t in_stride, int64_t num_slots,
+                    int32_t dtype, void* stream);
+
+/* Attention of single tokens over paged rows [k (HK heads of D) | v (HK of V)].  q (n, H, D); token i is
+ * the last of the context_lens[i] tokens of its sequence (0: inert, zeros) in row table_rows[i] (NULL:
+ * i) of table (B, NB); window, chunk, sinks, out_stride and out_scale as in zp_run_attention, with
+ * blocks counted from position 0.  `workspace`: zp_grouped_rows_workspace() bytes. */
+int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V,
+                                  int32_t window, int32_t chunk, int32_t NB, int32_t BS,
+                                  int32_t dtype);
+int zp_grouped_rows_attention(const void* q, const void* cache, const int32_t* table,
+                              const int32_t* context_lens, const int32_t* table_rows,
+                              const float* sinks, void* out, int32_t n, int32_t H, int32_t HK,
+                              int32_t D, int32_t V, int32_t BS, int32_t B, int32_t NB,
+                              int32_t num_pages, int32_t window, int32_t chunk, int64_t out_stride,
+                              float scale, float out_scale, int32_t dtype, void* workspace,
+                              int64_t workspace_bytes, void* stream);
+
+/* The runs of tokens a step holds, one per sequence: token rows row .. row + count - 1, the state slot,
+ * the position of the first token (0: the state starts at zero).  rows NULL: row i; max_count > 0 caps
+ * the counts; count 0 is inert. */
+typedef struct {
+  const int32_t *rows, *counts, *slots, *starts;
+  int32_t n, max_count, num_slots, num_rows;
+} zp_segments;
+
+/* Matrix memory with exponential gates, and the normed, gated read-out.  Rows `in` hold q, k (heads of
+ * dk), v, g (heads of dv) from columns q_at, k_at, v_at, g_at; gates (fp32) hold the input gates'
+ * and then the forget gates' pre-activations.  dk 32, 64, 128 or 256, dv a multiple of 32 up to 256, zero
+ * padded; the norm's mean runs over vdim.  state: (num_slots, heads, dk * dv + dk + 4) fp32. */
+typedef struct {
+  zp_segments seg;
+  const void* in;
+  const float *gates, *i_bias, *f_bias, *norm;
+  float* state;
+  void* out;
+  int64_t in_stride, gate_stride, out_stride;
+  int32_t heads, dk, dv, vdim, q_at, k_at, v_at, g_at;
+  float cap, q_scale, eps, out_scale;
+} zp_mlstm;
+int zp_mlstm_scan(const zp_mlstm* args, int32_t dtype, void* stream);
+
+/* Gated delta rule with a decay per key channel, its short convolutions and gates, and the normed, gated
+ * read-out.  Rows `in` hold the projections q, k (kv_heads of dk), v (heads of dv) and from column b_at
+ * the step sizes' pre-activations; rows `low` hold the decays' (heads of dk) and from column g_at the
+ * output gates' (heads of dv).  filters (taps, 2 * kv_heads * dk + heads * dv), the last tap is the
+ * current token's.  state: (num_slots, heads, dk, dv) fp32; conv_state: (num_slots, heads, taps - 1, 2
+ * dk + dv) of `dtype`. */
+typedef struct {
+  zp_segments seg;
+  const void *in, *low;
+  const float *filters, *a_log, *dt_bias, *norm;
+  float* state;
+  void *conv_state, *out;
+  int64_t in_stride, low_stride, out_stride;
+  int32_t heads, kv_heads, dk, dv, vdim, taps, b_at, g_at;
+  float q_scale, eps, out_scale;
+} zp_delta;
+int zp_delta_scan(const zp_delta* args, int32_t dtype, void* stream);
+
+/* out (n, M) fp32 = x (n, K) w (M, K)^T.  K a multiple of 32, M of 4. */
+int zp_small_linear(const void* x, const void* w, float* out, int32_t n, int32_t K, int32_t M,
+                    int64_t x_stride, int32_t dtype, void* stream);
+
+/* Per token: softmax over the E logits, the `keep` of `groups` groups with the largest single score, and
+ * the `top` best experts of those: ids and scores (n, top).  counts (E + 1) is cleared for the plan. */
+int zp_moe_select(const float* logits, int32_t* ids, float* weights, int32_t* counts, int32_t n,
+                  int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t logits_stride,
+                  void* stream);
+
+/* Assignments (token n, slot j), numbered n * (top + shared) + j, in the order of their experts, and the
+ * row tiles of the expert products: tiles (max_tiles, 4) of expert, first position in `sorted`, rows.
+ * Expert E is the shared one (slot `top` of every token).  zp_moe_tile_rows: rows per tile to plan
+ * for; zp_moe_max_tiles: the length of `tiles`. */
+int64_t zp_moe_tile_rows(int32_t n, int32_t E, int32_t top, int32_t dtype);
+int64_t zp_moe_max_tiles(int32_t n, int32_t E, int32_t top, int32_t shared, int32_t rows);
+int64_t zp_moe_plan_workspace(int32_t n, int32_t E, int32_t top);
+int zp_moe_plan(const int32_t* ids, int32_t* counts, int32_t* sorted, int32_t* tiles, int32_t* ntiles,
+                int32_t n, int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles,
+                void* workspace, int64_t workspace_bytes, void* stream);
+
+/* Expert products over a plan.  Weights in tile order: [out / 16][in / step][64 lanes][16 bytes], lane (g,
+ * r) = 16 g + r holding row r and the g-th 16 bytes of a step of 64 bytes; gate_up interleaves 16
+ * rows of the gate with the 16 of `up`.  out of gate_up, by position in `sorted`:
+ * weight * g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).  out of
+ * down: planes (slots, n, out_stride), an assignment's row in the plane of its slot.  K a multiple
+ * of 32, M of 16 (of 32 where it is a later K). */
+int zp_moe_gate_up(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
+                   const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n,
+                   int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K,
+                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
+                   float limit_shared, int32_t dtype, void* stream);
+int zp_moe_down(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
+                const int32_t* tiles, const int32_t* ntiles, int32_t n, int32_t E, int32_t top,
+                int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared,
+                int32_t M, int64_t x_stride, int64_t out_stride, int32_t dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -36,17 +36,31 @@ def test_library_exports_every_declared_symbol():
 
 def test_models_library_exports_every_declared_symbol():
     from zipage_amd import _lib
-    lib = _lib.load_models()
     names = _declared("zipage_models.h")
-    for name in names:
-        assert hasattr(lib, name), f"{name} declared in the header but not exported"
-    assert sorted(_lib.MODEL_EXPORTS) == names
+    assert sorted(n for names in _lib.MODEL_EXPORTS.values() for n in names) == names
+    for part, exported in _lib.MODEL_EXPORTS.items():
+        lib = _lib.load_models(part)
+        for name in exported:
+            assert hasattr(lib, name), f"{name} declared in the header but not exported"
+    lib = _lib.load_models("latent")
     # bad arguments are refused on the host, before any launch
     assert lib.zp_headwise_linear(None, None, None, 1, 2, 33, 16, 0, None) != 0
     assert b"multiple of 32" in lib.zp_last_error()
     assert lib.zp_latent_rows_attention(None, None, None, None, None, None, 1, 1, 32, 16, 1, 1, 1, -1, 1.0, 0,
                                         None, 0, None) == 1
-    assert lib.zp_embed_norm(None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1e-6, 0.0, 0, None) != 0
+    lib = _lib.load_models("models")
+    assert lib.zp_embed_norm(None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1.0, 1e-6, 0.0, 0, None) != 0
+    assert lib.zp_run_attention(None, None, None, None, None, None, 1, 4, 3, 32, 32, 0, 0, 1, 1, 128, 256, 128, 1.0, 1.0,
+                                0, None) == 1
+    lib = _lib.load_models("hybrid")
+    assert lib.zp_moe_select(None, None, None, None, 1, 12, 5, 3, 1, 12, None) == 1      # five of a group of four
+    assert lib.zp_small_linear(None, None, None, 1, 40, 4, 40, 0, None) != 0
+    bad = _lib.MlstmArgs(heads=2, dk=48, dv=32, vdim=32, cap=1.0, gate_stride=4, out_stride=64,
+                         seg=_lib.Segments(n=1, num_slots=1, num_rows=1))
+    assert lib.zp_mlstm_scan(ctypes.byref(bad), 0, None) != 0 and b"48" in lib.zp_last_error()
+    bad = _lib.DeltaArgs(heads=3, kv_heads=2, dk=32, dv=32, vdim=32, taps=4, out_stride=96,
+                         seg=_lib.Segments(n=1, num_slots=1, num_rows=1))
+    assert lib.zp_delta_scan(ctypes.byref(bad), 0, None) == 1
 
 
 def test_version_and_error_string():

@@ -129,7 +129,8 @@ def test_residual_linear_in_parts(dev, n):
 @pytest.mark.parametrize("dtype", DTYPES, ids=ids)
 @pytest.mark.parametrize("q,qp,r,rp", [(52, 64, 44, 64), (96, 96, 512, 512), (1536, 1536, 20, 32)])
 def test_latent_norm_store_and_gather(dev, dtype, q, qp, r, rp):
-    from zipage_amd.layers.latent import gather_rows, latent_norm_store
+    from zipage_amd.layers.latent import latent_norm_store
+    from zipage_amd.layers.runs import gather_rows
     n, pages, BS = 9, 4, 8
     down = _rand(dev, dtype, n, qp + rp, seed=1)
     down[:, q:qp] = 0

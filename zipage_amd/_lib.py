@@ -1,4 +1,4 @@
-"""ctypes binding of ``libzipage_hip.so`` and ``libzipage_models.so`` (the C ABIs in
+"""ctypes binding of ``libzipage_hip.so`` and of the model-side libraries (the C ABIs in
 ``include/zipage_hip.h`` and ``include/zipage_models.h``).
 
 The product path has no CPU fallback: if the shared object is missing or a symbol cannot
@@ -16,7 +16,6 @@ import torch
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libzipage_hip.so")
-MODELS_LIB_PATH = os.path.join(_HERE, "libzipage_models.so")
 
 ZP_BF16, ZP_F16, ZP_F32 = 0, 1, 2
 _DTYPES = {torch.bfloat16: ZP_BF16, torch.float16: ZP_F16, torch.float32: ZP_F32}
@@ -86,25 +85,70 @@ I64_RETURNING = {
 }
 EXPORTS = sorted(list(SIGNATURES) + list(I64_RETURNING) + ["zp_abi_version", "zp_last_error"])
 
-# the model-side library, in the order of include/zipage_models.h
-MODEL_SIGNATURES = {
-    "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, i32, ptr],
-    "zp_residual_norm": [ptr, ptr, i32, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32, f32,
-                         i32, ptr],
-    "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
-    "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, f32, i32, ptr],
-    "zp_gather_rows": [ptr, ptr, ptr, i32, i32, i64, ptr],
-    "zp_headwise_linear": [ptr, ptr, ptr, i32, i32, i32, i32, i32, ptr],
-    "zp_latent_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, f32,
-                                 i32, ptr, i64, ptr],
-    "zp_latent_tiles_attention": [ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, i64, i64, i64, f32,
-                                  i32, ptr],
+class Segments(C.Structure):
+    """zp_segments of include/zipage_models.h."""
+    _fields_ = [(n, ptr) for n in ("rows", "counts", "slots", "starts")] + \
+        [(n, i32) for n in ("n", "max_count", "num_slots", "num_rows")]
+
+
+class MlstmArgs(C.Structure):
+    """zp_mlstm."""
+    _fields_ = [("seg", Segments)] + \
+        [(n, ptr) for n in ("inp", "gates", "i_bias", "f_bias", "norm", "state", "out")] + \
+        [(n, i64) for n in ("in_stride", "gate_stride", "out_stride")] + \
+        [(n, i32) for n in ("heads", "dk", "dv", "vdim", "q_at", "k_at", "v_at", "g_at")] + \
+        [(n, f32) for n in ("cap", "q_scale", "eps", "out_scale")]
+
+
+class DeltaArgs(C.Structure):
+    """zp_delta."""
+    _fields_ = [("seg", Segments)] + \
+        [(n, ptr) for n in ("inp", "low", "filters", "a_log", "dt_bias", "norm", "state", "conv_state", "out")] + \
+        [(n, i64) for n in ("in_stride", "low_stride", "out_stride")] + \
+        [(n, i32) for n in ("heads", "kv_heads", "dk", "dv", "vdim", "taps", "b_at", "g_at")] + \
+        [(n, f32) for n in ("q_scale", "eps", "out_scale")]
+
+
+# the model-side libraries, in the order of include/zipage_models.h: name -> (entry points, those that
+# return an int64 count instead of a status)
+MODEL_LIBS = {
+    "models": ({
+        "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, i32, ptr],
+        "zp_residual_norm": [ptr, ptr, i32, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32,
+                             f32, i32, ptr],
+        "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
+        "zp_softcap": [ptr, ptr, i64, f32, i32, ptr],
+        "zp_gather_rows": [ptr, ptr, ptr, i32, i32, i64, ptr],
+        "zp_run_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i64, i64, i64, i64,
+                             i64, f32, f32, i32, ptr],
+    }, {}),
+    "latent": ({
+        "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, f32, i32, ptr],
+        "zp_headwise_linear": [ptr, ptr, ptr, i32, i32, i32, i32, i32, ptr],
+        "zp_latent_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, f32,
+                                     i32, ptr, i64, ptr],
+    }, {"zp_latent_rows_workspace": [i32, i32, i32, i32, i32, i32, i32]}),
+    "hybrid": ({
+        "zp_rotary_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i64, i64, i32, ptr],
+        "zp_grouped_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32,
+                                      i32, i32, i32, i64, f32, f32, i32, ptr, i64, ptr],
+        "zp_mlstm_scan": [C.POINTER(MlstmArgs), i32, ptr],
+        "zp_delta_scan": [C.POINTER(DeltaArgs), i32, ptr],
+        "zp_small_linear": [ptr, ptr, ptr, i32, i32, i32, i64, i32, ptr],
+        "zp_moe_select": [ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, ptr],
+        "zp_moe_plan": [ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, ptr, i64, ptr],
+        "zp_moe_gate_up": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, i64,
+                           i64, f32, f32, i32, ptr],
+        "zp_moe_down": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, i64, i64, i32,
+                        ptr],
+    }, {"zp_grouped_rows_workspace": [i32, i32, i32, i32, i32, i32, i32, i32, i32, i32],
+        "zp_moe_tile_rows": [i32, i32, i32, i32], "zp_moe_max_tiles": [i32, i32, i32, i32, i32], "zp_moe_plan_workspace": [i32, i32, i32]}),
 }
-MODEL_I64_RETURNING = {"zp_latent_rows_workspace": [i32, i32, i32, i32, i32, i32, i32]}
-MODEL_EXPORTS = sorted(list(MODEL_SIGNATURES) + list(MODEL_I64_RETURNING))
+MODEL_EXPORTS = {lib: sorted([*calls, *sizes]) for lib, (calls, sizes) in MODEL_LIBS.items()}
+_LIB_OF = {name: lib for lib, (calls, _) in MODEL_LIBS.items() for name in calls}
 
 _lib = None
-_models = None
+_models: dict[str, C.CDLL] = {}
 
 
 def _open(path: str, signatures: dict, i64_returning: dict) -> C.CDLL:
@@ -132,12 +176,15 @@ def load() -> C.CDLL:
     return _lib
 
 
-def load_models() -> C.CDLL:
-    """The same for the model-side library."""
-    global _models
-    if _models is None:
-        _models = _open(MODELS_LIB_PATH, MODEL_SIGNATURES, MODEL_I64_RETURNING)
-    return _models
+def model_lib_path(name: str) -> str:
+    return os.path.join(_HERE, f"libzipage_{name}.so")
+
+
+def load_models(name: str = "models") -> C.CDLL:
+    """The same for a model-side library."""
+    if name not in _models:
+        _models[name] = _open(model_lib_path(name), *MODEL_LIBS[name])
+    return _models[name]
 
 
 def _check(lib, name: str, rc: int) -> None:
@@ -151,7 +198,7 @@ def call(name: str, *args) -> None:
 
 
 def call_models(name: str, *args) -> None:
-    lib = load_models()
+    lib = load_models(_LIB_OF[name])
     _check(lib, name, getattr(lib, name)(*args))
 
 

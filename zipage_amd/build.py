@@ -1,9 +1,9 @@
 """Build the HIP libraries (gfx950) in-tree with hipcc.
 
-Run as ``python -m zipage_amd.build``.  Two shared objects with a plain C ABI, neither linked
-against torch: ``libzipage_hip.so`` (``include/zipage_hip.h``: the compression path and the kernels
-of the models that use it) and ``libzipage_models.so`` (``include/zipage_models.h``: the kernels of
-the other models), so that a model served without compression compiles only what it runs.
+Run as ``python -m zipage_amd.build``.  Shared objects with a plain C ABI, none linked against
+torch: ``libzipage_hip.so`` (``include/zipage_hip.h``: the compression path and the kernels of the
+models that use it) and, for the other models, ``libzipage_models.so``, ``libzipage_latent.so`` and
+``libzipage_hybrid.so`` (``include/zipage_models.h``), so that a model compiles only what it runs.
 """
 from __future__ import annotations
 
@@ -16,6 +16,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libzipage_hip.so")
 MODELS_LIB = os.path.join(HERE, "libzipage_models.so")
+LATENT_LIB = os.path.join(HERE, "libzipage_latent.so")
+HYBRID_LIB = os.path.join(HERE, "libzipage_hybrid.so")
 
 # packed fp32 VALU ops are disabled on purpose (some forms misbehave on this fleet)
 BASE_FLAGS = [
@@ -26,14 +28,23 @@ BASE_FLAGS = [
 # keep a*b+c as two roundings: the compression stages restate torch ops that round after each op
 FLAGS = BASE_FLAGS + ["-ffp-contract=off"]
 
-MODEL_SOURCES = ("latent.hip", "residual.hip")     # these and the error reporting
+# sources of the model-side libraries, beside the error reporting; the rest is the compression library
+MODEL_SOURCES = {
+    MODELS_LIB: ("residual.hip", "runs.hip"),
+    LATENT_LIB: ("latent.hip",),
+    HYBRID_LIB: ("grouped.hip", "mlstm.hip", "delta.hip", "moe.hip"),
+}
 COMMON_SOURCES = ("runtime.hip",)
+LIBS = (LIB, *MODEL_SOURCES)
 
 
-def sources(models: bool = False):
-    names = [f for f in os.listdir(CSRC) if f.endswith(".hip")]
-    keep = (lambda f: f in MODEL_SOURCES or f in COMMON_SOURCES) if models else (lambda f: f not in MODEL_SOURCES)
-    return sorted(os.path.join(CSRC, f) for f in names if keep(f))
+def sources(lib: str = LIB) -> list[str]:
+    if lib in MODEL_SOURCES:
+        names = [*MODEL_SOURCES[lib], *COMMON_SOURCES]
+    else:
+        others = {f for fs in MODEL_SOURCES.values() for f in fs}
+        names = [f for f in os.listdir(CSRC) if f.endswith(".hip") and f not in others]
+    return sorted(os.path.join(CSRC, f) for f in names)
 
 
 def _run(cmd, verbose):
@@ -48,18 +59,18 @@ def _run(cmd, verbose):
         print(err, file=sys.stderr)
 
 
-def build(verbose: bool = True, jobs: int | None = None, libs: tuple[str, ...] = (LIB, MODELS_LIB)) -> str:
+def build(verbose: bool = True, jobs: int | None = None, libs: tuple[str, ...] = LIBS) -> str:
     """Compile the sources of ``libs`` to object files (in parallel) and link the shared objects."""
     from concurrent.futures import ThreadPoolExecutor
     hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
     extra = os.environ.get("ZP_EXTRA_HIPCC_FLAGS", "").split()
     work, links = [], []
     for lib in libs:
-        models = lib == MODELS_LIB
-        objdir = os.path.join(HERE, "build", "models" if models else "")
+        models = lib in MODEL_SOURCES
+        objdir = os.path.join(HERE, "build", os.path.basename(lib)[len("libzipage_"):-3] if models else "")
         os.makedirs(objdir, exist_ok=True)
         objs = []
-        for src in sources(models):
+        for src in sources(lib):
             obj = os.path.join(objdir, os.path.basename(src)[:-4] + ".o")
             work.append([hipcc, *(BASE_FLAGS if models else FLAGS), *extra, "-c", src, "-o", obj])
             objs.append(obj)
@@ -73,16 +84,16 @@ def build(verbose: bool = True, jobs: int | None = None, libs: tuple[str, ...] =
     return libs[0]
 
 
-def ensure(lib: str) -> str:
-    """Build ``lib`` if it is not there yet (one process at a time)."""
-    if not os.path.exists(lib):
+def ensure(*libs: str) -> None:
+    """Build those of ``libs`` that are not there yet (one process at a time)."""
+    if not all(os.path.exists(lib) for lib in libs):
         import fcntl
         os.makedirs(os.path.join(HERE, "build"), exist_ok=True)
         with open(os.path.join(HERE, "build", ".lock"), "w") as lock:
             fcntl.flock(lock, fcntl.LOCK_EX)
-            if not os.path.exists(lib):
-                build(verbose=False, libs=(lib,))
-    return lib
+            missing = tuple(lib for lib in libs if not os.path.exists(lib))
+            if missing:
+                build(verbose=False, libs=missing)
 
 
 if __name__ == "__main__":

@@ -26,10 +26,11 @@ def _engine(folder: str, dtype: str, pages: int, page_size: int, slots: int, **k
     from zipage_amd.engine.registry import arch_for_shape, read_shape
     shape = read_shape(folder)
     arch = arch_for_shape(shape)
-    build.ensure(build.LIB if arch.model.compressible else build.MODELS_LIB)
+    build.ensure(*(getattr(build, lib) for lib in arch.libs))
     import torch
     from zipage_amd.engine import EngineConfig, ZipageEngine
-    limit = getattr(shape, "max_positions", None) or getattr(shape, "max_position", 8192)
+    # without a limit of its own a model takes what the pool holds
+    limit = getattr(shape, "max_positions", None) or getattr(shape, "max_position", pages * page_size)
     return ZipageEngine(EngineConfig(
         shape=shape, model_folder=folder if arch.loads_weights else None, dtype=getattr(torch, dtype),
         num_kvcache_blocks=pages, kvcache_block_size=page_size, max_concurrency=slots,

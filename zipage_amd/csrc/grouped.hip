@@ -1,0 +1,530 @@
+// Grouped-query attention over paged rows [keys of all heads | values of all heads] per token.
+//
+//   rotary_store    rotary positions on queries and keys; keys and values to their cache slot
+//   grouped_rows    attention of single tokens over the pages; the query heads of a key head share
+//                   one read of its keys and values
+//   grouped_plain   float32 form (true fp32 products), any sizes
+//
+// Attention of runs of prompt tokens is run_attention (runs.hip).  A token sees a window, its own
+// block of positions, or everything before it; a sink is a logit per head that joins the softmax's
+// denominator only.
+#include "mfma.h"
+
+namespace {
+
+// ------------------------------------------------------------------ rotary positions and the store
+struct RotaryArgs {
+  const void* in;           // token rows of in_st elements: q (H * D), k (HK * D), v (HK * V)
+  const int32_t* positions;
+  const float* freqs;       // (rot / 2,)
+  void* q_out;              // (n, H * D)
+  void* kv_out;             // (n, HK * (D + V)) or null
+  void* cache;              // (num_slots, HK * (D + V))
+  const int32_t* slots;     // (n,), -1 skips
+  int n, H, HK, D, V, half; // half = rotated dimensions / 2
+  int64_t in_st, num_slots;
+};
+constexpr int kRotTokens = 4;
+
+// Four tokens per workgroup: their angles once, in LDS, for all heads.  VEC elements per item; an
+// item of the rotated part is the pair (i .. i + VEC, i + half ..).
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  float2* cs = (float2*)lds_raw;            // [kRotTokens][half]
+  const int n0 = blockIdx.x * kRotTokens, tid = threadIdx.x;
+  for (int i = tid; i < kRotTokens * a.half; i += 256) {
+    const int tok = i / a.half;
+    if (n0 + tok < a.n) {
+      float s, c;
+      sincosf((float)a.positions[n0 + tok] * a.freqs[i - tok * a.half], &s, &c);
+      cs[i] = make_float2(c, s);
+    }
+  }
+  __syncthreads();
+  const int pairs = a.half / VEC, per_head = (a.D - a.half) / VEC;
+  const int heads = a.H + a.HK, rotated = heads * per_head, items = rotated + a.HK * a.V / VEC;
+  const int kvw = a.HK * (a.D + a.V);
+  for (int id = tid; id < kRotTokens * items; id += 256) {
+    const int tok = id / items, it = id - tok * items;
+    const int64_t row = n0 + tok;
+    if (row >= a.n) break;
+    float x[VEC], y[VEC];
+    auto load = [&](int64_t at, float* o) {
+      if constexpr (VEC == 8) Vec8<T>::ld(a.in, at, o); else o[0] = Elem<T>::ld(a.in, at);
+    };
+    int64_t slot = a.slots[row];
+    if (slot >= a.num_slots) slot = -1;
+    auto put = [&](int c, const float* o) {   // column of the row [q | k | v]
+      const int kc = c - a.H * a.D;
+      if (kc < 0) {
+        if constexpr (VEC == 8) Vec8<T>::st(a.q_out, row * a.H * a.D + c, o);
+        else Elem<T>::st(a.q_out, row * a.H * a.D + c, o[0]);
+        return;
+      }
+      if (a.kv_out) {
+        if constexpr (VEC == 8) Vec8<T>::st(a.kv_out, row * kvw + kc, o);
+        else Elem<T>::st(a.kv_out, row * kvw + kc, o[0]);
+      }
+      if (slot >= 0) {
+        if constexpr (VEC == 8) Vec8<T>::st(a.cache, slot * kvw + kc, o);
+        else Elem<T>::st(a.cache, slot * kvw + kc, o[0]);
+      }
+    };
+    if (it >= rotated) {
+      const int c = heads * a.D + (it - rotated) * VEC;
+      load(row * a.in_st + c, x);
+      put(c, x);
+      continue;
+    }
+    const int h = it / per_head, p = it - h * per_head;
+    if (p >= pairs) {                          // dimensions behind the rotated ones
+      const int c = h * a.D + (p + pairs) * VEC;
+      load(row * a.in_st + c, x);
+      put(c, x);
+      continue;
+    }
+    const int c = h * a.D + p * VEC;
+    load(row * a.in_st + c, x);
+    load(row * a.in_st + c + a.half, y);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const float2 r = cs[tok * a.half + p * VEC + i];
+      const float u = x[i], v = y[i];
+      x[i] = u * r.x - v * r.y;
+      y[i] = v * r.x + u * r.y;
+    }
+    put(c, x);
+    put(c + a.half, y);
+  }
+}
+
+// ------------------------------------------------------------------ single tokens over the pages
+struct RowsArgs {
+  const void* q;          // (n, H * D)
+  const void* cache;      // (pages, BS, HK * (D + V))
+  const int32_t* table;   // (B, NB) page ids
+  const int32_t* ctx;     // (n,) tokens of the sequence up to and including this one; 0 = inert
+  const int32_t* seq;     // (n,) row of table, or null: row i
+  const float* sinks;     // (H,) or null
+  void* out;              // token rows of o_st elements, head h at h * V
+  float* part;            // splits > 1: (n, H, splits, V) fp32, then (n, H, splits, 2) max and sum
+  int n, H, HK, D, V, BS, bs_shift, B, NB, num_pages;
+  int window, chunk;
+  int splits, htiles;     // key ranges, and tiles of 16 query heads per key head
+  int lds_pages;
+  int64_t o_st;
+  float scale, out_scale;
+};
+
+__device__ __forceinline__ int first_key(const RowsArgs& a, int n) {   // n tokens, the last one asks
+  if (a.window > 0) return max(0, n - a.window);
+  return a.chunk > 0 && n > 0 ? (n - 1) / a.chunk * a.chunk : 0;
+}
+
+// A workgroup owns one token, up to 16 query heads of one key head and one key range; its four waves
+// are flash loops of their own over every fourth 32-key step and meet in LDS at the end.  Keys are the
+// row operand straight from memory (64-byte pieces), values are loaded as rows and turned into column
+// operands by v_perm.  The next step's keys are requested once the scores are done, its values once the
+// value products are.
+template <int DKS, int VCB>
+__global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  int* const pg = (int*)lds_raw;
+  float* const merge = (float*)(lds_raw + ((a.lds_pages * 4 + 15) & ~15));
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+  int id = blockIdx.x;
+  const int split = id % a.splits;
+  id /= a.splits;
+  const int ht = id % a.htiles;
+  id /= a.htiles;
+  const int hk = id % a.HK, row = id / a.HK;
+  const int G = a.H / a.HK;
+  const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
+  const int n = min(a.ctx[row], a.NB * a.BS);
+  const int lo = first_key(a, n);
+  const int p0 = lo >> a.bs_shift;
+  // every entry gets a valid page, whatever the context length says: no address rests on it
+  for (int j = tid; j < a.lds_pages; j += 256) {
+    const int p = p0 + j < a.NB ? a.table[(int64_t)seq * a.NB + p0 + j] : 0;
+    pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
+  }
+  const int nks = a.D / 32;
+  const int head = hk * G + min(ht * 16 + l16, G - 1);
+  u32x4 qf[DKS];
+  const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + head) * a.D + g * 8;
+#pragma unroll
+  for (int ks = 0; ks < DKS; ++ks) {
+    qf[ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
+    if (ks >= nks) qf[ks] = u32x4{0u, 0u, 0u, 0u};
+  }
+  __syncthreads();
+  const int kvw = a.HK * (a.D + a.V), mask = a.BS - 1;
+  const uint16_t* const kc = (const uint16_t*)a.cache + hk * a.D + g * 8;
+  const uint16_t* const vc = (const uint16_t*)a.cache + a.HK * a.D + hk * a.V;
+  int col[VCB];
+#pragma unroll
+  for (int cb = 0; cb < VCB; ++cb) {
+    const int c = cb * 128 + l16 * 8;
+    col[cb] = c < a.V ? c : 0;
+  }
+  // keys outside the visible range repeat a visible row, with weight zero
+  auto row_at = [&](int key) -> int64_t {
+    key = min(max(key, lo), n - 1);
+    const int page = pg[min((key >> a.bs_shift) - p0, a.lds_pages - 1)];
+    return ((int64_t)page * a.BS + (key & mask)) * kvw;
+  };
+  u32x4 kf[2][DKS], vf[VCB][8];
+  auto load_keys = [&](int b) {
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) {
+      const uint16_t* k = kc + row_at(b * 32 + tt * 16 + l16);
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) kf[tt][ks] = *(const u32x4*)(k + (ks < nks ? ks * 32 : 0));
+    }
+  };
+  auto load_values = [&](int b) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const uint16_t* v = vc + row_at(b * 32 + step_key(g, i));
+#pragma unroll
+      for (int cb = 0; cb < VCB; ++cb) vf[cb][i] = *(const u32x4*)(v + col[cb]);
+    }
+  };
+  f32x4 o[VCB * 8];
+#pragma unroll
+  for (int i = 0; i < VCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  const float sc = a.scale * 1.44269504088896f;
+  const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = 4 * a.splits;
+  int b = (lo >> 5) + split * 4 + wave;
+  if (b <= b1) {
+    load_keys(b);
+    load_values(b);
+  }
+  for (; b <= b1; b += step) {
+    const int k0 = b * 32, next = min(b + step, b1);       // after the last step its own rows again, unused
+    f32x4 s[2];
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) {
+      s[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) s[tt] = mfma_bf16(kf[tt][ks], qf[ks], s[tt]);
+    }
+    load_keys(next);
+    float p[8], mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int key = k0 + step_key(g, i);
+      p[i] = key < lo || key >= n ? -INFINITY : s[i >> 2][i & 3] * sc;
+      mx = fmaxf(mx, p[i]);
+    }
+    mx = fmaxf(mx, lane_xor16(mx));
+    mx = fmaxf(mx, lane_xor32(mx));
+    const float mn = fmaxf(m, mx);                          // finite: every step holds a visible key
+    const float f = __builtin_amdgcn_exp2f(m - mn);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
+      sum += p[i];
+    }
+    l = l * f + sum;
+    m = mn;
+    if (__any(f != 1.f)) {
+#pragma unroll
+      for (int i = 0; i < VCB * 8; ++i) o[i] *= f;
+    }
+    const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]), pack_bf16(p[6], p[7])};
+#pragma unroll
+    for (int cb = 0; cb < VCB; ++cb)
+#pragma unroll
+      for (int t = 0; t < 8; ++t) o[cb * 8 + t] = mfma_bf16(column_of(vf[cb], t), pf, o[cb * 8 + t]);
+    load_values(next);
+  }
+  l += lane_xor16(l);
+  l += lane_xor32(l);
+  const int RS = a.V + 4, per = 16 * RS + 32;
+  float* const dst = merge + wave * per;
+  if (g == 0) { dst[16 * RS + l16] = m; dst[16 * RS + 16 + l16] = l; }
+#pragma unroll
+  for (int cb = 0; cb < VCB; ++cb)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = cb * 128 + (4 * g + i) * 8;
+      if (c < a.V) {
+        float* d = dst + l16 * RS + c;
+        const f32x4* t = o + cb * 8;
+        *(f32x4*)d = f32x4{t[0][i], t[1][i], t[2][i], t[3][i]};
+        *(f32x4*)(d + 4) = f32x4{t[4][i], t[5][i], t[6][i], t[7][i]};
+      }
+    }
+  __syncthreads();
+  if (tid < 16 && ht * 16 + tid < G) {
+    const int h = hk * G + ht * 16 + tid;
+    float* const src = merge + 16 * RS + tid;
+    float mx = fmaxf(fmaxf(src[0], src[per]), fmaxf(src[2 * per], src[3 * per]));
+    const float ms = mx == -INFINITY ? 0.f : mx;
+    float sum = 0.f, f[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      f[k] = __builtin_amdgcn_exp2f(src[k * per] - ms);
+      sum += src[k * per + 16] * f[k];
+    }
+    float inv = 1.f;
+    if (a.splits > 1) {
+      float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.V + (((int64_t)row * a.H + h) * a.splits + split) * 2;
+      ml[0] = mx;
+      ml[1] = sum;
+    } else {
+      if (a.sinks && mx != -INFINITY) sum += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - ms);
+      inv = sum > 0.f ? a.out_scale / sum : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) src[k * per] = f[k] * inv;
+  }
+  __syncthreads();
+  for (int it = tid; it < 16 * (a.V / 8); it += 256) {
+    const int hl = it / (a.V / 8), c = (it - hl * (a.V / 8)) * 8;
+    if (ht * 16 + hl >= G) continue;
+    const int h = hk * G + ht * 16 + hl;
+    float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float* part = merge + k * per;
+      const float f = part[16 * RS + hl];
+      float x[8];
+      Vec8<F32>::ld(part, hl * RS + c, x);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
+    }
+    if (a.splits == 1) Vec8<BF16>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, r);
+    else Vec8<F32>::st(a.part, (((int64_t)row * a.H + h) * a.splits + split) * a.V + c, r);
+  }
+}
+
+__global__ __launch_bounds__(64) void grouped_combine_kernel(RowsArgs a) {
+  const int64_t item = blockIdx.x;       // (row, head)
+  const int h = (int)(item % a.H);
+  const float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.V + item * a.splits * 2;
+  float mx = -INFINITY;
+  for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ml[2 * s]);
+  const bool any = mx != -INFINITY;
+  if (!any) mx = 0.f;
+  float l = 0.f;
+  for (int s = 0; s < a.splits; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - mx);
+  if (a.sinks && any) l += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - mx);
+  const float inv = l > 0.f ? a.out_scale / l : 0.f;
+  for (int c = threadIdx.x * 8; c < a.V; c += 512) {
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < a.splits; ++s) {
+      const float f = __builtin_amdgcn_exp2f(ml[2 * s] - mx) * inv;
+      float v[8];
+      Vec8<F32>::ld(a.part, (item * a.splits + s) * a.V + c, v);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc[i] += v[i] * f;
+    }
+    Vec8<BF16>::st(a.out, item / a.H * a.o_st + (int64_t)h * a.V + c, acc);
+  }
+}
+
+// One workgroup per (token, query head), plain fp32 arithmetic.
+template <typename T>
+__global__ __launch_bounds__(256) void grouped_plain_kernel(RowsArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  float* q = (float*)lds_raw;              // D
+  __shared__ float sc[256];
+  __shared__ float red[4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, hk = h / (a.H / a.HK);
+  const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
+  const int n = min(a.ctx[row], a.NB * a.BS);
+  const int lo = first_key(a, n);
+  for (int c = tid; c < a.D; c += 256) q[c] = Elem<T>::ld(a.q, (int64_t)blockIdx.x * a.D + c);
+  const int64_t kvw = (int64_t)a.HK * (a.D + a.V);
+  auto key_at = [&](int t) -> int64_t {
+    const int p = a.bs_shift >= 0 ? t >> a.bs_shift : t / a.BS;
+    int page = a.table[(int64_t)seq * a.NB + p];
+    if (page < 0 || page >= a.num_pages) page = 0;
+    return ((int64_t)page * a.BS + (t - p * a.BS)) * kvw;
+  };
+  constexpr int kCols = 4;                 // columns per thread: V <= 1024
+  float o[kCols] = {0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  for (int c0 = lo; c0 < n; c0 += 256) {
+    const int cnt = min(256, n - c0);
+    __syncthreads();                       // q is there; the last chunk's scores are used up
+    for (int j = wave; j < cnt; j += 4) {
+      const int64_t at = key_at(c0 + j) + hk * a.D;
+      float acc = 0.f;
+      for (int c = lane; c < a.D; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
+      acc = wave_sum(acc);
+      if (lane == 0) sc[j] = acc * a.scale;
+    }
+    __syncthreads();
+    float mx = tid < cnt ? sc[tid] : -INFINITY;
+    mx = wave_max(mx);
+    if (lane == 0) red[wave] = mx;
+    __syncthreads();
+    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    const float mn = fmaxf(m, mx);
+    const float f = expf(m - mn);
+    __syncthreads();
+    const float p = tid < cnt ? expf(sc[tid] - mn) : 0.f;
+    sc[tid] = p;
+    const float s = wave_sum(p);
+    if (lane == 0) red[wave] = s;
+    __syncthreads();
+    l = l * f + red[0] + red[1] + red[2] + red[3];
+    m = mn;
+#pragma unroll
+    for (int i = 0; i < kCols; ++i) o[i] *= f;
+    for (int j = 0; j < cnt; ++j) {
+      const int64_t at = key_at(c0 + j) + a.HK * a.D + hk * a.V;
+      const float pj = sc[j];
+#pragma unroll
+      for (int i = 0; i < kCols; ++i) {
+        const int c = tid + i * 256;
+        if (c < a.V) o[i] = fmaf(pj, Elem<T>::ld(a.cache, at + c), o[i]);
+      }
+    }
+  }
+  if (a.sinks && n > 0) l += expf(a.sinks[h] - m);
+  const float inv = l > 0.f ? a.out_scale / l : 0.f;
+#pragma unroll
+  for (int i = 0; i < kCols; ++i) {
+    const int c = tid + i * 256;
+    if (c < a.V) Elem<T>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, o[i] * inv);
+  }
+}
+
+constexpr int kMaxLdsPages = 4096;
+
+// Key ranges per token: enough workgroups to cover the chip, at least two steps per wave.
+int rows_splits(int n, int H, int HK, int window, int chunk, int NB, int BS) {
+  const int groups = n * HK * ((H / HK + 15) / 16);
+  int64_t keys = (int64_t)NB * BS;
+  if (window > 0 && window < keys) keys = window;
+  if (chunk > 0 && chunk < keys) keys = chunk;
+  const int steps = (int)((keys + 31) / 32);
+  int s = 512 / (groups > 0 ? groups : 1);
+  s = s < steps / 8 ? s : steps / 8;
+  s = s < 32 ? s : 32;
+  return s < 1 ? 1 : s;
+}
+
+template <int DKS, int VCB> int launch_rows(const RowsArgs& a, hipStream_t st) {
+  const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + 4 * sizeof(float) * (16 * (a.V + 4) + 32);
+  if (smem > 64 * 1024 &&
+      hipFuncSetAttribute((const void*)grouped_rows_kernel<DKS, VCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                          (int)smem) != hipSuccess) {
+    zp_set_error("grouped_rows_attention: cannot reserve %zu bytes of LDS", smem);
+    return ZP_EHIP;
+  }
+  hipLaunchKernelGGL((grouped_rows_kernel<DKS, VCB>), dim3((unsigned)a.n * a.HK * a.htiles * a.splits), dim3(256), smem, st, a);
+  ZP_LAUNCH_CHECK();
+  if (a.splits > 1) {
+    hipLaunchKernelGGL(grouped_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
+    ZP_LAUNCH_CHECK();
+  }
+  return ZP_OK;
+}
+
+}  // namespace
+
+extern "C" int zp_rotary_store(const void* in, const int32_t* positions, const float* freqs, void* q_out,
+                               void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
+                               int32_t HK, int32_t D, int32_t V, int32_t rot, int64_t in_stride,
+                               int64_t num_slots, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && D > 0 && V > 0 && rot >= 0 && rot % 2 == 0 && rot <= D && num_slots > 0 &&
+                 in_stride >= (int64_t)H * D + (int64_t)HK * (D + V), "rotary_store: bad dims");
+  ZP_MODEL_DTYPE("rotary_store");
+  if (D % 8 != 0 || V % 8 != 0 || in_stride % 8 != 0 || rot > 2048) {
+    zp_set_error("rotary_store: head sizes %d, %d (multiples of 8), %d rotated (<= 2048)", D, V, rot);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(in && positions && q_out && cache && slots && (rot == 0 || freqs), "rotary_store: null pointer");
+  ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache),
+             "rotary_store: tensors must be 16-byte aligned");
+  RotaryArgs a = {in, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, V, rot / 2, in_stride, num_slots};
+  const unsigned grid = (unsigned)((n + kRotTokens - 1) / kRotTokens);
+  const size_t smem = sizeof(float2) * kRotTokens * (rot / 2);
+  hipStream_t st = (hipStream_t)stream;
+#define ZP_ROTARY(T)                                                                                          \
+  do {                                                                                                        \
+    if (rot % 16 == 0) hipLaunchKernelGGL((rotary_store_kernel<T, 8>), dim3(grid), dim3(256), smem, st, a);   \
+    else hipLaunchKernelGGL((rotary_store_kernel<T, 1>), dim3(grid), dim3(256), smem, st, a);                 \
+  } while (0)
+  if (dtype == ZP_BF16) ZP_ROTARY(BF16); else ZP_ROTARY(F32);
+#undef ZP_ROTARY
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+static bool rows_need_plain(int D, int V, int BS, int dtype) {
+  return dtype == ZP_F32 || D > 256 || V > 256 || D % 32 != 0 || BS < 16 || (BS & (BS - 1)) != 0;
+}
+
+extern "C" int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V,
+                                             int32_t window, int32_t chunk, int32_t NB, int32_t BS,
+                                             int32_t dtype) {
+  if (n < 0 || H <= 0 || HK <= 0 || H % HK || V <= 0 || NB <= 0 || BS <= 0) return -1;
+  if (rows_need_plain(D, V, BS, dtype)) return 0;
+  const int s = rows_splits(n, H, HK, window, chunk, NB, BS);
+  return s == 1 ? 0 : (int64_t)n * H * s * (V + 2) * 4;
+}
+
+extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const int32_t* table,
+                                         const int32_t* context_lens, const int32_t* table_rows,
+                                         const float* sinks, void* out, int32_t n, int32_t H, int32_t HK,
+                                         int32_t D, int32_t V, int32_t BS, int32_t B, int32_t NB,
+                                         int32_t num_pages, int32_t window, int32_t chunk, int64_t out_stride,
+                                         float scale, float out_scale, int32_t dtype, void* workspace,
+                                         int64_t workspace_bytes, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && V > 0 && BS > 0 && B > 0 && NB > 0 &&
+                 num_pages > 0 && window >= 0 && chunk >= 0 && !(window && chunk), "grouped_rows_attention: bad dims");
+  ZP_MODEL_DTYPE("grouped_rows_attention");
+  if (D % 8 != 0 || V % 8 != 0 || V > 1024 || D > 4096) {
+    zp_set_error("grouped_rows_attention: head sizes %d, %d unsupported (multiples of 8, <= 4096, <= 1024)", D, V);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(q && cache && table && context_lens && out, "grouped_rows_attention: null pointer");
+  ZP_REQUIRE(table_rows || n <= B, "grouped_rows_attention: more tokens than table rows");
+  ZP_REQUIRE(aligned16(q) && aligned16(cache) && aligned16(out) && aligned16(workspace) && out_stride % 8 == 0 &&
+                 out_stride >= (int64_t)H * V, "grouped_rows_attention: tensors must be 16-byte aligned");
+  RowsArgs a = {};
+  a.q = q; a.cache = cache; a.table = table; a.ctx = context_lens; a.seq = table_rows; a.sinks = sinks; a.out = out;
+  a.part = (float*)workspace; a.n = n; a.H = H; a.HK = HK; a.D = D; a.V = V; a.BS = BS; a.B = B; a.NB = NB;
+  a.num_pages = num_pages; a.window = window; a.chunk = chunk; a.o_st = out_stride; a.scale = scale;
+  a.out_scale = out_scale; a.bs_shift = -1;
+  if ((BS & (BS - 1)) == 0)
+    for (a.bs_shift = 0; (1 << a.bs_shift) < BS; ++a.bs_shift) {}
+  int64_t pages = NB;
+  const int seen = window > 0 ? window : chunk;
+  if (seen > 0 && (seen - 1) / BS + 2 < pages) pages = (seen - 1) / BS + 2;
+  hipStream_t st = (hipStream_t)stream;
+  if (rows_need_plain(D, V, BS, dtype) || pages > kMaxLdsPages) {
+    const size_t smem = sizeof(float) * D;
+    if (dtype == ZP_BF16)
+      hipLaunchKernelGGL((grouped_plain_kernel<BF16>), dim3((unsigned)n * H), dim3(256), smem, st, a);
+    else
+      hipLaunchKernelGGL((grouped_plain_kernel<F32>), dim3((unsigned)n * H), dim3(256), smem, st, a);
+    ZP_LAUNCH_CHECK();
+    return ZP_OK;
+  }
+  a.htiles = (H / HK + 15) / 16;
+  a.lds_pages = (int)pages;
+  a.splits = rows_splits(n, H, HK, window, chunk, NB, BS);
+  ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_grouped_rows_workspace(n, H, HK, D, V, window, chunk, NB, BS, dtype)),
+             "grouped_rows_attention: workspace too small");
+  const int dk = D / 32;
+  if (V <= 128) {
+    if (dk <= 2) return launch_rows<2, 1>(a, st);
+    if (dk <= 4) return launch_rows<4, 1>(a, st);
+    return launch_rows<8, 1>(a, st);
+  }
+  if (dk <= 4) return launch_rows<4, 2>(a, st);
+  return launch_rows<8, 2>(a, st);
+}

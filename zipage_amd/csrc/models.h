@@ -3,6 +3,14 @@
 #include "common.h"
 #include "../../include/zipage_models.h"
 
+#define ZP_MODEL_DTYPE(name)                                       \
+  if (dtype != ZP_BF16 && dtype != ZP_F32) {                       \
+    zp_set_error(name ": bfloat16 and float32 only");              \
+    return ZP_EUNSUPPORTED;                                        \
+  }
+
+static inline bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
+
 typedef uint32_t zp_u32x4 __attribute__((ext_vector_type(4)));
 typedef float zp_f32x4 __attribute__((ext_vector_type(4)));
 

@@ -1,0 +1,528 @@
+// Mixture of experts, without a host decision anywhere: every launch shape follows from the number of
+// tokens, so a step can be captured into a graph.
+//
+//   small_linear     products with few outputs whose result stays in fp32 (router logits)
+//   moe_select       softmax, the best groups of experts, the best experts of those
+//   moe_plan         assignments in the order of their experts, and the list of row tiles
+//   moe_gate_up      both input products of an expert for a row tile, its activation and the weight
+//   moe_down         the output product; each assignment's row goes to the plane of its slot
+//
+// An assignment is (token n, slot j), written n * (top + 1) + j; slot `top` is the shared expert's,
+// which every token uses with weight 1 and which counts as expert E.  Without a shared expert slots
+// are 0 .. top - 1.
+//
+// Expert weights are kept in the order the matrix cores read them: [out / 16][in / step][lane][16
+// bytes], where lane (g, r) holds row r and elements g * 16 bytes .. of a step of 64 bytes per row; a
+// wave's operand is then one contiguous KB.  W is the row operand: a lane ends with four consecutive
+// outputs of one token.
+#include "mfma.h"
+
+namespace {
+
+template <typename T> struct Mma;
+template <> struct Mma<BF16> {
+  static constexpr int kStep = 32;
+  __device__ static __forceinline__ f32x4 go(const u32x4& w, const u32x4& x, const f32x4& c) { return mfma_bf16(w, x, c); }
+  __device__ static __forceinline__ void st4(void* p, int64_t i, const float* v) {
+    uint2 o;
+    o.x = pack_bf16(v[0], v[1]);
+    o.y = pack_bf16(v[2], v[3]);
+    *(uint2*)((uint16_t*)p + i) = o;
+  }
+};
+template <> struct Mma<F32> {
+  static constexpr int kStep = 16;
+  __device__ static __forceinline__ f32x4 go(const u32x4& w, const u32x4& x, f32x4 c) {
+    const f32x4 a = __builtin_bit_cast(f32x4, w), b = __builtin_bit_cast(f32x4, x);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+    return c;
+  }
+  __device__ static __forceinline__ void st4(void* p, int64_t i, const float* v) {
+    *(f32x4*)((float*)p + i) = f32x4{v[0], v[1], v[2], v[3]};
+  }
+};
+template <typename T> constexpr int kPiece = 16 / T::bytes;   // elements a lane holds per step
+
+// ------------------------------------------------------------------ few outputs, fp32
+struct SmallArgs {
+  const void* x;    // token rows of x_st elements
+  const void* w;    // (M, K)
+  float* out;       // (n, M)
+  int n, K, M;
+  int64_t x_st;
+};
+
+// 16 tokens x 16 * MT outputs per workgroup, its four waves share the contraction.
+template <typename T, int MT>
+__global__ __launch_bounds__(256) void small_linear_kernel(SmallArgs a) {
+  __shared__ float red[3][MT * 64 * 4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+  const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16 * MT;
+  const int steps = a.K / Mma<T>::kStep;
+  const char* x = (const char*)a.x + ((int64_t)min(n0 + l16, a.n - 1) * a.x_st + g * kPiece<T>) * T::bytes;
+  const char* w[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+    w[t] = (const char*)a.w + ((int64_t)min(m0 + t * 16 + l16, a.M - 1) * a.K + g * kPiece<T>) * T::bytes;
+  f32x4 acc[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int ks = wave; ks < steps; ks += 4) {
+    const u32x4 xf = *(const u32x4*)(x + (int64_t)ks * 64);
+#pragma unroll
+    for (int t = 0; t < MT; ++t) acc[t] = Mma<T>::go(*(const u32x4*)(w[t] + (int64_t)ks * 64), xf, acc[t]);
+  }
+  if (wave > 0) {
+#pragma unroll
+    for (int t = 0; t < MT; ++t) *(f32x4*)(red[wave - 1] + (t * 64 + lane) * 4) = acc[t];
+  }
+  __syncthreads();
+  if (wave > 0) return;
+  const int n = n0 + l16;
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+#pragma unroll
+    for (int k = 0; k < 3; ++k) acc[t] += *(const f32x4*)(red[k] + (t * 64 + lane) * 4);
+    const int m = m0 + t * 16 + g * 4;
+    if (n < a.n && m < a.M) *(f32x4*)(a.out + (int64_t)n * a.M + m) = acc[t];
+  }
+}
+
+// ------------------------------------------------------------------ selection
+constexpr int kMaxExperts = 1024;
+
+struct SelectArgs {
+  const float* z;     // (n, z_st) router logits
+  int32_t* ids;       // (n, top)
+  float* weights;     // (n, top)
+  int32_t* counts;    // (E + 1,), cleared here
+  int n, E, top, groups, keep, z_st;
+};
+
+__device__ __forceinline__ int lowest_holder(float best, const float* v, int per) {
+  // smallest index lane + 64 j whose value is `best`
+  for (int j = 0; j < per; ++j) {
+    const uint64_t b = __ballot(v[j] == best);
+    if (b) return j * 64 + __builtin_ctzll(b);
+  }
+  return 0;
+}
+
+// A wave per token.  PER values per lane: expert (or group) lane + 64 j.
+template <int PER>
+__global__ __launch_bounds__(256) void moe_select_kernel(SelectArgs a) {
+  extern __shared__ float lds[];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  if (blockIdx.x == 0)
+    for (int e = threadIdx.x; e <= a.E; e += 256) a.counts[e] = 0;
+  const int n = blockIdx.x * 4 + wave;
+  float* const zl = lds + wave * a.E;
+  float z[PER];
+  float mx = -INFINITY;
+  if (n < a.n) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int e = lane + 64 * j;
+      z[j] = e < a.E ? a.z[(int64_t)n * a.z_st + e] : -INFINITY;
+      if (e < a.E) zl[e] = z[j];
+      mx = fmaxf(mx, z[j]);
+    }
+  }
+  __syncthreads();
+  if (n >= a.n) return;
+  mx = wave_max(mx);
+  float sum = 0.f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) sum += expf(z[j] - mx);
+  const float inv = 1.f / wave_sum(sum);
+  const int gs = a.E / a.groups;
+  if (a.keep < a.groups) {
+    float gm[PER];
+    uint32_t kept = 0;                          // bit j: group lane + 64 j
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int gr = lane + 64 * j;
+      gm[j] = -INFINITY;
+      if (gr < a.groups)
+        for (int i = 0; i < gs; ++i) gm[j] = fmaxf(gm[j], zl[gr * gs + i]);
+    }
+    for (int k = 0; k < a.keep; ++k) {
+      float b = -INFINITY;
+#pragma unroll
+      for (int j = 0; j < PER; ++j) b = fmaxf(b, gm[j]);
+      b = wave_max(b);
+      const int gr = lowest_holder(b, gm, PER);
+#pragma unroll
+      for (int j = 0; j < PER; ++j)
+        if (gr == lane + 64 * j) { gm[j] = -INFINITY; kept |= 1u << j; }
+    }
+    // experts of the other groups leave: group g's bit is in lane g % 64
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int e = min(lane + 64 * j, a.E - 1), gr = e / gs;
+      const uint32_t bits = (uint32_t)__shfl((int)kept, gr & 63);
+      if (!((bits >> (gr >> 6)) & 1u)) z[j] = -INFINITY;
+    }
+  }
+  for (int k = 0; k < a.top; ++k) {
+    float b = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) b = fmaxf(b, z[j]);
+    b = wave_max(b);
+    const int e = lowest_holder(b, z, PER);
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (e == lane + 64 * j) z[j] = -INFINITY;
+    if (lane == 0) {
+      a.ids[(int64_t)n * a.top + k] = e;
+      a.weights[(int64_t)n * a.top + k] = expf(b - mx) * inv;
+    }
+  }
+}
+
+// ------------------------------------------------------------------ plan
+struct PlanArgs {
+  const int32_t* ids;     // (n, top)
+  int32_t* counts;        // (E + 1,) zero before the first plan launch (large plans)
+  int32_t* base;          // (blocks, E) large plans
+  int32_t* offsets;       // (E + 2,)
+  int32_t* sorted;        // (n * slots,) assignments by expert
+  int32_t* tiles;         // (max_tiles, 4): expert, first position in `sorted`, rows, 0
+  int32_t* ntiles;
+  int n, E, top, shared, rows, max_tiles;   // rows: most rows per tile
+};
+constexpr int kPlanThreads = 1024;
+constexpr int kPlanBlock = 4096;    // assignments per workgroup of a large plan
+
+// Exclusive prefix sum of one value per thread over the workgroup.
+__device__ __forceinline__ int block_prefix(int v, int* red) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int inc = wave_prefix_sum_incl(v);
+  __syncthreads();
+  if (lane == 63) red[wave] = inc;
+  __syncthreads();
+  int before = 0;
+  for (int w = 0; w < wave; ++w) before += red[w];
+  return before + inc - v;
+}
+
+// Offsets and tiles from the counts in LDS (E of them); the shared expert's rows follow the others'.
+__device__ __forceinline__ void offsets_and_tiles(const PlanArgs& a, const int* counts, int* offsets, int* red) {
+  const int e = threadIdx.x;
+  const int c = e < a.E ? counts[e] : (e == a.E && a.shared ? a.n : 0);
+  const int at = block_prefix(c, red);
+  const int t = (c + a.rows - 1) / a.rows;
+  const int first = block_prefix(t, red);
+  if (e <= a.E) {
+    offsets[e] = at;
+    for (int i = 0; i < t; ++i)
+      if (first + i < a.max_tiles)
+        *(int4*)(a.tiles + (int64_t)(first + i) * 4) = make_int4(e, at + i * a.rows, min(a.rows, c - i * a.rows), 0);
+    if (e == a.E) *a.ntiles = min(first + t, a.max_tiles);
+  }
+  __syncthreads();
+}
+
+__global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(PlanArgs a) {
+  __shared__ int counts[kMaxExperts], offsets[kMaxExperts + 1], red[kPlanThreads / 64];
+  const int tid = threadIdx.x, total = a.n * a.top, slots = a.top + a.shared;
+  counts[tid] = 0;
+  __syncthreads();
+  for (int i = tid; i < total; i += kPlanThreads) atomicAdd(&counts[min(max(a.ids[i], 0), a.E - 1)], 1);
+  __syncthreads();
+  offsets_and_tiles(a, counts, offsets, red);
+  for (int i = tid; i < total; i += kPlanThreads) {
+    const int e = min(max(a.ids[i], 0), a.E - 1);
+    const int n = i / a.top;
+    a.sorted[atomicAdd(&offsets[e], 1)] = n * slots + i - n * a.top;
+  }
+  if (a.shared)
+    for (int n = tid; n < a.n; n += kPlanThreads) a.sorted[total + n] = n * slots + a.top;
+}
+
+// Large plans in three launches: each workgroup's counts claim a place behind the counts of others;
+// offsets and tiles; placement.
+__global__ __launch_bounds__(kPlanThreads) void moe_count_kernel(PlanArgs a) {
+  __shared__ int counts[kMaxExperts];
+  const int tid = threadIdx.x, total = a.n * a.top, i0 = blockIdx.x * kPlanBlock;
+  counts[tid] = 0;
+  __syncthreads();
+  for (int i = i0 + tid; i < min(i0 + kPlanBlock, total); i += kPlanThreads)
+    atomicAdd(&counts[min(max(a.ids[i], 0), a.E - 1)], 1);
+  __syncthreads();
+  if (tid < a.E) a.base[(int64_t)blockIdx.x * a.E + tid] = atomicAdd(&a.counts[tid], counts[tid]);
+}
+__global__ __launch_bounds__(kPlanThreads) void moe_offsets_kernel(PlanArgs a) {
+  __shared__ int counts[kMaxExperts], offsets[kMaxExperts + 1], red[kPlanThreads / 64];
+  const int tid = threadIdx.x;
+  counts[tid] = tid < a.E ? a.counts[tid] : 0;
+  __syncthreads();
+  offsets_and_tiles(a, counts, offsets, red);
+  for (int e = tid; e <= a.E; e += kPlanThreads) a.offsets[e] = offsets[e];
+}
+__global__ __launch_bounds__(kPlanThreads) void moe_place_kernel(PlanArgs a) {
+  __shared__ int at[kMaxExperts];
+  const int tid = threadIdx.x, total = a.n * a.top, i0 = blockIdx.x * kPlanBlock, slots = a.top + a.shared;
+  if (tid < a.E) at[tid] = a.offsets[tid] + a.base[(int64_t)blockIdx.x * a.E + tid];
+  __syncthreads();
+  for (int i = i0 + tid; i < min(i0 + kPlanBlock, total); i += kPlanThreads) {
+    const int n = i / a.top;
+    a.sorted[atomicAdd(&at[min(max(a.ids[i], 0), a.E - 1)], 1)] = n * slots + i - n * a.top;
+  }
+  if (a.shared)
+    for (int n = blockIdx.x * kPlanThreads + tid; n < a.n; n += gridDim.x * kPlanThreads)
+      a.sorted[total + n] = n * slots + a.top;
+}
+
+// ------------------------------------------------------------------ expert products
+struct ExpertArgs {
+  const void* x;          // gate_up: (n, K) tokens; down: (n * slots, K) rows by position in `sorted`
+  const void* w;          // routed experts, back to back
+  const void* w_shared;
+  void* out;              // gate_up: (n * slots, o_st); down: planes (slots, n, o_st)
+  const int32_t* sorted;
+  const int32_t* tiles;
+  const int32_t* ntiles;
+  const float* weights;   // (n, top)
+  int n, E, top, slots, max_tiles;
+  int K, K_shared;        // contraction, routed and shared
+  int M, M_shared;        // outputs (gate_up: of the gate alone)
+  int64_t x_st, o_st, w_expert;   // w_expert: elements between experts
+  float limit, limit_shared;
+};
+
+// g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(1.702 g) (u + 1)
+template <typename T> __device__ __forceinline__ float gated(float gate, float up, float limit);
+template <> __device__ __forceinline__ float gated<F32>(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+}
+template <> __device__ __forceinline__ float gated<BF16>(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-1.702f * g)) * (u + 1.f);
+}
+
+// Few rows per expert: the weights are streamed straight into registers, each wave its own 32 rows of
+// W (gate_up: 16 of the gate and the 16 of `up` that belong to them) against 16 * MT tokens.
+template <typename T, int MT, bool UP>
+__global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const int tile = blockIdx.x % a.max_tiles, cb = blockIdx.x / a.max_tiles;
+  if (tile >= *a.ntiles) return;
+  const int4 t = *(const int4*)(a.tiles + (int64_t)tile * 4);
+  const bool shared = t.x == a.E;
+  const int M = shared ? a.M_shared : a.M, K = shared ? a.K_shared : a.K;
+  const int pair = cb * 4 + wave;                    // of 16-row tiles of W
+  if (pair * (UP ? 16 : 32) >= M) return;
+  const int steps = K / Mma<T>::kStep;
+  const char* w = (const char*)(shared ? a.w_shared : a.w) +
+                  ((shared ? 0 : t.x * a.w_expert) + (int64_t)pair * 32 * K) * T::bytes + lane * 16;
+  const bool two = UP || pair * 32 + 16 < M;         // outputs are a multiple of 16
+  const int64_t wt = two ? (int64_t)16 * K * T::bytes : 0;
+  const char* x[MT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const int pos = t.y + min(i * 16 + l16, t.z - 1);
+    const int64_t row = UP ? a.sorted[pos] / a.slots : pos;
+    x[i] = (const char*)a.x + (row * a.x_st + g * kPiece<T>) * T::bytes;
+  }
+  f32x4 acc[2][MT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i) acc[0][i] = acc[1][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int ks = 0; ks < steps; ++ks) {
+    const u32x4 w0 = *(const u32x4*)(w + (int64_t)ks * 1024), w1 = *(const u32x4*)(w + wt + (int64_t)ks * 1024);
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const u32x4 xf = *(const u32x4*)(x[i] + (int64_t)ks * 64);
+      acc[0][i] = Mma<T>::go(w0, xf, acc[0][i]);
+      acc[1][i] = Mma<T>::go(w1, xf, acc[1][i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    if (i * 16 + l16 >= t.z) continue;
+    const int pos = t.y + i * 16 + l16;
+    const int as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
+    if constexpr (UP) {
+      const float wgt = slot < a.top ? a.weights[(int64_t)n * a.top + slot] : 1.f;
+      const float lim = shared ? a.limit_shared : a.limit;
+      float r[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) r[k] = wgt * gated<T>(acc[0][i][k], acc[1][i][k], lim);
+      Mma<T>::st4(a.out, (int64_t)pos * a.o_st + pair * 16 + g * 4, r);
+    } else {
+      const int64_t at = ((int64_t)slot * a.n + n) * a.o_st + pair * 32 + g * 4;
+      float r[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) r[k] = acc[0][i][k];
+      Mma<T>::st4(a.out, at, r);
+      if (two) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) r[k] = acc[1][i][k];
+        Mma<T>::st4(a.out, at + 16, r);
+      }
+    }
+  }
+}
+
+template <bool UP> int launch_experts(const ExpertArgs& a, int rows, int dtype, hipStream_t st) {
+  const int per = UP ? 64 : 128;                     // outputs per workgroup
+  const int M = a.M > a.M_shared ? a.M : a.M_shared;
+  const int64_t grid = (int64_t)a.max_tiles * ((M + per - 1) / per);
+  if (grid >= (1ll << 31)) {
+    zp_set_error("moe: too many tiles");
+    return ZP_EUNSUPPORTED;
+  }
+#define ZP_EXPERTS(T, MT) hipLaunchKernelGGL((expert_rows_kernel<T, MT, UP>), dim3((unsigned)grid), dim3(256), 0, st, a)
+#define ZP_EXPERT_ROWS(T)                 \
+  do {                                    \
+    if (rows == 16) ZP_EXPERTS(T, 1);     \
+    else if (rows == 32) ZP_EXPERTS(T, 2);\
+    else ZP_EXPERTS(T, 4);                \
+  } while (0)
+  if (dtype == ZP_BF16) ZP_EXPERT_ROWS(BF16); else ZP_EXPERT_ROWS(F32);
+#undef ZP_EXPERT_ROWS
+#undef ZP_EXPERTS
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+// Rows per tile: enough for the average expert.
+int tile_rows(int n, int E, int top) {
+  const int64_t avg = ((int64_t)n * top + E - 1) / E;
+  return avg <= 12 ? 16 : (avg <= 24 ? 32 : 64);
+}
+int tile_bound(int n, int E, int top, int shared, int rows) {
+  const int64_t a = (int64_t)n * top;
+  const int64_t used = a < E ? a : E;
+  return (int)(a / rows + used + (shared ? (n + rows - 1) / rows : 0));
+}
+
+}  // namespace
+
+extern "C" int zp_small_linear(const void* x, const void* w, float* out, int32_t n, int32_t K, int32_t M,
+                               int64_t x_stride, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && K > 0 && M > 0 && x_stride >= K, "small_linear: bad dims");
+  ZP_MODEL_DTYPE("small_linear");
+  if (K % 32 != 0 || M % 4 != 0 || x_stride % 8 != 0) {
+    zp_set_error("small_linear: K %d, M %d unsupported (multiples of 32 and 4)", K, M);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(x && w && out && aligned16(x) && aligned16(w) && aligned16(out), "small_linear: null or unaligned pointer");
+  SmallArgs a = {x, w, out, n, K, M, x_stride};
+  hipStream_t st = (hipStream_t)stream;
+  const unsigned gx = (unsigned)((n + 15) / 16);
+  const bool wide = gx >= 256 && M > 16;
+  const dim3 grid(gx, (unsigned)(wide ? (M + 63) / 64 : (M + 15) / 16));
+#define ZP_SMALL(T)                                                                              \
+  do {                                                                                           \
+    if (wide) hipLaunchKernelGGL((small_linear_kernel<T, 4>), grid, dim3(256), 0, st, a);        \
+    else hipLaunchKernelGGL((small_linear_kernel<T, 1>), grid, dim3(256), 0, st, a);             \
+  } while (0)
+  if (dtype == ZP_BF16) ZP_SMALL(BF16); else ZP_SMALL(F32);
+#undef ZP_SMALL
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_moe_select(const float* logits, int32_t* ids, float* weights, int32_t* counts, int32_t n,
+                             int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t logits_stride,
+                             void* stream) {
+  ZP_REQUIRE(n >= 0 && E > 0 && top > 0 && groups > 0 && E % groups == 0 && keep > 0 && keep <= groups &&
+                 top <= E / groups * keep && logits_stride >= E, "moe_select: bad dims");
+  if (E > kMaxExperts - 1) {
+    zp_set_error("moe_select: %d experts (at most %d)", E, kMaxExperts - 1);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(logits && ids && weights && counts, "moe_select: null pointer");
+  SelectArgs a = {logits, ids, weights, counts, n, E, top, groups, keep, logits_stride};
+  const dim3 grid((unsigned)((n + 3) / 4));
+  const size_t smem = sizeof(float) * 4 * E;
+  hipStream_t st = (hipStream_t)stream;
+  if (E <= 64) hipLaunchKernelGGL((moe_select_kernel<1>), grid, dim3(256), smem, st, a);
+  else if (E <= 256) hipLaunchKernelGGL((moe_select_kernel<4>), grid, dim3(256), smem, st, a);
+  else hipLaunchKernelGGL((moe_select_kernel<16>), grid, dim3(256), smem, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int64_t zp_moe_tile_rows(int32_t n, int32_t E, int32_t top, int32_t dtype) {
+  (void)dtype;
+  return n <= 0 || E <= 0 || top <= 0 ? -1 : tile_rows(n, E, top);
+}
+extern "C" int64_t zp_moe_max_tiles(int32_t n, int32_t E, int32_t top, int32_t shared, int32_t rows) {
+  return n <= 0 || E <= 0 || top <= 0 || rows <= 0 ? -1 : tile_bound(n, E, top, shared, rows);
+}
+extern "C" int64_t zp_moe_plan_workspace(int32_t n, int32_t E, int32_t top) {
+  if (n <= 0 || E <= 0 || top <= 0) return -1;
+  return ((int64_t)(((int64_t)n * top + kPlanBlock - 1) / kPlanBlock) * E + E + 2) * 4;
+}
+
+extern "C" int zp_moe_plan(const int32_t* ids, int32_t* counts, int32_t* sorted, int32_t* tiles, int32_t* ntiles,
+                           int32_t n, int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles,
+                           void* workspace, int64_t workspace_bytes, void* stream) {
+  ZP_REQUIRE(n > 0 && E > 0 && E < kMaxExperts && top > 0 && rows > 0 && (shared == 0 || shared == 1) &&
+                 max_tiles >= tile_bound(n, E, top, shared, rows), "moe_plan: bad dims");
+  ZP_REQUIRE(ids && counts && sorted && tiles && ntiles && aligned16(tiles), "moe_plan: null or unaligned pointer");
+  ZP_REQUIRE((int64_t)n * (top + shared) < (1ll << 31), "moe_plan: too many tokens");
+  PlanArgs a = {ids, counts, nullptr, nullptr, sorted, tiles, ntiles, n, E, top, shared, rows, max_tiles};
+  hipStream_t st = (hipStream_t)stream;
+  if ((int64_t)n * top <= 2 * kPlanBlock) {
+    hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(kPlanThreads), 0, st, a);
+    ZP_LAUNCH_CHECK();
+    return ZP_OK;
+  }
+  ZP_REQUIRE(workspace && workspace_bytes >= zp_moe_plan_workspace(n, E, top), "moe_plan: workspace too small");
+  a.offsets = (int32_t*)workspace;
+  a.base = a.offsets + E + 2;
+  const unsigned blocks = (unsigned)(((int64_t)n * top + kPlanBlock - 1) / kPlanBlock);
+  hipLaunchKernelGGL(moe_count_kernel, dim3(blocks), dim3(kPlanThreads), 0, st, a);
+  hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(kPlanThreads), 0, st, a);
+  hipLaunchKernelGGL(moe_place_kernel, dim3(blocks), dim3(kPlanThreads), 0, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+static int experts(bool up, const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
+                   const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n, int32_t E,
+                   int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared,
+                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
+                   float limit_shared, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && E > 0 && top > 0 && max_tiles > 0 && K > 0 && M > 0 && (!shared || (K_shared > 0 && M_shared > 0)),
+             "moe experts: bad dims");
+  ZP_MODEL_DTYPE("moe experts");
+  if (K % 32 || K_shared % 32 || M % 16 || M_shared % 16 || x_stride % 8 || out_stride % 8 || (rows != 16 && rows != 32 && rows != 64)) {
+    zp_set_error("moe experts: sizes %d x %d, shared %d x %d, %d rows per tile unsupported", M, K, M_shared, K_shared, rows);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(x && w && (!shared || w_shared) && out && sorted && tiles && ntiles && (!up || weights), "moe experts: null pointer");
+  ZP_REQUIRE(aligned16(x) && aligned16(w) && aligned16(w_shared) && aligned16(out) && aligned16(tiles) &&
+                 x_stride >= (K > K_shared ? K : K_shared) && out_stride >= (M > M_shared ? M : M_shared),
+             "moe experts: unaligned or overlapping rows");
+  ExpertArgs a = {x, w, w_shared, out, sorted, tiles, ntiles, weights, n, E, top, top + shared, max_tiles, K, K_shared,
+                  M, shared ? M_shared : 0, x_stride, out_stride, (int64_t)M * K * (up ? 2 : 1), limit, limit_shared};
+  return up ? launch_experts<true>(a, rows, dtype, (hipStream_t)stream)
+            : launch_experts<false>(a, rows, dtype, (hipStream_t)stream);
+}
+
+extern "C" int zp_moe_gate_up(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
+                              const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n,
+                              int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K,
+                              int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
+                              float limit_shared, int32_t dtype, void* stream) {
+  return experts(true, x, w, w_shared, out, sorted, tiles, ntiles, weights, n, E, top, shared, rows, max_tiles, K, K,
+                 M, M_shared, x_stride, out_stride, limit, limit_shared, dtype, stream);
+}
+extern "C" int zp_moe_down(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
+                           const int32_t* tiles, const int32_t* ntiles, int32_t n, int32_t E, int32_t top,
+                           int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared, int32_t M,
+                           int64_t x_stride, int64_t out_stride, int32_t dtype, void* stream) {
+  return experts(false, x, w, w_shared, out, sorted, tiles, ntiles, nullptr, n, E, top, shared, rows, max_tiles, K,
+                 K_shared, M, M, x_stride, out_stride, 0.f, 0.f, dtype, stream);
+}

@@ -1,6 +1,7 @@
 // Row kernels of decoders that keep their residual stream in fp32 whatever the dtype of their
-// matrix products: token + learned-position embedding, residual add, depth average over all earlier
-// layer results, RMS norm, and the xIELU activation.  Each is one pass over its rows (HBM- or
+// matrix products: token + learned-position embedding, residual add (of a branch output as it is or
+// normed), depth average over all earlier layer results, RMS norm, the xIELU activation, and the
+// soft cap of logits.  Each is one pass over its rows (HBM- or
 // launch-bound): the stream is read once, and what the next matrix product needs leaves the same
 // launch in that product's dtype.
 #include "models.h"
@@ -21,6 +22,8 @@ struct RowArgs {
   const void* y;          // n_y planes of (n, width) T
   int64_t y_plane;
   int n_y;
+  const float* yw;        // (width,) weight of an RMS norm on y before the add, or null
+  float embed_scale;
   // depth average: result_new = sum_j mix[j] * hist[j] + mix[n_hist] * (x + y)
   const float* hist;      // n_hist planes of (n, width) fp32
   int64_t hist_plane;     // elements between planes
@@ -35,15 +38,58 @@ struct RowArgs {
 };
 
 // One workgroup of THREADS per row; the row lives in registers.
-template <typename T, int THREADS, bool EMBED>
+template <int kW> __device__ __forceinline__ float row_sum(float v, float* red, int tid) {
+  v = wave_sum(v);
+  if (kW > 1) {
+    if ((tid & 63) == 0) red[tid >> 6] = v;
+    __syncthreads();
+    v = 0.f;
+#pragma unroll
+    for (int i = 0; i < kW; ++i) v += red[i];
+  }
+  return v;
+}
+
+template <typename T, int THREADS, bool EMBED, bool BRANCH>
 __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
   constexpr int kW = THREADS / 64;
-  __shared__ float red[kW];
+  __shared__ float red[kW], red_y[kW];
   const int tid = threadIdx.x;
   const int64_t row = blockIdx.x;
   const int pieces = a.width / 8;
   float v[kMaxPieces][8];
   float ss = 0.f;
+  float y[BRANCH ? kMaxPieces : 1][8];     // the normed branch: its sum first, the stream joins later
+  float ry = 0.f;
+  if constexpr (BRANCH) {
+#pragma unroll
+    for (int k = 0; k < kMaxPieces; ++k) {
+      const int pc = tid + k * THREADS;
+      if (pc < pieces) {
+        const int64_t at = row * a.width + pc * 8;
+        Vec8<T>::ld(a.y, at, y[k]);
+        int j = 1;
+        for (; j + 4 <= a.n_y; j += 4) {
+          float r[4][8];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) Vec8<T>::ld(a.y, (j + u) * a.y_plane + at, r[u]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[k][i] += r[u][i];
+        }
+        for (; j < a.n_y; ++j) {
+          float r[8];
+          Vec8<T>::ld(a.y, j * a.y_plane + at, r);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) y[k][i] += r[i];
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ry += y[k][i] * y[k][i];
+      }
+    }
+    ry = 1.f / sqrtf(row_sum<kW>(ry, red_y, tid) / (float)a.norm_width + a.eps);
+  }
   int64_t tok = 0, ps = 0;
   if (EMBED) {
     tok = a.tokens[row];
@@ -61,6 +107,8 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
       float r[8];
       if (EMBED) {
         Vec8<T>::ld(a.embed, tok * a.width + pc * 8, v[k]);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[k][i] *= a.embed_scale;
         if (a.pos) {
           Vec8<T>::ld(a.pos, ps * a.width + pc * 8, r);
 #pragma unroll
@@ -68,7 +116,11 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
         }
       } else {
         Vec8<F32>::ld(a.x, at, v[k]);
-        for (int j = 0; j < a.n_y; ++j) {
+        if constexpr (BRANCH) {
+          Vec8<F32>::ld(a.yw, pc * 8, r);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) v[k][i] += y[k][i] * ry * r[i];
+        } else for (int j = 0; j < a.n_y; ++j) {
           Vec8<T>::ld(a.y, j * a.y_plane + at, r);
 #pragma unroll
           for (int i = 0; i < 8; ++i) v[k][i] += r[i];
@@ -105,14 +157,7 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
     }
   }
   if (!a.w) return;
-  ss = wave_sum(ss);
-  if (kW > 1) {
-    if ((tid & 63) == 0) red[tid >> 6] = ss;
-    __syncthreads();
-    ss = 0.f;
-#pragma unroll
-    for (int i = 0; i < kW; ++i) ss += red[i];
-  }
+  ss = row_sum<kW>(ss, red, tid);
   const float rs = 1.f / sqrtf(ss / (float)a.norm_width + a.eps);
 #pragma unroll
   for (int k = 0; k < kMaxPieces; ++k) {
@@ -127,13 +172,13 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
   }
 }
 
-template <bool EMBED>
+template <bool EMBED, bool BRANCH = false>
 int launch_rows(const RowArgs& a, int n, int dtype, hipStream_t st) {
   const bool small = a.width <= 512;
 #define ZP_ROWS(T)                                                                             \
   do {                                                                                         \
-    if (small) hipLaunchKernelGGL((row_kernel<T, 64, EMBED>), dim3(n), dim3(64), 0, st, a);    \
-    else hipLaunchKernelGGL((row_kernel<T, 256, EMBED>), dim3(n), dim3(256), 0, st, a);        \
+    if (small) hipLaunchKernelGGL((row_kernel<T, 64, EMBED, BRANCH>), dim3(n), dim3(64), 0, st, a);    \
+    else hipLaunchKernelGGL((row_kernel<T, 256, EMBED, BRANCH>), dim3(n), dim3(256), 0, st, a);        \
   } while (0)
   if (dtype == ZP_BF16) ZP_ROWS(BF16); else ZP_ROWS(F32);
 #undef ZP_ROWS
@@ -168,15 +213,25 @@ __global__ __launch_bounds__(256) void xielu_kernel(const void* in, void* out, i
   Vec8<T>::st(out, id * 8, z);
 }
 
-bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
+// ------------------------------------------------------------------ soft cap
+// Logits leave in fp32: cap * tanh(z / cap).
+template <typename T>
+__global__ __launch_bounds__(256) void softcap_kernel(const void* in, float* out, int64_t count, float cap, float inv) {
+  const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 8;
+  if (i >= count) return;
+  if (i + 8 <= count) {
+    float z[8];
+    Vec8<T>::ld(in, i, z);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) z[k] = cap * tanhf(z[k] * inv);
+    Vec8<F32>::st(out, i, z);
+  } else {
+    for (int64_t k = i; k < count; ++k) out[k] = cap * tanhf(Elem<T>::ld(in, k) * inv);
+  }
+}
 
 }  // namespace
 
-#define ZP_MODEL_DTYPE(name)                                       \
-  if (dtype != ZP_BF16 && dtype != ZP_F32) {                       \
-    zp_set_error(name ": bfloat16 and float32 only");              \
-    return ZP_EUNSUPPORTED;                                        \
-  }
 #define ZP_ROW_WIDTH(name)                                                                      \
   if (width % 8 != 0 || width > 8 * 256 * kMaxPieces) {                                         \
     zp_set_error(name ": width %d unsupported (multiple of 8, <= %d)", width, 8 * 256 * kMaxPieces); \
@@ -186,8 +241,8 @@ bool aligned16(const void* p) { return (uintptr_t)p % 16 == 0; }
 extern "C" int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* embed,
                              const void* pos, float* x, const float* norm_weight, void* out,
                              int32_t n, int32_t width, int32_t norm_width, int64_t vocab,
-                             int64_t max_positions, float eps, float weight_offset, int32_t dtype,
-                             void* stream) {
+                             int64_t max_positions, float embed_scale, float eps, float weight_offset,
+                             int32_t dtype, void* stream) {
   ZP_REQUIRE(n >= 0 && width > 0 && norm_width > 0 && norm_width <= width && vocab > 0,
              "embed_norm: bad dims");
   ZP_MODEL_DTYPE("embed_norm");
@@ -201,11 +256,12 @@ extern "C" int zp_embed_norm(const int64_t* tokens, const int32_t* positions, co
   a.tokens = tokens; a.positions = positions; a.embed = embed; a.pos = pos; a.vocab = vocab;
   a.max_positions = max_positions; a.x_out = x; a.w = norm_weight; a.out = out; a.width = width;
   a.norm_width = norm_width; a.eps = eps; a.offset = weight_offset; a.out_scale = 1.f;
+  a.embed_scale = embed_scale;
   return launch_rows<true>(a, n, dtype, (hipStream_t)stream);
 }
 
-extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* hist,
-                                int64_t hist_plane, const float* mix, int32_t n_hist,
+extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* y_weight,
+                                const float* hist, int64_t hist_plane, const float* mix, int32_t n_hist,
                                 float* result, float* x_out, const float* norm_weight, void* out,
                                 int32_t n, int32_t width, int32_t norm_width, float eps,
                                 float weight_offset, float out_scale, int32_t dtype, void* stream) {
@@ -217,13 +273,15 @@ extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, cons
   ZP_REQUIRE(x && y && (!norm_weight || out), "residual_norm: null pointer");
   ZP_REQUIRE(n_hist == 0 || (hist && mix && hist_plane >= (int64_t)n * width),
              "residual_norm: a depth average needs its weights and planes of n rows");
-  ZP_REQUIRE(aligned16(x) && aligned16(y) && aligned16(hist) && hist_plane % 4 == 0 && aligned16(result) &&
+  ZP_REQUIRE(aligned16(x) && aligned16(y) && aligned16(y_weight) && aligned16(hist) && hist_plane % 4 == 0 && aligned16(result) &&
                  aligned16(x_out) && aligned16(norm_weight) && aligned16(out),
              "residual_norm: tensors must be 16-byte aligned");
   RowArgs a = {};
   a.x = x; a.y = y; a.n_y = n_y; a.y_plane = (int64_t)n * width; a.hist = hist; a.hist_plane = hist_plane; a.mix = mix; a.n_hist = n_hist;
   a.result = result; a.x_out = x_out; a.w = norm_weight; a.out = out; a.width = width;
   a.norm_width = norm_width; a.eps = eps; a.offset = weight_offset; a.out_scale = out_scale;
+  a.yw = y_weight;
+  if (y_weight) return launch_rows<false, true>(a, n, dtype, (hipStream_t)stream);
   return launch_rows<false>(a, n, dtype, (hipStream_t)stream);
 }
 
@@ -240,6 +298,19 @@ extern "C" int zp_xielu(const void* in, void* out, int64_t count, float alpha_p,
     hipLaunchKernelGGL((xielu_kernel<BF16>), dim3(grid), dim3(256), 0, st, in, out, pieces, alpha_p, alpha_n);
   else
     hipLaunchKernelGGL((xielu_kernel<F32>), dim3(grid), dim3(256), 0, st, in, out, pieces, alpha_p, alpha_n);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_softcap(const void* in, float* out, int64_t count, float cap, int32_t dtype, void* stream) {
+  ZP_REQUIRE(count >= 0 && cap > 0.f, "softcap: bad arguments");
+  ZP_MODEL_DTYPE("softcap");
+  if (count == 0) return ZP_OK;
+  ZP_REQUIRE(in && out && aligned16(in) && aligned16(out), "softcap: null or unaligned pointer");
+  const unsigned grid = (unsigned)((count + 2047) / 2048);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == ZP_BF16) hipLaunchKernelGGL((softcap_kernel<BF16>), dim3(grid), dim3(256), 0, st, in, out, count, cap, 1.f / cap);
+  else hipLaunchKernelGGL((softcap_kernel<F32>), dim3(grid), dim3(256), 0, st, in, out, count, cap, 1.f / cap);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }

@@ -1,0 +1,283 @@
+// Attention of runs of prompt tokens, and the gather of the cached rows they look back on.
+#include "mfma.h"
+
+namespace {
+
+// ------------------------------------------------------------------ gather of cached rows
+__global__ __launch_bounds__(256) void gather_rows_kernel(const char* src, const int32_t* rows, char* out,
+                                                          int64_t total, int pieces, int64_t num_rows) {
+  const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (id >= total) return;
+  const int64_t r = id / pieces, pc = id - r * pieces;
+  int64_t s = rows[r];
+  if (s < 0 || s >= num_rows) s = 0;
+  ((u32x4*)out)[id] = ((const u32x4*)src)[s * pieces + pc];
+}
+
+// ------------------------------------------------------------------ runs of prompt tokens
+struct TilesArgs {
+  const uint16_t* q;      // token rows of q_st elements, head h at h * D
+  const uint16_t* k;      // key rows of kv_st elements, head h at h * D
+  const uint16_t* v;      // value rows of kv_st elements, head h at h * V
+  uint16_t* out;          // token rows of o_st elements, head h at h * V
+  const int32_t* tiles;   // (T, 4): first query row, queries, first key row of the run, position
+                          // of the first query counted from that key
+  const float* sinks;     // (H,) logits that only join the denominator, or null
+  int T, H, HK, D, V;     // HK key / value heads; query head h uses head h / (H / HK)
+  int window, chunk;      // at most one is set, see first_seen
+  int64_t q_rows, k_rows, q_st, kv_st, o_st;
+  float scale, out_scale;
+};
+
+constexpr int kTileQ = 128;   // queries per workgroup
+constexpr int kTileK = 64;    // keys per LDS tile
+
+// A workgroup owns up to 128 queries of one head; key and value tiles pass through LDS once for all of
+// them (double-buffered, the next tile's loads in flight during the products), a wave owns 16 * kQT
+// queries at a time and skips the 32-key steps none of them sees.
+// First key position a query sees: the last `window` up to and including its own, or those of its own
+// block of `chunk` positions (key 0 of the run starts a block), or all.
+__device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
+  if (window > 0) return max(0, pos - window + 1);
+  return chunk > 0 ? pos / chunk * chunk : 0;
+}
+
+template <int DKS, int VCB> struct TileStage {
+  static constexpr int kK = DKS * 32 + 8, kV = VCB * 128 + 8;    // row strides: rows 16 bytes apart in the banks
+  static constexpr int kElems = kTileK * (kK + kV);
+  static constexpr int kBytes = 2 * kElems * 2;
+};
+
+template <int DKS, int VCB, int kQT>
+__global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  typedef TileStage<DKS, VCB> Stage;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+  const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
+  const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
+  const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
+  // host-made descriptors: rows outside the buffers are not touched
+  if (q0 < 0 || kb < 0 || rel < 0 || (int64_t)q0 + nq > a.q_rows || (int64_t)kb + rel + nq > a.k_rows) return;
+  const int nks = a.D / 32;
+  const float sc = a.scale * 1.44269504088896f;
+  const int hk = h / (a.H / a.HK);
+  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + hk * a.D;
+  const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + hk * a.V;
+
+  for (int wg0 = 0; wg0 < nq; wg0 += 64 * kQT) {              // uniform in the workgroup
+    const int w0 = wg0 + wave * 16 * kQT;
+    const int last = rel + min(wg0 + 64 * kQT, nq) - 1;       // last key any query of the pass sees
+    const int first = first_seen(rel + wg0, a.window, a.chunk);
+    const int hi = w0 < nq ? rel + min(w0 + 16 * kQT, nq) - 1 : -1;      // the same for the wave
+    const int lo = first_seen(rel + w0, a.window, a.chunk);
+    const int lo_last = first_seen(rel + w0 + 16 * kQT - 1, a.window, a.chunk);
+
+    u32x4 qf[kQT][DKS];
+    int qpos[kQT], qlow[kQT];                                 // keys qlow .. qpos are seen
+#pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      const int qi = min(w0 + t * 16 + l16, nq - 1);
+      qpos[t] = rel + qi;
+      qlow[t] = first_seen(qpos[t], a.window, a.chunk);
+      const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + h * a.D + g * 8;
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) {
+        // D may end inside the last steps: they read the row's start, against zeros in q
+        qf[t][ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
+        if (ks >= nks) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
+      }
+    }
+    f32x4 o[kQT][VCB * 8];
+    float m[kQT], l[kQT];
+#pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      m[t] = -INFINITY;
+      l[t] = 0.f;
+#pragma unroll
+      for (int i = 0; i < VCB * 8; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+
+    u32x4 rk[DKS], rv[4 * VCB];                                // this thread's pieces of a tile
+    auto fetch = [&](int k0) {
+#pragma unroll
+      for (int j = 0; j < DKS; ++j) {
+        const int id = tid + 256 * j, r = id / (4 * DKS), c = (id % (4 * DKS)) * 8;
+        rk[j] = *(const u32x4*)(kbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.D ? c : 0));
+      }
+#pragma unroll
+      for (int j = 0; j < 4 * VCB; ++j) {
+        const int id = tid + 256 * j, r = id / (16 * VCB), c = (id % (16 * VCB)) * 8;
+        rv[j] = *(const u32x4*)(vbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.V ? c : 0));
+      }
+    };
+    fetch(first);
+    __syncthreads();                                           // a pass before this one still reads its tiles
+    int buf = 0;
+    for (int t0 = first; t0 <= last; t0 += kTileK, buf ^= 1) {
+      uint16_t* const ldsk = (uint16_t*)lds_raw + buf * Stage::kElems;
+      uint16_t* const ldsv = ldsk + kTileK * Stage::kK;
+#pragma unroll
+      for (int j = 0; j < DKS; ++j) {
+        const int id = tid + 256 * j;
+        *(u32x4*)(ldsk + id / (4 * DKS) * Stage::kK + (id % (4 * DKS)) * 8) = rk[j];
+      }
+#pragma unroll
+      for (int j = 0; j < 4 * VCB; ++j) {
+        const int id = tid + 256 * j;
+        *(u32x4*)(ldsv + id / (16 * VCB) * Stage::kV + (id % (16 * VCB)) * 8) = rv[j];
+      }
+      __syncthreads();
+      if (t0 + kTileK <= last) fetch(t0 + kTileK);
+#pragma unroll 1
+      for (int sub = 0; sub < kTileK; sub += 32) {
+        const int k0 = t0 + sub;
+        if (k0 > hi || k0 + 31 < lo) continue;                 // uniform in the wave
+        f32x4 s[kQT][2];
+#pragma unroll
+        for (int tt = 0; tt < 2; ++tt) {
+#pragma unroll
+          for (int t = 0; t < kQT; ++t) s[t][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int ks = 0; ks < DKS; ++ks) {
+            const u32x4 kf = *(const u32x4*)(ldsk + (sub + tt * 16 + l16) * Stage::kK + ks * 32 + g * 8);
+#pragma unroll
+            for (int t = 0; t < kQT; ++t) s[t][tt] = mfma_bf16(kf, qf[t][ks], s[t][tt]);
+          }
+        }
+        // every query of the wave sees all 32 keys: no masks
+        const bool inner = k0 + 31 <= rel + w0 && k0 >= lo_last;
+        u32x4 pf[kQT];
+#pragma unroll
+        for (int t = 0; t < kQT; ++t) {
+          float p[8], mx = -INFINITY;
+#pragma unroll
+          for (int i = 0; i < 8; ++i) p[i] = s[t][i >> 2][i & 3] * sc;
+          if (!inner) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+              const int key = k0 + step_key(g, i);
+              if (key > qpos[t] || key < qlow[t]) p[i] = -INFINITY;
+            }
+          }
+#pragma unroll
+          for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+          mx = fmaxf(mx, lane_xor16(mx));
+          mx = fmaxf(mx, lane_xor32(mx));
+          const float mn = fmaxf(m[t], mx);
+          const float ms = mn == -INFINITY ? 0.f : mn;          // a query whose window starts later
+          const float f = __builtin_amdgcn_exp2f(m[t] - ms);
+          float sum = 0.f;
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            p[i] = __builtin_amdgcn_exp2f(p[i] - ms);
+            sum += p[i];
+          }
+          l[t] = l[t] * f + sum;
+          m[t] = mn;
+          if (__any(f != 1.f)) {
+#pragma unroll
+            for (int i = 0; i < VCB * 8; ++i) o[t][i] *= f;
+          }
+          pf[t] = u32x4{pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]),
+                        pack_bf16(p[6], p[7])};
+        }
+#pragma unroll
+        for (int cb = 0; cb < VCB; ++cb) {
+          u32x4 v[8];
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            v[i] = *(const u32x4*)(ldsv + (sub + step_key(g, i)) * Stage::kV + cb * 128 + l16 * 8);
+#pragma unroll
+          for (int c = 0; c < 8; ++c) {
+            const u32x4 vf = column_of(v, c);
+#pragma unroll
+            for (int t = 0; t < kQT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
+          }
+        }
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < kQT; ++t) {
+      float lt = l[t];
+      lt += lane_xor16(lt);
+      lt += lane_xor32(lt);
+      if (a.sinks) lt += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - m[t]);
+      const float inv = lt > 0.f ? a.out_scale / lt : 0.f;
+      const int qi = w0 + t * 16 + l16;
+      if (qi >= nq) continue;
+      uint16_t* out = a.out + (int64_t)(q0 + qi) * a.o_st + h * a.V;
+#pragma unroll
+      for (int cb = 0; cb < VCB; ++cb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = cb * 128 + (4 * g + i) * 8;
+          if (col < a.V) {
+            float r[8];
+#pragma unroll
+            for (int c = 0; c < 8; ++c) r[c] = o[t][cb * 8 + c][i] * inv;
+            Vec8<BF16>::st(out, col, r);
+          }
+        }
+    }
+  }
+}
+
+template <int DKS, int VCB, int kQT> int launch_run_tiles(const TilesArgs& a, hipStream_t st) {
+  constexpr int smem = TileStage<DKS, VCB>::kBytes;
+  if (smem > 64 * 1024 &&
+      hipFuncSetAttribute((const void*)run_tiles_kernel<DKS, VCB, kQT>,
+                          hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
+    zp_set_error("run_attention: cannot reserve %d bytes of LDS", smem);
+    return ZP_EHIP;
+  }
+  hipLaunchKernelGGL((run_tiles_kernel<DKS, VCB, kQT>), dim3((unsigned)a.T * a.H), dim3(256), smem, st, a);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+}  // namespace
+
+extern "C" int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n,
+                              int32_t row_bytes, int64_t num_rows, void* stream) {
+  ZP_REQUIRE(n >= 0 && row_bytes > 0 && row_bytes % 16 == 0 && num_rows > 0, "gather_rows: bad dims");
+  if (n == 0) return ZP_OK;
+  ZP_REQUIRE(src && rows && out && aligned16(src) && aligned16(out), "gather_rows: null or unaligned pointer");
+  const int pieces = row_bytes / 16;
+  const int64_t total = (int64_t)n * pieces;
+  hipLaunchKernelGGL(gather_rows_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0,
+                     (hipStream_t)stream, (const char*)src, rows, (char*)out, total, pieces, num_rows);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_run_attention(const void* q, const void* k, const void* v, void* out,
+                                const int32_t* tiles, const float* sinks, int32_t T, int32_t H,
+                                int32_t HK, int32_t D, int32_t V, int32_t window, int32_t chunk,
+                                int64_t q_rows, int64_t k_rows, int64_t q_stride, int64_t kv_stride,
+                                int64_t out_stride, float scale, float out_scale, int32_t dtype,
+                                void* stream) {
+  ZP_REQUIRE(T >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && V > 0 && window >= 0 && chunk >= 0 &&
+                 !(window && chunk), "run_attention: bad dims");
+  if (dtype != ZP_BF16 || D % 32 != 0 || D > 256 || V % 8 != 0 || V > 256) {
+    zp_set_error("run_attention: bfloat16, D %d (multiple of 32, <= 256), V %d (multiple of 8, <= 256)", D, V);
+    return ZP_EUNSUPPORTED;
+  }
+  if (T == 0) return ZP_OK;
+  ZP_REQUIRE(q && k && v && out && tiles, "run_attention: null pointer");
+  ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && q_stride % 8 == 0 &&
+                 kv_stride % 8 == 0 && out_stride % 8 == 0 && q_stride >= (int64_t)H * D &&
+                 out_stride >= (int64_t)H * V && (int64_t)T * H < (1ll << 31),
+             "run_attention: unaligned rows or too many tiles");
+  TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (uint16_t*)out, tiles, sinks, T, H, HK,
+                 D, V, window, chunk, q_rows, k_rows, q_stride, kv_stride, out_stride, scale, out_scale};
+  hipStream_t st = (hipStream_t)stream;
+  const int dk = D / 32;
+  if (V <= 128) {
+    if (dk <= 2) return launch_run_tiles<2, 1, 2>(a, st);
+    if (dk <= 4) return launch_run_tiles<4, 1, 2>(a, st);
+    if (dk <= 6) return launch_run_tiles<6, 1, 2>(a, st);
+    return launch_run_tiles<8, 1, 2>(a, st);
+  }
+  if (dk <= 4) return launch_run_tiles<4, 2, 1>(a, st);
+  return launch_run_tiles<8, 2, 1>(a, st);
+}

@@ -1,4 +1,5 @@
 from .config import EngineConfig  # noqa: F401
+from .kapolorn import Kapolorn, KapolornShape  # noqa: F401
 from .llm import ZipageEngine  # noqa: F401
 from .pages import PagePool  # noqa: F401
 from .pedivik import Pedivik, PedivikLayer, PedivikShape  # noqa: F401

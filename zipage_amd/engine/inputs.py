@@ -5,6 +5,8 @@ from dataclasses import dataclass, field
 
 import numpy as np
 
+from zipage_amd.sight import first_seen
+
 from .sequence import Portion, Sequence
 
 HEADER_ROWS = 5   # query row, position, flat K/V slot, context length, token-log column
@@ -99,7 +101,7 @@ RUN_TILE = 128    # queries per entry of a run plan
 
 @dataclass
 class Runs:
-    """The multi-token portions of a step as the run attention reads them, for one window."""
+    """The multi-token portions of a step as the run attention reads them, for one kind of sight."""
     tiles: np.ndarray             # (T, 4): first query row, queries, first key row, rel. position
     key_slots: np.ndarray | None  # cache rows to gather as keys; None: the step's own tokens
 
@@ -114,16 +116,17 @@ class PortionPlan:
     table_rows: np.ndarray
     tables: np.ndarray            # (sequences, width), -1 where nothing is held
     first_row: list[int]          # token row where each portion starts, in the order given
+    segments: np.ndarray          # (4, portions): token row, tokens, query row, position of the first
     runs: dict = field(default_factory=dict)
 
 
-def plan_runs(portions: list[Portion], block_size: int, window: int | None) -> Runs:
+def plan_runs(portions: list[Portion], block_size: int, sight) -> Runs:
     """Key rows and query tiles of `portions`, whose tokens follow one another in the query rows.  A
-    run's keys start `window` - 1 tokens before its first token (at 0 without a window)."""
+    run's keys start with the first its first token sees."""
     tiles, slots, q, k = [], [], 0, 0
     own = True
     for p in portions:
-        k_first = 0 if window is None else max(0, p.start - window + 1)
+        k_first = first_seen(p.start, sight)
         own &= k_first == p.start
         for off in range(0, p.count, RUN_TILE):
             tiles.append((q + off, min(RUN_TILE, p.count - off), k, p.start - k_first + off))
@@ -136,7 +139,7 @@ def plan_runs(portions: list[Portion], block_size: int, window: int | None) -> R
                 None if own else np.concatenate(slots).astype(np.int32))
 
 
-def plan_portions(portions: list[Portion], block_size: int, windows, run_min: int | None) -> PortionPlan:
+def plan_portions(portions: list[Portion], block_size: int, sights, run_min: int | None) -> PortionPlan:
     """All inputs of a step that holds portions of any length.  Portions shorter than `run_min`
     (None: all) are attended token by token and come first."""
     short = [i for i, p in enumerate(portions) if run_min is None or p.count < run_min]
@@ -164,9 +167,11 @@ def plan_portions(portions: list[Portion], block_size: int, windows, run_min: in
         ctx.append(np.arange(p.start + 1, p.start + p.count + 1))
         trows.append(np.full(p.count, i))
     cat = lambda a: np.concatenate(a).astype(np.int32) if a else np.zeros(0, np.int32)
+    segments = np.array([[first_row[i], portions[i].count, portions[i].seq.query_id, portions[i].start]
+                         for i in short + long], np.int32).T
     plan = PortionPlan(np.asarray(ids, np.int32), np.asarray(rows, np.int32), cat(pos), cat(slots),
-                       cat(ctx), cat(trows), tables, first_row)
+                       cat(ctx), cat(trows), tables, first_row, segments)
     if long:
-        for w in windows:
+        for w in sights:
             plan.runs[w] = plan_runs([portions[i] for i in long], block_size, w)
     return plan

@@ -19,7 +19,7 @@ from zipage_amd.compress import StageTimer, compress_layers
 from .config import EngineConfig
 from .inputs import (Runs, encode_compress_tables, pack_decode, packed_words, plan_portions,
                      query_slot_mapping, unpack_views)
-from .qwen3 import StepContext
+from .qwen3 import Segments, StepContext
 from .registry import build_model
 from .sequence import Portion, Sequence
 
@@ -70,10 +70,11 @@ class ModelRunner:
     # ------------------------------------------------------------------ memory
     def allocate_kv_cache(self):
         """model_runner.py:219-307, with the page count given by the configuration.  A model that is
-        not compressed keeps its own kind of pages and no window queries."""
+        not compressed keeps its own kind of pages, or recurrent states by query row (with the scratch
+        row's), and no window queries."""
         cfg, s = self.cfg, self.cfg.shape
         if not self.model.compressible:
-            self.model.allocate_caches(cfg.num_kvcache_blocks, self.block_size)
+            self.model.allocate_caches(cfg.num_kvcache_blocks, self.block_size, cfg.max_concurrency + 1)
             return
         dt = self.model.dtype
         self.kv_cache = torch.zeros(2, s.layers, cfg.num_kvcache_blocks, self.block_size, s.kv_heads,
@@ -147,7 +148,8 @@ class ModelRunner:
     def _decode_hidden(self, buf: torch.Tensor, Bp: int, TW: int) -> torch.Tensor:
         """The part of the step a graph replays: embedding to final norm."""
         head, tables, triples = unpack_views(buf, Bp, TW)
-        ctx = StepContext(False, head[2], triples, head[3], tables, runs={})
+        ctx = StepContext(False, head[2], triples, head[3], tables, runs={},
+                          segments=Segments(None, head[3], head[0], head[1], max_count=1))
         return self.model.forward(self.last_token[head[0].long()], head[1].long(), ctx)
 
     def _decode_tail(self, buf: torch.Tensor, Bp: int, TW: int, hidden: torch.Tensor,
@@ -211,9 +213,9 @@ class ModelRunner:
     def prepare_portions(self, portions: list[Portion]):
         """One packed buffer for a step of portions: (ids, positions, ctx, first row per portion)."""
         m = self.model
-        plan = plan_portions(portions, self.block_size, m.windows, m.run_min)
+        plan = plan_portions(portions, self.block_size, m.sights, m.run_min)
         parts = [plan.ids, plan.rows, plan.positions, plan.slots, plan.context_lens, plan.table_rows,
-                 plan.tables.reshape(-1)]
+                 plan.tables.reshape(-1), *plan.segments]
         for r in plan.runs.values():
             parts += [r.tiles.reshape(-1)] + ([] if r.key_slots is None else [r.key_slots])
         host = torch.empty(sum(-(-len(a) // 4) * 4 for a in parts), dtype=torch.int32, pin_memory=True)
@@ -226,6 +228,7 @@ class ModelRunner:
         d = iter([buf[a:b] for a, b in spans])
         ids, rows, pos, slots, ctx_lens, table_rows = (next(d) for _ in range(6))
         tables = next(d).view(plan.tables.shape)
+        segments = Segments(*(next(d) for _ in range(4)))
         runs = {}
         for w, r in plan.runs.items():
             tiles = next(d).view(-1, 4)
@@ -233,7 +236,7 @@ class ModelRunner:
         ids = ids.long()
         if (plan.rows >= 0).any():
             ids = torch.where(rows >= 0, self.last_token[rows.clamp_min(0).long()], ids)
-        ctx = StepContext(False, slots, None, ctx_lens, tables, table_rows=table_rows, runs=runs)
+        ctx = StepContext(False, slots, None, ctx_lens, tables, table_rows=table_rows, runs=runs, segments=segments)
         return ids, pos, ctx, plan.first_row
 
     @staticmethod

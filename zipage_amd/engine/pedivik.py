@@ -16,7 +16,7 @@ import torch
 import torch.nn.functional as F
 
 from zipage_amd.layers.latent import LatentAttention
-from zipage_amd.layers.linear import ResidualLinear
+from zipage_amd.layers.linear import ResidualLinear, fit
 from zipage_amd.layers.residual import embed_norm, residual_norm, xielu
 
 
@@ -75,17 +75,12 @@ class PedivikShape:
         return cls(vocab, width, tuple(layers), max_positions, float(eps), float(logit_scale))
 
 
-def _pad_to(t: torch.Tensor, *shape: int) -> torch.Tensor:
-    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
-    out[tuple(slice(0, n) for n in t.shape)] = t
-    return out
-
-
 class Pedivik:
     # what the engine asks a model: no KV compression (every key inside the window counts), and
     # steps that hold portions of prompts beside decoded tokens
     compressible = False
     portions = True
+    recurrent = False
 
     def __init__(self, shape: PedivikShape, device, dtype=torch.bfloat16, seed: int = 0,
                  weights: dict[str, torch.Tensor] | None = None):
@@ -97,9 +92,9 @@ class Pedivik:
         self.vocab = shape.vocab
         self.mixers = [LatentAttention(shape.width, l.heads, l.dim, l.vdim, l.q_rank, l.kv_rank, l.scale,
                                        l.window, shape.eps) for l in shape.layers]
-        self.windows = sorted({l.window for l in shape.layers})
+        self.sights = sorted({l.window for l in shape.layers})
         # the furthest a token looks back, and the shortest portion attended as a run
-        self.lookback = max(self.windows, default=1)
+        self.lookback = max(self.sights, default=1)
         self.run_min = 16 if dtype == torch.bfloat16 and all(m.can_expand for m in self.mixers) else None
         self.caches: list[torch.Tensor] = []
         if weights is None:
@@ -123,9 +118,9 @@ class Pedivik:
 
         dev = lambda t, dt=None: t.to(device=self.device, dtype=dt or self.dtype).contiguous()
         f32 = lambda t: dev(t, torch.float32)
-        vec = lambda name: f32(_pad_to(get(name, s.width), W))
-        self.embed = dev(_pad_to(get("embed", s.vocab, s.width), s.vocab, W))
-        self.pos = dev(_pad_to(get("pos", s.max_positions, s.width), s.max_positions, W))
+        vec = lambda name: f32(fit(get(name, s.width), W))
+        self.embed = dev(fit(get("embed", s.vocab, s.width), s.vocab, W))
+        self.pos = dev(fit(get("pos", s.max_positions, s.width), s.max_positions, W))
         self.final_norm = vec("final.norm")
         self.layers = []
         for i, (l, mixer) in enumerate(zip(s.layers, self.mixers)):
@@ -138,8 +133,8 @@ class Pedivik:
             if l.ff is not None:
                 ffp = -(-l.ff // 8) * 8
                 p["norm2"] = vec(pre + "norm2")
-                p["up"] = dev(_pad_to(get(pre + "mlp.up", l.ff, s.width), ffp, W))
-                p["down"] = ResidualLinear(dev(_pad_to(get(pre + "mlp.down", s.width, l.ff), W, ffp)))
+                p["up"] = dev(fit(get(pre + "mlp.up", l.ff, s.width), ffp, W))
+                p["down"] = ResidualLinear(dev(fit(get(pre + "mlp.down", s.width, l.ff), W, ffp)))
                 act = get(pre + "mlp.act", 2).double().tolist()
                 softplus = lambda a: math.log1p(math.exp(-abs(a))) + max(a, 0.0)
                 p["act"] = (softplus(act[0]), 0.5 + softplus(act[1]))
@@ -155,8 +150,7 @@ class Pedivik:
         g = torch.Generator(device=self.device).manual_seed(seed)
         w = lambda *d: torch.empty(*d, device=self.device, dtype=self.dtype).normal_(0.0, std, generator=g)
         zeros = lambda: torch.zeros(W, device=self.device)
-        self.embed, self.pos = _pad_to(w(s.vocab, s.width), s.vocab, W), _pad_to(w(s.max_positions, s.width),
-                                                                              s.max_positions, W)
+        self.embed, self.pos = fit(w(s.vocab, s.width), s.vocab, W), fit(w(s.max_positions, s.width), s.max_positions, W)
         self.final_norm = zeros()
         self.layers = []
         for i, (l, mixer) in enumerate(zip(s.layers, self.mixers)):
@@ -164,12 +158,12 @@ class Pedivik:
             p = dict(norm1=zeros(), dwa=torch.tensor([0.1 / (i + 1)] * (i + 1) + [0.9], device=self.device))
             if l.ff is not None:
                 ffp = -(-l.ff // 8) * 8
-                p.update(norm2=zeros(), up=_pad_to(w(l.ff, s.width), ffp, W),
-                         down=ResidualLinear(_pad_to(w(s.width, l.ff), W, ffp)), act=(0.8, 1.3))
+                p.update(norm2=zeros(), up=fit(w(l.ff, s.width), ffp, W),
+                         down=ResidualLinear(fit(w(s.width, l.ff), W, ffp)), act=(0.8, 1.3))
             self.layers.append(p)
 
     # ------------------------------------------------------------------ cache
-    def allocate_caches(self, num_pages: int, page_size: int):
+    def allocate_caches(self, num_pages: int, page_size: int, num_slots: int):
         """One page pool per layer; a page holds page_size latents of that layer."""
         self.caches = [torch.zeros(num_pages, page_size, m.kv_rank_p, dtype=self.dtype, device=self.device)
                        for m in self.mixers]

@@ -43,6 +43,18 @@ QWEN3_0_6B = Qwen3Shape(28, 1024, 16, 8, 128, 3072, 151936)
 
 
 @dataclass
+class Segments:
+    """The portions of a step as recurrent layers read them, int32 arrays: first token row (None: the
+    portion's index), tokens (at most `max_count` when that is set; 0: inert), state slot, position of
+    the first token."""
+    rows: torch.Tensor | None
+    counts: torch.Tensor
+    slots: torch.Tensor
+    starts: torch.Tensor
+    max_count: int = 0
+
+
+@dataclass
 class StepContext:
     """Per-step attention metadata (the reference keeps it in a module-global context,
     zipage/utils/context.py; here it is passed explicitly so a captured graph can own one)."""
@@ -54,15 +66,17 @@ class StepContext:
     seq_lens_q: list[int] | None = None             # prefill: new tokens per sequence
     seq_lens_k: list[int] | None = None             # prefill: total tokens per sequence
     # steps of portions: the first context_lens.numel() tokens are attended one by one, token i over
-    # row table_rows[i] of block_tables (None: i); the rest belong to runs, planned per window
+    # row table_rows[i] of block_tables (None: i); the rest belong to runs, planned per kind of sight
     table_rows: torch.Tensor | None = None          # (singles,) int32
-    runs: dict | None = None                        # window -> inputs.Runs
+    runs: dict | None = None                        # sight -> inputs.Runs
+    segments: Segments | None = None                # the portions, for recurrent layers
 
 
 class Qwen3:
     # what the engine asks a model: its cache may be compressed; a step is whole prompts or decodes
     compressible = True
     portions = False
+    recurrent = False
 
     def __init__(self, shape: Qwen3Shape, device, dtype=torch.bfloat16, seed: int = 0,
                  init_std: float = 0.02):

@@ -6,6 +6,7 @@ import os
 from dataclasses import dataclass
 from typing import Any, Callable
 
+from .kapolorn import Kapolorn, KapolornShape
 from .pedivik import Pedivik, PedivikShape
 from .qwen3 import Qwen3, Qwen3Shape
 from .weights import read_folder
@@ -17,12 +18,14 @@ class Architecture:
     model: type
     shape: type
     from_config: Callable[[dict], Any]
+    libs: tuple[str, ...]                    # the kernels it needs (names in zipage_amd/build.py)
     loads_weights: bool = True
 
 
 ARCHITECTURES = {a.name: a for a in (
-    Architecture("Qwen3ForCausalLM", Qwen3, Qwen3Shape, Qwen3Shape.from_config, loads_weights=False),
-    Architecture("Pedivik", Pedivik, PedivikShape, PedivikShape.from_config),
+    Architecture("Qwen3ForCausalLM", Qwen3, Qwen3Shape, Qwen3Shape.from_config, ("LIB",), loads_weights=False),
+    Architecture("Pedivik", Pedivik, PedivikShape, PedivikShape.from_config, ("MODELS_LIB", "LATENT_LIB")),
+    Architecture("Kapolorn", Kapolorn, KapolornShape, KapolornShape.from_config, ("MODELS_LIB", "HYBRID_LIB")),
 )}
 
 

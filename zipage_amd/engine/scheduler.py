@@ -19,7 +19,9 @@ class Scheduler:
     def __init__(self, cfg: EngineConfig):
         self.cfg = cfg
         self.pool = PagePool(cfg.num_kvcache_blocks, cfg.kvcache_block_size,
-                             cfg.table_width, cfg.enable_prefix_cache)
+                             cfg.table_width,
+                             # a recurrent state cannot start behind tokens that did not run
+                             cfg.enable_prefix_cache and not cfg.arch.model.recurrent)
         self.waiting: deque[Sequence] = deque()
         self.running: deque[Sequence] = deque()
         self.free_rows: deque[int] = deque(range(cfg.max_concurrency))

@@ -9,7 +9,8 @@ import torch.nn.functional as F
 
 from zipage_amd import _lib
 
-from .linear import ResidualLinear
+from .linear import ResidualLinear, fit, pad_to_multiple
+from .runs import gather_rows, run_attention
 
 
 def latent_norm_store(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tensor, q_norm: int,
@@ -31,16 +32,6 @@ def latent_norm_store(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torc
                      _lib.dev_ptr(slot_mapping), N, qw, cw, q_norm, c_norm, cache.numel() // cw, float(eps),
                      _lib.dtype_tag(down), _lib.stream_ptr(down))
     return (q, c) if return_c else q
-
-
-def gather_rows(src: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
-    """src viewed as (slots, width): its rows `rows` (int32)."""
-    width = src.shape[-1]
-    assert src.is_contiguous() and rows.dtype == torch.int32 and rows.is_contiguous()
-    out = torch.empty((rows.numel(), width), dtype=src.dtype, device=src.device)
-    _lib.call_models("zp_gather_rows", _lib.dev_ptr(src), _lib.dev_ptr(rows), _lib.dev_ptr(out),
-                     rows.numel(), width * src.element_size(), src.numel() // width, _lib.stream_ptr(src))
-    return out
 
 
 def headwise_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
@@ -68,7 +59,7 @@ def latent_rows_attention(q: torch.Tensor, cache: torch.Tensor, block_tables: to
     B, NB = block_tables.shape
     pages, BS, _ = cache.shape
     w, tag = window or 0, _lib.dtype_tag(q)
-    size = _lib.load_models().zp_latent_rows_workspace(N, H, R, w, NB, BS, tag)
+    size = _lib.load_models("latent").zp_latent_rows_workspace(N, H, R, w, NB, BS, tag)
     ws = torch.empty(max(size, 0), dtype=torch.uint8, device=q.device) if size > 0 else None
     out = torch.empty_like(q)
     _lib.call_models("zp_latent_rows_attention", _lib.dev_ptr(q), _lib.dev_ptr(cache),
@@ -82,19 +73,7 @@ def latent_tiles_attention(q: torch.Tensor, kv: torch.Tensor, heads: int, dim: i
                            tiles: torch.Tensor, scale: float, window: int | None, out: torch.Tensor):
     """Runs of prompt tokens over expanded keys and values.  q (N, heads * dim); kv (Nk, heads * dim
     + heads * vdim); tiles (T, 4) int32 as `inputs.plan_runs` makes them; out (N, heads * vdim)."""
-    assert q.stride(1) == 1 and kv.is_contiguous() and out.is_contiguous()
-    assert kv.shape[1] == heads * (dim + vdim) and out.shape == (q.shape[0], heads * vdim)
-    assert tiles.dtype == torch.int32 and tiles.is_contiguous() and tiles.shape[1] == 4
-    v = kv[:, heads * dim:]
-    _lib.call_models("zp_latent_tiles_attention", _lib.dev_ptr(q), _lib.dev_ptr(kv), v.data_ptr(),
-                     _lib.dev_ptr(out), _lib.dev_ptr(tiles), tiles.shape[0], heads, dim, vdim, window or 0,
-                     q.shape[0], kv.shape[0], q.stride(0), kv.stride(0), float(scale), _lib.dtype_tag(q),
-                     _lib.stream_ptr(q))
-    return out
-
-
-def _pad(n: int, to: int) -> int:
-    return -(-n // to) * to
+    return run_attention(q, kv, heads, heads, dim, vdim, tiles, scale, out, window=window)
 
 
 class LatentAttention:
@@ -113,9 +92,9 @@ class LatentAttention:
                  scale: float, window: int | None, eps: float):
         self.width, self.heads, self.dim, self.vdim = width, heads, dim, vdim
         self.q_rank, self.kv_rank, self.scale, self.window, self.eps = q_rank, kv_rank, scale, window, eps
-        self.padded_width = _pad(width, 8)
-        self.dim_p, self.vdim_p = _pad(dim, 32), _pad(vdim, 16)
-        self.q_rank_p, self.kv_rank_p = _pad(q_rank, 32), _pad(kv_rank, 32)
+        self.padded_width = pad_to_multiple(width, 8)
+        self.dim_p, self.vdim_p = pad_to_multiple(dim, 32), pad_to_multiple(vdim, 16)
+        self.q_rank_p, self.kv_rank_p = pad_to_multiple(q_rank, 32), pad_to_multiple(kv_rank, 32)
 
     @property
     def can_expand(self) -> bool:
@@ -126,11 +105,6 @@ class LatentAttention:
         """w: dq, dq.norm, uq, dkv, dkv.norm, uk, uv, o as stored ([out, in], heads in order)."""
         H, D, V, R, Q, W = self.heads, self.dim, self.vdim, self.kv_rank, self.q_rank, self.width
         put = lambda t, dt=dtype: t.to(device=device, dtype=dt).contiguous()
-
-        def fit(t, *shape):
-            out = torch.zeros(shape, dtype=t.dtype, device=t.device)
-            out[tuple(slice(0, n) for n in t.shape)] = t
-            return out
 
         self.down = put(torch.cat([fit(w["dq"], self.q_rank_p, self.padded_width),
                                    fit(w["dkv"], self.kv_rank_p, self.padded_width)]))

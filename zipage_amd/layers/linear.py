@@ -5,6 +5,17 @@ import torch
 import torch.nn.functional as F
 
 
+def pad_to_multiple(n: int, to: int) -> int:
+    return -(-n // to) * to
+
+
+def fit(t: torch.Tensor, *shape: int) -> torch.Tensor:
+    """`t` in the corner of a zero tensor of `shape`."""
+    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
+    out[tuple(slice(0, n) for n in t.shape)] = t
+    return out
+
+
 class ResidualLinear:
     """y = W x, returned as planes of partial sums (planes, N, out) that `residual_norm` adds up in
     fp32.

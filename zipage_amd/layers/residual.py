@@ -15,8 +15,8 @@ def _rows(t: torch.Tensor | None, width: int):
 
 def embed_norm(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.Tensor,
                pos: torch.Tensor | None, x: torch.Tensor, norm_weight: torch.Tensor, eps: float,
-               norm_width: int, weight_offset: float = 0.0) -> torch.Tensor:
-    """x = embed[tokens] (+ pos[positions]) into `x`; returns its RMS norm times
+               norm_width: int, weight_offset: float = 0.0, embed_scale: float = 1.0) -> torch.Tensor:
+    """x = embed[tokens] * embed_scale (+ pos[positions]) into `x`; returns its RMS norm times
     (weight_offset + norm_weight) in the table's dtype.  tokens (N,) int64, positions (N,) int32."""
     N, W = x.shape
     assert tokens.dtype == torch.int64 and positions.dtype == torch.int32
@@ -26,7 +26,7 @@ def embed_norm(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.Tenso
     out = torch.empty((N, W), dtype=embed.dtype, device=x.device)
     _lib.call_models("zp_embed_norm", _lib.dev_ptr(tokens), _lib.dev_ptr(positions), _rows(embed, W),
                      _rows(pos, W), _rows(x, W), _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width,
-                     embed.shape[0], 0 if pos is None else pos.shape[0], float(eps), float(weight_offset),
+                     embed.shape[0], 0 if pos is None else pos.shape[0], float(embed_scale), float(eps), float(weight_offset),
                      _lib.dtype_tag(embed), _lib.stream_ptr(x))
     return out
 
@@ -34,13 +34,16 @@ def embed_norm(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.Tenso
 def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | None, eps: float,
                   norm_width: int, weight_offset: float = 0.0, out_scale: float = 1.0,
                   x_out: torch.Tensor | None = None, result: torch.Tensor | None = None,
-                  history: torch.Tensor | None = None, mix: torch.Tensor | None = None):
-    """r = x + y (y also as planes (P, N, width), all of them added), kept in `result`; with `mix`, r <- mix[-1] r + sum_j mix[j] history[j]; kept in
-    `x_out`; returns rmsnorm(r) * (weight_offset + norm_weight) * out_scale in y's dtype (None
+                  history: torch.Tensor | None = None, mix: torch.Tensor | None = None,
+                  y_weight: torch.Tensor | None = None):
+    """r = x + y (y also as planes (P, N, width), all of them added; with `y_weight` their sum is
+    RMS-normed, times that weight, before it joins x), kept in `result`; with `mix`,
+    r <- mix[-1] r + sum_j mix[j] history[j]; kept in `x_out`; returns rmsnorm(r) * (weight_offset + norm_weight) * out_scale in y's dtype (None
     without a norm).  history (planes, N, width) fp32, of which the first len(mix) - 1 are read."""
     N, W = x.shape
     y = y if y.dim() == 3 else y.unsqueeze(0)
     assert x.dtype == torch.float32 and y.shape[1:] == x.shape
+    assert y_weight is None or y_weight.dtype == torch.float32
     n_hist, plane = 0, 0
     if mix is not None:
         assert mix.dtype == torch.float32 and mix.is_contiguous()
@@ -50,7 +53,8 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
             plane = history.stride(0)
             assert history.stride(1) == W and history.stride(2) == 1
     out = torch.empty((N, W), dtype=y.dtype, device=x.device) if norm_weight is not None else None
-    _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), y.shape[0], _lib.dev_ptr(history if n_hist else None),
+    _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), y.shape[0], _rows(y_weight, W),
+                     _lib.dev_ptr(history if n_hist else None),
                      plane, _lib.dev_ptr(mix), n_hist, _rows(result, W), _rows(x_out, W),
                      _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width, float(eps),
                      float(weight_offset), float(out_scale), _lib.dtype_tag(y), _lib.stream_ptr(x))
@@ -63,4 +67,13 @@ def xielu(z: torch.Tensor, alpha_p: float, alpha_n: float) -> torch.Tensor:
     out = torch.empty_like(z)
     _lib.call_models("zp_xielu", _lib.dev_ptr(z), _lib.dev_ptr(out), z.numel(), float(alpha_p),
                      float(alpha_n), _lib.dtype_tag(z), _lib.stream_ptr(z))
+    return out
+
+
+def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap * tanh(z / cap) in fp32."""
+    assert z.is_contiguous()
+    out = torch.empty(z.shape, dtype=torch.float32, device=z.device)
+    _lib.call_models("zp_softcap", _lib.dev_ptr(z), _lib.dev_ptr(out), z.numel(), float(cap), _lib.dtype_tag(z),
+                     _lib.stream_ptr(z))
     return out
