@@ -18,7 +18,7 @@ through the decode engine as `end_to_end` (decode tokens/s and the compression s
 
   python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--no-cpu-baseline] [--no-e2e]
   python bench.py --config 5 [--requests R] [--prompt P] [--out-tokens T] [--sync-compress]
-  python bench.py --compare-models [--model-sizes 1k,4k]     (Pedivik beside Qwen3 at equal size)
+  python bench.py --compare-models [pedivik|kapolorn] [--model-sizes 1k,4k]     (the model beside Qwen3 at equal size)
 """
 from __future__ import annotations
 
@@ -413,9 +413,9 @@ def main():
     ap.add_argument("--traffic", type=float, default=None,
                     help="HBM bytes per compaction launch measured with rocprofv3 --pmc "
                          "(reported as roofline.traffic)")
-    ap.add_argument("--compare-models", action="store_true",
+    ap.add_argument("--compare-models", nargs="?", const="pedivik", choices=("pedivik", "kapolorn"),
                     help="instead of the compression workload: prefill and decode throughput of "
-                         "Pedivik beside Qwen3 at equal size, and their kernels against the roofline")
+                         "Pedivik or Kapolorn beside Qwen3 at equal size, and their kernels against the roofline")
     ap.add_argument("--model-sizes", default="1k,4k", help="sizes of --compare-models")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -432,13 +432,13 @@ def main():
     if args.compare_models:
         from zipage_amd.bench.model_compare import SIZES, compare
         sizes = args.model_sizes.split(",")
-        report = compare(sizes)
-        head = report["sizes"][sizes[-1]]["pedivik"]["256 x 2048"]
+        report = compare(args.compare_models, sizes)
+        head = report["sizes"][sizes[-1]][args.compare_models]["256 x 2048"]
         print(json.dumps({
             "metric": "decode tokens/sec", "value": head["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1,
             "steps": 63, "warmup": 2, "ms_per_step": head["ms_per_decode_step"], "higher_is_better": True,
             "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-            "config": {"workload": f"random-init Pedivik {sizes[-1]} (layer sizes {SIZES[sizes[-1]]}), 256 requests x "
+            "config": {"workload": f"random-init {args.compare_models.capitalize()} {sizes[-1]} (layer sizes {SIZES[sizes[-1]]}), 256 requests x "
                                    "2048-token prompts x 64 greedy tokens"}, "compare": report}))
         return
     if args.config == 5:

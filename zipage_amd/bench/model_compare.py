@@ -1,9 +1,10 @@
-"""Pedivik beside Qwen3 at equal size: prefill and decode throughput through the engine (random
-weights), and every kernel between the matrix products against its roofline, beside the kernel of
-the other model that does the like work.
+"""Pedivik or Kapolorn beside Qwen3 at equal size: prefill and decode throughput through the engine
+(random weights), and every kernel between the matrix products against its roofline, beside the kernel
+of the other model that does the like work.
 
 Equal size: same width, heads, head dimensions and vocabulary; Pedivik's ungated feed-forward is 1.5
-times as wide as Qwen3's gated one, so both hold the same parameters.  Kernels are timed as replays
+times as wide as Qwen3's gated one, so both hold the same parameters; a Kapolorn token passes three of 32
+experts and the shared one, each a quarter as wide as Qwen3's feed-forward.  Kernels are timed as replays
 of a graph of many launches over buffers that together exceed the caches.
 """
 from __future__ import annotations
@@ -14,6 +15,7 @@ import torch
 
 HBM = 8.0e12          # bytes/s
 MFMA = 2.5e15         # dense bf16 FLOP/s
+FP32 = 157e12         # fp32 FLOP/s, vector or matrix
 BF16 = torch.bfloat16
 
 SIZES = {
@@ -28,6 +30,17 @@ def shapes(size: str):
     W, H, HK, D, FF, L, V, QR, KR, win = SIZES[size]
     layer = PedivikLayer(H, D, D, QR, KR, D ** -0.5, win, FF * 3 // 2)
     return (PedivikShape(V, W, (layer,) * L, 8192, 1e-6, 1.0),
+            Qwen3Shape(L, W, H, HK, D, FF, V, max_position=8192))
+
+
+def kapolorn_shapes(size: str):
+    from zipage_amd.engine import KapolornShape, Qwen3Shape
+    from zipage_amd.engine.kapolorn import DeltaMixer, ExpertsShape, KapolornLayer, ParallelMixer
+    W, H, HK, D, FF, L, V, _, _, chunk = SIZES[size]
+    moe = ExpertsShape(32, 3, 4, 2, FF // 4, 7.0, FF // 4, 7.0)
+    par = KapolornLayer(ParallelMixer(H, HK, D, D, D ** -0.5, chunk, 1e6, D, 0.8, H // 2, D, D, 15.0, 1.1), moe)
+    delta = KapolornLayer(DeltaMixer(H, H // 2, D, D, 4), moe)
+    return (KapolornShape(V, W, (par, delta) * (L // 2), (0, 0, 1), 1e-6, 1.0, 15.0),
             Qwen3Shape(L, W, H, HK, D, FF, V, max_position=8192))
 
 
@@ -227,15 +240,166 @@ def kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dic
     return rows
 
 
-def compare(sizes=("1k", "4k"), out_tokens: int = 64) -> dict:
-    """The whole report.  The headline figure is Pedivik's decode rate at the largest size and batch."""
+def kapolorn_kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dict]:
+    """The same for Kapolorn's kernels.  Recurrences run in fp32: their roofline is that of fp32 arithmetic
+    (7 or 5 operations per state element and token) or of the state's bytes, whichever is longer."""
+    import torch.nn.functional as F
+    from zipage_amd.engine.inputs import plan_runs
+    from zipage_amd.engine.qwen3 import Segments
+    from zipage_amd.engine.sequence import Portion, Sequence
+    from zipage_amd.layers import (ChannelDelta, Experts, MatrixMemory, grouped_rows_attention, paged_decode_attention,
+                                   qk_norm_rope_store, residual_norm, rms_norm, rotary_store, run_attention,
+                                   silu_and_mul, small_linear, softcap)
+    from zipage_amd.layers.moe import Plan, moe_select
+    from zipage_amd.sight import Chunk
+    W, H, HK, D, FF, L, V, _, _, chunk = SIZES[size]
+    dev, BS = torch.device("cuda:0"), 256
+    rnd = lambda *s, dt=BF16: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    i32 = lambda a: torch.as_tensor(a, dtype=torch.int32, device=dev)
+    rows = []
+
+    def put(name, where, secs, byts, flops=0.0, peak=MFMA):
+        roof = max(byts / HBM, flops / peak)
+        bound = "hbm" if byts / HBM >= flops / peak else ("mfma" if peak == MFMA else "fp32")
+        rows.append({"kernel": name, "at": where, "us": round(secs * 1e6, 1), "bound": bound,
+                     "roofline_us": round(roof * 1e6, 1), "frac": round(roof / secs, 3)})
+
+    gen = torch.Generator(device=dev).manual_seed(0)
+    moe = Experts(W, 32, 3, FF // 4, 7.0, 4, 2, FF // 4, 7.0)
+    moe.random(BF16, dev, gen)
+    E, S = moe.experts, moe.top + 1
+    plan_of = lambda r: Plan(r[0], r[2], E, True, BF16)
+    gu, dn = [rnd(2 * FF, W) for _ in range(2)], [rnd(W, FF) for _ in range(2)]
+    for phase, N in (("decode", 64), ("decode", decode_batch), ("prefill", prompts * prompt)):
+        at, big = f"{phase}, {N} tokens", N * W
+        seqs = N if phase == "decode" else prompts
+        # norms of the stream
+        for planes in (1, S):
+            k = _sets(big * (10 + 2 * planes))
+            xs, ys = [rnd(N, W, dt=torch.float32) for _ in range(k)], [rnd(planes, N, W) for _ in range(k)]
+            w32, w16 = torch.ones(W, device=dev), torch.ones(W, device=dev, dtype=BF16)
+            put(f"residual_norm of a normed branch, {planes} planes", at,
+                timed(lambda i: residual_norm(xs[i], ys[i], w32, 1e-6, W, x_out=xs[i], y_weight=w32), k), big * (10 + 2 * planes))
+            if planes == 1:
+                rs = [rnd(N, W) for _ in range(k)]
+                put("like: add_rms_norm (16-bit stream)", at, timed(lambda i: rms_norm(ys[i][0], w16, 1e-6, rs[i]), k), big * 8)
+                del rs
+            del xs, ys
+        # rotary positions and the store
+        width = (H + 2 * HK) * D
+        slots, pos = torch.randperm(N, device=dev).int(), torch.arange(N, device=dev, dtype=torch.int32) % 4096
+        k = _sets(N * width * 4)
+        qkvs, caches = [rnd(N, width) for _ in range(k)], [rnd(-(-N // BS), BS, 2 * HK * D) for _ in range(k)]
+        freqs = rnd(D // 2, dt=torch.float32).abs()
+        put("rotary_store", at, timed(lambda i: rotary_store(qkvs[i], pos, freqs, H, HK, D, D, caches[i], slots), k), N * width * 4)
+        cos, sin, nw = rnd(8192, D // 2, dt=torch.float32), rnd(8192, D // 2, dt=torch.float32), torch.ones(D, device=dev, dtype=BF16)
+        kcs = [rnd(-(-N // BS), BS, HK, D) for _ in range(2 * k)]
+        put("like: qk_norm_rope_store", at,
+            timed(lambda i: qk_norm_rope_store(qkvs[i], pos, cos, sin, nw, nw, H, HK, D, 1e-6, kcs[2 * i], kcs[2 * i + 1], slots), k),
+            N * width * 4)
+        del qkvs, caches, kcs
+        # recurrences
+        n = N // seqs
+        seg = Segments(i32(range(0, N, n)), i32([n] * seqs), i32(torch.randperm(seqs)), i32([5] * seqs))
+        for name, mixer, ops in ((f"mlstm_scan, {H // 2} heads", MatrixMemory(W, H // 2, D, D, 15.0, 1e-6), 5),
+                                 (f"delta_scan, {H} heads", ChannelDelta(W, H, H // 2, D, D, 4, 1e-6), 7)):
+            small = {q: torch.randn(*s) * 0.02 for q, s in (mixer.shapes() if ops == 5 else mixer.shapes(128, 128)).items()}
+            mixer.load({q: t.to(BF16) for q, t in small.items()}, BF16, dev, W)
+            h = rnd(N, W)
+            k = 2
+            projs = [rnd(N, mixer.columns) for _ in range(k)]
+            states = [mixer.allocate(seqs + 1, BF16, dev) for _ in range(k)]
+            out = torch.empty(N, mixer.out_columns, device=dev, dtype=BF16)
+            state = 2 * seqs * mixer.heads * D * D * 4
+            inner = (lambda i: mixer.scan(h, projs[i], states[i], seg, out)) if ops == 5 else \
+                (lambda i: mixer.scan(projs[i], states[i], seg, out))
+            extra = timed((lambda i: small_linear(h, mixer.gates)) if ops == 5 else
+                          (lambda i: F.linear(projs[i][:, mixer.low_at:mixer.low_at + mixer.low_rank], mixer.low)), k, 6)
+            low = 0 if ops == 5 else N * H * 2 * D * 2
+            put(name, at, max(timed(inner, k, 6) - extra, 1e-9), state + N * (mixer.columns + mixer.out_columns) * 2 + low,
+                float(ops) * N * mixer.heads * D * D, FP32)
+            del projs, states, out
+        # experts
+        h = [rnd(N, W) for _ in range(2)]
+        put("small_linear (router)", at, timed(lambda i: small_linear(h[i], moe.router), 2), N * W * 2 + E * W * 2)
+        z = rnd(N, E, dt=torch.float32)
+        ids, wts, counts = moe_select(z, E, 3, 4, 2)
+        put("moe_select", at, timed(lambda i: moe_select(z, E, 3, 4, 2), 2), N * E * 4 + N * 24)
+        put("moe_plan (after moe_select)", at,
+            timed(lambda i: plan_of(moe_select(z, E, 3, 4, 2)), 2) - timed(lambda i: moe_select(z, E, 3, 4, 2), 2),
+            N * 3 * 12)
+        plan = plan_of((ids, wts, counts))
+        act = moe.gate_up_rows(h[0], plan, wts)
+        used = min(E, N * 3) + 1
+        fl = 2.0 * N * S * W * (FF // 4)
+        put("moe_gate_up", at, timed(lambda i: moe.gate_up_rows(h[i], plan, wts), 2, 6),
+            used * 2 * (FF // 4) * W * 2 + N * W * 2 + N * FF * 2, 2 * fl)
+        put("like: gate and up (library product), silu_and_mul", at, timed(lambda i: silu_and_mul(F.linear(h[i], gu[i])), 2, 6),
+            2 * FF * W * 2 + N * W * 2 + N * FF * 2, 2 * fl)
+        put("moe_down", at, timed(lambda i: moe.down_planes(act, plan), 2, 6),
+            used * (FF // 4) * W * 2 + N * FF * 2 + S * N * W * 2, fl)
+        full = rnd(N, FF)
+        put("like: down (library product)", at, timed(lambda i: F.linear(full, dn[i]), 2, 6), FF * W * 2 + N * FF * 2 + N * W * 2, fl)
+        del h, act, full
+        m = N if phase == "decode" else prompts
+        z = rnd(m, V)
+        put("softcap", f"{m} rows of logits", timed(lambda i: softcap(z, 15.0), 1), m * V * 6)
+    # ---- decode attention
+    per = -(-prompt // BS)
+    for B in (64, decode_batch):
+        for ctx_len in (chunk, prompt):
+            at = f"decode, {B} sequences, context {ctx_len}"
+            k = _sets(B * ctx_len * HK * D * 4)
+            caches = [rnd(B * per, BS, 2 * HK * D) for _ in range(k)]
+            tables, ctx = torch.randperm(B * per, device=dev).int().view(B, per), i32([ctx_len] * B)
+            q, sinks, out = rnd(B, H * D), rnd(H, dt=torch.float32), torch.empty(B, H * D, device=dev, dtype=BF16)
+            for name, size_ in ((f"grouped_rows_attention, chunk {chunk}", chunk), ("grouped_rows_attention, no limit", None)):
+                seen = ctx_len if size_ is None else (ctx_len - 1) % size_ + 1
+                put(name, at, timed(lambda i: grouped_rows_attention(q, caches[i], H, HK, D, D, tables, ctx, D ** -0.5, out,
+                                                                     chunk=size_, sinks=sinks), k),
+                    2 * B * seen * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * seen * D)
+            del caches
+            kcs = [rnd(B * per, BS, HK, D) for _ in range(2 * k)]
+            qd = rnd(B, H, D)
+            put("like: paged_decode_attention", at,
+                timed(lambda i: paged_decode_attention(qd, kcs[2 * i], kcs[2 * i + 1], ctx, tables, D ** -0.5), k),
+                2 * B * ctx_len * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * ctx_len * D)
+            del kcs
+    # ---- prefill attention
+    N, at, k = prompts * prompt, f"prefill, {prompts} x {prompt} tokens", 2
+    parts = []
+    for _ in range(prompts):
+        s = Sequence([0] * prompt)
+        s.block_table = list(range(per))
+        parts.append(Portion(s, 0, prompt))
+    qs, kvs = [rnd(N, H * D) for _ in range(k)], [rnd(N, 2 * HK * D) for _ in range(k)]
+    out = torch.empty(N, H * D, device=dev, dtype=BF16)
+    for name, size_ in ((f"run_attention, chunk {chunk}", chunk), ("run_attention, no limit", None)):
+        tiles = i32(plan_runs(parts, BS, None if size_ is None else Chunk(size_)).tiles)
+        pairs = sum((i % size_ if size_ else i) + 1 for i in range(prompt)) * prompts
+        put(name, at, timed(lambda i: run_attention(qs[i], kvs[i], H, HK, D, D, tiles, D ** -0.5, out, chunk=size_, sinks=sinks), k, 6),
+            N * (2 * H + 2 * HK) * D * 2, 4.0 * pairs * H * D)
+    ks = [rnd(prompts, prompt, HK, D) for _ in range(2 * k)]
+    put("like: scaled_dot_product_attention (library, causal)", at,
+        timed(lambda i: F.scaled_dot_product_attention(
+            qs[i].view(prompts, prompt, H, D).transpose(1, 2), ks[2 * i].transpose(1, 2), ks[2 * i + 1].transpose(1, 2),
+            is_causal=True, enable_gqa=True), k, 6), N * (2 * H + 2 * HK) * D * 2, 4.0 * prompt * (prompt + 1) / 2 * prompts * H * D)
+    return rows
+
+
+MODELS = {"pedivik": (shapes, kernels), "kapolorn": (kapolorn_shapes, kapolorn_kernels)}
+
+
+def compare(model: str = "pedivik", sizes=("1k", "4k"), out_tokens: int = 64) -> dict:
+    """The whole report.  The headline figure is the model's decode rate at the largest size and batch."""
     report = {"sizes": {}}
+    make, table = MODELS[model]
     for size in sizes:
-        pedivik, qwen = shapes(size)
-        entry = {"pedivik": {}, "qwen3": {}}
+        own, qwen = make(size)
+        entry = {model: {}, "qwen3": {}}
         for batch, prompt in ((1, 2048), (64, 2048), (256, 2048)):
-            for name, shape in (("pedivik", pedivik), ("qwen3", qwen)):
+            for name, shape in ((model, own), ("qwen3", qwen)):
                 entry[name][f"{batch} x {prompt}"] = throughput(shape, batch, prompt, out_tokens)
-        entry["kernels"] = kernels(size, 256, 8, 2048)
+        entry["kernels"] = table(size, 256, 8, 2048)
         report["sizes"][size] = entry
     return report

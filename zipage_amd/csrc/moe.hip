@@ -211,8 +211,10 @@ __device__ __forceinline__ int block_prefix(int v, int* red) {
 // Offsets and tiles from the counts in LDS (E of them); the shared expert's rows follow the others'.
 __device__ __forceinline__ void offsets_and_tiles(const PlanArgs& a, const int* counts, int* offsets, int* red) {
   const int e = threadIdx.x;
-  const int c = e < a.E ? counts[e] : (e == a.E && a.shared ? a.n : 0);
-  const int at = block_prefix(c, red);
+  int c = e < a.E ? counts[e] : (e == a.E && a.shared ? a.n : 0);
+  int at = block_prefix(c, red);
+  at = min(at, a.n * (a.top + a.shared));             // counters that were not cleared stay in bounds
+  c = min(c, a.n * (a.top + a.shared) - at);
   const int t = (c + a.rows - 1) / a.rows;
   const int first = block_prefix(t, red);
   if (e <= a.E) {
@@ -236,7 +238,7 @@ __global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(PlanArgs a) {
   for (int i = tid; i < total; i += kPlanThreads) {
     const int e = min(max(a.ids[i], 0), a.E - 1);
     const int n = i / a.top;
-    a.sorted[atomicAdd(&offsets[e], 1)] = n * slots + i - n * a.top;
+    a.sorted[min(atomicAdd(&offsets[e], 1), total - 1)] = n * slots + i - n * a.top;
   }
   if (a.shared)
     for (int n = tid; n < a.n; n += kPlanThreads) a.sorted[total + n] = n * slots + a.top;
@@ -269,7 +271,7 @@ __global__ __launch_bounds__(kPlanThreads) void moe_place_kernel(PlanArgs a) {
   __syncthreads();
   for (int i = i0 + tid; i < min(i0 + kPlanBlock, total); i += kPlanThreads) {
     const int n = i / a.top;
-    a.sorted[atomicAdd(&at[min(max(a.ids[i], 0), a.E - 1)], 1)] = n * slots + i - n * a.top;
+    a.sorted[min(atomicAdd(&at[min(max(a.ids[i], 0), a.E - 1)], 1), total - 1)] = n * slots + i - n * a.top;
   }
   if (a.shared)
     for (int n = blockIdx.x * kPlanThreads + tid; n < a.n; n += gridDim.x * kPlanThreads)
