@@ -370,7 +370,130 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
   }
 }
 
+// Many rows per expert: 128 tokens x 256 rows of W per workgroup, both streamed straight into LDS in the
+// order the matrix cores read them, 32 of the contraction at a time, two stages ahead of the products; one
+// barrier per stage.  A wave owns 64 tokens x 128 rows of W.
+typedef __attribute__((address_space(3))) void* lds_ptr_t;
+constexpr int kBlockRows = 128;                        // tokens
+constexpr int kBlockW = 16;                            // 16-row tiles of W
+constexpr int kStageBytes = (kBlockRows / 16 + kBlockW) * 1024, kStages = 3;
+
+template <bool UP>
+__global__ __launch_bounds__(256, 2) void expert_tiles_kernel(ExpertArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, g = lane >> 4;
+  // An XCD takes a contiguous share of the (tile, column block) pairs, in squares of eight by eight, so that
+  // what is in flight on it shares rows of x and of W in its L2.
+  const int nt = *a.ntiles;
+  const int Mx = max(a.M, a.M_shared) * (UP ? 2 : 1), cols = (Mx + 16 * kBlockW - 1) / (16 * kBlockW);
+  const int groups = (nt + 7) / 8, i_xcd = blockIdx.x >> 3;
+  if (i_xcd >= groups * cols) return;
+  const int lin = (blockIdx.x & 7) * groups * cols + i_xcd;
+  const int tg = lin / (8 * cols), rem = lin - tg * 8 * cols;
+  const int tile = tg * 8 + (rem & 7), cb = rem >> 3;
+  if (tile >= nt) return;
+  const int4 t = *(const int4*)(a.tiles + (int64_t)tile * 4);
+  const bool shared = t.x == a.E;
+  const int wtiles = (shared ? a.M_shared : a.M) / 16 * (UP ? 2 : 1), K = shared ? a.K_shared : a.K;
+  const int w0 = cb * kBlockW;
+  if (w0 >= wtiles) return;
+  const int steps = K / 32;
+  const char* wbase = (const char*)(shared ? a.w_shared : a.w) + (shared ? 0 : t.x * a.w_expert) * 2;
+  const __amdgpu_buffer_rsrc_t rw = __builtin_amdgcn_make_buffer_rsrc((void*)(wbase + (int64_t)w0 * steps * 1024), 0,
+                                                                      min(kBlockW, wtiles - w0) * steps * 1024, 0x00020000);
+  const int rows = UP ? a.n : a.n * a.slots;
+  const __amdgpu_buffer_rsrc_t rx =
+      __builtin_amdgcn_make_buffer_rsrc((void*)a.x, 0, (int)min((int64_t)rows * a.x_st * 2, (int64_t)0x7fffffff), 0x00020000);
+  // this wave's loads of a stage: two of the eight 16-token tiles, four of the sixteen of W
+  int xoff[2], woff[4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int pos = t.y + min((wave * 2 + i) * 16 + l16, t.z - 1);
+    xoff[i] = (int)((UP ? a.sorted[pos] / a.slots : pos) * a.x_st * 2) + g * 16;
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) woff[i] = min(wave * 4 + i, wtiles - w0 - 1) * steps * 1024;
+  auto request = [&](int ks) {
+    char* const st = lds_raw + (ks % kStages) * kStageBytes;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      __builtin_amdgcn_raw_ptr_buffer_load_lds(rx, (lds_ptr_t)(st + (wave * 2 + i) * 1024), 16, xoff[i], ks * 64, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      __builtin_amdgcn_raw_ptr_buffer_load_lds(rw, (lds_ptr_t)(st + (8 + wave * 4 + i) * 1024), 16, lane * 16,
+                                               woff[i] + ks * 1024, 0, 0);
+  };
+  const int th = wave & 1, wh = wave >> 1;
+  f32x4 acc[8][4];
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  request(0);
+  if (steps > 1) request(1);
+#pragma unroll 1
+  for (int ks = 0; ks < steps; ++ks) {
+    if (ks + 1 < steps) asm volatile("s_waitcnt vmcnt(6)" ::: "memory");
+    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();                        // everyone's part of the stage is there
+    if (ks + 2 < steps) request(ks + 2);                 // over the stage that was used up before the barrier
+    const char* const st = lds_raw + (ks % kStages) * kStageBytes + lane * 16;
+    u32x4 xf[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xf[j] = *(const u32x4*)(st + (th * 4 + j) * 1024);
+    u32x4 wf[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) wf[i] = *(const u32x4*)(st + (8 + wh * 8 + i) * 1024);
+    __builtin_amdgcn_sched_barrier(0);                   // all reads on their way before the first product
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = mfma_bf16(wf[i], xf[j], acc[i][j]);
+    __builtin_amdgcn_sched_barrier(0);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = (th * 4 + j) * 16 + l16;
+    if (r >= t.z) continue;
+    const int pos = t.y + r, as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
+    if constexpr (UP) {
+      const float wgt = slot < a.top ? a.weights[(int64_t)n * a.top + slot] : 1.f;
+      const float lim = shared ? a.limit_shared : a.limit;
+#pragma unroll
+      for (int i = 0; i < 8; i += 2) {
+        const int wt = w0 + wh * 8 + i;
+        if (wt >= wtiles) break;
+        float v[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[k] = wgt * gated<BF16>(acc[i][j][k], acc[i + 1][j][k], lim);
+        Mma<BF16>::st4(a.out, (int64_t)pos * a.o_st + wt * 8 + g * 4, v);
+      }
+    } else {
+      const int64_t at = ((int64_t)slot * a.n + n) * a.o_st;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int wt = w0 + wh * 8 + i;
+        if (wt >= wtiles) break;
+        const float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+        Mma<BF16>::st4(a.out, at + wt * 16 + g * 4, v);
+      }
+    }
+  }
+}
+
 template <bool UP> int launch_experts(const ExpertArgs& a, int rows, int dtype, hipStream_t st) {
+  if (rows == kBlockRows) {
+    const int Mx = (a.M > a.M_shared ? a.M : a.M_shared) * (UP ? 2 : 1);
+    const int64_t grid = (int64_t)((a.max_tiles + 7) / 8) * 8 * ((Mx + 16 * kBlockW - 1) / (16 * kBlockW));
+    constexpr int smem = kStages * kStageBytes;
+    if (hipFuncSetAttribute((const void*)expert_tiles_kernel<UP>, hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
+      zp_set_error("moe: cannot reserve %d bytes of LDS", smem);
+      return ZP_EHIP;
+    }
+    hipLaunchKernelGGL((expert_tiles_kernel<UP>), dim3((unsigned)grid), dim3(256), smem, st, a);
+    ZP_LAUNCH_CHECK();
+    return ZP_OK;
+  }
   const int per = UP ? 64 : 128;                     // outputs per workgroup
   const int M = a.M > a.M_shared ? a.M : a.M_shared;
   const int64_t grid = (int64_t)a.max_tiles * ((M + per - 1) / per);
@@ -393,8 +516,9 @@ template <bool UP> int launch_experts(const ExpertArgs& a, int rows, int dtype, 
 }
 
 // Rows per tile: enough for the average expert.
-int tile_rows(int n, int E, int top) {
+int tile_rows(int n, int E, int top, int dtype) {
   const int64_t avg = ((int64_t)n * top + E - 1) / E;
+  if (dtype == ZP_BF16 && avg > 48) return kBlockRows;
   return avg <= 12 ? 16 : (avg <= 24 ? 32 : 64);
 }
 int tile_bound(int n, int E, int top, int shared, int rows) {
@@ -454,8 +578,7 @@ extern "C" int zp_moe_select(const float* logits, int32_t* ids, float* weights, 
 }
 
 extern "C" int64_t zp_moe_tile_rows(int32_t n, int32_t E, int32_t top, int32_t dtype) {
-  (void)dtype;
-  return n <= 0 || E <= 0 || top <= 0 ? -1 : tile_rows(n, E, top);
+  return n <= 0 || E <= 0 || top <= 0 ? -1 : tile_rows(n, E, top, dtype);
 }
 extern "C" int64_t zp_moe_max_tiles(int32_t n, int32_t E, int32_t top, int32_t shared, int32_t rows) {
   return n <= 0 || E <= 0 || top <= 0 || rows <= 0 ? -1 : tile_bound(n, E, top, shared, rows);
@@ -498,7 +621,8 @@ static int experts(bool up, const void* x, const void* w, const void* w_shared, 
   ZP_REQUIRE(n >= 0 && E > 0 && top > 0 && max_tiles > 0 && K > 0 && M > 0 && (!shared || (K_shared > 0 && M_shared > 0)),
              "moe experts: bad dims");
   ZP_MODEL_DTYPE("moe experts");
-  if (K % 32 || K_shared % 32 || M % 16 || M_shared % 16 || x_stride % 8 || out_stride % 8 || (rows != 16 && rows != 32 && rows != 64)) {
+  if (K % 32 || K_shared % 32 || M % 16 || M_shared % 16 || x_stride % 8 || out_stride % 8 ||
+      (rows != 16 && rows != 32 && rows != 64 && (rows != kBlockRows || dtype != ZP_BF16))) {
     zp_set_error("moe experts: sizes %d x %d, shared %d x %d, %d rows per tile unsupported", M, K, M_shared, K_shared, rows);
     return ZP_EUNSUPPORTED;
   }
@@ -507,6 +631,13 @@ static int experts(bool up, const void* x, const void* w, const void* w_shared, 
   ZP_REQUIRE(aligned16(x) && aligned16(w) && aligned16(w_shared) && aligned16(out) && aligned16(tiles) &&
                  x_stride >= (K > K_shared ? K : K_shared) && out_stride >= (M > M_shared ? M : M_shared),
              "moe experts: unaligned or overlapping rows");
+  if (rows == kBlockRows) {       // 31-bit byte offsets into x and into a block of W
+    const int64_t xr = up ? n : (int64_t)n * (top + shared), kx = K > K_shared ? K : K_shared;
+    if (xr * x_stride * 2 >= (1ll << 31) || kx * 512 >= (1ll << 31)) {
+      zp_set_error("moe experts: %lld rows of %lld elements in one step", (long long)xr, (long long)x_stride);
+      return ZP_EUNSUPPORTED;
+    }
+  }
   ExpertArgs a = {x, w, w_shared, out, sorted, tiles, ntiles, weights, n, E, top, top + shared, max_tiles, K, K_shared,
                   M, shared ? M_shared : 0, x_stride, out_stride, (int64_t)M * K * (up ? 2 : 1), limit, limit_shared};
   return up ? launch_experts<true>(a, rows, dtype, (hipStream_t)stream)
