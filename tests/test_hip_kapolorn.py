@@ -2,6 +2,7 @@
 cut and batched, and generation through the engine."""
 import io
 import json
+import types
 
 import pytest
 import torch
@@ -224,17 +225,22 @@ def test_run_attention(dev, H, G, D, V, window, chunk):
 
 
 # ------------------------------------------------------------------ recurrences
-def _segments(dev, parts):
-    """parts: (row, count, slot, start)"""
+def _segments(dev, parts, run_min=None):
+    """parts: (row, count, slot, start), those of run_min tokens and more behind the others."""
     from zipage_amd.engine.qwen3 import Segments
-    t = torch.tensor(parts, dtype=torch.int32).T.contiguous().to(dev)
-    return Segments(t[0], t[1], t[2], t[3])
+    made = []
+    for some in ([p for p in parts if run_min is None or p[1] < run_min], [p for p in parts if run_min and p[1] >= run_min]):
+        t = torch.tensor(some, dtype=torch.int32).view(-1, 4).T.contiguous().to(dev)
+        # steps of single tokens only take the kernels of decoding
+        made.append(Segments(*t, first_row=some[0][0], longest=max(p[1] for p in some),
+                             max_count=int(all(p[1] == 1 for p in parts))) if some else None)
+    return types.SimpleNamespace(segments=made[0], run_segments=made[1])
 
 
-CUTS = [[40], [1] * 40, [2, 3, 16, 17, 1, 1], [15, 25], [16, 16, 8], [33, 7]]
+CUTS = [[70], [1], [2, 3, 16, 17, 1, 1], [15, 25, 30], [16, 16, 8], [33, 7]]
 
 
-def _scan_in_cuts(dev, step, n, cuts, slots, seed):
+def _scan_in_cuts(dev, step, n, cuts, slots, run_min):
     """Sequences of n tokens run together, each cut its own way, states in the given slots; step(rows of the
     sequences, segments) -> output rows.  Returns the outputs in sequence order."""
     seqs = len(cuts)
@@ -242,17 +248,18 @@ def _scan_in_cuts(dev, step, n, cuts, slots, seed):
     turn = 0
     while any(a < n for a in at):
         parts, rows, row = [], [], 0
-        for s in range(seqs):
+        count = lambda s: min(cuts[s][len(out[s]) % len(cuts[s])], n - at[s])
+        for s in sorted(range(seqs), key=lambda s: run_min is not None and count(s) >= run_min):
             if at[s] == n or (turn + s) % 4 == 3:            # it pauses
                 continue
-            c = min(cuts[s][len(out[s]) % len(cuts[s])], n - at[s])
+            c = count(s)
             parts.append((row, c, slots[s], at[s]))
             rows += [(s, t) for t in range(at[s], at[s] + c)]
             row += c
         turn += 1
         if not parts:
             continue
-        got = step(rows, _segments(dev, parts))
+        got = step(rows, _segments(dev, parts, run_min))
         for (r, c, slot, _), s in zip(parts, [slots.index(p[2]) for p in parts]):
             out[s].append(got[r:r + c])
             at[s] += c
@@ -260,11 +267,13 @@ def _scan_in_cuts(dev, step, n, cuts, slots, seed):
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=ids)
-@pytest.mark.parametrize("H,D,V", [(3, 20, 24), (2, 64, 64), (1, 128, 128), (2, 40, 136), (1, 130, 250)])
-def test_matrix_memory(dev, dtype, H, D, V):
-    """Prompts against token by token against portions, states in slots that others used before."""
+@pytest.mark.parametrize("run_min", [None, 16, 2])
+@pytest.mark.parametrize("H,D,V", [(3, 20, 24), (2, 64, 64), (1, 128, 128), (300, 32, 40), (2, 40, 136), (1, 130, 250)])
+def test_matrix_memory(dev, dtype, run_min, H, D, V):
+    """Prompts against token by token against portions, in blocks and token by token, states in slots that
+    others used before."""
     from zipage_amd.layers import MatrixMemory
-    W, n, cap, eps = 64, 40, 3.0, 1e-3
+    W, n, cap, eps = 64, 70, 3.0, 1e-3
     r = lambda *s, seed, std=1.0: _rand("cpu", dtype, *s, seed=seed, std=std)
     w = {"q": r(H * D, W, seed=1, std=.2), "k": r(H * D, W, seed=2, std=.2), "v": r(H * V, W, seed=3, std=.2),
          "g": r(H * V, W, seed=4, std=.2), "o": r(W, H * V, seed=5), "norm": 1 + r(H * V, seed=6, std=.3),
@@ -285,7 +294,7 @@ def test_matrix_memory(dev, dtype, H, D, V):
         assert (out[:, H * Vp:] == 7).all()
         return out[:, :H * Vp].view(len(rows), H, Vp)[..., :V].clone()
     for round_, slots in enumerate(([3, 0, 6, 1, 5, 2], [0, 1, 2, 3, 4, 5])):
-        got = _scan_in_cuts(dev, step, n, CUTS, slots, round_)
+        got = _scan_in_cuts(dev, step, n, CUTS, slots, run_min)
         for s in range(len(CUTS)):
             P = proj[s].double().cpu()
             part = lambda at, d, dp: P[:, at:at + H * dp].view(n, H, dp)[..., :d]
@@ -299,16 +308,19 @@ def test_matrix_memory(dev, dtype, H, D, V):
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=ids)
-@pytest.mark.parametrize("H,G,D,V,taps", [(6, 2, 24, 40, 3), (2, 2, 64, 64, 4), (2, 1, 128, 128, 4), (1, 1, 40, 136, 1), (2, 2, 200, 250, 8)])
-def test_channel_delta(dev, dtype, H, G, D, V, taps):
+@pytest.mark.parametrize("run_min", [None, 16, 7])
+@pytest.mark.parametrize("H,G,D,V,taps", [(6, 2, 24, 40, 3), (2, 2, 64, 64, 4), (2, 1, 128, 128, 8), (200, 50, 32, 32, 2), (1, 1, 40, 136, 1),
+                                          (2, 2, 200, 250, 8)])
+def test_channel_delta(dev, dtype, run_min, H, G, D, V, taps):
+    """As above; some channels keep everything, others forget within a token."""
     from zipage_amd.layers import ChannelDelta
-    W, n, eps = 64, 40, 1e-3
+    W, n, eps = 64, 70, 1e-3
     r = lambda *s, seed, std=1.0: _rand("cpu", dtype, *s, seed=seed, std=std)
     ra, rg = 5, 11
     w = {"q": r(G * D, W, seed=1, std=.2), "k": r(G * D, W, seed=2, std=.2), "v": r(H * V, W, seed=3, std=.2),
          "q.conv": r(G * D, taps, seed=4), "k.conv": r(G * D, taps, seed=5), "v.conv": r(H * V, taps, seed=6),
          "b": r(H, W, seed=7, std=.2), "A_log": r(H, seed=8, std=.5), "norm": 1 + r(V, seed=9, std=.3),
-         "a1": r(ra, W, seed=10, std=.1), "a2": r(H * D, ra, seed=11, std=.4), "dt_bias": -3 + 2 * r(H * D, seed=12),
+         "a1": r(ra, W, seed=10, std=.1), "a2": r(H * D, ra, seed=11, std=.4), "dt_bias": -3 + 6 * r(H * D, seed=12),
          "g1": r(rg, W, seed=13, std=.1), "g2": r(H * V, rg, seed=14, std=.4), "o": r(W, H * V, seed=15)}
     assert {k: tuple(t.shape) for k, t in w.items()} == ChannelDelta(W, H, G, D, V, taps, eps).shapes(ra, rg)
     m = ChannelDelta(W, H, G, D, V, taps, eps, out_scale=1.5)
@@ -326,7 +338,7 @@ def test_channel_delta(dev, dtype, H, G, D, V, taps):
         return out.view(len(rows), H, Vp)[..., :V].clone()
     head = torch.arange(H) // (H // G)
     for round_, slots in enumerate(([3, 0, 6, 1, 5, 2], [0, 1, 2, 3, 4, 5])):
-        got = _scan_in_cuts(dev, step, n, CUTS, slots, round_)
+        got = _scan_in_cuts(dev, step, n, CUTS, slots, run_min)
         for s in range(len(CUTS)):
             P = proj[s].double().cpu()
             part = lambda at, k, d, dp: P[:, at:at + k * dp].reshape(n, k, dp)[..., :d].reshape(n, k * d)
@@ -356,7 +368,8 @@ def test_inert_segments_leave_states_alone(dev, dtype):
     proj, state = (h.float() @ into.to(dev).float().T).to(dtype), m.allocate(5, dtype, dev)
     t = lambda *a: torch.tensor(a, dtype=torch.int32, device=dev)
     out = torch.full((4, 64), 9.0, dtype=dtype, device=dev)
-    m.scan(h, proj, state, Segments(None, t(1, 0, 900, 0), t(1, 4, 2, 4), t(0, 0, 0, 0), max_count=1), out)
+    m.scan(h, proj, state, types.SimpleNamespace(
+        segments=Segments(None, t(1, 0, 900, 0), t(1, 4, 2, 4), t(0, 0, 0, 0), max_count=1), run_segments=None), out)
     assert not out[1].any() and not out[3].any() and out[0].any() and out[2].any()
     assert not state[[0, 3, 4]].any() and state[1].any() and state[2].any()
 

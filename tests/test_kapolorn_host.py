@@ -251,6 +251,7 @@ def test_portion_plan_names_the_segments():
     a.block_table, b.block_table, c.block_table = [5, 6], [-1, 1, 2, 3], [9]
     plan = plan_portions([Portion(b, 20, 30), Portion(a, 19, 1), Portion(c, 5, 3)], 16, [Chunk(33)], 16)
     assert plan.first_row == [4, 0, 1]
+    assert plan.short == 2
     assert plan.segments.tolist() == [[0, 1, 4], [1, 3, 30], [3, 2, 1], [19, 5, 20]]
 
 

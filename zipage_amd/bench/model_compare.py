@@ -10,6 +10,7 @@ of a graph of many launches over buffers that together exceed the caches.
 from __future__ import annotations
 
 import time
+from types import SimpleNamespace
 
 import torch
 
@@ -300,7 +301,9 @@ def kapolorn_kernels(size: str, decode_batch: int, prompts: int, prompt: int) ->
         del qkvs, caches, kcs
         # recurrences
         n = N // seqs
-        seg = Segments(i32(range(0, N, n)), i32([n] * seqs), i32(torch.randperm(seqs)), i32([5] * seqs))
+        seg = Segments(i32(range(0, N, n)), i32([n] * seqs), i32(torch.randperm(seqs)), i32([5] * seqs), longest=n,
+                       max_count=int(n == 1))
+        seg = SimpleNamespace(segments=seg if n < 16 else None, run_segments=None if n < 16 else seg)
         for name, mixer, ops in ((f"mlstm_scan, {H // 2} heads", MatrixMemory(W, H // 2, D, D, 15.0, 1e-6), 5),
                                  (f"delta_scan, {H} heads", ChannelDelta(W, H, H // 2, D, D, 4, 1e-6), 7)):
             small = {q: torch.randn(*s) * 0.02 for q, s in (mixer.shapes() if ops == 5 else mixer.shapes(128, 128)).items()}

@@ -32,7 +32,8 @@ FLAGS = BASE_FLAGS + ["-ffp-contract=off"]
 MODEL_SOURCES = {
     MODELS_LIB: ("residual.hip", "runs.hip"),
     LATENT_LIB: ("latent.hip",),
-    HYBRID_LIB: ("grouped.hip", "mlstm.hip", "delta.hip", "moe.hip"),
+    HYBRID_LIB: ("grouped.hip", "mlstm.hip", "mlstm_runs.hip", "delta.hip", "delta_runs.hip",
+                 "moe.hip"),
 }
 COMMON_SOURCES = ("runtime.hip",)
 LIBS = (LIB, *MODEL_SOURCES)

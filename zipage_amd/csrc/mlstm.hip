@@ -143,9 +143,106 @@ __global__ __launch_bounds__(64 * NW) void mlstm_scan_kernel(zp_mlstm a) {
   if (tid == 0) nstate[dk] = m;
 }
 
+// One token per segment (decoding): the state passes through once, nothing is staged.
+template <typename T, int RL, int NW>
+__global__ __launch_bounds__(64 * NW) void mlstm_step_kernel(zp_mlstm a) {
+  __shared__ float red[NW];
+  const int dk = 8 * RL, dv = a.dv;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
+  const int cq = lane_cq(), rg = lane_rg();
+  const int h = blockIdx.x % a.heads;
+  const Segment sg = segment_of(a.seg, blockIdx.x / a.heads);
+  const int col = wave * 32 + cq * 4;
+  const int64_t out_at = sg.row * a.out_stride + h * dv + col;
+  if (sg.count <= 0) {
+    if (a.seg.rows == nullptr && sg.row < a.seg.num_rows && rg == 0) store4<T>(a.out, out_at, f32x4{0.f, 0.f, 0.f, 0.f});
+    return;
+  }
+  const int64_t src = sg.row * a.in_stride + h * dk, vsrc = sg.row * a.in_stride + h * dv + col;
+  float* const state = a.state + ((int64_t)sg.slot * a.heads + h) * ((int64_t)dk * dv + dk + 4);
+  float* const nstate = state + (int64_t)dk * dv;
+  const bool fresh = sg.start == 0;
+  constexpr int kN = (RL * 8 + 63) / 64;
+  f32x4 S[RL], q[RL / 4], k[RL / 4];
+#pragma unroll
+  for (int j = 0; j < RL / 4; ++j) {
+    q[j] = load4<T>(a.in, src + a.q_at + 4 * (8 * j + rg));
+    k[j] = load4<T>(a.in, src + a.k_at + 4 * (8 * j + rg));
+  }
+  f32x4 v = load4<T>(a.in, vsrc + a.v_at);
+  const f32x4 gate = load4<T>(a.in, vsrc + a.g_at);
+  float nv[kN], nk[kN], nq[kN];
+#pragma unroll
+  for (int j = 0; j < kN; ++j) {
+    const int c = lane + 64 * j;
+    nv[j] = !fresh && c < dk ? nstate[c] : 0.f;
+    nk[j] = c < dk ? Elem<T>::ld(a.in, src + a.k_at + c) : 0.f;
+    nq[j] = c < dk ? Elem<T>::ld(a.in, src + a.q_at + c) : 0.f;
+  }
+  const float m0 = fresh ? 0.f : nstate[dk];
+  const float zi = a.gates[sg.row * a.gate_stride + h], zf = a.gates[sg.row * a.gate_stride + a.heads + h];
+#pragma unroll
+  for (int r = 0; r < RL; ++r) {
+    S[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (!fresh) S[r] = *(const f32x4*)(state + (int64_t)(4 * (8 * (r >> 2) + rg) + (r & 3)) * dv + col);
+  }
+  const float gi = a.cap * tanhf((zi + a.i_bias[h]) / a.cap), x = a.cap * tanhf((zf + a.f_bias[h]) / a.cap);
+  const float gf = fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
+  const float m = fmaxf(gf + m0, gi), kp = expf(gf + m0 - m), w = expf(gi - m);
+  float d = 0.f;
+#pragma unroll
+  for (int j = 0; j < kN; ++j) {
+    nv[j] = fmaf(w, nk[j], nv[j] * kp);
+    d = fmaf(nv[j], nq[j], d);
+  }
+  d = wave_sum(d) * a.q_scale;
+  const float f = a.q_scale / (fmaxf(fabsf(d), expf(-m)) + 1e-6f);
+  v *= w;
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < RL; ++r) {
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      S[r][c] = fmaf(k[r >> 2][r & 3], v[c], S[r][c] * kp);
+      o[c] = fmaf(S[r][c], q[r >> 2][r & 3], o[c]);
+    }
+    *(f32x4*)(state + (int64_t)(4 * (8 * (r >> 2) + rg) + (r & 3)) * dv + col) = S[r];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < 4; ++c) {
+    o[c] = rows_sum(o[c]) * f;
+    ss = fmaf(o[c], o[c], ss);
+  }
+  ss = quads_sum(ss);
+  if (lane == 0) red[wave] = ss;
+  __syncthreads();                            // also: every wave has read n and m
+  ss = 0.f;
+  for (int i = 0; i < nw; ++i) ss += red[i];
+  const float rs = a.out_scale / sqrtf(ss / (float)a.vdim + a.eps);
+  if (rg == 0) {
+    const f32x4 wn = *(const f32x4*)(a.norm + h * dv + col);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) o[c] *= rs * wn[c] * sigmoid_f(gate[c]);
+    store4<T>(a.out, out_at, o);
+  }
+  if (wave == nw - 1) {
+#pragma unroll
+    for (int j = 0; j < kN; ++j)
+      if (lane + 64 * j < dk) nstate[lane + 64 * j] = nv[j];
+    if (lane == 0) nstate[dk] = m;
+  }
+}
+
 template <typename T, int RL> int launch_mlstm(const zp_mlstm& a, hipStream_t st) {
   const size_t smem = sizeof(float) * kScanTokens * (2 * a.dk + a.dv + 3);
   const dim3 grid((unsigned)((int64_t)a.seg.n * a.heads)), block(a.dv * 2);
+  if (a.seg.max_count == 1) {
+    if (a.dv <= 128) hipLaunchKernelGGL((mlstm_step_kernel<T, RL, 4>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((mlstm_step_kernel<T, RL, 8>), grid, block, 0, st, a);
+    ZP_LAUNCH_CHECK();
+    return ZP_OK;
+  }
   const void* fn = a.dv <= 128 ? (const void*)mlstm_scan_kernel<T, RL, 4> : (const void*)mlstm_scan_kernel<T, RL, 8>;
   if (smem > 64 * 1024 && hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) != hipSuccess) {
     zp_set_error("mlstm: cannot reserve %zu bytes of LDS", smem);
@@ -166,13 +263,13 @@ extern "C" int zp_mlstm_scan(const zp_mlstm* args, int32_t dtype, void* stream) 
                  a.gate_stride >= 2 * a.heads && a.out_stride >= (int64_t)a.heads * a.dv, "mlstm: bad dims");
   ZP_MODEL_DTYPE("mlstm");
   if ((a.dk != 32 && a.dk != 64 && a.dk != 128 && a.dk != 256) || a.dv % 32 || a.dv > 256 || a.in_stride % 8 ||
-      a.q_at % 8 || a.k_at % 8 || a.v_at % 8) {
+      a.q_at % 8 || a.k_at % 8 || a.v_at % 8 || a.g_at % 8 || a.out_stride % 8) {
     zp_set_error("mlstm: head sizes %d (32, 64, 128, 256) and %d (a multiple of 32, <= 256) unsupported", a.dk, a.dv);
     return ZP_EUNSUPPORTED;
   }
   if (a.seg.n == 0) return ZP_OK;
   ZP_REQUIRE(a.in && a.gates && a.i_bias && a.f_bias && a.norm && a.state && a.out && a.seg.counts && a.seg.slots &&
-                 a.seg.starts && aligned16(a.in) && aligned16(a.state), "mlstm: null or unaligned pointer");
+                 a.seg.starts && aligned16(a.in) && aligned16(a.state) && aligned16(a.norm) && aligned16(a.out), "mlstm: null or unaligned pointer");
   hipStream_t st = (hipStream_t)stream;
 #define ZP_MLSTM(T)                                    \
   switch (a.dk) {                                      \

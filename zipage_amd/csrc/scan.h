@@ -41,6 +41,34 @@ __device__ __forceinline__ float rows_sum(float v) {
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
+// Sum over the eight column quads of a wave (lanes of one row group), in every one of them.
+__device__ __forceinline__ float quads_sum(float v) {
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x141, 0xf, 0xf, false));  // half mirror
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xf, 0xf, false));   // [1,0,3,2]
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xf, 0xf, false));   // [2,3,0,1]
+  return v;
+}
+
+// Four consecutive elements as fp32.
+template <typename T> __device__ __forceinline__ f32x4 load4(const void* p, int64_t i);
+template <> __device__ __forceinline__ f32x4 load4<BF16>(const void* p, int64_t i) {
+  const uint2 v = *(const uint2*)((const uint16_t*)p + i);
+  return f32x4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+               __uint_as_float(v.y & 0xffff0000u)};
+}
+template <> __device__ __forceinline__ f32x4 load4<F32>(const void* p, int64_t i) {
+  return *(const f32x4*)((const float*)p + i);
+}
+template <typename T> __device__ __forceinline__ void store4(void* p, int64_t i, const f32x4& v);
+template <> __device__ __forceinline__ void store4<BF16>(void* p, int64_t i, const f32x4& v) {
+  const zp_f32x2 a = {v[0], v[1]}, b = {v[2], v[3]};
+  uint2 o;
+  o.x = __builtin_bit_cast(uint32_t, __builtin_convertvector(a, zp_bf16x2));
+  o.y = __builtin_bit_cast(uint32_t, __builtin_convertvector(b, zp_bf16x2));
+  *(uint2*)((uint16_t*)p + i) = o;
+}
+template <> __device__ __forceinline__ void store4<F32>(void* p, int64_t i, const f32x4& v) { *(f32x4*)((float*)p + i) = v; }
+
 constexpr int kScanTokens = 16;   // tokens staged in LDS at a time
 
 // Readout of one token by one wave: o (dv values in LDS, the mean over vdim) normed, weighted, gated.

@@ -117,6 +117,7 @@ class PortionPlan:
     tables: np.ndarray            # (sequences, width), -1 where nothing is held
     first_row: list[int]          # token row where each portion starts, in the order given
     segments: np.ndarray          # (4, portions): token row, tokens, query row, position of the first
+    short: int                    # so many of them, which come first, are attended one by one
     runs: dict = field(default_factory=dict)
 
 
@@ -170,7 +171,7 @@ def plan_portions(portions: list[Portion], block_size: int, sights, run_min: int
     segments = np.array([[first_row[i], portions[i].count, portions[i].seq.query_id, portions[i].start]
                          for i in short + long], np.int32).T
     plan = PortionPlan(np.asarray(ids, np.int32), np.asarray(rows, np.int32), cat(pos), cat(slots),
-                       cat(ctx), cat(trows), tables, first_row, segments)
+                       cat(ctx), cat(trows), tables, first_row, segments, len(short))
     if long:
         for w in sights:
             plan.runs[w] = plan_runs([portions[i] for i in long], block_size, w)

@@ -164,7 +164,7 @@ class Parallel:
     def mix(self, h, proj, positions, cache, ctx, out):
         cut, edge = self.left.columns, self.left.out_columns
         self.left.attend(proj[:, :cut], positions, cache[0], ctx, out[:, :edge])
-        self.right.scan(h, proj[:, cut:], cache[1], ctx.segments, out[:, edge:])
+        self.right.scan(h, proj[:, cut:], cache[1], ctx, out[:, edge:])
 
 
 class Delta:
@@ -187,7 +187,7 @@ class Delta:
         return self.core.allocate(num_slots, dtype, device)
 
     def mix(self, h, proj, positions, cache, ctx, out):
-        self.core.scan(proj, cache, ctx.segments, out)
+        self.core.scan(proj, cache, ctx, out)
 
 
 class Kapolorn:

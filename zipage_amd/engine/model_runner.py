@@ -228,7 +228,10 @@ class ModelRunner:
         d = iter([buf[a:b] for a, b in spans])
         ids, rows, pos, slots, ctx_lens, table_rows = (next(d) for _ in range(6))
         tables = next(d).view(plan.tables.shape)
-        segments = Segments(*(next(d) for _ in range(4)))
+        seg, k = [next(d) for _ in range(4)], plan.short
+        segments = Segments(*(a[:k] for a in seg)) if k else None
+        long = Segments(*(a[k:] for a in seg), first_row=int(plan.segments[0, k]),
+                        longest=int(plan.segments[1, k:].max())) if k < len(portions) else None
         runs = {}
         for w, r in plan.runs.items():
             tiles = next(d).view(-1, 4)
@@ -236,7 +239,8 @@ class ModelRunner:
         ids = ids.long()
         if (plan.rows >= 0).any():
             ids = torch.where(rows >= 0, self.last_token[rows.clamp_min(0).long()], ids)
-        ctx = StepContext(False, slots, None, ctx_lens, tables, table_rows=table_rows, runs=runs, segments=segments)
+        ctx = StepContext(False, slots, None, ctx_lens, tables, table_rows=table_rows, runs=runs, segments=segments,
+                          run_segments=long)
         return ids, pos, ctx, plan.first_row
 
     @staticmethod

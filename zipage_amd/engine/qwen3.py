@@ -46,12 +46,14 @@ QWEN3_0_6B = Qwen3Shape(28, 1024, 16, 8, 128, 3072, 151936)
 class Segments:
     """The portions of a step as recurrent layers read them, int32 arrays: first token row (None: the
     portion's index), tokens (at most `max_count` when that is set; 0: inert), state slot, position of
-    the first token."""
+    the first token.  Long runs also name the first row of all and the length of the longest."""
     rows: torch.Tensor | None
     counts: torch.Tensor
     slots: torch.Tensor
     starts: torch.Tensor
     max_count: int = 0
+    first_row: int = 0
+    longest: int = 0
 
 
 @dataclass
@@ -69,7 +71,9 @@ class StepContext:
     # row table_rows[i] of block_tables (None: i); the rest belong to runs, planned per kind of sight
     table_rows: torch.Tensor | None = None          # (singles,) int32
     runs: dict | None = None                        # sight -> inputs.Runs
-    segments: Segments | None = None                # the portions, for recurrent layers
+    # the same portions for recurrent layers: those attended one by one, and the runs
+    segments: Segments | None = None
+    run_segments: Segments | None = None
 
 
 class Qwen3:

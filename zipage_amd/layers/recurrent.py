@@ -1,6 +1,6 @@
 """Recurrent mixers: a matrix memory with exponential gates, and a gated delta rule with a decay per key
 channel.  Both keep a float32 matrix per head and sequence slot; a step hands them its portions as
-segments (`StepContext.segments`)."""
+segments (`StepContext.segments`, and `.run_segments` where 16 tokens at a time pay)."""
 from __future__ import annotations
 
 import ctypes
@@ -72,18 +72,27 @@ class MatrixMemory:
         return torch.zeros(num_slots, self.heads, self.dim_p * self.vdim_p + self.dim_p + 4, dtype=torch.float32,
                            device=device)
 
-    def scan(self, h: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, segments, out: torch.Tensor):
+    @property
+    def can_run(self) -> bool:
+        """Sizes the blocked kernel covers; others run token by token."""
+        return self.dim_p <= 128 and self.vdim_p <= 128
+
+    def scan(self, h: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor):
         """h: the mixer's input (for the gates, which stay in fp32), proj: this mixer's columns of the
         projections, out: of the output rows."""
         H, D, V = self.heads, self.dim_p, self.vdim_p
         gates = small_linear(h, self.gates)
         assert proj.stride(1) == out.stride(1) == 1 and proj.dtype == out.dtype and state.is_contiguous()
-        args = _lib.MlstmArgs(
-            _segments(segments, state.shape[0], h.shape[0]), _lib.dev_ptr(proj), _lib.dev_ptr(gates),
-            _lib.dev_ptr(self.i_bias), _lib.dev_ptr(self.f_bias), _lib.dev_ptr(self.norm), _lib.dev_ptr(state),
-            _lib.dev_ptr(out), proj.stride(0), gates.stride(0), out.stride(0), H, D, V, self.vdim, 0, H * D, 2 * H * D,
-            2 * H * D + H * V, self.gate_cap, self.dim ** -0.5, self.eps, self.out_scale)
-        _lib.call_models("zp_mlstm_scan", ctypes.byref(args), _lib.dtype_tag(proj), _lib.stream_ptr(proj))
+        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run)):
+            if segments is None:
+                continue
+            args = _lib.MlstmArgs(
+                _segments(segments, state.shape[0], h.shape[0]), _lib.dev_ptr(proj), _lib.dev_ptr(gates),
+                _lib.dev_ptr(self.i_bias), _lib.dev_ptr(self.f_bias), _lib.dev_ptr(self.norm), _lib.dev_ptr(state),
+                _lib.dev_ptr(out), proj.stride(0), gates.stride(0), out.stride(0), H, D, V, self.vdim, 0, H * D,
+                2 * H * D, 2 * H * D + H * V, self.gate_cap, self.dim ** -0.5, self.eps, self.out_scale)
+            _lib.call_models("zp_mlstm_runs" if runs else "zp_mlstm_scan", ctypes.byref(args), _lib.dtype_tag(proj),
+                             _lib.stream_ptr(proj))
 
 
 class ChannelDelta:
@@ -141,16 +150,32 @@ class ChannelDelta:
                 torch.zeros(num_slots, self.heads, self.taps - 1, 2 * self.dim_p + self.vdim_p, dtype=dtype,
                             device=device))
 
-    def scan(self, proj: torch.Tensor, state, segments, out: torch.Tensor):
+    @property
+    def can_run(self) -> bool:
+        """Sizes the blocked kernels cover; others run token by token."""
+        return self.dim_p <= 128 and self.vdim_p <= 128
+
+    def scan(self, proj: torch.Tensor, state, ctx, out: torch.Tensor):
         """proj: this mixer's columns of the projections, out: of the output rows."""
         S, tail = state
         H, D = self.heads, self.dim_p
         assert proj.stride(1) == out.stride(1) == 1 and proj.dtype == out.dtype == tail.dtype and S.is_contiguous()
         low = F.linear(proj[:, self.low_at:self.low_at + self.low_rank], self.low)
-        args = _lib.DeltaArgs(
-            _segments(segments, S.shape[0], proj.shape[0]), _lib.dev_ptr(proj), _lib.dev_ptr(low),
-            _lib.dev_ptr(self.filters), _lib.dev_ptr(self.a_log), _lib.dev_ptr(self.dt_bias), _lib.dev_ptr(self.norm),
-            _lib.dev_ptr(S), _lib.dev_ptr(tail), _lib.dev_ptr(out), proj.stride(0), low.stride(0), out.stride(0), H,
-            self.kv_heads, D, self.vdim_p, self.vdim, self.taps, self.b_at, H * D, self.dim ** -0.5, self.eps,
-            self.out_scale)
-        _lib.call_models("zp_delta_scan", ctypes.byref(args), _lib.dtype_tag(proj), _lib.stream_ptr(proj))
+        tag, stream = _lib.dtype_tag(proj), _lib.stream_ptr(proj)
+        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run)):
+            if segments is None:
+                continue
+            args = _lib.DeltaArgs(
+                _segments(segments, S.shape[0], proj.shape[0]), _lib.dev_ptr(proj), _lib.dev_ptr(low),
+                _lib.dev_ptr(self.filters), _lib.dev_ptr(self.a_log), _lib.dev_ptr(self.dt_bias), _lib.dev_ptr(self.norm),
+                _lib.dev_ptr(S), _lib.dev_ptr(tail), _lib.dev_ptr(out), proj.stride(0), low.stride(0), out.stride(0), H,
+                self.kv_heads, D, self.vdim_p, self.vdim, self.taps, self.b_at, H * D, self.dim ** -0.5, self.eps,
+                self.out_scale)
+            if not runs:
+                _lib.call_models("zp_delta_scan", ctypes.byref(args), tag, stream)
+                continue
+            size = _lib.load_models("hybrid").zp_delta_runs_workspace(proj.shape[0] - segments.first_row,
+                                                                      segments.counts.numel(), H, D, self.vdim_p)
+            ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
+            _lib.call_models("zp_delta_runs", ctypes.byref(args), segments.first_row, segments.longest,
+                             _lib.dev_ptr(ws), size, tag, stream)
