@@ -135,9 +135,12 @@ typedef struct {
   float cap, q_scale, eps, out_scale;
 } zp_mlstm;
 int zp_mlstm_scan(const zp_mlstm* args, int32_t dtype, void* stream);
-/* The same for long runs, 16 tokens at a time on the matrix cores (fp32): dk 32, 64 or 128, dv up to 128,
- * rows given. */
-int zp_mlstm_runs(const zp_mlstm* args, int32_t dtype, void* stream);
+/* The same for long runs, 16 tokens at a time on the matrix cores (fp32): bfloat16, dk 32, 64 or 128, dv up
+ * to 128, rows given in rising order from first_row on, none longer than `longest`.  `workspace`:
+ * zp_mlstm_runs_workspace() bytes for the rows from first_row to the end. */
+int64_t zp_mlstm_runs_workspace(int32_t rows, int32_t segments, int32_t heads);
+int zp_mlstm_runs(const zp_mlstm* args, int32_t first_row, int32_t longest, void* workspace,
+                  int64_t workspace_bytes, int32_t dtype, void* stream);
 
 /* Gated delta rule with a decay per key channel, its short convolutions and gates, and the normed, gated
  * read-out.  Rows `in` hold the projections q, k (kv_heads of dk), v (heads of dv) and from column b_at
@@ -156,8 +159,8 @@ typedef struct {
   float q_scale, eps, out_scale;
 } zp_delta;
 int zp_delta_scan(const zp_delta* args, int32_t dtype, void* stream);
-/* The same for long runs (of taps - 1 tokens at least), 16 tokens at a time on the matrix cores (fp32): dk
- * 32, 64 or 128, dv up to 128, rows given in rising order from first_row on, none longer than
+/* The same for long runs (of taps - 1 tokens at least), 16 tokens at a time on the matrix cores (fp32):
+ * bfloat16, dk 32, 64 or 128, dv up to 128, rows given in rising order from first_row on, none longer than
  * `longest`.  `workspace`: zp_delta_runs_workspace() bytes for the rows from first_row to the end. */
 int64_t zp_delta_runs_workspace(int32_t rows, int32_t segments, int32_t heads, int32_t dk, int32_t dv);
 int zp_delta_runs(const zp_delta* args, int32_t first_row, int32_t longest, void* workspace,

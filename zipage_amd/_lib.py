@@ -133,7 +133,7 @@ MODEL_LIBS = {
         "zp_grouped_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32,
                                       i32, i32, i32, i64, f32, f32, i32, ptr, i64, ptr],
         "zp_mlstm_scan": [C.POINTER(MlstmArgs), i32, ptr],
-        "zp_mlstm_runs": [C.POINTER(MlstmArgs), i32, ptr],
+        "zp_mlstm_runs": [C.POINTER(MlstmArgs), i32, i32, ptr, i64, i32, ptr],
         "zp_delta_scan": [C.POINTER(DeltaArgs), i32, ptr],
         "zp_delta_runs": [C.POINTER(DeltaArgs), i32, i32, ptr, i64, i32, ptr],
         "zp_small_linear": [ptr, ptr, ptr, i32, i32, i32, i64, i32, ptr],
@@ -144,7 +144,7 @@ MODEL_LIBS = {
         "zp_moe_down": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, i64, i64, i32,
                         ptr],
     }, {"zp_grouped_rows_workspace": [i32, i32, i32, i32, i32, i32, i32, i32, i32, i32],
-        "zp_delta_runs_workspace": [i32, i32, i32, i32, i32], "zp_moe_tile_rows": [i32, i32, i32, i32],
+        "zp_mlstm_runs_workspace": [i32, i32, i32], "zp_delta_runs_workspace": [i32, i32, i32, i32, i32], "zp_moe_tile_rows": [i32, i32, i32, i32],
         "zp_moe_max_tiles": [i32, i32, i32, i32, i32], "zp_moe_plan_workspace": [i32, i32, i32]}),
 }
 MODEL_EXPORTS = {lib: sorted([*calls, *sizes]) for lib, (calls, sizes) in MODEL_LIBS.items()}

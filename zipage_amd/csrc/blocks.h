@@ -61,4 +61,69 @@ __device__ __forceinline__ f32x4 block_squares_total(const float* red, int nw) {
   return ss;
 }
 
+// Forms for 16-bit models on the hardware's exponential, logarithm, reciprocal and reciprocal square root,
+// each within a unit or two of the last of 24 bits.
+__device__ __forceinline__ float fast_sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+__device__ __forceinline__ float fast_softplus(float x) {
+  const float y = __expf(-fabsf(x));
+  // log(1 + y) as it stands loses a small y's digits
+  const float l = y < 0.03125f ? y * (1.f - y * (0.5f - y * (1.f / 3.f - y * 0.25f))) : __logf(1.f + y);
+  return fmaxf(x, 0.f) + l;
+}
+
+// Element (row 4 g + r, column col) of 16 token rows of bf16, for r = 0 .. 3; rows behind the last read as zero
+// and are not written.
+struct BlockRows {
+  __amdgpu_buffer_rsrc_t rs;
+  __device__ __forceinline__ BlockRows(const void* base, int64_t row, int cnt, int64_t stride)
+      : rs(__builtin_amdgcn_make_buffer_rsrc((void*)((char*)base + row * stride * 2), 0, (int)(cnt * stride * 2), 0x00020000)) {}
+  // as it is in memory: converting it is left to its use, so that nothing waits for the load before
+  __device__ __forceinline__ uint16_t ld(int offset, int col) const {
+    return __builtin_amdgcn_raw_buffer_load_b16(rs, offset, col * 2, 0);
+  }
+  __device__ __forceinline__ void st(int offset, int col, float v) const {
+    __builtin_amdgcn_raw_buffer_store_b16(float_to_bf16_bits(v), rs, offset, col * 2, 0);
+  }
+};
+
+// Columns of a 4 x 16 block of 16-bit values in LDS: lane i of a group of sixteen names row i / 4, values 4 (i % 4)
+// on, and receives column i.
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ f32x4 read_columns(const char* p) {
+  const s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)p);
+  return f32x4{bf16_bits_to_float((uint16_t)v[0]), bf16_bits_to_float((uint16_t)v[1]), bf16_bits_to_float((uint16_t)v[2]),
+               bf16_bits_to_float((uint16_t)v[3])};
+}
+
+// Loads straight into LDS: lane l's 16 bytes from `base` + offset (+ uniform) to `lds` + 16 l.  Written out,
+// because the compiler, which cannot tell the stage being filled from the stage being read, would wait for
+// them at the next LDS read; wait_and_meet() waits for them.
+typedef __attribute__((address_space(3))) void* lds_ptr_t;
+struct StageLoads {
+  u32x4 rs;
+  __device__ __forceinline__ StageLoads(const void* base, int64_t bytes) {
+    const uint64_t p = (uint64_t)base;
+    rs = u32x4{(uint32_t)__builtin_amdgcn_readfirstlane((int)(uint32_t)p),
+               (uint32_t)__builtin_amdgcn_readfirstlane((int)((uint32_t)(p >> 32) & 0xffffu)),
+               (uint32_t)__builtin_amdgcn_readfirstlane((int)bytes), 0x00020000u};
+  }
+  __device__ __forceinline__ void ld(void* lds, int offset, int uniform) const {
+    const uint32_t to = (uint32_t)__builtin_amdgcn_readfirstlane((int)(uint32_t)(uintptr_t)(lds_ptr_t)lds);
+    const int so = __builtin_amdgcn_readfirstlane(uniform);
+    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds"
+                 :: "s"(to), "v"(offset), "s"(rs), "s"(so) : "memory", "m0");
+  }
+};
+__device__ __forceinline__ void wait_and_meet() {
+  asm volatile("" ::: "memory");
+  __builtin_amdgcn_s_waitcnt(0);               // as a builtin: the compiler then knows that nothing is outstanding
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
+// Blocks of segment i start at slot (row - row0) / 16 + i: enough room, whatever the counts are.
+__device__ __forceinline__ int64_t block_slot(int row0, const Segment& sg, int seg, int b) {
+  return (sg.row - row0) / kBlock + seg + b;
+}
+
 }  // namespace

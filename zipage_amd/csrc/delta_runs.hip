@@ -7,7 +7,8 @@
 //
 // delta_prepare computes everything without S for all blocks at once and leaves it in the order of the
 // matrix operands; ratios of decays are running products of the decays themselves, so nothing is divided
-// and nothing overflows.  delta_blocks walks a head's blocks with S in registers.  All fp32.
+// and nothing overflows.  delta_blocks walks a head's blocks with S in registers.  All fp32; projections in
+// bfloat16.
 #include "blocks.h"
 
 namespace {
@@ -20,14 +21,19 @@ struct RunArgs {
   int row0;      // first token row of the first segment
 };
 
-__host__ __device__ inline int block_floats(int dk, int dv) { return kBlock * (3 * dk + dv) + kBlock * kBlock + dk; }
-// Blocks of segment i start at slot (row - row0) / 16 + i: enough room, whatever the counts are.
-__device__ __forceinline__ int64_t block_slot(const RunArgs& a, const Segment& sg, int seg, int b) {
-  return (sg.row - a.row0) / kBlock + seg + b;
+// [-W | G q] and the keys as left operands, U0 as a result tile, P, the block's decays; whole KBs
+__host__ __device__ inline int block_floats(int dk, int dv) {
+  return (kBlock * (3 * dk + dv) + kBlock * kBlock + dk + 255) / 256 * 256;
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void delta_prepare_kernel(RunArgs ra) {
+__device__ __forceinline__ void load2(const char* p, float& x, float& y) {
+  const uint32_t v = *(const uint32_t*)p;
+  x = __uint_as_float(v << 16);
+  y = __uint_as_float(v & 0xffff0000u);
+}
+
+template <int TAPS>
+__global__ __launch_bounds__(256, 3) void delta_prepare_kernel(RunArgs ra) {
   extern __shared__ __align__(16) float lds[];
   const zp_delta& a = ra.d;
   const int dk = a.dk, dv = a.dv, taps = a.taps;
@@ -46,48 +52,57 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(RunArgs ra) {
   float* const outs = beta + kBlock;           // W and G q in operand order, 4 floats of padding per 64
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int cw = 2 * dk + dv;
-  const char* const tail = (const char*)a.conv_state + ((int64_t)sg.slot * a.heads + h) * (taps - 1) * cw * T::bytes;
+  const char* const tail = (const char*)a.conv_state + ((int64_t)sg.slot * a.heads + h) * (taps - 1) * cw * 2;
   const float rate = expf(a.a_log[h]);
   const int channels = 2 * a.kv_heads * dk + a.heads * dv;
   auto place = [&](int c) -> int {
     return c < dk ? hk * dk + c : (c < 2 * dk ? a.kv_heads * dk + hk * dk + c - dk : 2 * a.kv_heads * dk + h * dv + c - 2 * dk);
   };
-  // ---- convolutions: a thread's channel, the block's 16 tokens from a sliding window
-  for (int c = tid; c < cw; c += 256) {
+  // ---- convolutions: a thread's two channels, the block's 16 tokens from a sliding window
+  for (int c = 2 * tid; c < cw; c += 512) {
     const int at = place(c);
-    float x[kBlock + kMaxTaps - 1], f[kMaxTaps];
+    float f[2][TAPS], x[2][kBlock + TAPS - 1];
 #pragma unroll
-    for (int j = 0; j < kMaxTaps; ++j) f[j] = j < taps ? a.filters[(int64_t)(taps - 1 - j) * channels + at] : 0.f;   // f[j]: j tokens back
+    for (int j = 0; j < TAPS; ++j)                            // f[.][j]: j tokens back
 #pragma unroll
-    for (int i = 0; i < kBlock + kMaxTaps - 1; ++i) {
-      const int u = t0 + i - (kMaxTaps - 1);
-      x[i] = 0.f;
-      if (i >= kMaxTaps - taps && u < t0 + cnt) {
-        if (u >= 0) x[i] = Elem<T>::ld(a.in, (int64_t)(sg.row + u) * a.in_stride + at);
-        else if (sg.start > 0) x[i] = Elem<T>::ld(tail, (int64_t)(taps - 1 + u) * cw + c);
+      for (int e = 0; e < 2; ++e) f[e][j] = j < taps ? a.filters[(int64_t)(taps - 1 - j) * channels + at + e] : 0.f;
+    const char* const first = (const char*)a.in + ((int64_t)(sg.row + t0) * a.in_stride + at) * 2;
+#pragma unroll
+    for (int i = 0; i < kBlock + TAPS - 1; ++i) {
+      const int u = t0 + i - (TAPS - 1);
+      x[0][i] = x[1][i] = 0.f;
+      if (i >= TAPS - taps && u < t0 + cnt) {
+        if (u >= 0) load2(first + (int64_t)(i - (TAPS - 1)) * a.in_stride * 2, x[0][i], x[1][i]);
+        else if (sg.start > 0) load2(tail + ((int64_t)(taps - 1 + u) * cw + c) * 2, x[0][i], x[1][i]);
       }
     }
     float* const dst = c < dk ? qs + c : (c < 2 * dk ? ks + c - dk : vs + c - 2 * dk);
     const int st = c < 2 * dk ? dk : dv;
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
-      float y = 0.f;
+      float2 y = {0.f, 0.f};
 #pragma unroll
-      for (int j = 0; j < kMaxTaps; ++j) y = fmaf(f[j], x[t + kMaxTaps - 1 - j], y);
-      dst[t * st] = t < cnt ? y * sigmoid_f(y) : 0.f;
+      for (int j = 0; j < TAPS; ++j) {
+        y.x = fmaf(f[0][j], x[0][t + TAPS - 1 - j], y.x);
+        y.y = fmaf(f[1][j], x[1][t + TAPS - 1 - j], y.y);
+      }
+      y.x = t < cnt ? y.x * fast_sigmoid(y.x) : 0.f;
+      y.y = t < cnt ? y.y * fast_sigmoid(y.y) : 0.f;
+      *(float2*)(dst + t * st) = y;
     }
   }
-  for (int i = tid; i < kBlock * dk; i += 256) {
-    const int t = i / dk, c = i - t * dk;
-    float g = 1.f;
+  for (int i = tid; i < kBlock * dk / 4; i += 256) {
+    const int t = i / (dk / 4), c = (i - t * (dk / 4)) * 4;
+    f32x4 g = {1.f, 1.f, 1.f, 1.f};
     if (t < cnt) {
-      const float z = Elem<T>::ld(a.low, (int64_t)(sg.row + t0 + t) * a.low_stride + h * dk + c) + a.dt_bias[h * dk + c];
-      g = expf(-rate * softplus_f(z));
+      const f32x4 z = load4<BF16>(a.low, (int64_t)(sg.row + t0 + t) * a.low_stride + h * dk + c) + *(const f32x4*)(a.dt_bias + h * dk + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[e] = __expf(-rate * fast_softplus(z[e]));
     }
-    gs[i] = g;
+    *(f32x4*)(gs + t * dk + c) = g;
   }
   if (tid < kBlock)
-    beta[tid] = tid < cnt ? sigmoid_f(Elem<T>::ld(a.in, (int64_t)(sg.row + t0 + tid) * a.in_stride + a.b_at + h)) : 0.f;
+    beta[tid] = tid < cnt ? fast_sigmoid(Elem<BF16>::ld(a.in, (int64_t)(sg.row + t0 + tid) * a.in_stride + a.b_at + h)) : 0.f;
   __syncthreads();
   // ---- unit vectors: a wave its four tokens
 #pragma unroll
@@ -141,46 +156,51 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(RunArgs ra) {
         As[t * kBlock + s] = t > s ? sa * beta[t] : 0.f;
         Ps[t * kBlock + s] = t >= s ? sp : 0.f;
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
   }
   __syncthreads();
   // ---- columns: forward substitution, and the block's decays
-  const int64_t base = (block_slot(ra, sg, blockIdx.z, blockIdx.x) * a.heads + h) * block_floats(dk, dv);
+  const int64_t base = (block_slot(ra.row0, sg, blockIdx.z, blockIdx.x) * a.heads + h) * block_floats(dk, dv);
   float* const oWQ = ra.ws + base;             // [2][dk / 16][64 lanes][4]
   float* const oK = oWQ + 2 * kBlock * dk;     // [dk / 16][64][4]
   float* const oU = oK + kBlock * dk;          // [dv / 16][64][4]
   float* const oP = oU + kBlock * dv;          // [64][4]
   float* const oG = oP + kBlock * kBlock;      // [dk]
   for (int c = tid; c < dk + dv; c += 256) {
+    // a token at a time: its factors and values must not all sit in registers
     float w[kBlock];
-    if (c < dk) {
-      float G = 1.f;
-      const int at = (c >> 4) * 272 + ((c & 15) >> 2) * 68 + (c & 3);      // 256 and 64 floats, padded
+    const bool key = c < dk;
+    const float* const src = key ? ks + c : vs + c - dk;
+    const int st = key ? dk : dv, o_at = (c >> 4) * 272 + ((c & 15) >> 2) * 68 + (c & 3);      // 256 and 64 floats, padded
+    float G = 1.f;
 #pragma unroll
-      for (int t = 0; t < kBlock; ++t) {
+    for (int t = 0; t < kBlock; ++t) {
+      if (key) {
         G *= gs[t * dk + c];
-        w[t] = beta[t] * ks[t * dk + c] * G;
-        outs[(dk / 16) * 272 + at + t * 4] = qs[t * dk + c] * G;
+        outs[(dk / 16) * 272 + o_at + t * 4] = qs[t * dk + c] * G;
       }
-      oG[c] = G;
-    } else {
+      float x = beta[t] * src[t * st] * G;
 #pragma unroll
-      for (int t = 0; t < kBlock; ++t) w[t] = beta[t] * vs[t * dv + c - dk];
+      for (int s = 0; s < t; s += 4) {
+        const f32x4 A = *(const f32x4*)(As + t * kBlock + s);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (s + i < t) x = fmaf(-A[i], w[s + i], x);
+      }
+      w[t] = x;
+      __builtin_amdgcn_sched_barrier(0);
     }
-#pragma unroll
-    for (int t = 1; t < kBlock; ++t) {
-#pragma unroll
-      for (int s = 0; s < t; ++s) w[t] = fmaf(-As[t * kBlock + s], w[s], w[t]);
-    }
+    if (key) oG[c] = G;
     if (c < dk) {
-      const int at = (c >> 4) * 272 + ((c & 15) >> 2) * 68 + (c & 3);
 #pragma unroll
-      for (int t = 0; t < kBlock; ++t) outs[at + t * 4] = -w[t];
+      for (int t = 0; t < kBlock; ++t) outs[o_at + t * 4] = -w[t];
       float R = 1.f;
 #pragma unroll
       for (int t = kBlock - 1; t >= 0; --t) {
         w[t] = ks[t * dk + c] * R;
         R *= gs[t * dk + c];
+        if (t % 4 == 0) __builtin_amdgcn_sched_barrier(0);
       }
 #pragma unroll
       for (int g = 0; g < 4; ++g)
@@ -200,12 +220,16 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(RunArgs ra) {
   }
 }
 
-template <typename T, int KT, int NC>
-__global__ __launch_bounds__(NC == 2 ? 256 : 512) void delta_blocks_kernel(RunArgs ra) {
+// A head's blocks, one after the other: a block's operands come straight into LDS while the block before it is
+// worked on; its rows are normed and stored behind the next meeting of the waves, which the norm needs too.
+template <int KT, int NC>
+__global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(RunArgs ra) {
+  extern __shared__ __align__(16) float lds[];
   const zp_delta& a = ra.d;
-  __shared__ float red[2][16 * kBlock];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
-  const int dk = 16 * KT, dv = a.dv;
+  const int tid = threadIdx.x, lane = tid & 63, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int dk = 16 * KT, dv = a.dv, size = block_floats(dk, dv);
+  float* const red = lds + 2 * size;           // [2][8 * 16]
   const int h = blockIdx.x % a.heads, seg = blockIdx.x / a.heads;
   const Segment sg = segment_of(a.seg, seg);
   if (sg.count <= 0 || sg.row < ra.row0) return;
@@ -217,112 +241,127 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void delta_blocks_kernel(RunAr
   float nrm[NC];
 #pragma unroll
   for (int nc = 0; nc < NC; ++nc) nrm[nc] = a.norm[h * dv + col0 + nc * 16 + l16] * a.out_scale;
-  const int64_t stride = (int64_t)a.heads * block_floats(dk, dv);
-  const float* blk = ra.ws + (block_slot(ra, sg, seg, 0) * a.heads + h) * block_floats(dk, dv) + lane * 4;
+  const float* const base = ra.ws + (block_slot(ra.row0, sg, seg, 0) * a.heads + h) * size;
+  const int64_t stride = (int64_t)a.heads * size;
   const int blocks = (sg.count + kBlock - 1) / kBlock;
-  f32x4 W[KT], Q[KT], U[NC];
-  auto fetch = [&](const float* p) {
+  auto request = [&](int b) {
+    const StageLoads from(base + b * stride, size * 4);
+    for (int i = wave; i < size / 256; i += nw) from.ld(lds + (b & 1) * size + i * 256, lane * 16, i * 1024);
+  };
+  f32x4 O[NC];
+  uint16_t gate[NC][4];
+  const float inv_v = 1.f / (float)a.vdim;
+  const int out_at = (4 * g * (int)a.out_stride + h * dv + col0 + l16) * 2;
+  const int low_at = (4 * g * (int)a.low_stride + a.g_at + h * dv + col0 + l16) * 2;
+  auto finish = [&](int b) {                   // rows of block b, whose squares are in red
+    const f32x4 ss = block_squares_total(red + (b & 1) * 8 * kBlock, nw);
+    const int cnt = min(kBlock, sg.count - b * kBlock);
+    const BlockRows out(a.out, sg.row + b * kBlock, cnt, a.out_stride);
 #pragma unroll
-    for (int kt = 0; kt < KT; ++kt) {
-      W[kt] = *(const f32x4*)(p + kt * 256);
-      Q[kt] = *(const f32x4*)(p + (KT + kt) * 256);
+    for (int r = 0; r < 4; ++r) {
+      const float rs = __builtin_amdgcn_rsqf(ss[r] * inv_v + a.eps);
+#pragma unroll
+      for (int nc = 0; nc < NC; ++nc)
+        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, O[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
+    }
+  };
+  request(0);
+  __builtin_amdgcn_s_waitcnt(0);               // the state is there: the loop's first use of it must not wait in every pass
+#pragma unroll 1
+  for (int b = 0; b < blocks; ++b) {
+    wait_and_meet();
+    if (b + 1 < blocks) request(b + 1);
+    if (b > 0) finish(b - 1);
+    const int cnt = min(kBlock, sg.count - b * kBlock);
+    const BlockRows low(a.low, sg.row + b * kBlock, cnt, a.low_stride);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int nc = 0; nc < NC; ++nc) gate[nc][r] = low.ld(low_at + r * (int)a.low_stride * 2, nc * 16);
+    const float* const blk = lds + (b & 1) * size + lane * 4;
+    f32x4 U[NC];
+#pragma unroll
+    for (int nc = 0; nc < NC; ++nc) {
+      U[nc] = *(const f32x4*)(blk + 3 * kBlock * dk + (wave * NC + nc) * 256);
+      O[nc] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 #pragma unroll
-    for (int nc = 0; nc < NC; ++nc) U[nc] = *(const f32x4*)(p + 3 * kBlock * dk + (wave * NC + nc) * 256);
-  };
-  fetch(blk);
-  for (int b = 0; b < blocks; ++b, blk += stride) {
-    f32x4 K[KT];
-#pragma unroll
-    for (int kt = 0; kt < KT; ++kt) K[kt] = *(const f32x4*)(blk + (2 * KT + kt) * 256);
-    const f32x4 P = *(const f32x4*)(blk + kBlock * (3 * dk + dv));
-    const float* const dec = blk - lane * 4 + kBlock * (3 * dk + dv) + kBlock * kBlock + 4 * g;
-    const int cnt = min(kBlock, sg.count - b * kBlock);
-    const int64_t row = sg.row + b * kBlock;
-    float gate[NC][4];
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        gate[nc][r] = Elem<T>::ld(a.low, (row + min(4 * g + r, cnt - 1)) * a.low_stride + a.g_at + h * dv + col0 + nc * 16 + l16);
-    f32x4 O[NC];
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc) O[nc] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int kt = 0; kt < KT; ++kt)
+    for (int kt = 0; kt < KT; ++kt) {
+      const f32x4 W = *(const f32x4*)(blk + kt * 256), Q = *(const f32x4*)(blk + (KT + kt) * 256);
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int nc = 0; nc < NC; ++nc) {
-          U[nc] = mfma_f32_step(W[kt][j], S[kt][nc][j], U[nc]);
-          O[nc] = mfma_f32_step(Q[kt][j], S[kt][nc][j], O[nc]);
+          U[nc] = mfma_f32_step(W[j], S[kt][nc][j], U[nc]);
+          O[nc] = mfma_f32_step(Q[j], S[kt][nc][j], O[nc]);
         }
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc) mfma_f32_16(P, U[nc], O[nc]);
-    f32x4 u[NC];
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc) u[nc] = U[nc];
-    fetch(b + 1 < blocks ? blk + stride : blk);
+    }
+    const f32x4 P = *(const f32x4*)(blk + kBlock * (3 * dk + dv));
+    const float* const dec = blk - lane * 4 + kBlock * (3 * dk + dv) + kBlock * kBlock + 4 * g;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
-      const f32x4 d = *(const f32x4*)(dec + 16 * kt);
+      const f32x4 d = *(const f32x4*)(dec + 16 * kt), K = *(const f32x4*)(blk + (2 * KT + kt) * 256);
 #pragma unroll
       for (int nc = 0; nc < NC; ++nc) {
         S[kt][nc] *= d;
-        mfma_f32_16(K[kt], u[nc], S[kt][nc]);
+        mfma_f32_16(K, U[nc], S[kt][nc]);
       }
     }
-    block_squares<NC>(O, red[b & 1]);
-    __syncthreads();
-    const f32x4 ss = block_squares_total(red[b & 1], nw);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float rs = 1.f / sqrtf(ss[r] / (float)a.vdim + a.eps);
-      if (4 * g + r < cnt) {
-#pragma unroll
-        for (int nc = 0; nc < NC; ++nc)
-          Elem<T>::st(a.out, (row + 4 * g + r) * a.out_stride + h * dv + col0 + nc * 16 + l16,
-                      O[nc][r] * rs * nrm[nc] * sigmoid_f(gate[nc][r]));
-      }
-    }
+    for (int nc = 0; nc < NC; ++nc) mfma_f32_16(P, U[nc], O[nc]);
+    block_squares<NC>(O, red + (b & 1) * 8 * kBlock);
   }
+  wait_and_meet();
+  finish(blocks - 1);
   store_state<KT, NC>(S, state, dv, col0);
   // the last inputs of the head's convolutions (runs are longer than a filter)
   const int taps = a.taps, cw = 2 * dk + dv, hk = h / (a.heads / a.kv_heads);
-  char* const tail = (char*)a.conv_state + item * (taps - 1) * cw * T::bytes;
+  char* const tail = (char*)a.conv_state + item * (taps - 1) * cw * 2;
   for (int i = tid; i < (taps - 1) * cw; i += blockDim.x) {
     const int e = i / cw, c = i - e * cw;
     const int at = c < dk ? hk * dk + c : (c < 2 * dk ? a.kv_heads * dk + hk * dk + c - dk : 2 * a.kv_heads * dk + h * dv + c - 2 * dk);
-    Elem<T>::st(tail, i, Elem<T>::ld(a.in, (int64_t)(sg.row + max(sg.count - (taps - 1) + e, 0)) * a.in_stride + at));
+    Elem<BF16>::st(tail, i, Elem<BF16>::ld(a.in, (int64_t)(sg.row + max(sg.count - (taps - 1) + e, 0)) * a.in_stride + at));
   }
 }
 
-template <typename T, int KT> int launch_blocks(const RunArgs& ra, hipStream_t st) {
+template <int KT> int launch_blocks(const RunArgs& ra, hipStream_t st) {
   const zp_delta& a = ra.d;
   const unsigned grid = (unsigned)((int64_t)a.seg.n * a.heads);
-  // few heads: half the columns per wave, twice the waves
-  const bool narrow = (int64_t)grid * (a.dv / 32) < 1024;
-  if (narrow) hipLaunchKernelGGL((delta_blocks_kernel<T, KT, 1>), dim3(grid), dim3(a.dv * 4), 0, st, ra);
-  else hipLaunchKernelGGL((delta_blocks_kernel<T, KT, 2>), dim3(grid), dim3(a.dv * 2), 0, st, ra);
+  const bool narrow = a.dv % 64 != 0 && a.dv < 128;          // few columns: more, smaller waves
+  const int smem = (2 * block_floats(a.dk, a.dv) + 2 * 8 * kBlock) * 4;
+  const void* fn = narrow ? (const void*)delta_blocks_kernel<KT, 1> : (const void*)delta_blocks_kernel<KT, 2>;
+  if (smem > 60 * 1024 && hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
+    zp_set_error("delta_runs: cannot reserve %d bytes of LDS", smem);
+    return ZP_EHIP;
+  }
+  if (narrow) hipLaunchKernelGGL((delta_blocks_kernel<KT, 1>), dim3(grid), dim3(a.dv * 4), smem, st, ra);
+  else hipLaunchKernelGGL((delta_blocks_kernel<KT, 2>), dim3(grid), dim3(a.dv * 2), smem, st, ra);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }
 
-template <typename T> int launch_runs(const RunArgs& ra, int longest, hipStream_t st) {
+template <int TAPS> int launch_prepare(const RunArgs& ra, int longest, hipStream_t st) {
   const zp_delta& a = ra.d;
   const size_t smem = sizeof(float) * (kBlock * (3 * a.dk + a.dv) + 2 * kBlock * kBlock + kBlock + 2 * (a.dk / 16) * 272);
-  if (smem > 64 * 1024 && hipFuncSetAttribute((const void*)delta_prepare_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize,
+  if (smem > 60 * 1024 && hipFuncSetAttribute((const void*)delta_prepare_kernel<TAPS>, hipFuncAttributeMaxDynamicSharedMemorySize,
                                               (int)smem) != hipSuccess) {
     zp_set_error("delta_runs: cannot reserve %zu bytes of LDS", smem);
     return ZP_EHIP;
   }
-  hipLaunchKernelGGL((delta_prepare_kernel<T>), dim3((unsigned)((longest + kBlock - 1) / kBlock), (unsigned)a.heads, (unsigned)a.seg.n),
+  hipLaunchKernelGGL((delta_prepare_kernel<TAPS>), dim3((unsigned)((longest + kBlock - 1) / kBlock), (unsigned)a.heads, (unsigned)a.seg.n),
                      dim3(256), smem, st, ra);
   ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+int launch_runs(const RunArgs& ra, int longest, hipStream_t st) {
+  const zp_delta& a = ra.d;
+  const int rc = a.taps <= 4 ? launch_prepare<4>(ra, longest, st) : launch_prepare<kMaxTaps>(ra, longest, st);
+  if (rc != ZP_OK) return rc;
   switch (a.dk) {
-    case 32: return launch_blocks<T, 2>(ra, st);
-    case 64: return launch_blocks<T, 4>(ra, st);
-    default: return launch_blocks<T, 8>(ra, st);
+    case 32: return launch_blocks<2>(ra, st);
+    case 64: return launch_blocks<4>(ra, st);
+    default: return launch_blocks<8>(ra, st);
   }
 }
 
@@ -340,20 +379,20 @@ extern "C" int zp_delta_runs(const zp_delta* args, int32_t first_row, int32_t lo
   ZP_REQUIRE(a.seg.n >= 0 && a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0 && a.vdim > 0 && a.vdim <= a.dv &&
                  a.seg.num_slots > 0 && a.out_stride >= (int64_t)a.heads * a.dv && first_row >= 0 && longest >= 0 &&
                  first_row <= a.seg.num_rows, "delta_runs: bad dims");
-  ZP_MODEL_DTYPE("delta_runs");
-  if ((a.dk != 32 && a.dk != 64 && a.dk != 128) || a.dv % 32 || a.dv > 128 || a.taps < 1 || a.taps > kMaxTaps || a.heads > 65535 ||
-      a.seg.n > 65535) {
-    zp_set_error("delta_runs: head sizes %d (32, 64, 128) and %d (a multiple of 32, <= 128), %d taps (1 .. %d) unsupported",
+  if (dtype != ZP_BF16 || (a.dk != 32 && a.dk != 64 && a.dk != 128) || a.dv % 32 || a.dv > 128 || a.taps < 1 || a.taps > kMaxTaps || a.heads > 65535 ||
+      a.seg.n > 65535 || a.in_stride % 8 || a.low_stride % 8 || a.out_stride >= (1 << 24) || a.low_stride >= (1 << 24)) {
+    zp_set_error("delta_runs: bfloat16, head sizes %d (32, 64, 128) and %d (a multiple of 32, <= 128), %d taps (1 .. %d) unsupported",
                  a.dk, a.dv, a.taps, kMaxTaps);
     return ZP_EUNSUPPORTED;
   }
   if (a.seg.n == 0 || longest == 0) return ZP_OK;
   ZP_REQUIRE(a.in && a.low && a.filters && a.a_log && a.dt_bias && a.norm && a.state && (a.conv_state || a.taps == 1) && a.out &&
-                 a.seg.rows && a.seg.counts && a.seg.slots && a.seg.starts && aligned16(a.state) && aligned16(workspace),
+                 a.seg.rows && a.seg.counts && a.seg.slots && a.seg.starts && aligned16(a.state) && aligned16(a.in) && aligned16(a.low) &&
+                 aligned16(a.dt_bias) && aligned16(workspace),
              "delta_runs: null or unaligned pointer");
   ZP_REQUIRE(workspace && workspace_bytes >= zp_delta_runs_workspace(a.seg.num_rows - first_row, a.seg.n, a.heads, a.dk, a.dv),
              "delta_runs: workspace too small");
   RunArgs ra = {a, (float*)workspace, first_row};
   ra.d.seg.max_count = longest;               // no segment has more blocks than were prepared
-  return dtype == ZP_BF16 ? launch_runs<BF16>(ra, longest, (hipStream_t)stream) : launch_runs<F32>(ra, longest, (hipStream_t)stream);
+  return launch_runs(ra, longest, (hipStream_t)stream);
 }

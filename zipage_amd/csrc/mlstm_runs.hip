@@ -5,256 +5,309 @@
 //   O = a (Q S) + D V,   n . q_t = a_t (n . q_t) + sum_s D[t, s]
 //   S <- e^{F_15 + m_0 - m_15} S + sum_s e^{F_15 + x_s - m_15} k_s v_s^T,  n likewise with k alone
 //
-// One workgroup per (segment, head) walks the blocks with S in registers; all fp32 (the products q . k on
-// the bf16 matrix cores are exact products of the projections, added up in fp32).
+//   mlstm_gates     gates and the running maximum, one wave per head and sequence
+//   mlstm_prepare   D and the block's factors, for all blocks at once
+//   mlstm_blocks    a head's blocks one after the other, S in registers
+//
+// All fp32: the products q . k on the bf16 matrix cores are exact products of the projections, added up in
+// fp32; those with S run on the fp32 ones.  Projections in bfloat16.
 #include "blocks.h"
 
 namespace {
 
-template <typename T, int KT, int NC>
-__global__ __launch_bounds__(NC == 2 ? 256 : 512) void mlstm_blocks_kernel(zp_mlstm a) {
-  extern __shared__ __align__(16) float lds[];
-  __shared__ float red[2][16 * kBlock];
-  constexpr int dk = 16 * KT, kKs = dk + 4;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
-  const int dv = a.dv;
-  const int h = blockIdx.x % a.heads;
+struct RunArgs {
+  zp_mlstm d;
+  float* aux;    // per block and head: kAux floats
+  float4* scal;  // per token row from row0 on and head: F, x, m, m before the block
+  int row0;
+};
+// D as a left operand (256), then a, write factors, e^{-m}, row sums of D (16 each), the keep factor
+constexpr int kAux = 512, kInter = 256, kWrite = 272, kFloor = 288, kSum = 304, kKeep = 320;
+
+__device__ __forceinline__ float lane_value(float v, int lane) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
+}
+
+// lane i <- lane i - N of its row of 16, or `edge`
+template <int N> __device__ __forceinline__ float row_shr(float v, float edge) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, edge), __builtin_bit_cast(int, v), 0x110 + N,
+                                                               0xf, 0xf, false));
+}
+
+__global__ __launch_bounds__(64) void mlstm_gates_kernel(RunArgs ra) {
+  const zp_mlstm& a = ra.d;
+  const int lane = threadIdx.x, h = blockIdx.x % a.heads;
   const Segment sg = segment_of(a.seg, blockIdx.x / a.heads);
-  if (sg.count <= 0) return;
-  float* const kl = lds;                       // [2][16][kKs] keys of the block
-  float* const nl = kl + 2 * kBlock * kKs;     // [2][dk] normaliser
+  if (sg.count <= 0 || sg.row < ra.row0) return;
+  float* const mstate = a.state + ((int64_t)sg.slot * a.heads + h) * ((int64_t)a.dk * a.dv + a.dk + 4) + (int64_t)a.dk * a.dv + a.dk;
+  float m = sg.start == 0 ? 0.f : *mstate;
+  const float icap = 1.f / a.cap, ib = a.i_bias[h], fb = a.f_bias[h];
+  float zi = 0.f, zf = 0.f;
+  auto fetch = [&](int t0) {
+    const int64_t src = (int64_t)(sg.row + min(t0 + lane, sg.count - 1)) * a.gate_stride + h;
+    zi = a.gates[src];
+    zf = a.gates[src + a.heads];
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < sg.count; t0 += 64) {
+    const int cnt = min(64, sg.count - t0);
+    const float gi = a.cap * tanhf((zi + ib) * icap), x = a.cap * tanhf((zf + fb) * icap);
+    const float gf = fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
+    fetch(t0 + 64);
+    // sums and maxima inside each block of 16 lanes: m_t = F_t + max(m before the block, max_{s <= t} x_s)
+    float F = lane < cnt ? gf : 0.f;
+    F += row_shr<1>(F, 0.f);
+    F += row_shr<2>(F, 0.f);
+    F += row_shr<4>(F, 0.f);
+    F += row_shr<8>(F, 0.f);
+    const float xs = lane < cnt ? gi - F : -INFINITY;
+    float top = xs;
+    top = fmaxf(top, row_shr<1>(top, -INFINITY));
+    top = fmaxf(top, row_shr<2>(top, -INFINITY));
+    top = fmaxf(top, row_shr<4>(top, -INFINITY));
+    top = fmaxf(top, row_shr<8>(top, -INFINITY));
+    float m0 = m;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (lane >> 4 == r) m0 = m;
+      m = lane_value(F, r * 16 + 15) + fmaxf(m, lane_value(top, r * 16 + 15));     // rows behind the end change nothing
+    }
+    const float mine_m = F + fmaxf(m0, top);
+    if (lane < cnt)
+      ra.scal[(int64_t)(sg.row + t0 + lane - ra.row0) * a.heads + h] = make_float4(F, xs, mine_m, m0);
+  }
+  if (lane == 0) *mstate = m;
+}
+
+// A wave per (block, head).
+template <int KT>
+__global__ __launch_bounds__(256) void mlstm_prepare_kernel(RunArgs ra) {
+  const zp_mlstm& a = ra.d;
+  const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4, h = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const Segment sg = segment_of(a.seg, blockIdx.z);
+  const int t0 = blockIdx.x * kBlock;
+  if (t0 >= sg.count || sg.row < ra.row0 || h >= a.heads) return;
+  const int cnt = min(kBlock, sg.count - t0);
+  const int64_t mine = sg.row + t0 + min(l16, cnt - 1);
+  const float4 sc = ra.scal[(mine - ra.row0) * a.heads + h];
+  const uint16_t* const in = (const uint16_t*)a.in + mine * a.in_stride + h * (16 * KT) + g * 8;
+  f32x4 P = {0.f, 0.f, 0.f, 0.f};              // rows s = 4 g + r, column t = l16
+#pragma unroll
+  for (int ks = 0; ks < KT / 2; ++ks)
+    P = mfma_bf16(*(const u32x4*)(in + a.k_at + ks * 32), *(const u32x4*)(in + a.q_at + ks * 32), P);
+  float sum = 0.f;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int s = 4 * g + r;
+    const float xs = __shfl(sc.y, s);
+    P[r] = s <= l16 && s < cnt && l16 < cnt ? P[r] * expf(sc.x + xs - sc.z) : 0.f;
+    sum += P[r];
+  }
+  sum += lane_xor16(sum);
+  sum += lane_xor32(sum);
+  const float F_end = lane_value(sc.x, cnt - 1), m_end = lane_value(sc.z, cnt - 1);
+  float* const aux = ra.aux + (block_slot(ra.row0, sg, blockIdx.z, blockIdx.x) * a.heads + h) * kAux;
+  *(f32x4*)(aux + lane * 4) = P;
+  if (g == 0) {
+    aux[kInter + l16] = expf(sc.x + sc.w - sc.z);
+    aux[kWrite + l16] = l16 < cnt ? expf(F_end + sc.y - m_end) : 0.f;
+    aux[kFloor + l16] = expf(-sc.z);
+    aux[kSum + l16] = sum;
+    if (l16 == 0) aux[kKeep] = expf(F_end + sc.w - m_end);
+  }
+}
+
+// LDS of a stage: Q and K rows, their 16-byte pieces xor-ed with the row so that neither operand order meets
+// bank conflicts; V rows; the block's factors.  The next stage comes in while this one is worked on.
+template <int KT, int NC>
+__global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void mlstm_blocks_kernel(RunArgs ra) {
+  extern __shared__ __align__(16) char lds_raw[];
+  const zp_mlstm& a = ra.d;
+  constexpr int dk = 16 * KT, PR = dk / 8;     // pieces per row
+  const int tid = threadIdx.x, lane = tid & 63, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int dv = a.dv, h = blockIdx.x % a.heads, seg = blockIdx.x / a.heads;
+  const Segment sg = segment_of(a.seg, seg);
+  if (sg.count <= 0 || sg.row < ra.row0) return;
+  float (*const red)[8 * kBlock] = (float (*)[8 * kBlock])(lds_raw + 2 * (2 * kBlock * dk * 2 + kBlock * dv * 2 + kAux * 4));
+  float (*const den)[kBlock] = (float (*)[kBlock])(red + 2);
+  float (*const nl)[dk] = (float (*)[dk])(den + 2);
+  const int v_bytes = kBlock * dv * 2, stage = 2 * kBlock * dk * 2 + v_bytes + kAux * 4;
   float* const state = a.state + ((int64_t)sg.slot * a.heads + h) * ((int64_t)dk * dv + dk + 4);
   float* const nstate = state + (int64_t)dk * dv;
   const bool fresh = sg.start == 0;
   const int col0 = wave * 16 * NC;
   f32x4 S[KT][NC];
   load_state<KT, NC>(S, state, dv, col0, fresh);
-  for (int c = tid; c < dk; c += blockDim.x) nl[c] = fresh ? 0.f : nstate[c];
-  float m = fresh ? 0.f : nstate[dk];
+  for (int c = tid; c < dk; c += blockDim.x) nl[0][c] = fresh ? 0.f : nstate[c];
   float nrm[NC];
 #pragma unroll
   for (int nc = 0; nc < NC; ++nc) nrm[nc] = a.norm[h * dv + col0 + nc * 16 + l16] * a.out_scale;
-  const float icap = 1.f / a.cap, ib = a.i_bias[h], fb = a.f_bias[h];
   const int blocks = (sg.count + kBlock - 1) / kBlock;
-
-  // what a block reads: its token l16's gates and query, keys for the stage, values
-  float zi, zf;
-  f32x4 q[KT];
-  float v[NC][4];
-  constexpr int kPieces = kBlock * dk / 4 / 256 > 0 ? kBlock * dk / 4 / 256 : 1;
-  f32x4 kp[kPieces];
-  auto fetch = [&](int b) {
+  const float* const aux0 = ra.aux + (block_slot(ra.row0, sg, seg, 0) * a.heads + h) * kAux;
+  constexpr int kQK = KT / 2;                  // KBs of Q, and of K
+  const int vkb = dv / 32, loads = 2 * kQK + vkb + 2;
+  auto request = [&](int b) {
+    char* const st = lds_raw + (b & 1) * stage;
     const int cnt = min(kBlock, sg.count - b * kBlock);
-    const int64_t row = sg.row + b * kBlock, mine = row + min(l16, cnt - 1);
-    zi = a.gates[mine * a.gate_stride + h];
-    zf = a.gates[mine * a.gate_stride + a.heads + h];
-#pragma unroll
-    for (int kt = 0; kt < KT; ++kt) q[kt] = load4<T>(a.in, mine * a.in_stride + a.q_at + h * dk + kt * 16 + 4 * g);
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        v[nc][r] = Elem<T>::ld(a.in, (row + min(4 * g + r, cnt - 1)) * a.in_stride + a.v_at + h * dv + col0 + nc * 16 + l16);
-#pragma unroll
-    for (int i = 0; i < kPieces; ++i) {
-      const int p = tid + i * blockDim.x;
-      if (p < kBlock * dk / 4) {
-        const int t = p / (dk / 4), c = (p % (dk / 4)) * 4;
-        kp[i] = load4<T>(a.in, (row + min(t, cnt - 1)) * a.in_stride + a.k_at + h * dk + c);
+    const StageLoads rows((const char*)a.in + (int64_t)(sg.row + b * kBlock) * a.in_stride * 2, cnt * a.in_stride * 2);
+    const StageLoads aux(aux0 + (int64_t)b * a.heads * kAux, kAux * 4);
+    for (int i = wave; i < loads; i += nw) {
+      if (i < 2 * kQK) {
+        const int s = (i < kQK ? i : i - kQK) * 64 + lane, row = s / PR, pc = (s % PR) ^ (row & (PR - 1));
+        rows.ld(st + i * 1024, min(row, cnt - 1) * (int)a.in_stride * 2 + pc * 16, ((i < kQK ? a.q_at : a.k_at) + h * dk) * 2);
+      } else if (i < 2 * kQK + vkb) {
+        const int s = (i - 2 * kQK) * 64 + lane, row = s / (dv / 8), pc = s - row * (dv / 8);
+        rows.ld(st + i * 1024, min(row, cnt - 1) * (int)a.in_stride * 2 + pc * 16, (a.v_at + h * dv) * 2);
+      } else {
+        aux.ld(st + i * 1024, lane * 16, (i - 2 * kQK - vkb) * 1024);
       }
     }
   };
-  auto stage = [&](int buf, int b) {
-    (void)b;
-#pragma unroll
-    for (int i = 0; i < kPieces; ++i) {
-      const int p = tid + i * blockDim.x;
-      if (p < kBlock * dk / 4) *(f32x4*)(kl + (buf * kBlock + p / (dk / 4)) * kKs + (p % (dk / 4)) * 4) = kp[i];
-    }
-    // workgroups of fewer threads than pieces: the rest straight from memory
-    for (int p = tid + kPieces * blockDim.x; p < kBlock * dk / 4; p += blockDim.x) {
-      const int cnt = min(kBlock, sg.count - b * kBlock), t = p / (dk / 4), c = (p % (dk / 4)) * 4;
-      *(f32x4*)(kl + (buf * kBlock + t) * kKs + c) =
-          load4<T>(a.in, (sg.row + b * kBlock + min(t, cnt - 1)) * a.in_stride + a.k_at + h * dk + c);
-    }
-  };
-  fetch(0);
-  stage(0, 0);
-  __syncthreads();
-  for (int b = 0; b < blocks; ++b) {
-    const int cnt = min(kBlock, sg.count - b * kBlock), buf = b & 1;
-    const int64_t row = sg.row + b * kBlock;
-    float gate[NC][4];
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        gate[nc][r] = Elem<T>::ld(a.in, (row + min(4 * g + r, cnt - 1)) * a.in_stride + a.g_at + h * dv + col0 + nc * 16 + l16);
-    // ---- gates of token l16
-    float gi = -INFINITY, gf = 0.f;
-    if (l16 < cnt) {
-      gi = a.cap * tanhf((zi + ib) * icap);
-      const float x = a.cap * tanhf((zf + fb) * icap);
-      gf = fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
-    }
-    const float m0 = m;
-    float F = 0.f, F_all = 0.f, mt = 0.f;
-#pragma unroll
-    for (int t = 0; t < kBlock; ++t) {
-      const float ft = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, gf), t));
-      const float it = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, gi), t));
-      m = fmaxf(ft + m, it);
-      F_all += ft;
-      if (l16 == t) { F = F_all; mt = m; }
-    }
-    const float x = gi - F;                                   // -inf behind the last token
-    const float inter = expf(F + m0 - mt), keep = expf(F_all + m0 - m), wr = expf(F_all + x - m), floor_ = expf(-mt);
-    // ---- q . k and its weights: rows s = 4 g + r, column t = l16
-    f32x4 P = {0.f, 0.f, 0.f, 0.f};
-    const float* const kb = kl + buf * kBlock * kKs;
-    if constexpr (T::bytes == 2) {
-      // the same bf16 values as in memory: 32 channels per product, in the order lane group g holds them
-#pragma unroll
-      for (int kt = 0; kt < KT; kt += 2) {
-        const f32x4 k0 = *(const f32x4*)(kb + l16 * kKs + kt * 16 + 4 * g), k1 = *(const f32x4*)(kb + l16 * kKs + kt * 16 + 16 + 4 * g);
-        const u32x4 kf = {pack_bf16(k0[0], k0[1]), pack_bf16(k0[2], k0[3]), pack_bf16(k1[0], k1[1]), pack_bf16(k1[2], k1[3])};
-        const u32x4 qf = {pack_bf16(q[kt][0], q[kt][1]), pack_bf16(q[kt][2], q[kt][3]), pack_bf16(q[kt + 1][0], q[kt + 1][1]),
-                          pack_bf16(q[kt + 1][2], q[kt + 1][3])};
-        P = mfma_bf16(kf, qf, P);
-      }
-    } else {
-#pragma unroll
-      for (int kt = 0; kt < KT; ++kt) {
-        const f32x4 k0 = *(const f32x4*)(kb + l16 * kKs + kt * 16 + 4 * g);
-        mfma_f32_16(k0, q[kt], P);
-      }
-    }
-    float nq = 0.f;
-    const float* const nb = nl + buf * dk;
-#pragma unroll
-    for (int kt = 0; kt < KT; ++kt) {
-      const f32x4 n4 = *(const f32x4*)(nb + kt * 16 + 4 * g);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) nq = fmaf(q[kt][j], n4[j], nq);
-    }
-    nq *= inter;
-    float wrow[4], irow[4];
+  f32x4 O[NC];
+  uint16_t gate[NC][4];
+  const float inv_v = 1.f / (float)a.vdim;
+  const int out_at = (4 * g * (int)a.out_stride + h * dv + col0 + l16) * 2;
+  const int gate_at = (4 * g * (int)a.in_stride + a.g_at + h * dv + col0 + l16) * 2;
+  auto finish = [&](int b) {                   // rows of block b, whose squares and denominators are in LDS
+    f32x4 ss = block_squares_total(red[b & 1], nw);
+    const f32x4 dn = *(const f32x4*)(den[b & 1] + 4 * g);
+    const int cnt = min(kBlock, sg.count - b * kBlock);
+    const BlockRows out(a.out, sg.row + b * kBlock, cnt, a.out_stride);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int s = 4 * g + r;
-      const float xs = __shfl(x, s);
-      wrow[r] = __shfl(wr, s);
-      irow[r] = __shfl(inter, s);
-      P[r] = s <= l16 && s < cnt ? P[r] * expf(F + xs - mt) : 0.f;
-      nq += P[r];
+      const float f = a.q_scale * __builtin_amdgcn_rcpf(dn[r]), rs = f * __builtin_amdgcn_rsqf(ss[r] * f * f * inv_v + a.eps);
+#pragma unroll
+      for (int nc = 0; nc < NC; ++nc)
+        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, O[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
     }
-    nq += lane_xor16(nq);
-    nq += lane_xor32(nq);
-    const float den = fmaxf(fabsf(nq) * a.q_scale, floor_) + 1e-6f;
-    const float unden = 1.f / den;
+  };
+  auto half = [](uint16_t v) { return bf16_bits_to_float(v); };
+  request(0);
+  __builtin_amdgcn_s_waitcnt(0);               // the state is there: the loop's first use of it must not wait in every pass
+#pragma unroll 1
+  for (int b = 0; b < blocks; ++b) {
+    wait_and_meet();
+    if (b + 1 < blocks) request(b + 1);
+    if (b > 0) finish(b - 1);
+    const int cnt = min(kBlock, sg.count - b * kBlock);
+    const BlockRows gp(a.in, sg.row + b * kBlock, cnt, a.in_stride);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int nc = 0; nc < NC; ++nc) gate[nc][r] = gp.ld(gate_at + r * (int)a.in_stride * 2, nc * 16);
+    const char* const st = lds_raw + (b & 1) * stage;
+    const char* const ks = st + kBlock * dk * 2;
+    const uint16_t* const vs = (const uint16_t*)(ks + kBlock * dk * 2);
+    const float* const aux = (const float*)((const char*)vs + v_bytes);
     // ---- read-outs
-    f32x4 O[NC];
 #pragma unroll
     for (int nc = 0; nc < NC; ++nc) O[nc] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int kt = 0; kt < KT; ++kt)
+    for (int kt = 0; kt < KT; ++kt) {
+      const f32x4 q = load4<BF16>(st + l16 * dk * 2 + (((2 * kt + (g >> 1)) ^ (l16 & (PR - 1))) * 16) + (g & 1) * 8, 0);
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
-        for (int nc = 0; nc < NC; ++nc) O[nc] = mfma_f32_step(q[kt][j], S[kt][nc][j], O[nc]);
+        for (int nc = 0; nc < NC; ++nc) O[nc] = mfma_f32_step(q[j], S[kt][nc][j], O[nc]);
+    }
+    const f32x4 P = *(const f32x4*)(aux + lane * 4), inter = *(const f32x4*)(aux + kInter + 4 * g), wr = *(const f32x4*)(aux + kWrite + 4 * g);
+    const float keep = aux[kKeep];
+    f32x4 v[NC];
 #pragma unroll
     for (int nc = 0; nc < NC; ++nc) {
-      const f32x4 vt = {v[nc][0], v[nc][1], v[nc][2], v[nc][3]};
-#pragma unroll
-      for (int r = 0; r < 4; ++r) O[nc][r] *= irow[r];
-      mfma_f32_16(P, vt, O[nc]);
+      v[nc] = read_columns((const char*)(vs + (4 * g + (l16 >> 2)) * dv + col0 + nc * 16 + (l16 & 3) * 4));
+      O[nc] *= inter;
+      mfma_f32_16(P, v[nc], O[nc]);
+      v[nc] *= wr;
     }
-    // ---- state and normaliser behind the block
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) v[nc][r] *= wrow[r];
-    f32x4 vw[NC];
-#pragma unroll
-    for (int nc = 0; nc < NC; ++nc) vw[nc] = f32x4{v[nc][0], v[nc][1], v[nc][2], v[nc][3]};
-    fetch(min(b + 1, blocks - 1));
+    // ---- the state behind the block
+    const int kr = 4 * g + (l16 >> 2), kz = ((l16 & 3) >> 1) ^ (kr & (PR - 1));
+    const char* const krow = ks + kr * dk * 2 + (l16 & 1) * 8;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
-      f32x4 kT;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) kT[j] = kb[(4 * g + j) * kKs + kt * 16 + l16];
+      const f32x4 kT = read_columns(krow + (((2 * kt) ^ kz) * 16));
 #pragma unroll
       for (int nc = 0; nc < NC; ++nc) {
         S[kt][nc] *= keep;
-        mfma_f32_16(kT, vw[nc], S[kt][nc]);
+        mfma_f32_16(kT, v[nc], S[kt][nc]);
       }
+    }
+    block_squares<NC>(O, red[b & 1]);
+    // ---- the normaliser: 16 lanes a token
+    const float* const n = nl[b & 1];
+    for (int t = tid >> 4; t < kBlock; t += blockDim.x >> 4) {
+      float d = 0.f;
+      if (l16 < PR) {
+        float q[8];
+        Vec8<BF16>::ld(st + t * dk * 2 + ((l16 ^ (t & (PR - 1))) * 16), 0, q);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) d = fmaf(q[i], n[l16 * 8 + i], d);
+      }
+      d = row16_sum(d);
+      if (l16 == 0) den[b & 1][t] = fmaxf(fabsf(fmaf(aux[kInter + t], d, aux[kSum + t])) * a.q_scale, aux[kFloor + t]) + 1e-6f;
     }
     for (int c = tid; c < dk; c += blockDim.x) {
-      float n = nb[c] * keep;
+      float x = n[c] * keep;
 #pragma unroll
       for (int s = 0; s < kBlock; ++s)
-        n = fmaf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, wr), s)), kb[s * kKs + c], n);
-      nl[(buf ^ 1) * dk + c] = n;
-    }
-    stage(buf ^ 1, min(b + 1, blocks - 1));
-    // ---- norm, gate, store
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float f = __shfl(unden, 4 * g + r) * a.q_scale;
-#pragma unroll
-      for (int nc = 0; nc < NC; ++nc) O[nc][r] *= f;
-    }
-    block_squares<NC>(O, red[buf]);
-    __syncthreads();
-    const f32x4 ss = block_squares_total(red[buf], nw);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float rs = 1.f / sqrtf(ss[r] / (float)a.vdim + a.eps);
-      if (4 * g + r < cnt) {
-#pragma unroll
-        for (int nc = 0; nc < NC; ++nc)
-          Elem<T>::st(a.out, (row + 4 * g + r) * a.out_stride + h * dv + col0 + nc * 16 + l16,
-                      O[nc][r] * rs * nrm[nc] * sigmoid_f(gate[nc][r]));
-      }
+        x = fmaf(aux[kWrite + s], half(*(const uint16_t*)(ks + s * dk * 2 + (((c >> 3) ^ (s & (PR - 1))) * 16) + (c & 7) * 2)), x);
+      nl[(b + 1) & 1][c] = x;
     }
   }
+  wait_and_meet();
+  finish(blocks - 1);
   store_state<KT, NC>(S, state, dv, col0);
-  for (int c = tid; c < dk; c += blockDim.x) nstate[c] = nl[(blocks & 1) * dk + c];
-  if (tid == 0) nstate[dk] = m;
+  for (int c = tid; c < dk; c += blockDim.x) nstate[c] = nl[blocks & 1][c];
 }
 
-template <typename T, int KT> int launch_blocks(const zp_mlstm& a, hipStream_t st) {
+template <int KT> int launch_runs(const RunArgs& ra, int longest, hipStream_t st) {
+  const zp_mlstm& a = ra.d;
   const unsigned grid = (unsigned)((int64_t)a.seg.n * a.heads);
-  const size_t smem = sizeof(float) * (2 * kBlock * (16 * KT + 4) + 2 * 16 * KT);
-  const bool narrow = (int64_t)grid * (a.dv / 32) < 1024;      // half the columns per wave, twice the waves
-  if (narrow) hipLaunchKernelGGL((mlstm_blocks_kernel<T, KT, 1>), dim3(grid), dim3(a.dv * 4), smem, st, a);
-  else hipLaunchKernelGGL((mlstm_blocks_kernel<T, KT, 2>), dim3(grid), dim3(a.dv * 2), smem, st, a);
+  hipLaunchKernelGGL(mlstm_gates_kernel, dim3(grid), dim3(64), 0, st, ra);
+  hipLaunchKernelGGL((mlstm_prepare_kernel<KT>), dim3((unsigned)((longest + kBlock - 1) / kBlock), (unsigned)((a.heads + 3) / 4), (unsigned)a.seg.n),
+                     dim3(256), 0, st, ra);
+  ZP_LAUNCH_CHECK();
+  const size_t smem = 2 * (size_t)(2 * kBlock * a.dk * 2 + kBlock * a.dv * 2 + kAux * 4) + 2 * 4 * (8 * kBlock + kBlock + a.dk);
+  const bool narrow = a.dv % 64 != 0 && a.dv < 128;            // few columns: more, smaller waves
+  if (narrow) hipLaunchKernelGGL((mlstm_blocks_kernel<KT, 1>), dim3(grid), dim3(a.dv * 4), smem, st, ra);
+  else hipLaunchKernelGGL((mlstm_blocks_kernel<KT, 2>), dim3(grid), dim3(a.dv * 2), smem, st, ra);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }
 
 }  // namespace
 
-extern "C" int zp_mlstm_runs(const zp_mlstm* args, int32_t dtype, void* stream) {
+extern "C" int64_t zp_mlstm_runs_workspace(int32_t rows, int32_t segments, int32_t heads) {
+  if (rows < 0 || segments < 0 || heads <= 0) return -1;
+  return (((int64_t)rows / kBlock + segments) * kAux + (int64_t)rows * 4) * heads * 4;
+}
+
+extern "C" int zp_mlstm_runs(const zp_mlstm* args, int32_t first_row, int32_t longest, void* workspace,
+                             int64_t workspace_bytes, int32_t dtype, void* stream) {
   ZP_REQUIRE(args, "mlstm_runs: null arguments");
   const zp_mlstm& a = *args;
   ZP_REQUIRE(a.seg.n >= 0 && a.heads > 0 && a.vdim > 0 && a.vdim <= a.dv && a.cap > 0.f && a.seg.num_slots > 0 &&
-                 a.gate_stride >= 2 * a.heads && a.out_stride >= (int64_t)a.heads * a.dv, "mlstm_runs: bad dims");
-  ZP_MODEL_DTYPE("mlstm_runs");
-  if ((a.dk != 32 && a.dk != 64 && a.dk != 128) || a.dv % 32 || a.dv > 128 || a.in_stride % 8 || a.q_at % 8 || a.k_at % 8) {
-    zp_set_error("mlstm_runs: head sizes %d (32, 64, 128) and %d (a multiple of 32, <= 128) unsupported", a.dk, a.dv);
+                 a.gate_stride >= 2 * a.heads && a.out_stride >= (int64_t)a.heads * a.dv && first_row >= 0 && longest >= 0 &&
+                 first_row <= a.seg.num_rows, "mlstm_runs: bad dims");
+  if (dtype != ZP_BF16 || (a.dk != 32 && a.dk != 64 && a.dk != 128) || a.dv % 32 || a.dv > 128 || a.in_stride % 8 || a.q_at % 8 ||
+      a.k_at % 8 || a.v_at % 8 || a.in_stride >= (1 << 24) || a.out_stride >= (1 << 24) || a.heads > 65535 || a.seg.n > 65535) {
+    zp_set_error("mlstm_runs: bfloat16, head sizes %d (32, 64, 128) and %d (a multiple of 32, <= 128) unsupported", a.dk, a.dv);
     return ZP_EUNSUPPORTED;
   }
-  if (a.seg.n == 0) return ZP_OK;
+  if (a.seg.n == 0 || longest == 0) return ZP_OK;
   ZP_REQUIRE(a.in && a.gates && a.i_bias && a.f_bias && a.norm && a.state && a.out && a.seg.rows && a.seg.counts &&
-                 a.seg.slots && a.seg.starts && aligned16(a.in) && aligned16(a.state), "mlstm_runs: null or unaligned pointer");
+                 a.seg.slots && a.seg.starts && aligned16(a.in) && aligned16(a.state) && aligned16(workspace),
+             "mlstm_runs: null or unaligned pointer");
+  ZP_REQUIRE(workspace && workspace_bytes >= zp_mlstm_runs_workspace(a.seg.num_rows - first_row, a.seg.n, a.heads),
+             "mlstm_runs: workspace too small");
+  RunArgs ra = {a, (float*)workspace, nullptr, first_row};
+  ra.scal = (float4*)(ra.aux + ((int64_t)(a.seg.num_rows - first_row) / kBlock + a.seg.n) * a.heads * kAux);
+  ra.d.seg.max_count = longest;               // no segment has more blocks than were prepared
   hipStream_t st = (hipStream_t)stream;
-#define ZP_MLSTM(T)                                    \
-  switch (a.dk) {                                      \
-    case 32: return launch_blocks<T, 2>(a, st);        \
-    case 64: return launch_blocks<T, 4>(a, st);        \
-    default: return launch_blocks<T, 8>(a, st);        \
+  switch (a.dk) {
+    case 32: return launch_runs<2>(ra, longest, st);
+    case 64: return launch_runs<4>(ra, longest, st);
+    default: return launch_runs<8>(ra, longest, st);
   }
-  if (dtype == ZP_BF16) { ZP_MLSTM(BF16); } else { ZP_MLSTM(F32); }
-#undef ZP_MLSTM
 }

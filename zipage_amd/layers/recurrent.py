@@ -83,7 +83,8 @@ class MatrixMemory:
         H, D, V = self.heads, self.dim_p, self.vdim_p
         gates = small_linear(h, self.gates)
         assert proj.stride(1) == out.stride(1) == 1 and proj.dtype == out.dtype and state.is_contiguous()
-        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run)):
+        tag, stream = _lib.dtype_tag(proj), _lib.stream_ptr(proj)
+        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run and proj.dtype == torch.bfloat16)):
             if segments is None:
                 continue
             args = _lib.MlstmArgs(
@@ -91,8 +92,14 @@ class MatrixMemory:
                 _lib.dev_ptr(self.i_bias), _lib.dev_ptr(self.f_bias), _lib.dev_ptr(self.norm), _lib.dev_ptr(state),
                 _lib.dev_ptr(out), proj.stride(0), gates.stride(0), out.stride(0), H, D, V, self.vdim, 0, H * D,
                 2 * H * D, 2 * H * D + H * V, self.gate_cap, self.dim ** -0.5, self.eps, self.out_scale)
-            _lib.call_models("zp_mlstm_runs" if runs else "zp_mlstm_scan", ctypes.byref(args), _lib.dtype_tag(proj),
-                             _lib.stream_ptr(proj))
+            if not runs:
+                _lib.call_models("zp_mlstm_scan", ctypes.byref(args), tag, stream)
+                continue
+            size = _lib.load_models("hybrid").zp_mlstm_runs_workspace(h.shape[0] - segments.first_row,
+                                                                      segments.counts.numel(), H)
+            ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
+            _lib.call_models("zp_mlstm_runs", ctypes.byref(args), segments.first_row, segments.longest, _lib.dev_ptr(ws),
+                             size, tag, stream)
 
 
 class ChannelDelta:
@@ -162,7 +169,7 @@ class ChannelDelta:
         assert proj.stride(1) == out.stride(1) == 1 and proj.dtype == out.dtype == tail.dtype and S.is_contiguous()
         low = F.linear(proj[:, self.low_at:self.low_at + self.low_rank], self.low)
         tag, stream = _lib.dtype_tag(proj), _lib.stream_ptr(proj)
-        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run)):
+        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run and proj.dtype == torch.bfloat16)):
             if segments is None:
                 continue
             args = _lib.DeltaArgs(
