@@ -43,10 +43,10 @@ template <int KT, int NC> __device__ __forceinline__ void store_state(const f32x
       for (int r = 0; r < 4; ++r) state[(int64_t)(16 * kt + 4 * g + r) * dv + col0 + nc * 16 + l16] = S[kt][nc][r];
 }
 
-// Sum of squares of each of the block's 16 tokens over the wave's columns; lane l16 == 0 of group g ends
-// with tokens 4 g .. 4 g + 3 in `red` (16 floats per wave).
-template <int NC> __device__ __forceinline__ void block_squares(const f32x4 (&o)[NC], float* red) {
-  const int l16 = threadIdx.x & 15, g = (threadIdx.x & 63) >> 4, wave = threadIdx.x >> 6;
+// Sum of squares of each of the block's 16 tokens over the wave's columns; lane l16 == 0 of group g leaves
+// tokens 4 g .. 4 g + 3 in `red` (16 floats per wave).
+template <int NC> __device__ __forceinline__ void block_squares(const f32x4 (&o)[NC], float* red, int wave) {
+  const int l16 = threadIdx.x & 15, g = (threadIdx.x & 63) >> 4;
   f32x4 ss = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int nc = 0; nc < NC; ++nc) ss += o[nc] * o[nc];
@@ -54,10 +54,11 @@ template <int NC> __device__ __forceinline__ void block_squares(const f32x4 (&o)
   for (int r = 0; r < 4; ++r) ss[r] = row16_sum(ss[r]);
   if (l16 == 0) *(f32x4*)(red + wave * kBlock + 4 * g) = ss;
 }
-__device__ __forceinline__ f32x4 block_squares_total(const float* red, int nw) {
+template <int NW> __device__ __forceinline__ f32x4 block_squares_total(const float* red) {
   const int g = (threadIdx.x & 63) >> 4;
   f32x4 ss = {0.f, 0.f, 0.f, 0.f};
-  for (int w = 0; w < nw; ++w) ss += *(const f32x4*)(red + w * kBlock + 4 * g);
+#pragma unroll
+  for (int w = 0; w < NW; ++w) ss += *(const f32x4*)(red + w * kBlock + 4 * g);
   return ss;
 }
 

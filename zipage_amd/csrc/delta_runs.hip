@@ -22,7 +22,7 @@ struct RunArgs {
 };
 
 // [-W | G q] and the keys as left operands, U0 as a result tile, P, the block's decays; whole KBs
-__host__ __device__ inline int block_floats(int dk, int dv) {
+__host__ __device__ inline constexpr int block_floats(int dk, int dv) {
   return (kBlock * (3 * dk + dv) + kBlock * kBlock + dk + 255) / 256 * 256;
 }
 
@@ -222,14 +222,14 @@ __global__ __launch_bounds__(256, 3) void delta_prepare_kernel(RunArgs ra) {
 
 // A head's blocks, one after the other: a block's operands come straight into LDS while the block before it is
 // worked on; its rows are normed and stored behind the next meeting of the waves, which the norm needs too.
-template <int KT, int NC>
-__global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(RunArgs ra) {
+template <int KT, int NW>
+__global__ __launch_bounds__(64 * NW, 2) void delta_blocks_kernel(RunArgs ra) {
   extern __shared__ __align__(16) float lds[];
   const zp_delta& a = ra.d;
-  const int tid = threadIdx.x, lane = tid & 63, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
+  constexpr int NC = 2, dk = 16 * KT, dv = 32 * NW, size = block_floats(dk, dv);
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int dk = 16 * KT, dv = a.dv, size = block_floats(dk, dv);
-  float* const red = lds + 2 * size;           // [2][8 * 16]
+  float* const red = lds + 2 * size;           // [2][NW * 16]
   const int h = blockIdx.x % a.heads, seg = blockIdx.x / a.heads;
   const Segment sg = segment_of(a.seg, seg);
   if (sg.count <= 0 || sg.row < ra.row0) return;
@@ -244,25 +244,30 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(Ru
   const float* const base = ra.ws + (block_slot(ra.row0, sg, seg, 0) * a.heads + h) * size;
   const int64_t stride = (int64_t)a.heads * size;
   const int blocks = (sg.count + kBlock - 1) / kBlock;
-  auto request = [&](int b) {
-    const StageLoads from(base + b * stride, size * 4);
-    for (int i = wave; i < size / 256; i += nw) from.ld(lds + (b & 1) * size + i * 256, lane * 16, i * 1024);
+  auto request = [&](int b) {                  // a block behind the last: nothing is read
+    const StageLoads from(base + b * stride, b < blocks ? size * 4 : 0);
+#pragma unroll
+    for (int u = 0; u < (size / 256 + NW - 1) / NW; ++u) {
+      const int i = min(wave + u * NW, size / 256 - 1);            // the last may come twice
+      from.ld(lds + (b & 1) * size + i * 256, lane * 16, i * 1024);
+    }
   };
   f32x4 O[NC];
   uint16_t gate[NC][4];
   const float inv_v = 1.f / (float)a.vdim;
   const int out_at = (4 * g * (int)a.out_stride + h * dv + col0 + l16) * 2;
   const int low_at = (4 * g * (int)a.low_stride + a.g_at + h * dv + col0 + l16) * 2;
-  auto finish = [&](int b) {                   // rows of block b, whose squares are in red
-    const f32x4 ss = block_squares_total(red + (b & 1) * 8 * kBlock, nw);
-    const int cnt = min(kBlock, sg.count - b * kBlock);
+  f32x4 done[NC];
+  auto finish = [&](int b) {                   // rows of block b, whose squares are in red; none of block -1
+    const f32x4 ss = block_squares_total<NW>(red + (b & 1) * NW * kBlock);
+    const int cnt = b < 0 ? 0 : min(kBlock, sg.count - b * kBlock);
     const BlockRows out(a.out, sg.row + b * kBlock, cnt, a.out_stride);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const float rs = __builtin_amdgcn_rsqf(ss[r] * inv_v + a.eps);
 #pragma unroll
       for (int nc = 0; nc < NC; ++nc)
-        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, O[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
+        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, done[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
     }
   };
   request(0);
@@ -270,8 +275,8 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(Ru
 #pragma unroll 1
   for (int b = 0; b < blocks; ++b) {
     wait_and_meet();
-    if (b + 1 < blocks) request(b + 1);
-    if (b > 0) finish(b - 1);
+    request(b + 1);
+    finish(b - 1);
     const int cnt = min(kBlock, sg.count - b * kBlock);
     const BlockRows low(a.low, sg.row + b * kBlock, cnt, a.low_stride);
 #pragma unroll
@@ -309,7 +314,9 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(Ru
     }
 #pragma unroll
     for (int nc = 0; nc < NC; ++nc) mfma_f32_16(P, U[nc], O[nc]);
-    block_squares<NC>(O, red + (b & 1) * 8 * kBlock);
+    block_squares<NC>(O, red + (b & 1) * NW * kBlock, wave);
+#pragma unroll
+    for (int nc = 0; nc < NC; ++nc) done[nc] = O[nc];
   }
   wait_and_meet();
   finish(blocks - 1);
@@ -324,20 +331,24 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void delta_blocks_kernel(Ru
   }
 }
 
-template <int KT> int launch_blocks(const RunArgs& ra, hipStream_t st) {
-  const zp_delta& a = ra.d;
-  const unsigned grid = (unsigned)((int64_t)a.seg.n * a.heads);
-  const bool narrow = a.dv % 64 != 0 && a.dv < 128;          // few columns: more, smaller waves
-  const int smem = (2 * block_floats(a.dk, a.dv) + 2 * 8 * kBlock) * 4;
-  const void* fn = narrow ? (const void*)delta_blocks_kernel<KT, 1> : (const void*)delta_blocks_kernel<KT, 2>;
-  if (smem > 60 * 1024 && hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
+template <int KT, int NW> int launch_blocks(const RunArgs& ra, hipStream_t st) {
+  constexpr int smem = (2 * block_floats(16 * KT, 32 * NW) + 2 * NW * kBlock) * 4;
+  if (smem > 60 * 1024 && hipFuncSetAttribute((const void*)delta_blocks_kernel<KT, NW>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                              smem) != hipSuccess) {
     zp_set_error("delta_runs: cannot reserve %d bytes of LDS", smem);
     return ZP_EHIP;
   }
-  if (narrow) hipLaunchKernelGGL((delta_blocks_kernel<KT, 1>), dim3(grid), dim3(a.dv * 4), smem, st, ra);
-  else hipLaunchKernelGGL((delta_blocks_kernel<KT, 2>), dim3(grid), dim3(a.dv * 2), smem, st, ra);
+  hipLaunchKernelGGL((delta_blocks_kernel<KT, NW>), dim3((unsigned)((int64_t)ra.d.seg.n * ra.d.heads)), dim3(64 * NW), smem, st, ra);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
+}
+template <int KT> int launch_blocks(const RunArgs& ra, hipStream_t st) {
+  switch (ra.d.dv / 32) {
+    case 1: return launch_blocks<KT, 1>(ra, st);
+    case 2: return launch_blocks<KT, 2>(ra, st);
+    case 3: return launch_blocks<KT, 3>(ra, st);
+    default: return launch_blocks<KT, 4>(ra, st);
+  }
 }
 
 template <int TAPS> int launch_prepare(const RunArgs& ra, int longest, hipStream_t st) {

@@ -12,6 +12,7 @@
 // All fp32: the products q . k on the bf16 matrix cores are exact products of the projections, added up in
 // fp32; those with S run on the fp32 ones.  Projections in bfloat16.
 #include "blocks.h"
+#include <type_traits>
 
 namespace {
 
@@ -119,20 +120,20 @@ __global__ __launch_bounds__(256) void mlstm_prepare_kernel(RunArgs ra) {
 
 // LDS of a stage: Q and K rows, their 16-byte pieces xor-ed with the row so that neither operand order meets
 // bank conflicts; V rows; the block's factors.  The next stage comes in while this one is worked on.
-template <int KT, int NC>
-__global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void mlstm_blocks_kernel(RunArgs ra) {
+template <int KT, int NW>
+__global__ __launch_bounds__(64 * NW, 2) void mlstm_blocks_kernel(RunArgs ra) {
   extern __shared__ __align__(16) char lds_raw[];
   const zp_mlstm& a = ra.d;
-  constexpr int dk = 16 * KT, PR = dk / 8;     // pieces per row
-  const int tid = threadIdx.x, lane = tid & 63, nw = blockDim.x >> 6, l16 = lane & 15, g = lane >> 4;
+  constexpr int NC = 2, dk = 16 * KT, dv = 32 * NW, PR = dk / 8;     // PR: pieces per row of Q and K
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int dv = a.dv, h = blockIdx.x % a.heads, seg = blockIdx.x / a.heads;
+  const int h = blockIdx.x % a.heads, seg = blockIdx.x / a.heads;
   const Segment sg = segment_of(a.seg, seg);
   if (sg.count <= 0 || sg.row < ra.row0) return;
-  float (*const red)[8 * kBlock] = (float (*)[8 * kBlock])(lds_raw + 2 * (2 * kBlock * dk * 2 + kBlock * dv * 2 + kAux * 4));
+  constexpr int v_bytes = kBlock * dv * 2, stage = 2 * kBlock * dk * 2 + v_bytes + kAux * 4;
+  float (*const red)[NW * kBlock] = (float (*)[NW * kBlock])(lds_raw + 2 * stage);
   float (*const den)[kBlock] = (float (*)[kBlock])(red + 2);
   float (*const nl)[dk] = (float (*)[dk])(den + 2);
-  const int v_bytes = kBlock * dv * 2, stage = 2 * kBlock * dk * 2 + v_bytes + kAux * 4;
   float* const state = a.state + ((int64_t)sg.slot * a.heads + h) * ((int64_t)dk * dv + dk + 4);
   float* const nstate = state + (int64_t)dk * dv;
   const bool fresh = sg.start == 0;
@@ -146,50 +147,54 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void mlstm_blocks_kernel(Ru
   const int blocks = (sg.count + kBlock - 1) / kBlock;
   const float* const aux0 = ra.aux + (block_slot(ra.row0, sg, seg, 0) * a.heads + h) * kAux;
   constexpr int kQK = KT / 2;                  // KBs of Q, and of K
-  const int vkb = dv / 32, loads = 2 * kQK + vkb + 2;
-  auto request = [&](int b) {
-    char* const st = lds_raw + (b & 1) * stage;
-    const int cnt = min(kBlock, sg.count - b * kBlock);
-    const StageLoads rows((const char*)a.in + (int64_t)(sg.row + b * kBlock) * a.in_stride * 2, cnt * a.in_stride * 2);
-    const StageLoads aux(aux0 + (int64_t)b * a.heads * kAux, kAux * 4);
-    for (int i = wave; i < loads; i += nw) {
-      if (i < 2 * kQK) {
-        const int s = (i < kQK ? i : i - kQK) * 64 + lane, row = s / PR, pc = (s % PR) ^ (row & (PR - 1));
-        rows.ld(st + i * 1024, min(row, cnt - 1) * (int)a.in_stride * 2 + pc * 16, ((i < kQK ? a.q_at : a.k_at) + h * dk) * 2);
-      } else if (i < 2 * kQK + vkb) {
-        const int s = (i - 2 * kQK) * 64 + lane, row = s / (dv / 8), pc = s - row * (dv / 8);
-        rows.ld(st + i * 1024, min(row, cnt - 1) * (int)a.in_stride * 2 + pc * 16, (a.v_at + h * dv) * 2);
-      } else {
-        aux.ld(st + i * 1024, lane * 16, (i - 2 * kQK - vkb) * 1024);
-      }
-    }
+  // a share of `kbs` KBs; the last may come twice
+  auto share = [&](auto kbs, auto ld) {
+#pragma unroll
+    for (int u = 0; u < (kbs.value + NW - 1) / NW; ++u) ld(min(wave + u * NW, kbs.value - 1));
   };
+  auto request = [&](int b) {                  // of a block behind the last nothing is read
+    char* const st = lds_raw + (b & 1) * stage;
+    const int cnt = b < blocks ? min(kBlock, sg.count - b * kBlock) : 0;
+    const StageLoads rows((const char*)a.in + (int64_t)(sg.row + b * kBlock) * a.in_stride * 2, cnt * a.in_stride * 2);
+    const StageLoads aux(aux0 + (int64_t)b * a.heads * kAux, cnt > 0 ? kAux * 4 : 0);
+    share(std::integral_constant<int, kQK>(), [&](int i) {
+      const int s = i * 64 + lane, row = s / PR, pc = (s % PR) ^ (row & (PR - 1));
+      const int at = max(min(row, cnt - 1), 0) * (int)a.in_stride * 2 + pc * 16;
+      rows.ld(st + i * 1024, at, (a.q_at + h * dk) * 2);
+      rows.ld(st + (kQK + i) * 1024, at, (a.k_at + h * dk) * 2);
+    });
+    share(std::integral_constant<int, NW>(), [&](int i) {
+      const int s = i * 64 + lane, row = s / (dv / 8), pc = s - row * (dv / 8);
+      rows.ld(st + (2 * kQK + i) * 1024, max(min(row, cnt - 1), 0) * (int)a.in_stride * 2 + pc * 16, (a.v_at + h * dv) * 2);
+    });
+    share(std::integral_constant<int, 2>(), [&](int i) { aux.ld(st + (2 * kQK + NW + i) * 1024, lane * 16, i * 1024); });
+  };
+  f32x4 done[NC];
   f32x4 O[NC];
   uint16_t gate[NC][4];
   const float inv_v = 1.f / (float)a.vdim;
   const int out_at = (4 * g * (int)a.out_stride + h * dv + col0 + l16) * 2;
   const int gate_at = (4 * g * (int)a.in_stride + a.g_at + h * dv + col0 + l16) * 2;
-  auto finish = [&](int b) {                   // rows of block b, whose squares and denominators are in LDS
-    f32x4 ss = block_squares_total(red[b & 1], nw);
+  auto finish = [&](int b) {                   // rows of block b, whose squares and denominators are in LDS; none of block -1
+    const f32x4 ss = block_squares_total<NW>(red[b & 1]);
     const f32x4 dn = *(const f32x4*)(den[b & 1] + 4 * g);
-    const int cnt = min(kBlock, sg.count - b * kBlock);
+    const int cnt = b < 0 ? 0 : min(kBlock, sg.count - b * kBlock);
     const BlockRows out(a.out, sg.row + b * kBlock, cnt, a.out_stride);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const float f = a.q_scale * __builtin_amdgcn_rcpf(dn[r]), rs = f * __builtin_amdgcn_rsqf(ss[r] * f * f * inv_v + a.eps);
 #pragma unroll
       for (int nc = 0; nc < NC; ++nc)
-        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, O[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
+        out.st(out_at + r * (int)a.out_stride * 2, nc * 16, done[nc][r] * rs * nrm[nc] * fast_sigmoid(bf16_bits_to_float(gate[nc][r])));
     }
   };
-  auto half = [](uint16_t v) { return bf16_bits_to_float(v); };
   request(0);
   __builtin_amdgcn_s_waitcnt(0);               // the state is there: the loop's first use of it must not wait in every pass
 #pragma unroll 1
   for (int b = 0; b < blocks; ++b) {
     wait_and_meet();
-    if (b + 1 < blocks) request(b + 1);
-    if (b > 0) finish(b - 1);
+    request(b + 1);
+    finish(b - 1);
     const int cnt = min(kBlock, sg.count - b * kBlock);
     const BlockRows gp(a.in, sg.row + b * kBlock, cnt, a.in_stride);
 #pragma unroll
@@ -233,32 +238,49 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512, 2) void mlstm_blocks_kernel(Ru
         mfma_f32_16(kT, v[nc], S[kt][nc]);
       }
     }
-    block_squares<NC>(O, red[b & 1]);
+    block_squares<NC>(O, red[b & 1], wave);
+#pragma unroll
+    for (int nc = 0; nc < NC; ++nc) done[nc] = O[nc];
     // ---- the normaliser: 16 lanes a token
     const float* const n = nl[b & 1];
-    for (int t = tid >> 4; t < kBlock; t += blockDim.x >> 4) {
-      float d = 0.f;
-      if (l16 < PR) {
-        float q[8];
-        Vec8<BF16>::ld(st + t * dk * 2 + ((l16 ^ (t & (PR - 1))) * 16), 0, q);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) d = fmaf(q[i], n[l16 * 8 + i], d);
-      }
-      d = row16_sum(d);
-      if (l16 == 0) den[b & 1][t] = fmaxf(fabsf(fmaf(aux[kInter + t], d, aux[kSum + t])) * a.q_scale, aux[kFloor + t]) + 1e-6f;
+    for (int u = 0; u < (kBlock + 4 * NW - 1) / (4 * NW); ++u) {
+      const int t = min((tid >> 4) + u * 4 * NW, kBlock - 1), pc = min(l16, PR - 1);
+      float q[8], d = 0.f;
+      Vec8<BF16>::ld(st + t * dk * 2 + ((pc ^ (t & (PR - 1))) * 16), 0, q);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) d = fmaf(q[i], n[pc * 8 + i], d);
+      d = row16_sum(l16 < PR ? d : 0.f);
+      const float x = fmaxf(fabsf(fmaf(aux[kInter + t], d, aux[kSum + t])) * a.q_scale, aux[kFloor + t]) + 1e-6f;
+      if (l16 == 0) den[b & 1][t] = x;
     }
-    for (int c = tid; c < dk; c += blockDim.x) {
-      float x = n[c] * keep;
 #pragma unroll
-      for (int s = 0; s < kBlock; ++s)
-        x = fmaf(aux[kWrite + s], half(*(const uint16_t*)(ks + s * dk * 2 + (((c >> 3) ^ (s & (PR - 1))) * 16) + (c & 7) * 2)), x);
-      nl[(b + 1) & 1][c] = x;
+    for (int u = 0; u < (KT + 4 * NW - 1) / (4 * NW); ++u) {
+      const int kt = min(wave * 4 + g + u * 4 * NW, KT - 1);         // channel 16 kt + l16
+      float x = n[kt * 16 + l16] * keep;
+#pragma unroll
+      for (int s4 = 0; s4 < 4; ++s4) {
+        const int r = 4 * s4 + (l16 >> 2);
+        const f32x4 k4 = read_columns(ks + r * dk * 2 + (((2 * kt + ((l16 & 3) >> 1)) ^ (r & (PR - 1))) * 16) + (l16 & 1) * 8);
+        const f32x4 w4 = *(const f32x4*)(aux + kWrite + 4 * s4);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) x = fmaf(w4[i], k4[i], x);
+      }
+      nl[(b + 1) & 1][kt * 16 + l16] = x;
     }
   }
   wait_and_meet();
   finish(blocks - 1);
   store_state<KT, NC>(S, state, dv, col0);
   for (int c = tid; c < dk; c += blockDim.x) nstate[c] = nl[blocks & 1][c];
+}
+
+template <int KT, int NW> int launch_blocks(const RunArgs& ra, hipStream_t st) {
+  constexpr int dk = 16 * KT, dv = 32 * NW;
+  constexpr size_t smem = 2 * (2 * kBlock * dk * 2 + kBlock * dv * 2 + kAux * 4) + 2 * 4 * (NW * kBlock + kBlock + dk);
+  hipLaunchKernelGGL((mlstm_blocks_kernel<KT, NW>), dim3((unsigned)((int64_t)ra.d.seg.n * ra.d.heads)), dim3(64 * NW), smem, st, ra);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
 }
 
 template <int KT> int launch_runs(const RunArgs& ra, int longest, hipStream_t st) {
@@ -268,12 +290,12 @@ template <int KT> int launch_runs(const RunArgs& ra, int longest, hipStream_t st
   hipLaunchKernelGGL((mlstm_prepare_kernel<KT>), dim3((unsigned)((longest + kBlock - 1) / kBlock), (unsigned)((a.heads + 3) / 4), (unsigned)a.seg.n),
                      dim3(256), 0, st, ra);
   ZP_LAUNCH_CHECK();
-  const size_t smem = 2 * (size_t)(2 * kBlock * a.dk * 2 + kBlock * a.dv * 2 + kAux * 4) + 2 * 4 * (8 * kBlock + kBlock + a.dk);
-  const bool narrow = a.dv % 64 != 0 && a.dv < 128;            // few columns: more, smaller waves
-  if (narrow) hipLaunchKernelGGL((mlstm_blocks_kernel<KT, 1>), dim3(grid), dim3(a.dv * 4), smem, st, ra);
-  else hipLaunchKernelGGL((mlstm_blocks_kernel<KT, 2>), dim3(grid), dim3(a.dv * 2), smem, st, ra);
-  ZP_LAUNCH_CHECK();
-  return ZP_OK;
+  switch (a.dv / 32) {
+    case 1: return launch_blocks<KT, 1>(ra, st);
+    case 2: return launch_blocks<KT, 2>(ra, st);
+    case 3: return launch_blocks<KT, 3>(ra, st);
+    default: return launch_blocks<KT, 4>(ra, st);
+  }
 }
 
 }  // namespace
