@@ -26,197 +26,210 @@ __host__ __device__ inline constexpr int block_floats(int dk, int dv) {
   return (kBlock * (3 * dk + dv) + kBlock * kBlock + dk + 255) / 256 * 256;
 }
 
-__device__ __forceinline__ void load2(const char* p, float& x, float& y) {
-  const uint32_t v = *(const uint32_t*)p;
-  x = __uint_as_float(v << 16);
-  y = __uint_as_float(v & 0xffff0000u);
-}
-
 template <int TAPS>
-__global__ __launch_bounds__(256, 3) void delta_prepare_kernel(RunArgs ra) {
+__global__ __launch_bounds__(256, 4) void delta_prepare_kernel(RunArgs ra) {
   extern __shared__ __align__(16) float lds[];
   const zp_delta& a = ra.d;
+  constexpr int ld = 132;                      // every row: reads across tokens meet no conflicts, offsets are constants
   const int dk = a.dk, dv = a.dv, taps = a.taps;
   const Segment sg = segment_of(a.seg, blockIdx.z);
   const int t0 = blockIdx.x * kBlock;
   if (t0 >= sg.count || sg.row < ra.row0) return;
   const int cnt = min(kBlock, sg.count - t0);
   const int h = blockIdx.y, hk = h / (a.heads / a.kv_heads);
-  float* const qs = lds;                       // [16][dk]
-  float* const ks = qs + kBlock * dk;
-  float* const gs = ks + kBlock * dk;
-  float* const vs = gs + kBlock * dk;          // [16][dv]
-  float* const As = vs + kBlock * dv;          // [16][16]
+  float* const qs = lds;                       // [16][ld], later G q
+  float* const ks = qs + kBlock * ld;
+  float* const gs = ks + kBlock * ld;          // decays, later -W
+  float* const vs = gs + kBlock * ld;
+  float* const As = vs + kBlock * ld;          // [16][16]
   float* const Ps = As + kBlock * kBlock;      // [16][16]
   float* const beta = Ps + kBlock * kBlock;
-  float* const outs = beta + kBlock;           // W and G q in operand order, 4 floats of padding per 64
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int cw = 2 * dk + dv;
   const char* const tail = (const char*)a.conv_state + ((int64_t)sg.slot * a.heads + h) * (taps - 1) * cw * 2;
-  const float rate = expf(a.a_log[h]);
   const int channels = 2 * a.kv_heads * dk + a.heads * dv;
   auto place = [&](int c) -> int {
     return c < dk ? hk * dk + c : (c < 2 * dk ? a.kv_heads * dk + hk * dk + c - dk : 2 * a.kv_heads * dk + h * dv + c - 2 * dk);
   };
+  // ---- requests first: the decays' pre-activations (two pieces a thread at most), the step sizes'
+  f32x4 z[2], zb[2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int i = tid + u * 256, t = i / (dk / 4), c = (i - t * (dk / 4)) * 4;
+    z[u] = zb[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (t < cnt) {
+      z[u] = load4<BF16>(a.low, (int64_t)(sg.row + t0 + t) * a.low_stride + h * dk + c);
+      zb[u] = *(const f32x4*)(a.dt_bias + h * dk + c);
+    }
+  }
+  const float b_in = tid < cnt ? Elem<BF16>::ld(a.in, (int64_t)(sg.row + t0 + tid) * a.in_stride + a.b_at + h) : 0.f;
+  const float rate = __expf(a.a_log[h]);
   // ---- convolutions: a thread's two channels, the block's 16 tokens from a sliding window
+  // rows from t0 - (TAPS - 1) on; those outside the run read as zero, those before it come from the history
+  const int back = min(TAPS - 1, t0);
+  const __amdgpu_buffer_rsrc_t rows = __builtin_amdgcn_make_buffer_rsrc(
+      (void*)((const char*)a.in + (int64_t)(sg.row + t0 - back) * a.in_stride * 2), 0, (int)((cnt + back) * a.in_stride * 2), 0x00020000);
   for (int c = 2 * tid; c < cw; c += 512) {
     const int at = place(c);
-    float f[2][TAPS], x[2][kBlock + TAPS - 1];
+    uint32_t x[kBlock + TAPS - 1];             // two channels' bf16
+#pragma unroll
+    for (int i = 0; i < kBlock + TAPS - 1; ++i) {
+      const int u = i - (TAPS - 1) + back;     // row of the buffer
+      x[i] = u >= 0 ? (uint32_t)__builtin_amdgcn_raw_buffer_load_b32(rows, at * 2, u * (int)a.in_stride * 2, 0) : 0u;
+    }
+    if (t0 == 0 && sg.start > 0) {
+#pragma unroll
+      for (int i = 0; i < TAPS - 1; ++i)
+        if (i >= TAPS - taps) x[i] = *(const uint32_t*)(tail + ((int64_t)(taps - TAPS + i) * cw + c) * 2);
+    }
+    float f[2][TAPS];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j)                            // f[.][j]: j tokens back
 #pragma unroll
       for (int e = 0; e < 2; ++e) f[e][j] = j < taps ? a.filters[(int64_t)(taps - 1 - j) * channels + at + e] : 0.f;
-    const char* const first = (const char*)a.in + ((int64_t)(sg.row + t0) * a.in_stride + at) * 2;
-#pragma unroll
-    for (int i = 0; i < kBlock + TAPS - 1; ++i) {
-      const int u = t0 + i - (TAPS - 1);
-      x[0][i] = x[1][i] = 0.f;
-      if (i >= TAPS - taps && u < t0 + cnt) {
-        if (u >= 0) load2(first + (int64_t)(i - (TAPS - 1)) * a.in_stride * 2, x[0][i], x[1][i]);
-        else if (sg.start > 0) load2(tail + ((int64_t)(taps - 1 + u) * cw + c) * 2, x[0][i], x[1][i]);
-      }
-    }
     float* const dst = c < dk ? qs + c : (c < 2 * dk ? ks + c - dk : vs + c - 2 * dk);
-    const int st = c < 2 * dk ? dk : dv;
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
       float2 y = {0.f, 0.f};
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
-        y.x = fmaf(f[0][j], x[0][t + TAPS - 1 - j], y.x);
-        y.y = fmaf(f[1][j], x[1][t + TAPS - 1 - j], y.y);
+        const uint32_t v = x[t + TAPS - 1 - j];
+        y.x = fmaf(f[0][j], __uint_as_float(v << 16), y.x);
+        y.y = fmaf(f[1][j], __uint_as_float(v & 0xffff0000u), y.y);
       }
       y.x = t < cnt ? y.x * fast_sigmoid(y.x) : 0.f;
       y.y = t < cnt ? y.y * fast_sigmoid(y.y) : 0.f;
-      *(float2*)(dst + t * st) = y;
+      *(float2*)(dst + t * ld) = y;
+      if (t % 4 == 3) __builtin_amdgcn_sched_barrier(0);
     }
   }
-  for (int i = tid; i < kBlock * dk / 4; i += 256) {
-    const int t = i / (dk / 4), c = (i - t * (dk / 4)) * 4;
-    f32x4 g = {1.f, 1.f, 1.f, 1.f};
-    if (t < cnt) {
-      const f32x4 z = load4<BF16>(a.low, (int64_t)(sg.row + t0 + t) * a.low_stride + h * dk + c) + *(const f32x4*)(a.dt_bias + h * dk + c);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) g[e] = __expf(-rate * fast_softplus(z[e]));
-    }
-    *(f32x4*)(gs + t * dk + c) = g;
-  }
-  if (tid < kBlock)
-    beta[tid] = tid < cnt ? fast_sigmoid(Elem<BF16>::ld(a.in, (int64_t)(sg.row + t0 + tid) * a.in_stride + a.b_at + h)) : 0.f;
-  __syncthreads();
-  // ---- unit vectors: a wave its four tokens
+  for (int u = 0; u < 2; ++u) {
+    const int i = tid + u * 256, t = i / (dk / 4), c = (i - t * (dk / 4)) * 4;
+    if (t < kBlock) {
+      f32x4 g = {1.f, 1.f, 1.f, 1.f};
+      if (t < cnt) {
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int t = wave * 4 + i;
-    float q2 = 0.f, k2 = 0.f;
-    for (int c = lane; c < dk; c += 64) {
-      const float q = qs[t * dk + c], k = ks[t * dk + c];
-      q2 = fmaf(q, q, q2);
-      k2 = fmaf(k, k, k2);
-    }
-    const float rq = a.q_scale / sqrtf(wave_sum(q2) + 1e-6f), rk = 1.f / sqrtf(wave_sum(k2) + 1e-6f);
-    for (int c = lane; c < dk; c += 64) {
-      qs[t * dk + c] *= rq;
-      ks[t * dk + c] *= rk;
+        for (int e = 0; e < 4; ++e) g[e] = __expf(-rate * fast_softplus(z[u][e] + zb[u][e]));
+      }
+      *(f32x4*)(gs + t * ld + c) = g;
     }
   }
+  if (tid < kBlock) beta[tid] = tid < cnt ? fast_sigmoid(b_in) : 0.f;
   __syncthreads();
-  // ---- A and P: lane group (lane / 16) of wave w walks k_s, s = 4 w + group, down the tokens; 16 lanes share
-  // its channels in pieces of four
+  // ---- unit vectors: a wave its four tokens, 16 lanes each
   {
-    const int l16 = lane & 15, s = wave * 4 + (lane >> 4), pieces = dk / 4;
+    const int t = wave * 4 + (lane >> 4), l16 = lane & 15, pieces = dk / 4;
+    f32x4 q[2], k[2], q2 = {0.f, 0.f, 0.f, 0.f}, k2 = q2;
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      const int pc = min(l16 + 16 * p, pieces - 1);
+      q[p] = *(const f32x4*)(qs + t * ld + pc * 4);
+      k[p] = *(const f32x4*)(ks + t * ld + pc * 4);
+      if (l16 + 16 * p < pieces) {
+        q2 += q[p] * q[p];
+        k2 += k[p] * k[p];
+      }
+    }
+    const float rq = a.q_scale / sqrtf(row16_sum(q2[0] + q2[1] + q2[2] + q2[3]) + 1e-6f);
+    const float rk = 1.f / sqrtf(row16_sum(k2[0] + k2[1] + k2[2] + k2[3]) + 1e-6f);
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      const int pc = l16 + 16 * p;
+      if (pc < pieces) {
+        *(f32x4*)(qs + t * ld + pc * 4) = q[p] * rq;
+        *(f32x4*)(ks + t * ld + pc * 4) = k[p] * rk;
+      }
+    }
+  }
+  __syncthreads();
+  // ---- A and P: 16 lanes walk k_s down the tokens, in pieces of four channels; group i of wave w takes s = w + 4 i
+  {
+    const int l16 = lane & 15, s = wave + 4 * (lane >> 4), pieces = dk / 4;
+    int at[2];
     f32x4 kk[2];
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
       const int pc = l16 + 16 * p;
-      kk[p] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (pc < pieces) kk[p] = *(const f32x4*)(ks + s * dk + pc * 4);
+      at[p] = min(pc, pieces - 1) * 4;
+      kk[p] = *(const f32x4*)(ks + s * ld + at[p]);
+      if (pc >= pieces) kk[p] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
-      float sa = 0.f, sp = 0.f;
-      if (t >= wave * 4) {                    // uniform in the wave
+      f32x4 pa = {0.f, 0.f, 0.f, 0.f}, pp = pa;
 #pragma unroll
-        for (int p = 0; p < 2; ++p) {
-          const int pc = l16 + 16 * p;
-          if (pc < pieces) {
-            if (t > s) kk[p] *= *(const f32x4*)(gs + t * dk + pc * 4);
-            const f32x4 kt = *(const f32x4*)(ks + t * dk + pc * 4), qt = *(const f32x4*)(qs + t * dk + pc * 4);
+      for (int p = 0; p < 2; ++p) {
+        const f32x4 gt = *(const f32x4*)(gs + t * ld + at[p]);
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              sa = fmaf(kk[p][i], kt[i], sa);
-              sp = fmaf(kk[p][i], qt[i], sp);
-            }
-          }
-        }
-        sa = row16_sum(sa);
-        sp = row16_sum(sp);
+        for (int e = 0; e < 4; ++e) kk[p][e] *= t > s ? gt[e] : 1.f;
+        pa += kk[p] * *(const f32x4*)(ks + t * ld + at[p]);
+        pp += kk[p] * *(const f32x4*)(qs + t * ld + at[p]);
       }
-      if (l16 == 0) {
-        As[t * kBlock + s] = t > s ? sa * beta[t] : 0.f;
-        Ps[t * kBlock + s] = t >= s ? sp : 0.f;
-      }
-      __builtin_amdgcn_sched_barrier(0);
+      const float sa = row16_sum((pa[0] + pa[1]) + (pa[2] + pa[3])), sp = row16_sum((pp[0] + pp[1]) + (pp[2] + pp[3]));
+      As[t * kBlock + s] = t > s ? sa * beta[t] : 0.f;         // all 16 lanes, the same value
+      Ps[t * kBlock + s] = t >= s ? sp : 0.f;
+      if (t % 2 == 1) __builtin_amdgcn_sched_barrier(0);       // not all tokens' rows in registers at once
     }
   }
   __syncthreads();
-  // ---- columns: forward substitution, and the block's decays
+  // ---- columns: forward substitution, and the block's decays.  A thread reads and writes its own column only.
   const int64_t base = (block_slot(ra.row0, sg, blockIdx.z, blockIdx.x) * a.heads + h) * block_floats(dk, dv);
   float* const oWQ = ra.ws + base;             // [2][dk / 16][64 lanes][4]
   float* const oK = oWQ + 2 * kBlock * dk;     // [dk / 16][64][4]
   float* const oU = oK + kBlock * dk;          // [dv / 16][64][4]
   float* const oP = oU + kBlock * dv;          // [64][4]
   float* const oG = oP + kBlock * kBlock;      // [dk]
-  for (int c = tid; c < dk + dv; c += 256) {
-    // a token at a time: its factors and values must not all sit in registers
-    float w[kBlock];
-    const bool key = c < dk;
-    const float* const src = key ? ks + c : vs + c - dk;
-    const int st = key ? dk : dv, o_at = (c >> 4) * 272 + ((c & 15) >> 2) * 68 + (c & 3);      // 256 and 64 floats, padded
+  float w[kBlock];
+  auto substitute = [&](int t, float b) {      // w_t = b - sum_{s < t} A[t, s] w_s
+    float x[4] = {b, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < t; s += 4) {
+      const f32x4 A = *(const f32x4*)(As + t * kBlock + s);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (s + i < t) x[i] = fmaf(-A[i], w[s + i], x[i]);
+    }
+    w[t] = (x[0] + x[1]) + (x[2] + x[3]);
+    if (t % 2 == 1) __builtin_amdgcn_sched_barrier(0);
+  };
+  for (int c = tid; c < dk; c += 256) {
     float G = 1.f;
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
-      if (key) {
-        G *= gs[t * dk + c];
-        outs[(dk / 16) * 272 + o_at + t * 4] = qs[t * dk + c] * G;
-      }
-      float x = beta[t] * src[t * st] * G;
+      G *= gs[t * ld + c];
+      qs[t * ld + c] *= G;
+      substitute(t, beta[t] * ks[t * ld + c] * G);
+    }
+    oG[c] = G;
+    asm volatile("" ::: "memory");            // keys and decays are read again rather than kept
+    float R = 1.f;
 #pragma unroll
-      for (int s = 0; s < t; s += 4) {
-        const f32x4 A = *(const f32x4*)(As + t * kBlock + s);
+    for (int g = 3; g >= 0; --g) {
+      f32x4 x;
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (s + i < t) x = fmaf(-A[i], w[s + i], x);
+      for (int r = 3; r >= 0; --r) {
+        const int t = 4 * g + r;
+        x[r] = ks[t * ld + c] * R;
+        R *= gs[t * ld + c];
+        gs[t * ld + c] = -w[t];
       }
-      w[t] = x;
+      *(f32x4*)(oK + ((c >> 4) * 64 + g * 16 + (c & 15)) * 4) = x;
       __builtin_amdgcn_sched_barrier(0);
     }
-    if (key) oG[c] = G;
-    if (c < dk) {
+  }
+  for (int v = (tid + 256 - dk) % 256; v < dv; v += 256) {      // on the threads the keys leave free, as far as they go
 #pragma unroll
-      for (int t = 0; t < kBlock; ++t) outs[o_at + t * 4] = -w[t];
-      float R = 1.f;
+    for (int t = 0; t < kBlock; ++t) substitute(t, beta[t] * vs[t * ld + v]);
 #pragma unroll
-      for (int t = kBlock - 1; t >= 0; --t) {
-        w[t] = ks[t * dk + c] * R;
-        R *= gs[t * dk + c];
-        if (t % 4 == 0) __builtin_amdgcn_sched_barrier(0);
-      }
-#pragma unroll
-      for (int g = 0; g < 4; ++g)
-        *(f32x4*)(oK + ((c >> 4) * 64 + g * 16 + (c & 15)) * 4) = f32x4{w[4 * g], w[4 * g + 1], w[4 * g + 2], w[4 * g + 3]};
-    } else {
-      const int v = c - dk;
-#pragma unroll
-      for (int g = 0; g < 4; ++g)
-        *(f32x4*)(oU + ((v >> 4) * 64 + g * 16 + (v & 15)) * 4) = f32x4{w[4 * g], w[4 * g + 1], w[4 * g + 2], w[4 * g + 3]};
-    }
+    for (int g = 0; g < 4; ++g)
+      *(f32x4*)(oU + ((v >> 4) * 64 + g * 16 + (v & 15)) * 4) = f32x4{w[4 * g], w[4 * g + 1], w[4 * g + 2], w[4 * g + 3]};
   }
   if (tid < 64) *(f32x4*)(oP + tid * 4) = *(const f32x4*)(Ps + (tid & 15) * kBlock + (tid >> 4) * 4);
   __syncthreads();
-  for (int i = tid; i < 2 * kBlock * dk / 4; i += 256) {
-    const int x = i * 4, tile = x >> 8, in = x & 255;
-    *(f32x4*)(oWQ + x) = *(const f32x4*)(outs + tile * 272 + (in >> 6) * 68 + (in & 63));
+  for (int i = tid; i < 2 * kBlock * dk / 4; i += 256) {       // lane (g, row) of tile kt: columns 16 kt + 4 g ..
+    const int tile = i >> 6, l = i & 63, kt = tile & (dk / 16 - 1);
+    *(f32x4*)(oWQ + i * 4) = *(const f32x4*)((tile < dk / 16 ? gs : qs) + (l & 15) * ld + kt * 16 + (l >> 4) * 4);
   }
 }
 
@@ -353,7 +366,7 @@ template <int KT> int launch_blocks(const RunArgs& ra, hipStream_t st) {
 
 template <int TAPS> int launch_prepare(const RunArgs& ra, int longest, hipStream_t st) {
   const zp_delta& a = ra.d;
-  const size_t smem = sizeof(float) * (kBlock * (3 * a.dk + a.dv) + 2 * kBlock * kBlock + kBlock + 2 * (a.dk / 16) * 272);
+  const size_t smem = sizeof(float) * (kBlock * 4 * 132 + 2 * kBlock * kBlock + kBlock);
   if (smem > 60 * 1024 && hipFuncSetAttribute((const void*)delta_prepare_kernel<TAPS>, hipFuncAttributeMaxDynamicSharedMemorySize,
                                               (int)smem) != hipSuccess) {
     zp_set_error("delta_runs: cannot reserve %zu bytes of LDS", smem);
