@@ -333,7 +333,7 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
   f32x4 acc[2][MT];
 #pragma unroll
   for (int i = 0; i < MT; ++i) acc[0][i] = acc[1][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 8
   for (int ks = 0; ks < steps; ++ks) {
     const u32x4 w0 = *(const u32x4*)(w + (int64_t)ks * 1024), w1 = *(const u32x4*)(w + wt + (int64_t)ks * 1024);
 #pragma unroll
@@ -401,15 +401,15 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(ExpertArgs a) {
   const char* wbase = (const char*)(shared ? a.w_shared : a.w) + (shared ? 0 : t.x * a.w_expert) * 2;
   const __amdgpu_buffer_rsrc_t rw = __builtin_amdgcn_make_buffer_rsrc((void*)(wbase + (int64_t)w0 * steps * 1024), 0,
                                                                       min(kBlockW, wtiles - w0) * steps * 1024, 0x00020000);
-  const int rows = UP ? a.n : a.n * a.slots;
-  const __amdgpu_buffer_rsrc_t rx =
-      __builtin_amdgcn_make_buffer_rsrc((void*)a.x, 0, (int)min((int64_t)rows * a.x_st * 2, (int64_t)0x7fffffff), 0x00020000);
+  // gate_up gathers tokens from all of x, down reads consecutive rows
+  const char* const xbase = (const char*)a.x + (UP ? 0 : t.y * a.x_st * 2);
+  const __amdgpu_buffer_rsrc_t rx = __builtin_amdgcn_make_buffer_rsrc((void*)xbase, 0, (int)((UP ? a.n : t.z) * a.x_st * 2), 0x00020000);
   // this wave's loads of a stage: two of the eight 16-token tiles, four of the sixteen of W
   int xoff[2], woff[4];
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
-    const int pos = t.y + min((wave * 2 + i) * 16 + l16, t.z - 1);
-    xoff[i] = (int)((UP ? a.sorted[pos] / a.slots : pos) * a.x_st * 2) + g * 16;
+    const int r = min((wave * 2 + i) * 16 + l16, t.z - 1);
+    xoff[i] = (int)((UP ? a.sorted[t.y + r] / a.slots : r) * a.x_st * 2) + g * 16;
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) woff[i] = min(wave * 4 + i, wtiles - w0 - 1) * steps * 1024;
@@ -451,31 +451,38 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(ExpertArgs a) {
       for (int j = 0; j < 4; ++j) acc[i][j] = mfma_bf16(wf[i], xf[j], acc[i][j]);
     __builtin_amdgcn_sched_barrier(0);
   }
+  // Two result tiles side by side hold 4 outputs per lane each; lanes of neighbouring groups swap halves, so that
+  // each ends with 8 consecutive outputs of one of them: group g has tile (g & 1), outputs 8 (g >> 1) on.
+  auto store8 = [&](const float* lo, const float* hi, int64_t at, int tile, int tiles, bool row) {
+    const auto a0 = __builtin_amdgcn_permlane16_swap(pack_bf16(lo[0], lo[1]), pack_bf16(hi[0], hi[1]), false, false);
+    const auto a1 = __builtin_amdgcn_permlane16_swap(pack_bf16(lo[2], lo[3]), pack_bf16(hi[2], hi[3]), false, false);
+    if (row && tile + (g & 1) < tiles)
+      *(u32x4*)((uint16_t*)a.out + at + (tile + (g & 1)) * 16 + (g >> 1) * 8) = u32x4{a0[0], a1[0], a0[1], a1[1]};
+  };
+  const int out_tiles = UP ? wtiles / 2 : wtiles;
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int r = (th * 4 + j) * 16 + l16;
-    if (r >= t.z) continue;
-    const int pos = t.y + r, as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
+    const bool row = r < t.z;                          // every lane takes part in the swaps
+    const int pos = t.y + min(r, t.z - 1), as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
     if constexpr (UP) {
       const float wgt = slot < a.top ? a.weights[(int64_t)n * a.top + slot] : 1.f;
       const float lim = shared ? a.limit_shared : a.limit;
 #pragma unroll
-      for (int i = 0; i < 8; i += 2) {
-        const int wt = w0 + wh * 8 + i;
-        if (wt >= wtiles) break;
-        float v[4];
+      for (int i = 0; i < 8; i += 4) {
+        float v[2][4];
 #pragma unroll
-        for (int k = 0; k < 4; ++k) v[k] = wgt * gated<BF16>(acc[i][j][k], acc[i + 1][j][k], lim);
-        Mma<BF16>::st4(a.out, (int64_t)pos * a.o_st + wt * 8 + g * 4, v);
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int k = 0; k < 4; ++k) v[u][k] = wgt * gated<BF16>(acc[i + 2 * u][j][k], acc[i + 2 * u + 1][j][k], lim);
+        store8(v[0], v[1], (int64_t)pos * a.o_st, (w0 + wh * 8 + i) / 2, out_tiles, row);
       }
     } else {
-      const int64_t at = ((int64_t)slot * a.n + n) * a.o_st;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int wt = w0 + wh * 8 + i;
-        if (wt >= wtiles) break;
-        const float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
-        Mma<BF16>::st4(a.out, at + wt * 16 + g * 4, v);
+      for (int i = 0; i < 8; i += 2) {
+        const float lo[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+        const float hi[4] = {acc[i + 1][j][0], acc[i + 1][j][1], acc[i + 1][j][2], acc[i + 1][j][3]};
+        store8(lo, hi, ((int64_t)slot * a.n + n) * a.o_st, w0 + wh * 8 + i, out_tiles, row);
       }
     }
   }
@@ -632,7 +639,7 @@ static int experts(bool up, const void* x, const void* w, const void* w_shared, 
                  x_stride >= (K > K_shared ? K : K_shared) && out_stride >= (M > M_shared ? M : M_shared),
              "moe experts: unaligned or overlapping rows");
   if (rows == kBlockRows) {       // 31-bit byte offsets into x and into a block of W
-    const int64_t xr = up ? n : (int64_t)n * (top + shared), kx = K > K_shared ? K : K_shared;
+    const int64_t xr = up ? n : kBlockRows, kx = K > K_shared ? K : K_shared;
     if (xr * x_stride * 2 >= (1ll << 31) || kx * 512 >= (1ll << 31)) {
       zp_set_error("moe experts: %lld rows of %lld elements in one step", (long long)xr, (long long)x_stride);
       return ZP_EUNSUPPORTED;
