@@ -306,23 +306,27 @@ template <> __device__ __forceinline__ float gated<BF16>(float gate, float up, f
   return g * __builtin_amdgcn_rcpf(1.f + __expf(-1.702f * g)) * (u + 1.f);
 }
 
-// Few rows per expert: the weights are streamed straight into registers, each wave its own 32 rows of
-// W (gate_up: 16 of the gate and the 16 of `up` that belong to them) against 16 * MT tokens.
+// Few rows per expert: the weights are streamed straight into registers.  A workgroup owns 64 rows of W (gate_up:
+// two 16-row tiles of the gate and the two of `up` that belong to them) and up to 16 * MT tokens; its four waves
+// take every fourth step of the contraction and meet in LDS.
+constexpr int kRowsW = 4;                              // 16-row tiles of W
 template <typename T, int MT, bool UP>
 __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  __shared__ __align__(16) float part[4][kRowsW * MT * 256];
+  const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int tile = blockIdx.x % a.max_tiles, cb = blockIdx.x / a.max_tiles;
   if (tile >= *a.ntiles) return;
   const int4 t = *(const int4*)(a.tiles + (int64_t)tile * 4);
   const bool shared = t.x == a.E;
-  const int M = shared ? a.M_shared : a.M, K = shared ? a.K_shared : a.K;
-  const int pair = cb * 4 + wave;                    // of 16-row tiles of W
-  if (pair * (UP ? 16 : 32) >= M) return;
+  const int wtiles = (shared ? a.M_shared : a.M) / 16 * (UP ? 2 : 1), K = shared ? a.K_shared : a.K;
+  const int w0 = cb * kRowsW;
+  if (w0 >= wtiles) return;
   const int steps = K / Mma<T>::kStep;
-  const char* w = (const char*)(shared ? a.w_shared : a.w) +
-                  ((shared ? 0 : t.x * a.w_expert) + (int64_t)pair * 32 * K) * T::bytes + lane * 16;
-  const bool two = UP || pair * 32 + 16 < M;         // outputs are a multiple of 16
-  const int64_t wt = two ? (int64_t)16 * K * T::bytes : 0;
+  const char* const w = (const char*)(shared ? a.w_shared : a.w) + (shared ? 0 : t.x * a.w_expert) * T::bytes + lane * 16;
+  const char* wp[kRowsW];
+#pragma unroll
+  for (int i = 0; i < kRowsW; ++i) wp[i] = w + (int64_t)min(w0 + i, wtiles - 1) * steps * 1024;
   const char* x[MT];
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
@@ -330,42 +334,55 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
     const int64_t row = UP ? a.sorted[pos] / a.slots : pos;
     x[i] = (const char*)a.x + (row * a.x_st + g * kPiece<T>) * T::bytes;
   }
-  f32x4 acc[2][MT];
+  f32x4 acc[kRowsW][MT];
 #pragma unroll
-  for (int i = 0; i < MT; ++i) acc[0][i] = acc[1][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-  for (int ks = 0; ks < steps; ++ks) {
-    const u32x4 w0 = *(const u32x4*)(w + (int64_t)ks * 1024), w1 = *(const u32x4*)(w + wt + (int64_t)ks * 1024);
+  for (int k = 0; k < kRowsW; ++k)
 #pragma unroll
-    for (int i = 0; i < MT; ++i) {
-      const u32x4 xf = *(const u32x4*)(x[i] + (int64_t)ks * 64);
-      acc[0][i] = Mma<T>::go(w0, xf, acc[0][i]);
-      acc[1][i] = Mma<T>::go(w1, xf, acc[1][i]);
+    for (int i = 0; i < MT; ++i) acc[k][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int ks = wave; ks < steps; ks += 4) {
+    u32x4 wf[kRowsW], xf[MT];
+#pragma unroll
+    for (int k = 0; k < kRowsW; ++k) {
+      const u32x4* const p = (const u32x4*)(wp[k] + (int64_t)ks * 1024);
+      if constexpr (MT == 1) wf[k] = __builtin_nontemporal_load(p);       // hardly any expert has a second tile
+      else wf[k] = *p;
     }
+#pragma unroll
+    for (int i = 0; i < MT; ++i) xf[i] = *(const u32x4*)(x[i] + (int64_t)ks * 64);
+#pragma unroll
+    for (int k = 0; k < kRowsW; ++k)
+#pragma unroll
+      for (int i = 0; i < MT; ++i) acc[k][i] = Mma<T>::go(wf[k], xf[i], acc[k][i]);
   }
 #pragma unroll
-  for (int i = 0; i < MT; ++i) {
-    if (i * 16 + l16 >= t.z) continue;
-    const int pos = t.y + i * 16 + l16;
-    const int as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
+  for (int k = 0; k < kRowsW; ++k)
+#pragma unroll
+    for (int i = 0; i < MT; ++i) *(f32x4*)(part[wave] + ((k * MT + i) * 64 + lane) * 4) = acc[k][i];
+  __syncthreads();
+  auto total = [&](int k, int i) {
+    f32x4 r = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int v = 0; v < 4; ++v) r += *(const f32x4*)(part[v] + ((k * MT + i) * 64 + lane) * 4);
+    return r;
+  };
+  for (int u = wave; u < (UP ? kRowsW / 2 : kRowsW) * MT; u += 4) {
+    const int i = u % MT, k = u / MT * (UP ? 2 : 1), wt = w0 + k;
+    if (wt >= wtiles || i * 16 + l16 >= t.z) continue;
+    const int pos = t.y + i * 16 + l16, as = a.sorted[pos], n = as / a.slots, slot = as - n * a.slots;
+    const f32x4 first = total(k, i);
+    float r[4];
     if constexpr (UP) {
+      const f32x4 second = total(k + 1, i);
       const float wgt = slot < a.top ? a.weights[(int64_t)n * a.top + slot] : 1.f;
       const float lim = shared ? a.limit_shared : a.limit;
-      float r[4];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) r[k] = wgt * gated<T>(acc[0][i][k], acc[1][i][k], lim);
-      Mma<T>::st4(a.out, (int64_t)pos * a.o_st + pair * 16 + g * 4, r);
+      for (int e = 0; e < 4; ++e) r[e] = wgt * gated<T>(first[e], second[e], lim);
+      Mma<T>::st4(a.out, (int64_t)pos * a.o_st + wt * 8 + g * 4, r);
     } else {
-      const int64_t at = ((int64_t)slot * a.n + n) * a.o_st + pair * 32 + g * 4;
-      float r[4];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) r[k] = acc[0][i][k];
-      Mma<T>::st4(a.out, at, r);
-      if (two) {
-#pragma unroll
-        for (int k = 0; k < 4; ++k) r[k] = acc[1][i][k];
-        Mma<T>::st4(a.out, at + 16, r);
-      }
+      for (int e = 0; e < 4; ++e) r[e] = first[e];
+      Mma<T>::st4(a.out, ((int64_t)slot * a.n + n) * a.o_st + wt * 16 + g * 4, r);
     }
   }
 }
@@ -501,9 +518,8 @@ template <bool UP> int launch_experts(const ExpertArgs& a, int rows, int dtype, 
     ZP_LAUNCH_CHECK();
     return ZP_OK;
   }
-  const int per = UP ? 64 : 128;                     // outputs per workgroup
-  const int M = a.M > a.M_shared ? a.M : a.M_shared;
-  const int64_t grid = (int64_t)a.max_tiles * ((M + per - 1) / per);
+  const int Mw = (a.M > a.M_shared ? a.M : a.M_shared) * (UP ? 2 : 1);
+  const int64_t grid = (int64_t)a.max_tiles * ((Mw + 16 * kRowsW - 1) / (16 * kRowsW));
   if (grid >= (1ll << 31)) {
     zp_set_error("moe: too many tiles");
     return ZP_EUNSUPPORTED;
@@ -526,7 +542,7 @@ template <bool UP> int launch_experts(const ExpertArgs& a, int rows, int dtype, 
 int tile_rows(int n, int E, int top, int dtype) {
   const int64_t avg = ((int64_t)n * top + E - 1) / E;
   if (dtype == ZP_BF16 && avg > 48) return kBlockRows;
-  return avg <= 12 ? 16 : (avg <= 24 ? 32 : 64);
+  return avg <= 8 ? 16 : (avg <= 16 ? 32 : 64);       // a second tile reads an expert's weights again
 }
 int tile_bound(int n, int E, int top, int shared, int rows) {
   const int64_t a = (int64_t)n * top;
