@@ -53,10 +53,10 @@ struct SmallArgs {
   int64_t x_st;
 };
 
-// 16 tokens x 16 * MT outputs per workgroup, its four waves share the contraction.
-template <typename T, int MT>
-__global__ __launch_bounds__(256) void small_linear_kernel(SmallArgs a) {
-  __shared__ float red[3][MT * 64 * 4];
+// 16 tokens x 16 * MT outputs per workgroup, its NW waves share the contraction.
+template <typename T, int MT, int NW>
+__global__ __launch_bounds__(64 * NW) void small_linear_kernel(SmallArgs a) {
+  __shared__ float red[NW - 1][MT * 64 * 4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16 * MT;
   const int steps = a.K / Mma<T>::kStep;
@@ -69,7 +69,7 @@ __global__ __launch_bounds__(256) void small_linear_kernel(SmallArgs a) {
 #pragma unroll
   for (int t = 0; t < MT; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
-  for (int ks = wave; ks < steps; ks += 4) {
+  for (int ks = wave; ks < steps; ks += NW) {
     const u32x4 xf = *(const u32x4*)(x + (int64_t)ks * 64);
 #pragma unroll
     for (int t = 0; t < MT; ++t) acc[t] = Mma<T>::go(*(const u32x4*)(w[t] + (int64_t)ks * 64), xf, acc[t]);
@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void small_linear_kernel(SmallArgs a) {
 #pragma unroll
   for (int t = 0; t < MT; ++t) {
 #pragma unroll
-    for (int k = 0; k < 3; ++k) acc[t] += *(const f32x4*)(red[k] + (t * 64 + lane) * 4);
+    for (int k = 0; k < NW - 1; ++k) acc[t] += *(const f32x4*)(red[k] + (t * 64 + lane) * 4);
     const int m = m0 + t * 16 + g * 4;
     if (n < a.n && m < a.M) *(f32x4*)(a.out + (int64_t)n * a.M + m) = acc[t];
   }
@@ -569,8 +569,8 @@ extern "C" int zp_small_linear(const void* x, const void* w, float* out, int32_t
   const dim3 grid(gx, (unsigned)(wide ? (M + 63) / 64 : (M + 15) / 16));
 #define ZP_SMALL(T)                                                                              \
   do {                                                                                           \
-    if (wide) hipLaunchKernelGGL((small_linear_kernel<T, 4>), grid, dim3(256), 0, st, a);        \
-    else hipLaunchKernelGGL((small_linear_kernel<T, 1>), grid, dim3(256), 0, st, a);             \
+    if (wide) hipLaunchKernelGGL((small_linear_kernel<T, 4, 4>), grid, dim3(256), 0, st, a);     \
+    else hipLaunchKernelGGL((small_linear_kernel<T, 1, 16>), grid, dim3(1024), 0, st, a);        \
   } while (0)
   if (dtype == ZP_BF16) ZP_SMALL(BF16); else ZP_SMALL(F32);
 #undef ZP_SMALL
