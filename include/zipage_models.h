@@ -1,8 +1,8 @@
 /* C ABI of the model-side kernels of decoders that need more than the compression library's layer
- * kernels.  Three shared objects, so that a model compiles only what it runs: libzipage_models.so (an
+ * kernels.  Five shared objects, so that a model compiles only what it runs: libzipage_models.so (an
  * fp32 residual stream, attention of prompt runs), libzipage_latent.so (latent attention over pages of
- * latents) and libzipage_hybrid.so (grouped-query attention with sinks, recurrent mixers, mixtures of
- * experts).  Status codes, dtype tags and conventions are those of
+ * latents), libzipage_grouped.so (grouped-query attention, with sinks or of two maps),
+ * libzipage_recurrent.so (recurrent mixers) and libzipage_moe.so (mixtures of experts).  Status codes, dtype tags and conventions are those of
  * zipage_hip.h; every entry point here takes ZP_BF16 or ZP_F32 (true 32-bit products), enqueues on
  * `stream`, allocates nothing and may be captured into a HIP graph. */
 #ifndef ZIPAGE_MODELS_H
@@ -16,28 +16,35 @@ extern "C" {
 /* ------------------------------------------------------------------ libzipage_models.so */
 
 /* x = embed[tokens] * embed_scale (+ pos[positions] when pos is given), fp32; with norm_weight also
- * out = x / sqrt(mean(x^2) + eps) * (weight_offset + norm_weight).  Rows are `width` long (multiple
+ * out = x / sqrt(mean(x^2) + eps) * (weight_offset + norm_weight) or, with norm_bias,
+ * out = tanh(norm_alpha * x) * (weight_offset + norm_weight) + norm_bias.  Rows are `width` long (multiple
  * of 8, zero padded), the mean runs over norm_width.  embed (vocab, width), pos (max_positions,
  * width) and out are of `dtype`; indices are clamped to the tables. */
 int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* embed, const void* pos,
-                  float* x, const float* norm_weight, void* out, int32_t n, int32_t width,
-                  int32_t norm_width, int64_t vocab, int64_t max_positions,
-                  float embed_scale, float eps, float weight_offset, int32_t dtype, void* stream);
+                  float* x, const float* norm_weight, const float* norm_bias, void* out, int32_t n,
+                  int32_t width, int32_t norm_width, int64_t vocab, int64_t max_positions,
+                  float embed_scale, float eps, float weight_offset, float norm_alpha, int32_t dtype,
+                  void* stream);
 
 /* r = x + the sum of y's n_y planes (x (n, width) fp32; y (n_y, n, width) of dtype), where with
  * y_weight the sum is RMS-normed times y_weight before it is added; written to `result` when given; with a depth average
  * r <- mix[n_hist] * r + sum_{j < n_hist} mix[j] * hist[j] (hist: planes of (n, width) fp32,
  * hist_plane elements apart); written to `x_out` when given; with norm_weight also
- * out = rmsnorm(r) * (weight_offset + norm_weight) * out_scale.  mix NULL: no average. */
+ * out = rmsnorm(r) * (weight_offset + norm_weight) * out_scale, or with norm_bias
+ * out = (tanh(norm_alpha * r) * (weight_offset + norm_weight) + norm_bias) * out_scale.
+ * mix NULL: no average. */
 int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* y_weight,
                      const float* hist, int64_t hist_plane, const float* mix, int32_t n_hist, float* result, float* x_out,
-                     const float* norm_weight, void* out, int32_t n, int32_t width,
-                     int32_t norm_width, float eps, float weight_offset, float out_scale,
-                     int32_t dtype, void* stream);
+                     const float* norm_weight, const float* norm_bias, void* out, int32_t n,
+                     int32_t width, int32_t norm_width, float eps, float weight_offset,
+                     float norm_alpha, float out_scale, int32_t dtype, void* stream);
 
 /* z > 0: alpha_p z^2 + z / 2;  z <= 0: alpha_n (exp(z) - 1 - z) + z / 2.  count % 8 == 0. */
 int zp_xielu(const void* in, void* out, int64_t count, float alpha_p, float alpha_n, int32_t dtype,
              void* stream);
+
+/* max(z, 0)^2.  count % 8 == 0. */
+int zp_relu_square(const void* in, void* out, int64_t count, int32_t dtype, void* stream);
 
 /* out (fp32) = cap * tanh(in / cap). */
 int zp_softcap(const void* in, float* out, int64_t count, float cap, int32_t dtype, void* stream);
@@ -46,6 +53,22 @@ int zp_softcap(const void* in, float* out, int64_t count, float cap, int32_t dty
 int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n, int32_t row_bytes,
                    int64_t num_rows, void* stream);
 
+/* What an attention does beyond the softmax of scaled products; NULL stands for {0, 1}.
+ * softcap > 0: scores s (after the scale) enter the softmax as softcap * tanh(s / softcap).
+ * maps 2 (differential attention): a query head holds two queries of D and a key head two keys of D, back to
+ * back; both softmaxes weight the same values, and with their results o1, o2 the output is
+ *   rms(o1 - balance * o2) * out_scale * sigmoid(gate),  rms over the first `vdim` values with eps,
+ * gate (rows gate_stride elements apart, heads of V back to back, of the call's dtype) or NULL: no gate.
+ * Sinks are for one map only. */
+typedef struct {
+  float softcap;
+  int32_t maps;
+  float balance, eps;
+  int32_t vdim;
+  const void* gate;
+  int64_t gate_stride;
+} zp_attention_form;
+
 /* Attention of runs of tokens, bfloat16.  tiles (T, 4) int32, one entry per up to 128 queries of one
  * sequence: first query row, number of queries, row of the run's first key, position of the first
  * query counted from that key (key rows of a run are consecutive positions).  Query head h reads key
@@ -53,64 +76,79 @@ int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n, i
  * `window` (0: no limit) or, with `chunk`, in its own block of `chunk` positions (the run's first key
  * starts a block); at most one of the two is set.  sinks (H,) or NULL: a logit per head that joins the
  * denominator only.  q rows q_stride, k and v rows kv_stride, out rows out_stride elements apart, heads
- * back to back; out is multiplied by out_scale. */
-int zp_run_attention(const void* q, const void* k, const void* v, void* out, const int32_t* tiles,
-                     const float* sinks, int32_t T, int32_t H, int32_t HK, int32_t D, int32_t V,
-                     int32_t window, int32_t chunk, int64_t q_rows, int64_t k_rows, int64_t q_stride,
-                     int64_t kv_stride, int64_t out_stride, float scale, float out_scale,
+ * back to back; out is multiplied by out_scale.  With k_shared (rows shared_stride apart) a query head is
+ * D + P long and its last P elements meet the row of k_shared, whatever the head. */
+int zp_run_attention(const void* q, const void* k, const void* v, const void* k_shared, void* out,
+                     const int32_t* tiles, const float* sinks, const zp_attention_form* form, int32_t T,
+                     int32_t H, int32_t HK, int32_t D, int32_t P, int32_t V, int32_t window,
+                     int32_t chunk, int64_t q_rows, int64_t k_rows, int64_t q_stride, int64_t kv_stride,
+                     int64_t shared_stride, int64_t out_stride, float scale, float out_scale,
                      int32_t dtype, void* stream);
 
 /* ------------------------------------------------------------------ libzipage_latent.so */
 
-/* in (n, q_width + c_width): the first part RMS-normed times q_weight goes to q_out, the second
- * times c_weight to slot slots[i] of the cache (-1 skips) and to c_out when given.  The means run
- * over q_norm and c_norm elements; widths are multiples of 8, zero padded. */
+/* in (n, q_width + c_width + p_width): the first part RMS-normed times q_weight goes to q_out; the second
+ * times c_weight, and behind it the third, of which the first `rot` elements turn by positions[i] * freqs[.]
+ * (j with j + rot / 2), go to slot slots[i] of the cache (-1 skips) and to c_out when given.  The means run
+ * over q_norm and c_norm elements; widths are multiples of 8, zero padded.  c_width and p_width 0: the
+ * first part alone. */
 int zp_latent_norm_store(const void* in, const float* q_weight, const float* c_weight, void* q_out,
-                         void* c_out, void* cache, const int32_t* slots, int32_t n, int32_t q_width,
-                         int32_t c_width, int32_t q_norm, int32_t c_norm, int64_t num_slots, float eps,
-                         int32_t dtype, void* stream);
+                         void* c_out, void* cache, const int32_t* slots, const int32_t* positions,
+                         const float* freqs, int32_t n, int32_t q_width, int32_t c_width,
+                         int32_t p_width, int32_t q_norm, int32_t c_norm, int32_t rot,
+                         int64_t num_slots, float eps, int32_t dtype, void* stream);
 
-/* out[n, h, :] = w[h] (M, K) in[n, h, :]; K a multiple of 32, M of 16. */
-int zp_headwise_linear(const void* in, const void* w, void* out, int32_t n, int32_t H, int32_t K,
-                       int32_t M, int32_t dtype, void* stream);
+/* x[i, h * head + at ...]: `rot` elements turn in place by positions[i] * freqs[.], j with j + rot / 2. */
+int zp_rotate_heads(void* x, const int32_t* positions, const float* freqs, int32_t n, int32_t H,
+                    int32_t head, int32_t at, int32_t rot, int64_t x_stride, int32_t dtype,
+                    void* stream);
 
-/* Attention of single tokens over paged latents.  q (n, H, R); cache (num_pages, BS, R); token i
+/* out[n, h, :M] = w[h] (M, K) in[n, h, :K]; heads of K + tail and M + tail elements.  The tail passes, its
+ * first `rot` elements turned as in zp_rotate_heads.  K a multiple of 32, M of 16, tail of 8. */
+int zp_headwise_linear(const void* in, const void* w, void* out, const int32_t* positions,
+                       const float* freqs, int32_t n, int32_t H, int32_t K, int32_t M, int32_t tail,
+                       int32_t rot, int32_t dtype, void* stream);
+
+/* Attention of single tokens over paged latents.  q (n, H, R + P); cache (num_pages, BS, R + P); token i
  * sees the tokens [max(0, c - window), c) of its sequence, c = context_lens[i] (window 0: all;
  * c = 0: inert, zeros), through row table_rows[i] (NULL: i) of table (B, NB).
- * out[n, h] = sum_j softmax_j(scale * q[n, h] . c_j) c_j.  R a multiple of 32.  `workspace`:
- * zp_latent_rows_workspace() bytes, 16-byte aligned. */
+ * out[n, h] (R) = sum_j softmax_j(scale * q[n, h] . row_j) row_j[:R].  R a multiple of 32, P of 8.
+ * `workspace`: zp_latent_rows_workspace() bytes, 16-byte aligned. */
 int64_t zp_latent_rows_workspace(int32_t n, int32_t H, int32_t R, int32_t window, int32_t NB,
                                  int32_t BS, int32_t dtype);
 int zp_latent_rows_attention(const void* q, const void* cache, const int32_t* table,
                              const int32_t* context_lens, const int32_t* table_rows, void* out,
-                             int32_t n, int32_t H, int32_t R, int32_t BS, int32_t B, int32_t NB,
-                             int32_t num_pages, int32_t window, float scale, int32_t dtype,
+                             int32_t n, int32_t H, int32_t R, int32_t P, int32_t BS, int32_t B,
+                             int32_t NB, int32_t num_pages, int32_t window, float scale, int32_t dtype,
                              void* workspace, int64_t workspace_bytes, void* stream);
 
-/* ------------------------------------------------------------------ libzipage_hybrid.so */
+/* ------------------------------------------------------------------ libzipage_grouped.so */
 
-/* Rows `in` (in_stride elements apart) hold q (H heads of D), k (HK of D), v (HK of V).  The first `rot`
- * dimensions of q's and k's heads turn by positions[i] * freqs[.], dimension j with j + rot / 2.  q goes
- * to q_out, [k | v] to slot slots[i] of the cache (-1 skips) and to kv_out when given. */
-int zp_rotary_store(const void* in, const int32_t* positions, const float* freqs, void* q_out,
-                    void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H, int32_t HK,
-                    int32_t D, int32_t V, int32_t rot, int64_t in_stride, int64_t num_slots,
-                    int32_t dtype, void* stream);
+/* Rows `in` (in_stride elements apart) hold q (H heads of D), k (HK of D) and VT value columns; with `bias`
+ * (a row of them) it is added first.  The first `rot` dimensions of q's and k's heads turn by positions[i] *
+ * freqs[.], dimension j with j + rot / 2.  q goes to q_out, [k | v] to slot slots[i] of the cache (-1
+ * skips) and to kv_out when given. */
+int zp_rotary_store(const void* in, const float* bias, const int32_t* positions, const float* freqs,
+                    void* q_out, void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
+                    int32_t HK, int32_t D, int32_t VT, int32_t rot, int64_t in_stride,
+                    int64_t num_slots, int32_t dtype, void* stream);
 
-/* Attention of single tokens over paged rows [k (HK heads of D) | v (HK of V)].  q (n, H, D); token i is
- * the last of the context_lens[i] tokens of its sequence (0: inert, zeros) in row table_rows[i] (NULL:
- * i) of table (B, NB); window, chunk, sinks, out_stride and out_scale as in zp_run_attention, with
- * blocks counted from position 0.  `workspace`: zp_grouped_rows_workspace() bytes. */
-int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V,
+/* Attention of single tokens over paged rows [k (HK heads of maps * D) | v (HK of V)].  q (n, H, maps * D);
+ * token i is the last of the context_lens[i] tokens of its sequence (0: inert, zeros) in row table_rows[i]
+ * (NULL: i) of table (B, NB); window, chunk, sinks, form, out_stride and out_scale as in zp_run_attention,
+ * with blocks counted from position 0.  `workspace`: zp_grouped_rows_workspace() bytes. */
+int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V, int32_t maps,
                                   int32_t window, int32_t chunk, int32_t NB, int32_t BS,
                                   int32_t dtype);
 int zp_grouped_rows_attention(const void* q, const void* cache, const int32_t* table,
                               const int32_t* context_lens, const int32_t* table_rows,
-                              const float* sinks, void* out, int32_t n, int32_t H, int32_t HK,
-                              int32_t D, int32_t V, int32_t BS, int32_t B, int32_t NB,
-                              int32_t num_pages, int32_t window, int32_t chunk, int64_t out_stride,
-                              float scale, float out_scale, int32_t dtype, void* workspace,
-                              int64_t workspace_bytes, void* stream);
+                              const float* sinks, const zp_attention_form* form, void* out, int32_t n,
+                              int32_t H, int32_t HK, int32_t D, int32_t V, int32_t BS, int32_t B,
+                              int32_t NB, int32_t num_pages, int32_t window, int32_t chunk,
+                              int64_t out_stride, float scale, float out_scale, int32_t dtype,
+                              void* workspace, int64_t workspace_bytes, void* stream);
+
+/* ------------------------------------------------------------------ libzipage_recurrent.so */
 
 /* The runs of tokens a step holds, one per sequence: token rows row .. row + count - 1, the state slot,
  * the position of the first token (0: the state starts at zero).  rows NULL: row i; max_count > 0 caps
@@ -166,15 +204,19 @@ int64_t zp_delta_runs_workspace(int32_t rows, int32_t segments, int32_t heads, i
 int zp_delta_runs(const zp_delta* args, int32_t first_row, int32_t longest, void* workspace,
                   int64_t workspace_bytes, int32_t dtype, void* stream);
 
+/* ------------------------------------------------------------------ libzipage_moe.so */
+
 /* out (n, M) fp32 = x (n, K) w (M, K)^T.  K a multiple of 32, M of 4. */
 int zp_small_linear(const void* x, const void* w, float* out, int32_t n, int32_t K, int32_t M,
                     int64_t x_stride, int32_t dtype, void* stream);
 
-/* Per token: softmax over the E logits, the `keep` of `groups` groups with the largest single score, and
- * the `top` best experts of those: ids and scores (n, top).  counts (E + 1) is cleared for the plan. */
+/* Per token: scores of the E logits (softmax over them, or each one's sigmoid), the `keep` of `groups` groups
+ * with the largest single score, and the `top` best experts of those: ids and scores (n, top).  counts (E +
+ * 1) is cleared for the plan. */
+enum { ZP_SCORE_SOFTMAX = 0, ZP_SCORE_SIGMOID = 1 };
 int zp_moe_select(const float* logits, int32_t* ids, float* weights, int32_t* counts, int32_t n,
-                  int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t logits_stride,
-                  void* stream);
+                  int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t score,
+                  int32_t logits_stride, void* stream);
 
 /* Assignments (token n, slot j), numbered n * (top + shared) + j, in the order of their experts, and the
  * row tiles of the expert products: tiles (max_tiles, 4) of expert, first position in `sorted`, rows.
@@ -189,15 +231,18 @@ int zp_moe_plan(const int32_t* ids, int32_t* counts, int32_t* sorted, int32_t* t
 
 /* Expert products over a plan.  Weights in tile order: [out / 16][in / step][64 lanes][16 bytes], lane (g,
  * r) = 16 g + r holding row r and the g-th 16 bytes of a step of 64 bytes; gate_up interleaves 16
- * rows of the gate with the 16 of `up`.  out of gate_up, by position in `sorted`:
- * weight * g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).  out of
- * down: planes (slots, n, out_stride), an assignment's row in the plane of its slot.  K a multiple
+ * rows of the gate with the 16 of `up`.  out of gate_up, by position in `sorted`, with the assignment's
+ * weight w (1 for the shared expert):
+ *   ZP_GATE_CLAMPED  w g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+ *   ZP_GATE_SILU     g sigmoid(g) u, g = w gate, u = w up: the weight on the expert's input
+ * out of down: planes (slots, n, out_stride), an assignment's row in the plane of its slot.  K a multiple
  * of 32, M of 16 (of 32 where it is a later K). */
+enum { ZP_GATE_CLAMPED = 0, ZP_GATE_SILU = 1 };
 int zp_moe_gate_up(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
                    const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n,
                    int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K,
-                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
-                   float limit_shared, int32_t dtype, void* stream);
+                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, int32_t act,
+                   float limit, float limit_shared, int32_t dtype, void* stream);
 int zp_moe_down(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
                 const int32_t* tiles, const int32_t* ntiles, int32_t n, int32_t E, int32_t top,
                 int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared,

@@ -44,17 +44,23 @@ def test_models_library_exports_every_declared_symbol():
             assert hasattr(lib, name), f"{name} declared in the header but not exported"
     lib = _lib.load_models("latent")
     # bad arguments are refused on the host, before any launch
-    assert lib.zp_headwise_linear(None, None, None, 1, 2, 33, 16, 0, None) != 0
-    assert b"multiple of 32" in lib.zp_last_error()
-    assert lib.zp_latent_rows_attention(None, None, None, None, None, None, 1, 1, 32, 16, 1, 1, 1, -1, 1.0, 0,
+    assert lib.zp_headwise_linear(None, None, None, None, None, 1, 2, 33, 16, 0, 0, 0, None) != 0
+    assert b"multiples of 32" in lib.zp_last_error()
+    assert lib.zp_latent_rows_attention(None, None, None, None, None, None, 1, 1, 32, 0, 16, 1, 1, 1, -1, 1.0, 0,
                                         None, 0, None) == 1
     lib = _lib.load_models("models")
-    assert lib.zp_embed_norm(None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1.0, 1e-6, 0.0, 0, None) != 0
-    assert lib.zp_run_attention(None, None, None, None, None, None, 1, 4, 3, 32, 32, 0, 0, 1, 1, 128, 256, 128, 1.0, 1.0,
-                                0, None) == 1
-    lib = _lib.load_models("hybrid")
-    assert lib.zp_moe_select(None, None, None, None, 1, 12, 5, 3, 1, 12, None) == 1      # five of a group of four
+    assert lib.zp_embed_norm(None, None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1.0, 1e-6, 0.0, 0.0, 0, None) != 0
+    assert lib.zp_run_attention(None, None, None, None, None, None, None, None, 1, 4, 3, 32, 0, 32, 0, 0, 1, 1, 128, 256, 0,
+                                128, 1.0, 1.0, 0, None) == 1
+    lib = _lib.load_models("grouped")
+    two = _lib.AttentionForm(0.0, 2, 0.5, 1e-6, 0, None, 0)                              # a mean over nothing
+    assert lib.zp_grouped_rows_attention(1, 1, 1, 1, 1, None, ctypes.byref(two), 1, 1, 2, 2, 32, 32, 16, 1, 1, 1, 0, 0,
+                                         64, 1.0, 1.0, 0, None, 0, None) == 1
+    assert b"mean over the values" in lib.zp_last_error()
+    lib = _lib.load_models("moe")
+    assert lib.zp_moe_select(None, None, None, None, 1, 12, 5, 3, 1, 0, 12, None) == 1      # five of a group of four
     assert lib.zp_small_linear(None, None, None, 1, 40, 4, 40, 0, None) != 0
+    lib = _lib.load_models("recurrent")
     bad = _lib.MlstmArgs(heads=2, dk=48, dv=32, vdim=32, cap=1.0, gate_stride=4, out_stride=64,
                          seg=_lib.Segments(n=1, num_slots=1, num_rows=1))
     assert lib.zp_mlstm_scan(ctypes.byref(bad), 0, None) != 0 and b"48" in lib.zp_last_error()

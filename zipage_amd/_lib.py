@@ -109,43 +109,59 @@ class DeltaArgs(C.Structure):
         [(n, f32) for n in ("q_scale", "eps", "out_scale")]
 
 
+class AttentionForm(C.Structure):
+    """zp_attention_form."""
+    _fields_ = [("softcap", f32), ("maps", i32), ("balance", f32), ("eps", f32), ("vdim", i32), ("gate", ptr),
+                ("gate_stride", i64)]
+
+
+SCORE_SOFTMAX, SCORE_SIGMOID = 0, 1      # ZP_SCORE_*
+GATE_CLAMPED, GATE_SILU = 0, 1           # ZP_GATE_*
+form_ptr = C.POINTER(AttentionForm)
+
 # the model-side libraries, in the order of include/zipage_models.h: name -> (entry points, those that
 # return an int64 count instead of a status)
 MODEL_LIBS = {
     "models": ({
-        "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, i32, ptr],
-        "zp_residual_norm": [ptr, ptr, i32, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32,
-                             f32, i32, ptr],
+        "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, f32, i32, ptr],
+        "zp_residual_norm": [ptr, ptr, i32, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32,
+                             f32, f32, i32, ptr],
         "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
+        "zp_relu_square": [ptr, ptr, i64, i32, ptr],
         "zp_softcap": [ptr, ptr, i64, f32, i32, ptr],
         "zp_gather_rows": [ptr, ptr, ptr, i32, i32, i64, ptr],
-        "zp_run_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i64, i64, i64, i64,
-                             i64, f32, f32, i32, ptr],
+        "zp_run_attention": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, form_ptr, i32, i32, i32, i32, i32, i32, i32, i32, i64,
+                             i64, i64, i64, i64, i64, f32, f32, i32, ptr],
     }, {}),
     "latent": ({
-        "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, f32, i32, ptr],
-        "zp_headwise_linear": [ptr, ptr, ptr, i32, i32, i32, i32, i32, ptr],
-        "zp_latent_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, f32,
+        "zp_latent_norm_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i64,
+                                 f32, i32, ptr],
+        "zp_rotate_heads": [ptr, ptr, ptr, i32, i32, i32, i32, i32, i64, i32, ptr],
+        "zp_headwise_linear": [ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, ptr],
+        "zp_latent_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, f32,
                                      i32, ptr, i64, ptr],
     }, {"zp_latent_rows_workspace": [i32, i32, i32, i32, i32, i32, i32]}),
-    "hybrid": ({
-        "zp_rotary_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i64, i64, i32, ptr],
-        "zp_grouped_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32,
-                                      i32, i32, i32, i64, f32, f32, i32, ptr, i64, ptr],
+    "grouped": ({
+        "zp_rotary_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i64, i64, i32, ptr],
+        "zp_grouped_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, form_ptr, ptr, i32, i32, i32, i32, i32, i32, i32,
+                                      i32, i32, i32, i32, i64, f32, f32, i32, ptr, i64, ptr],
+    }, {"zp_grouped_rows_workspace": [i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32]}),
+    "recurrent": ({
         "zp_mlstm_scan": [C.POINTER(MlstmArgs), i32, ptr],
         "zp_mlstm_runs": [C.POINTER(MlstmArgs), i32, i32, ptr, i64, i32, ptr],
         "zp_delta_scan": [C.POINTER(DeltaArgs), i32, ptr],
         "zp_delta_runs": [C.POINTER(DeltaArgs), i32, i32, ptr, i64, i32, ptr],
+    }, {"zp_mlstm_runs_workspace": [i32, i32, i32], "zp_delta_runs_workspace": [i32, i32, i32, i32, i32]}),
+    "moe": ({
         "zp_small_linear": [ptr, ptr, ptr, i32, i32, i32, i64, i32, ptr],
-        "zp_moe_select": [ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, ptr],
+        "zp_moe_select": [ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, ptr],
         "zp_moe_plan": [ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, ptr, i64, ptr],
         "zp_moe_gate_up": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, i64,
-                           i64, f32, f32, i32, ptr],
+                           i64, i32, f32, f32, i32, ptr],
         "zp_moe_down": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, i32, i32, i64, i64, i32,
                         ptr],
-    }, {"zp_grouped_rows_workspace": [i32, i32, i32, i32, i32, i32, i32, i32, i32, i32],
-        "zp_mlstm_runs_workspace": [i32, i32, i32], "zp_delta_runs_workspace": [i32, i32, i32, i32, i32], "zp_moe_tile_rows": [i32, i32, i32, i32],
-        "zp_moe_max_tiles": [i32, i32, i32, i32, i32], "zp_moe_plan_workspace": [i32, i32, i32]}),
+    }, {"zp_moe_tile_rows": [i32, i32, i32, i32], "zp_moe_max_tiles": [i32, i32, i32, i32, i32],
+        "zp_moe_plan_workspace": [i32, i32, i32]}),
 }
 MODEL_EXPORTS = {lib: sorted([*calls, *sizes]) for lib, (calls, sizes) in MODEL_LIBS.items()}
 _LIB_OF = {name: lib for lib, (calls, _) in MODEL_LIBS.items() for name in calls}

@@ -2,8 +2,9 @@
 
 Run as ``python -m zipage_amd.build``.  Shared objects with a plain C ABI, none linked against
 torch: ``libzipage_hip.so`` (``include/zipage_hip.h``: the compression path and the kernels of the
-models that use it) and, for the other models, ``libzipage_models.so``, ``libzipage_latent.so`` and
-``libzipage_hybrid.so`` (``include/zipage_models.h``), so that a model compiles only what it runs.
+models that use it) and, for the other models, ``libzipage_models.so``, ``libzipage_latent.so``,
+``libzipage_grouped.so``, ``libzipage_recurrent.so`` and ``libzipage_moe.so``
+(``include/zipage_models.h``), so that a model compiles only what it runs.
 """
 from __future__ import annotations
 
@@ -17,7 +18,9 @@ CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libzipage_hip.so")
 MODELS_LIB = os.path.join(HERE, "libzipage_models.so")
 LATENT_LIB = os.path.join(HERE, "libzipage_latent.so")
-HYBRID_LIB = os.path.join(HERE, "libzipage_hybrid.so")
+GROUPED_LIB = os.path.join(HERE, "libzipage_grouped.so")
+RECURRENT_LIB = os.path.join(HERE, "libzipage_recurrent.so")
+MOE_LIB = os.path.join(HERE, "libzipage_moe.so")
 
 # packed fp32 VALU ops are disabled on purpose (some forms misbehave on this fleet)
 BASE_FLAGS = [
@@ -32,8 +35,9 @@ FLAGS = BASE_FLAGS + ["-ffp-contract=off"]
 MODEL_SOURCES = {
     MODELS_LIB: ("residual.hip", "runs.hip"),
     LATENT_LIB: ("latent.hip",),
-    HYBRID_LIB: ("grouped.hip", "mlstm.hip", "mlstm_runs.hip", "delta.hip", "delta_runs.hip",
-                 "moe.hip"),
+    GROUPED_LIB: ("grouped.hip",),
+    RECURRENT_LIB: ("mlstm.hip", "mlstm_runs.hip", "delta.hip", "delta_runs.hip"),
+    MOE_LIB: ("moe.hip",),
 }
 COMMON_SOURCES = ("runtime.hip",)
 LIBS = (LIB, *MODEL_SOURCES)

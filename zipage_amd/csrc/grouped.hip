@@ -7,21 +7,24 @@
 //
 // Attention of runs of prompt tokens is run_attention (runs.hip).  A token sees a window, its own
 // block of positions, or everything before it; a sink is a logit per head that joins the softmax's
-// denominator only.
+// denominator only.  A head may hold two maps over the same values (differential attention): in
+// grouped_rows they are two query columns of a key head of twice the length, each with zeros where the
+// other one's elements are, so that keys and values are still read once.
 #include "mfma.h"
 
 namespace {
 
 // ------------------------------------------------------------------ rotary positions and the store
 struct RotaryArgs {
-  const void* in;           // token rows of in_st elements: q (H * D), k (HK * D), v (HK * V)
+  const void* in;           // token rows of in_st elements: q (H * D), k (HK * D), v (VT)
+  const float* bias;        // the same row, added before the turn; or null
   const int32_t* positions;
   const float* freqs;       // (rot / 2,)
   void* q_out;              // (n, H * D)
-  void* kv_out;             // (n, HK * (D + V)) or null
-  void* cache;              // (num_slots, HK * (D + V))
+  void* kv_out;             // (n, HK * D + VT) or null
+  void* cache;              // (num_slots, HK * D + VT)
   const int32_t* slots;     // (n,), -1 skips
-  int n, H, HK, D, V, half; // half = rotated dimensions / 2
+  int n, H, HK, D, VT, half; // half = rotated dimensions / 2
   int64_t in_st, num_slots;
 };
 constexpr int kRotTokens = 4;
@@ -36,22 +39,27 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
   for (int i = tid; i < kRotTokens * a.half; i += 256) {
     const int tok = i / a.half;
     if (n0 + tok < a.n) {
-      float s, c;
-      sincosf((float)a.positions[n0 + tok] * a.freqs[i - tok * a.half], &s, &c);
-      cs[i] = make_float2(c, s);
+      cs[i] = rotary_turn(a.positions[n0 + tok], a.freqs[i - tok * a.half]);
     }
   }
   __syncthreads();
   const int pairs = a.half / VEC, per_head = (a.D - a.half) / VEC;
-  const int heads = a.H + a.HK, rotated = heads * per_head, items = rotated + a.HK * a.V / VEC;
-  const int kvw = a.HK * (a.D + a.V);
+  const int heads = a.H + a.HK, rotated = heads * per_head, items = rotated + a.VT / VEC;
+  const int kvw = a.HK * a.D + a.VT;
   for (int id = tid; id < kRotTokens * items; id += 256) {
     const int tok = id / items, it = id - tok * items;
     const int64_t row = n0 + tok;
     if (row >= a.n) break;
     float x[VEC], y[VEC];
-    auto load = [&](int64_t at, float* o) {
+    auto load = [&](int c, float* o) {
+      const int64_t at = row * a.in_st + c;
       if constexpr (VEC == 8) Vec8<T>::ld(a.in, at, o); else o[0] = Elem<T>::ld(a.in, at);
+      if (a.bias) {
+        float b[VEC];
+        if constexpr (VEC == 8) Vec8<F32>::ld(a.bias, c, b); else b[0] = a.bias[c];
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) o[i] += b[i];
+      }
     };
     int64_t slot = a.slots[row];
     if (slot >= a.num_slots) slot = -1;
@@ -73,20 +81,20 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
     };
     if (it >= rotated) {
       const int c = heads * a.D + (it - rotated) * VEC;
-      load(row * a.in_st + c, x);
+      load(c, x);
       put(c, x);
       continue;
     }
     const int h = it / per_head, p = it - h * per_head;
     if (p >= pairs) {                          // dimensions behind the rotated ones
       const int c = h * a.D + (p + pairs) * VEC;
-      load(row * a.in_st + c, x);
+      load(c, x);
       put(c, x);
       continue;
     }
     const int c = h * a.D + p * VEC;
-    load(row * a.in_st + c, x);
-    load(row * a.in_st + c + a.half, y);
+    load(c, x);
+    load(c + a.half, y);
 #pragma unroll
     for (int i = 0; i < VEC; ++i) {
       const float2 r = cs[tok * a.half + p * VEC + i];
@@ -101,7 +109,7 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
 
 // ------------------------------------------------------------------ single tokens over the pages
 struct RowsArgs {
-  const void* q;          // (n, H * D)
+  const void* q;          // (n, H * D / maps)
   const void* cache;      // (pages, BS, HK * (D + V))
   const int32_t* table;   // (B, NB) page ids
   const int32_t* ctx;     // (n,) tokens of the sequence up to and including this one; 0 = inert
@@ -109,13 +117,32 @@ struct RowsArgs {
   const float* sinks;     // (H,) or null
   void* out;              // token rows of o_st elements, head h at h * V
   float* part;            // splits > 1: (n, H, splits, V) fp32, then (n, H, splits, 2) max and sum
-  int n, H, HK, D, V, BS, bs_shift, B, NB, num_pages;
+  int n, H, HK, D, V, BS, bs_shift, B, NB, num_pages;   // H counts the maps of a head, D is a key head's length
   int window, chunk;
   int splits, htiles;     // key ranges, and tiles of 16 query heads per key head
   int lds_pages;
   int64_t o_st;
   float scale, out_scale;
+  float cap;              // > 0: soft cap of the scores
+  // two maps: rms(o1 - balance * o2) * out_scale * sigmoid(gate), the mean over vdim
+  float balance, eps;
+  int vdim;
+  const void* gate;       // token rows of g_st elements, head h at h * V; or null
+  int64_t g_st;
 };
+
+// A piece of a head's result, normed: scale and gate it, and store it.
+template <typename T> __device__ __forceinline__ void store_gated(const RowsArgs& a, int64_t row, int head, int c, float* r, float scale) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) r[i] *= scale;
+  if (a.gate) {
+    float z[8];
+    Vec8<T>::ld(a.gate, row * a.g_st + (int64_t)head * a.V + c, z);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) r[i] *= sigmoid_of<T>(z[i]);
+  }
+  Vec8<T>::st(a.out, row * a.o_st + (int64_t)head * a.V + c, r);
+}
 
 __device__ __forceinline__ int first_key(const RowsArgs& a, int n) {   // n tokens, the last one asks
   if (a.window > 0) return max(0, n - a.window);
@@ -127,7 +154,7 @@ __device__ __forceinline__ int first_key(const RowsArgs& a, int n) {   // n toke
 // row operand straight from memory (64-byte pieces), values are loaded as rows and turned into column
 // operands by v_perm.  The next step's keys are requested once the scores are done, its values once the
 // value products are.
-template <int DKS, int VCB>
+template <int DKS, int VCB, int MAPS>
 __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
   int* const pg = (int*)lds_raw;
@@ -149,15 +176,18 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
     const int p = p0 + j < a.NB ? a.table[(int64_t)seq * a.NB + p0 + j] : 0;
     pg[j] = (p >= 0 && p < a.num_pages) ? p : 0;
   }
-  const int nks = a.D / 32;
-  const int head = hk * G + min(ht * 16 + l16, G - 1);
+  const int head = hk * G + min(ht * 16 + l16, G - 1), qd = a.D / MAPS;
   u32x4 qf[DKS];
-  const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + head) * a.D + g * 8;
+  const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * a.H + head) * qd;
 #pragma unroll
   for (int ks = 0; ks < DKS; ++ks) {
-    qf[ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
-    if (ks >= nks) qf[ks] = u32x4{0u, 0u, 0u, 0u};
+    const int c = ks * 32 + g * 8 - (MAPS == 2 ? (head & 1) * qd : 0);     // element of this map
+    const bool own = c >= 0 && c < qd;
+    qf[ks] = *(const u32x4*)(q + (own ? c : 0));
+    if (!own) qf[ks] = u32x4{0u, 0u, 0u, 0u};
   }
+  // key columns past the head's end repeat its start, against zeros in q
+  const int nks = a.D / 32, past = -g * 8, tail = nks * 32 + g * 8 < a.D ? nks * 32 : past;
   __syncthreads();
   const int kvw = a.HK * (a.D + a.V), mask = a.BS - 1;
   const uint16_t* const kc = (const uint16_t*)a.cache + hk * a.D + g * 8;
@@ -180,7 +210,7 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
     for (int tt = 0; tt < 2; ++tt) {
       const uint16_t* k = kc + row_at(b * 32 + tt * 16 + l16);
 #pragma unroll
-      for (int ks = 0; ks < DKS; ++ks) kf[tt][ks] = *(const u32x4*)(k + (ks < nks ? ks * 32 : 0));
+      for (int ks = 0; ks < DKS; ++ks) kf[tt][ks] = *(const u32x4*)(k + (ks < nks ? ks * 32 : (ks == nks ? tail : past)));
     }
   };
   auto load_values = [&](int b) {
@@ -195,7 +225,8 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
 #pragma unroll
   for (int i = 0; i < VCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  const float sc = a.scale * 1.44269504088896f;
+  const float sc = a.cap > 0.f ? a.scale / a.cap : a.scale * 1.44269504088896f;
+  const float capl2 = a.cap * 1.44269504088896f;
   const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = 4 * a.splits;
   int b = (lo >> 5) + split * 4 + wave;
   if (b <= b1) {
@@ -216,7 +247,9 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int key = k0 + step_key(g, i);
-      p[i] = key < lo || key >= n ? -INFINITY : s[i >> 2][i & 3] * sc;
+      p[i] = s[i >> 2][i & 3] * sc;
+      if (a.cap > 0.f) p[i] = capl2 * fast_tanh(p[i]);
+      if (key < lo || key >= n) p[i] = -INFINITY;
       mx = fmaxf(mx, p[i]);
     }
     mx = fmaxf(mx, lane_xor16(mx));
@@ -278,12 +311,35 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
       ml[1] = sum;
     } else {
       if (a.sinks && mx != -INFINITY) sum += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - ms);
-      inv = sum > 0.f ? a.out_scale / sum : 0.f;
+      inv = sum > 0.f ? (MAPS == 1 ? a.out_scale : 1.f) / sum : 0.f;
     }
 #pragma unroll
     for (int k = 0; k < 4; ++k) src[k * per] = f[k] * inv;
   }
   __syncthreads();
+  if (MAPS == 2 && a.splits == 1) {              // a wave per head, a lane per eight columns
+    for (int pr = wave; pr < 8 && ht * 16 + 2 * pr < G; pr += 4) {
+      const int c = lane * 8;
+      float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, ss = 0.f;
+      if (c < a.V) {
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {            // four waves' parts of the two maps
+          const float* part = merge + (k >> 1) * per;
+          const int hl = 2 * pr + (k & 1);
+          const float f = part[16 * RS + hl] * ((k & 1) ? -a.balance : 1.f);
+          float x[8];
+          Vec8<F32>::ld(part, hl * RS + c, x);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += r[i] * r[i];
+      }
+      ss = wave_sum(ss);
+      if (c < a.V) store_gated<BF16>(a, row, (hk * G + ht * 16) / 2 + pr, c, r, a.out_scale / sqrtf(ss / (float)a.vdim + a.eps));
+    }
+    return;
+  }
   for (int it = tid; it < 16 * (a.V / 8); it += 256) {
     const int hl = it / (a.V / 8), c = (it - hl * (a.V / 8)) * 8;
     if (ht * 16 + hl >= G) continue;
@@ -328,19 +384,46 @@ __global__ __launch_bounds__(64) void grouped_combine_kernel(RowsArgs a) {
   }
 }
 
-// One workgroup per (token, query head), plain fp32 arithmetic.
-template <typename T>
+// The two maps of a head (V <= 512).
+__global__ __launch_bounds__(64) void grouped_pair_combine_kernel(RowsArgs a) {
+  const int heads = a.H / 2, row = blockIdx.x / heads, head = blockIdx.x - row * heads;
+  const int c = threadIdx.x * 8;
+  float r[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, ss = 0.f;
+  for (int map = 0; map < 2; ++map) {
+    const int64_t item = (int64_t)row * a.H + head * 2 + map;
+    const float* ml = a.part + (int64_t)a.n * a.H * a.splits * a.V + item * a.splits * 2;
+    float mx = -INFINITY, l = 0.f;
+    for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ml[2 * s]);
+    if (mx == -INFINITY) mx = 0.f;
+    for (int s = 0; s < a.splits; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - mx);
+    const float inv = l > 0.f ? (map ? -a.balance : 1.f) / l : 0.f;
+    if (c < a.V)
+      for (int s = 0; s < a.splits; ++s) {
+        const float f = __builtin_amdgcn_exp2f(ml[2 * s] - mx) * inv;
+        float v[8];
+        Vec8<F32>::ld(a.part, (item * a.splits + s) * a.V + c, v);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) r[i] += v[i] * f;
+      }
+  }
+#pragma unroll
+  for (int i = 0; i < 8; ++i) ss += r[i] * r[i];
+  ss = wave_sum(ss);
+  if (c < a.V) store_gated<BF16>(a, row, head, c, r, a.out_scale / sqrtf(ss / (float)a.vdim + a.eps));
+}
+
+// One workgroup per (token, head), plain fp32 arithmetic; two maps one after the other.
+template <typename T, int MAPS>
 __global__ __launch_bounds__(256) void grouped_plain_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
   float* q = (float*)lds_raw;              // D
   __shared__ float sc[256];
   __shared__ float red[4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, hk = h / (a.H / a.HK);
+  const int heads = a.H / MAPS, row = blockIdx.x / heads, h = blockIdx.x - row * heads, hk = h / (heads / a.HK);
   const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
-  const int n = min(a.ctx[row], a.NB * a.BS);
+  const int n = min(a.ctx[row], a.NB * a.BS), qd = a.D / MAPS;
   const int lo = first_key(a, n);
-  for (int c = tid; c < a.D; c += 256) q[c] = Elem<T>::ld(a.q, (int64_t)blockIdx.x * a.D + c);
   const int64_t kvw = (int64_t)a.HK * (a.D + a.V);
   auto key_at = [&](int t) -> int64_t {
     const int p = a.bs_shift >= 0 ? t >> a.bs_shift : t / a.BS;
@@ -349,52 +432,75 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(RowsArgs a) {
     return ((int64_t)page * a.BS + (t - p * a.BS)) * kvw;
   };
   constexpr int kCols = 4;                 // columns per thread: V <= 1024
-  float o[kCols] = {0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  for (int c0 = lo; c0 < n; c0 += 256) {
-    const int cnt = min(256, n - c0);
-    __syncthreads();                       // q is there; the last chunk's scores are used up
-    for (int j = wave; j < cnt; j += 4) {
-      const int64_t at = key_at(c0 + j) + hk * a.D;
-      float acc = 0.f;
-      for (int c = lane; c < a.D; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
-      acc = wave_sum(acc);
-      if (lane == 0) sc[j] = acc * a.scale;
-    }
-    __syncthreads();
-    float mx = tid < cnt ? sc[tid] : -INFINITY;
-    mx = wave_max(mx);
-    if (lane == 0) red[wave] = mx;
-    __syncthreads();
-    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
-    const float mn = fmaxf(m, mx);
-    const float f = expf(m - mn);
-    __syncthreads();
-    const float p = tid < cnt ? expf(sc[tid] - mn) : 0.f;
-    sc[tid] = p;
-    const float s = wave_sum(p);
-    if (lane == 0) red[wave] = s;
-    __syncthreads();
-    l = l * f + red[0] + red[1] + red[2] + red[3];
-    m = mn;
+  float total[kCols] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 1
+  for (int map = 0; map < MAPS; ++map) {
+    __syncthreads();                       // the map before is done with q and its scores
+    for (int c = tid; c < qd; c += 256) q[c] = Elem<T>::ld(a.q, ((int64_t)blockIdx.x * MAPS + map) * qd + c);
+    float o[kCols] = {0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;
+    for (int c0 = lo; c0 < n; c0 += 256) {
+      const int cnt = min(256, n - c0);
+      __syncthreads();                     // q is there; the last chunk's scores are used up
+      for (int j = wave; j < cnt; j += 4) {
+        const int64_t at = key_at(c0 + j) + hk * a.D + map * qd;
+        float acc = 0.f;
+        for (int c = lane; c < qd; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
+        acc = wave_sum(acc) * a.scale;
+        if (a.cap > 0.f) acc = a.cap * tanhf(acc / a.cap);
+        if (lane == 0) sc[j] = acc;
+      }
+      __syncthreads();
+      float mx = tid < cnt ? sc[tid] : -INFINITY;
+      mx = wave_max(mx);
+      if (lane == 0) red[wave] = mx;
+      __syncthreads();
+      mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+      const float mn = fmaxf(m, mx);
+      const float f = expf(m - mn);
+      __syncthreads();
+      const float p = tid < cnt ? expf(sc[tid] - mn) : 0.f;
+      sc[tid] = p;
+      const float s = wave_sum(p);
+      if (lane == 0) red[wave] = s;
+      __syncthreads();
+      l = l * f + red[0] + red[1] + red[2] + red[3];
+      m = mn;
 #pragma unroll
-    for (int i = 0; i < kCols; ++i) o[i] *= f;
-    for (int j = 0; j < cnt; ++j) {
-      const int64_t at = key_at(c0 + j) + a.HK * a.D + hk * a.V;
-      const float pj = sc[j];
+      for (int i = 0; i < kCols; ++i) o[i] *= f;
+      for (int j = 0; j < cnt; ++j) {
+        const int64_t at = key_at(c0 + j) + a.HK * a.D + hk * a.V;
+        const float pj = sc[j];
 #pragma unroll
-      for (int i = 0; i < kCols; ++i) {
-        const int c = tid + i * 256;
-        if (c < a.V) o[i] = fmaf(pj, Elem<T>::ld(a.cache, at + c), o[i]);
+        for (int i = 0; i < kCols; ++i) {
+          const int c = tid + i * 256;
+          if (c < a.V) o[i] = fmaf(pj, Elem<T>::ld(a.cache, at + c), o[i]);
+        }
       }
     }
+    if (MAPS == 1 && a.sinks && n > 0) l += expf(a.sinks[h] - m);
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+    for (int i = 0; i < kCols; ++i) total[i] += o[i] * inv * (map ? -a.balance : 1.f);
   }
-  if (a.sinks && n > 0) l += expf(a.sinks[h] - m);
-  const float inv = l > 0.f ? a.out_scale / l : 0.f;
+  float scale = a.out_scale;
+  if constexpr (MAPS == 2) {
+    float ss = 0.f;                        // columns past V are zero
+#pragma unroll
+    for (int i = 0; i < kCols; ++i) ss += total[i] * total[i];
+    ss = wave_sum(ss);
+    __syncthreads();
+    if (lane == 0) red[wave] = ss;
+    __syncthreads();
+    scale /= sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.vdim + a.eps);
+  }
 #pragma unroll
   for (int i = 0; i < kCols; ++i) {
     const int c = tid + i * 256;
-    if (c < a.V) Elem<T>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, o[i] * inv);
+    if (c >= a.V) continue;
+    float r = total[i] * scale;
+    if (MAPS == 2 && a.gate) r *= sigmoid_of<T>(Elem<T>::ld(a.gate, row * a.g_st + (int64_t)h * a.V + c));
+    Elem<T>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, r);
   }
 }
 
@@ -413,41 +519,52 @@ int rows_splits(int n, int H, int HK, int window, int chunk, int NB, int BS) {
   return s < 1 ? 1 : s;
 }
 
-template <int DKS, int VCB> int launch_rows(const RowsArgs& a, hipStream_t st) {
+template <int DKS, int VCB, int MAPS> int launch_rows(const RowsArgs& a, hipStream_t st) {
   const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + 4 * sizeof(float) * (16 * (a.V + 4) + 32);
   if (smem > 64 * 1024 &&
-      hipFuncSetAttribute((const void*)grouped_rows_kernel<DKS, VCB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+      hipFuncSetAttribute((const void*)grouped_rows_kernel<DKS, VCB, MAPS>, hipFuncAttributeMaxDynamicSharedMemorySize,
                           (int)smem) != hipSuccess) {
     zp_set_error("grouped_rows_attention: cannot reserve %zu bytes of LDS", smem);
     return ZP_EHIP;
   }
-  hipLaunchKernelGGL((grouped_rows_kernel<DKS, VCB>), dim3((unsigned)a.n * a.HK * a.htiles * a.splits), dim3(256), smem, st, a);
+  hipLaunchKernelGGL((grouped_rows_kernel<DKS, VCB, MAPS>), dim3((unsigned)a.n * a.HK * a.htiles * a.splits), dim3(256), smem, st, a);
   ZP_LAUNCH_CHECK();
   if (a.splits > 1) {
-    hipLaunchKernelGGL(grouped_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
+    if (MAPS == 2) hipLaunchKernelGGL(grouped_pair_combine_kernel, dim3((unsigned)a.n * a.H / 2), dim3(64), 0, st, a);
+    else hipLaunchKernelGGL(grouped_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
     ZP_LAUNCH_CHECK();
   }
   return ZP_OK;
 }
+template <int MAPS> int dispatch_rows(const RowsArgs& a, hipStream_t st) {
+  const int dk = (a.D + 31) / 32;
+  if (a.V <= 128) {
+    if (dk <= 2) return launch_rows<2, 1, MAPS>(a, st);
+    if (dk <= 4) return launch_rows<4, 1, MAPS>(a, st);
+    return launch_rows<8, 1, MAPS>(a, st);
+  }
+  if (dk <= 4) return launch_rows<4, 2, MAPS>(a, st);
+  return launch_rows<8, 2, MAPS>(a, st);
+}
 
 }  // namespace
 
-extern "C" int zp_rotary_store(const void* in, const int32_t* positions, const float* freqs, void* q_out,
-                               void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
-                               int32_t HK, int32_t D, int32_t V, int32_t rot, int64_t in_stride,
+extern "C" int zp_rotary_store(const void* in, const float* bias, const int32_t* positions, const float* freqs,
+                               void* q_out, void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
+                               int32_t HK, int32_t D, int32_t VT, int32_t rot, int64_t in_stride,
                                int64_t num_slots, int32_t dtype, void* stream) {
-  ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && D > 0 && V > 0 && rot >= 0 && rot % 2 == 0 && rot <= D && num_slots > 0 &&
-                 in_stride >= (int64_t)H * D + (int64_t)HK * (D + V), "rotary_store: bad dims");
+  ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && D > 0 && VT > 0 && rot >= 0 && rot % 2 == 0 && rot <= D && num_slots > 0 &&
+                 in_stride >= (int64_t)(H + HK) * D + VT, "rotary_store: bad dims");
   ZP_MODEL_DTYPE("rotary_store");
-  if (D % 8 != 0 || V % 8 != 0 || in_stride % 8 != 0 || rot > 2048) {
-    zp_set_error("rotary_store: head sizes %d, %d (multiples of 8), %d rotated (<= 2048)", D, V, rot);
+  if (D % 8 != 0 || VT % 8 != 0 || in_stride % 8 != 0 || rot > 2048) {
+    zp_set_error("rotary_store: head size %d, value columns %d (multiples of 8), %d rotated (<= 2048)", D, VT, rot);
     return ZP_EUNSUPPORTED;
   }
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(in && positions && q_out && cache && slots && (rot == 0 || freqs), "rotary_store: null pointer");
-  ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache),
+  ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache) && aligned16(bias),
              "rotary_store: tensors must be 16-byte aligned");
-  RotaryArgs a = {in, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, V, rot / 2, in_stride, num_slots};
+  RotaryArgs a = {in, bias, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, VT, rot / 2, in_stride, num_slots};
   const unsigned grid = (unsigned)((n + kRotTokens - 1) / kRotTokens);
   const size_t smem = sizeof(float2) * kRotTokens * (rot / 2);
   hipStream_t st = (hipStream_t)stream;
@@ -462,28 +579,32 @@ extern "C" int zp_rotary_store(const void* in, const int32_t* positions, const f
   return ZP_OK;
 }
 
+// D: length of a key head, all its maps together
 static bool rows_need_plain(int D, int V, int BS, int dtype) {
-  return dtype == ZP_F32 || D > 256 || V > 256 || D % 32 != 0 || BS < 16 || (BS & (BS - 1)) != 0;
+  return dtype == ZP_F32 || D > 256 || V > 256 || BS < 16 || (BS & (BS - 1)) != 0;
 }
 
-extern "C" int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V,
+extern "C" int64_t zp_grouped_rows_workspace(int32_t n, int32_t H, int32_t HK, int32_t D, int32_t V, int32_t maps,
                                              int32_t window, int32_t chunk, int32_t NB, int32_t BS,
                                              int32_t dtype) {
-  if (n < 0 || H <= 0 || HK <= 0 || H % HK || V <= 0 || NB <= 0 || BS <= 0) return -1;
-  if (rows_need_plain(D, V, BS, dtype)) return 0;
-  const int s = rows_splits(n, H, HK, window, chunk, NB, BS);
-  return s == 1 ? 0 : (int64_t)n * H * s * (V + 2) * 4;
+  if (n < 0 || H <= 0 || HK <= 0 || H % HK || V <= 0 || NB <= 0 || BS <= 0 || (maps != 1 && maps != 2)) return -1;
+  if (rows_need_plain(D * maps, V, BS, dtype)) return 0;
+  const int s = rows_splits(n, H * maps, HK, window, chunk, NB, BS);
+  return s == 1 ? 0 : (int64_t)n * H * maps * s * (V + 2) * 4;
 }
 
 extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const int32_t* table,
                                          const int32_t* context_lens, const int32_t* table_rows,
-                                         const float* sinks, void* out, int32_t n, int32_t H, int32_t HK,
-                                         int32_t D, int32_t V, int32_t BS, int32_t B, int32_t NB,
-                                         int32_t num_pages, int32_t window, int32_t chunk, int64_t out_stride,
-                                         float scale, float out_scale, int32_t dtype, void* workspace,
-                                         int64_t workspace_bytes, void* stream) {
+                                         const float* sinks, const zp_attention_form* form, void* out, int32_t n,
+                                         int32_t H, int32_t HK, int32_t D, int32_t V, int32_t BS, int32_t B,
+                                         int32_t NB, int32_t num_pages, int32_t window, int32_t chunk,
+                                         int64_t out_stride, float scale, float out_scale, int32_t dtype,
+                                         void* workspace, int64_t workspace_bytes, void* stream) {
+  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0}, f = form ? *form : plain;
+  const bool two = f.maps == 2;
   ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && V > 0 && BS > 0 && B > 0 && NB > 0 &&
-                 num_pages > 0 && window >= 0 && chunk >= 0 && !(window && chunk), "grouped_rows_attention: bad dims");
+                 num_pages > 0 && window >= 0 && chunk >= 0 && !(window && chunk) && (f.maps == 1 || two) &&
+                 f.softcap >= 0.f, "grouped_rows_attention: bad dims");
   ZP_MODEL_DTYPE("grouped_rows_attention");
   if (D % 8 != 0 || V % 8 != 0 || V > 1024 || D > 4096) {
     zp_set_error("grouped_rows_attention: head sizes %d, %d unsupported (multiples of 8, <= 4096, <= 1024)", D, V);
@@ -492,39 +613,41 @@ extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(q && cache && table && context_lens && out, "grouped_rows_attention: null pointer");
   ZP_REQUIRE(table_rows || n <= B, "grouped_rows_attention: more tokens than table rows");
-  ZP_REQUIRE(aligned16(q) && aligned16(cache) && aligned16(out) && aligned16(workspace) && out_stride % 8 == 0 &&
-                 out_stride >= (int64_t)H * V, "grouped_rows_attention: tensors must be 16-byte aligned");
+  ZP_REQUIRE(!two || (!sinks && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
+             "grouped_rows_attention: two maps go without sinks, with a mean over the values");
+  ZP_REQUIRE(aligned16(q) && aligned16(cache) && aligned16(out) && aligned16(workspace) && aligned16(f.gate) &&
+                 f.gate_stride % 8 == 0 && out_stride % 8 == 0 && out_stride >= (int64_t)H * V,
+             "grouped_rows_attention: tensors must be 16-byte aligned");
+  const int DK = D * f.maps;
   RowsArgs a = {};
   a.q = q; a.cache = cache; a.table = table; a.ctx = context_lens; a.seq = table_rows; a.sinks = sinks; a.out = out;
-  a.part = (float*)workspace; a.n = n; a.H = H; a.HK = HK; a.D = D; a.V = V; a.BS = BS; a.B = B; a.NB = NB;
+  a.part = (float*)workspace; a.n = n; a.H = H * f.maps; a.HK = HK; a.D = DK; a.V = V; a.BS = BS; a.B = B; a.NB = NB;
   a.num_pages = num_pages; a.window = window; a.chunk = chunk; a.o_st = out_stride; a.scale = scale;
-  a.out_scale = out_scale; a.bs_shift = -1;
+  a.out_scale = out_scale; a.bs_shift = -1; a.cap = f.softcap; a.balance = f.balance; a.eps = f.eps; a.vdim = f.vdim;
+  a.gate = f.gate; a.g_st = f.gate_stride;
   if ((BS & (BS - 1)) == 0)
     for (a.bs_shift = 0; (1 << a.bs_shift) < BS; ++a.bs_shift) {}
   int64_t pages = NB;
   const int seen = window > 0 ? window : chunk;
   if (seen > 0 && (seen - 1) / BS + 2 < pages) pages = (seen - 1) / BS + 2;
   hipStream_t st = (hipStream_t)stream;
-  if (rows_need_plain(D, V, BS, dtype) || pages > kMaxLdsPages) {
+  if (rows_need_plain(DK, V, BS, dtype) || pages > kMaxLdsPages) {
     const size_t smem = sizeof(float) * D;
-    if (dtype == ZP_BF16)
-      hipLaunchKernelGGL((grouped_plain_kernel<BF16>), dim3((unsigned)n * H), dim3(256), smem, st, a);
-    else
-      hipLaunchKernelGGL((grouped_plain_kernel<F32>), dim3((unsigned)n * H), dim3(256), smem, st, a);
+    const dim3 grid((unsigned)n * H);
+#define ZP_PLAIN(T)                                                                              \
+  do {                                                                                           \
+    if (two) hipLaunchKernelGGL((grouped_plain_kernel<T, 2>), grid, dim3(256), smem, st, a);     \
+    else hipLaunchKernelGGL((grouped_plain_kernel<T, 1>), grid, dim3(256), smem, st, a);         \
+  } while (0)
+    if (dtype == ZP_BF16) ZP_PLAIN(BF16); else ZP_PLAIN(F32);
+#undef ZP_PLAIN
     ZP_LAUNCH_CHECK();
     return ZP_OK;
   }
-  a.htiles = (H / HK + 15) / 16;
+  a.htiles = (a.H / HK + 15) / 16;
   a.lds_pages = (int)pages;
-  a.splits = rows_splits(n, H, HK, window, chunk, NB, BS);
-  ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_grouped_rows_workspace(n, H, HK, D, V, window, chunk, NB, BS, dtype)),
+  a.splits = rows_splits(n, a.H, HK, window, chunk, NB, BS);
+  ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_grouped_rows_workspace(n, H, HK, D, V, f.maps, window, chunk, NB, BS, dtype)),
              "grouped_rows_attention: workspace too small");
-  const int dk = D / 32;
-  if (V <= 128) {
-    if (dk <= 2) return launch_rows<2, 1>(a, st);
-    if (dk <= 4) return launch_rows<4, 1>(a, st);
-    return launch_rows<8, 1>(a, st);
-  }
-  if (dk <= 4) return launch_rows<4, 2>(a, st);
-  return launch_rows<8, 2>(a, st);
+  return two ? dispatch_rows<2>(a, st) : dispatch_rows<1>(a, st);
 }

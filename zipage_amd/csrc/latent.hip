@@ -1,10 +1,13 @@
 // Latent attention: keys and values of all heads are linear images of one cached vector c per token
-// (R elements), so the cache holds c alone.
+// (R elements), so the cache holds c alone, or c and a rotated key part (P elements) that all heads share.
 //
-//   latent_norm_store   RMS norms of the two low-rank projections of a token; c goes to its slot
-//   headwise            per-head product out[n, h] = W[h] in[n, h]  (q -> W_uk^T q, sum p c -> W_uv sum p c)
+//   latent_norm_store   RMS norms of the two low-rank projections of a token; c, and the key part turned by
+//                       the token's position, go to its slot
+//   headwise            per-head product out[n, h] = W[h] in[n, h]  (q -> W_uk^T q, sum p c -> W_uv sum p c);
+//                       a tail behind each head's part passes beside it, turned
+//   rotate_heads        rotary positions on a part of every head, in place
 //   latent_rows         attention of single tokens over the paged latents, all heads of a token on
-//                       one read of its context: score = (W_uk^T q) . c, out = sum p c
+//                       one read of its context: score = (W_uk^T q) . c + turned q . turned k, out = sum p c
 //   latent_plain        float32 form of latent_rows (true fp32 products), any sizes
 //
 // The attention of runs of prompt tokens over expanded keys and values is in runs.hip.
@@ -23,30 +26,32 @@ namespace {
 
 // ------------------------------------------------------------------ norms of the low-rank rows
 struct NormStoreArgs {
-  const void* in;        // (n, q_width + c_width) T
+  const void* in;        // (n, q_width + c_width + p_width) T
   const float* wq;       // (q_width,)
   const float* wc;       // (c_width,)
   void* q_out;           // (n, q_width) T
-  void* c_out;           // (n, c_width) T or null
-  void* cache;           // (num_slots, c_width) T
+  void* c_out;           // (n, c_width + p_width) T or null
+  void* cache;           // (num_slots, c_width + p_width) T
   const int32_t* slots;  // (n,), -1 skips
-  int n, q_width, c_width, q_norm, c_norm;
+  const int32_t* positions;
+  const float* freqs;    // (half,)
+  int n, q_width, c_width, p_width, q_norm, c_norm, half;   // half: rotated pairs of the last part
   int64_t num_slots;
   float eps;
 };
 constexpr int kNormPieces = 8;   // 8-element pieces per lane: ranks up to 4096
 
-// One wave per (token, part).
+// One wave per (token, part); without a second part, per token.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_norm_store_kernel(NormStoreArgs a) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int row = item >> 1;
+  const int row = a.c_width ? item >> 1 : item;
   if (row >= a.n) return;
-  const bool is_c = item & 1;
-  const int width = is_c ? a.c_width : a.q_width;
+  const bool is_c = a.c_width && (item & 1);
+  const int width = is_c ? a.c_width : a.q_width, held = a.c_width + a.p_width;
   const int pieces = width / 8;
-  const int64_t src = (int64_t)row * (a.q_width + a.c_width) + (is_c ? a.q_width : 0);
+  const int64_t src = (int64_t)row * (a.q_width + held) + (is_c ? a.q_width : 0);
   const float* w = is_c ? a.wc : a.wq;
   float v[kNormPieces][8];
   float ss = 0.f;
@@ -72,21 +77,84 @@ __global__ __launch_bounds__(256) void latent_norm_store_kernel(NormStoreArgs a)
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[k][i] = v[k][i] * rs * wv[i];
       if (is_c) {
-        if (slot >= 0) Vec8<T>::st(a.cache, slot * width + pc * 8, v[k]);
-        if (a.c_out) Vec8<T>::st(a.c_out, (int64_t)row * width + pc * 8, v[k]);
+        if (slot >= 0) Vec8<T>::st(a.cache, slot * held + pc * 8, v[k]);
+        if (a.c_out) Vec8<T>::st(a.c_out, (int64_t)row * held + pc * 8, v[k]);
       } else {
         Vec8<T>::st(a.q_out, (int64_t)row * width + pc * 8, v[k]);
       }
     }
   }
+  if (!is_c) return;
+  // the key part: pairs (i, half + i) turn, what follows them passes
+  const int rest = a.p_width - 2 * a.half;
+  for (int i = lane; i < a.half + rest; i += 64) {
+    float x[2];
+    int at[2] = {i, i + a.half};
+    const int cnt = i < a.half ? 2 : 1;
+    if (cnt == 1) at[0] = i + a.half;
+    for (int k = 0; k < cnt; ++k) x[k] = Elem<T>::ld(a.in, src + width + at[k]);
+    if (cnt == 2) {
+      const float2 r = rotary_turn(a.positions[row], a.freqs[i]);
+      const float u = x[0], w2 = x[1];
+      x[0] = u * r.x - w2 * r.y;
+      x[1] = w2 * r.x + u * r.y;
+    }
+    for (int k = 0; k < cnt; ++k) {
+      if (slot >= 0) Elem<T>::st(a.cache, slot * held + width + at[k], x[k]);
+      if (a.c_out) Elem<T>::st(a.c_out, (int64_t)row * held + width + at[k], x[k]);
+    }
+  }
+}
+
+// ------------------------------------------------------------------ rotary positions in place
+struct RotateArgs {
+  void* x;                  // token rows of x_st elements; head h's part at h * head + at
+  const int32_t* positions;
+  const float* freqs;
+  int n, H, head, at, half;
+  int64_t x_st;
+};
+constexpr int kRotTokens = 4;
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void rotate_heads_kernel(RotateArgs a) {
+  extern __shared__ __align__(16) char lds_raw[];
+  float2* cs = (float2*)lds_raw;            // [kRotTokens][half]
+  const int n0 = blockIdx.x * kRotTokens;
+  for (int i = threadIdx.x; i < kRotTokens * a.half; i += 256) {
+    const int tok = i / a.half;
+    if (n0 + tok < a.n) cs[i] = rotary_turn(a.positions[n0 + tok], a.freqs[i - tok * a.half]);
+  }
+  __syncthreads();
+  const int per_head = a.half / VEC, items = a.H * per_head;
+  for (int id = threadIdx.x; id < kRotTokens * items; id += 256) {
+    const int tok = id / items, it = id - tok * items;
+    if (n0 + tok >= a.n) break;
+    const int h = it / per_head, p = (it - h * per_head) * VEC;
+    const int64_t at = (n0 + tok) * a.x_st + (int64_t)h * a.head + a.at + p;
+    float u[VEC], v[VEC];
+    if constexpr (VEC == 8) { Vec8<T>::ld(a.x, at, u); Vec8<T>::ld(a.x, at + a.half, v); }
+    else { u[0] = Elem<T>::ld(a.x, at); v[0] = Elem<T>::ld(a.x, at + a.half); }
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const float2 r = cs[tok * a.half + p + i];
+      const float x = u[i], y = v[i];
+      u[i] = x * r.x - y * r.y;
+      v[i] = y * r.x + x * r.y;
+    }
+    if constexpr (VEC == 8) { Vec8<T>::st(a.x, at, u); Vec8<T>::st(a.x, at + a.half, v); }
+    else { Elem<T>::st(a.x, at, u[0]); Elem<T>::st(a.x, at + a.half, v[0]); }
+  }
 }
 
 // ------------------------------------------------------------------ per-head product
 struct HeadArgs {
-  const void* in;   // (n, H, K) T
+  const void* in;   // (n, H, K + tail) T
   const void* w;    // (H, M, K) T
-  void* out;        // (n, H, M) T
-  int n, H, K, M;
+  void* out;        // (n, H, M + tail) T
+  const int32_t* positions;
+  const float* freqs;
+  int n, H, K, M, tail, half;   // behind each head's part `tail` elements, of which 2 * half turn
 };
 
 // A wave owns 16 outputs of one head for 16 * kTokTiles tokens: W is the row operand, so a lane ends
@@ -97,6 +165,22 @@ __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
   const int m0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16;
   const int h = blockIdx.y;
   const int n0 = blockIdx.z * 16 * kTokTiles;
+  if (a.tail && blockIdx.x == 0) {
+    const int rest = a.tail - a.half;             // items of a token: the pairs, then what follows them
+    for (int it = threadIdx.x; it < 16 * kTokTiles * rest; it += 256) {
+      const int tok = it / rest, i = it - tok * rest, n = n0 + tok;
+      if (n >= a.n) break;
+      const int64_t from = ((int64_t)n * a.H + h) * (a.K + a.tail) + a.K, to = ((int64_t)n * a.H + h) * (a.M + a.tail) + a.M;
+      if (i < a.half) {
+        const float2 r = rotary_turn(a.positions[n], a.freqs[i]);
+        const float u = Elem<T>::ld(a.in, from + i), v = Elem<T>::ld(a.in, from + i + a.half);
+        Elem<T>::st(a.out, to + i, u * r.x - v * r.y);
+        Elem<T>::st(a.out, to + i + a.half, v * r.x + u * r.y);
+      } else {
+        Elem<T>::st(a.out, to + i + a.half, Elem<T>::ld(a.in, from + i + a.half));
+      }
+    }
+  }
   if (m0 >= a.M) return;
   f32x4 acc[kTokTiles];
 #pragma unroll
@@ -105,7 +189,7 @@ __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
   int64_t xrow[kTokTiles];
 #pragma unroll
   for (int t = 0; t < kTokTiles; ++t)
-    xrow[t] = ((int64_t)min(n0 + t * 16 + l16, a.n - 1) * a.H + h) * a.K;
+    xrow[t] = ((int64_t)min(n0 + t * 16 + l16, a.n - 1) * a.H + h) * (a.K + a.tail);
   if constexpr (T::bytes == 2) {
     const uint16_t* w = (const uint16_t*)a.w;
     const uint16_t* x = (const uint16_t*)a.in;
@@ -134,7 +218,7 @@ __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
   for (int t = 0; t < kTokTiles; ++t) {
     const int n = n0 + t * 16 + l16;
     if (n < a.n) {
-      const int64_t at = ((int64_t)n * a.H + h) * a.M + m0 + g * 4;
+      const int64_t at = ((int64_t)n * a.H + h) * (a.M + a.tail) + m0 + g * 4;
       if constexpr (T::bytes == 2) {
         uint2 o;
         o.x = pack_bf16(acc[t][0], acc[t][1]);
@@ -149,14 +233,14 @@ __global__ __launch_bounds__(256) void headwise_kernel(HeadArgs a) {
 
 // ------------------------------------------------------------------ single tokens over the pages
 struct RowsArgs {
-  const void* q;          // (n, H, R) T
-  const void* cache;      // (pages, BS, R) T
+  const void* q;          // (n, H, R + P) T
+  const void* cache;      // (pages, BS, R + P) T
   const int32_t* table;   // (B, NB) page ids
   const int32_t* ctx;     // (n,) tokens of the sequence up to and including this one; 0 = inert
   const int32_t* seq;     // (n,) row of table, or null: row i
   void* out;              // (n, H, R) T
   float* part;            // splits > 1: (n, H, splits, R) fp32, then (n, H, splits, 2) max and sum
-  int n, H, R, BS, bs_shift, B, NB, num_pages;
+  int n, H, R, P, BS, bs_shift, B, NB, num_pages;   // P: elements that only join the scores
   int window;             // a token sees the last `window` tokens including itself; 0 = all
   int splits;             // key ranges handled by different workgroups
   int hw;                 // waves of a workgroup on different heads (1, 2, 4); the others split keys
@@ -176,17 +260,20 @@ __device__ __forceinline__ int page_of(const RowsArgs& a, int t) {
 // columns per MFMA) would touch 16 cache lines per 16 lanes if it were read from memory, so the wave
 // passes each half of the block through an LDS stage of its own.  The next block's pieces are
 // requested as the value products free their registers.  No barrier until the waves meet at the end.
-template <int NCB> struct RowsLds {
+// The rotated part (PK MFMA steps) is a key only, never a value: it is read as a key operand straight from
+// memory, P elements of a key per four lanes.
+template <int NCB, int PK> struct RowsLds {
   static constexpr int kStride = NCB * 128 + 8;                  // elements: rows 16 bytes apart in the banks
   static constexpr int kStage = 16 * kStride * 2;                // bytes per wave: 16 keys
-  static constexpr int kQ = 16 * kStride * 2;                    // bytes per 16 heads
+  static constexpr int kQStride = kStride + PK * 32;             // with 64 more: an odd number of 16 bytes still
+  static constexpr int kQ = 16 * kQStride * 2;                   // bytes per 16 heads
 };
 __host__ __device__ inline int rows_merge_floats(int R) { return 16 * (R + 4) + 32; }   // per wave
 
-template <int NCB, int HT>
+template <int NCB, int HT, int PK>
 __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
-  typedef RowsLds<NCB> Lds;
+  typedef RowsLds<NCB, PK> Lds;
   int* pg = (int*)lds_raw;
   char* const shared = lds_raw + ((a.lds_pages * 4 + 15) & ~15);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -202,12 +289,15 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
   const int row = id / hgroups;
   const int head0 = hg * hw * HT * 16;
   // queries to LDS, zeros past R and past the last head
-  for (int it = tid; it < hw * HT * 16 * NCB * 16; it += 256) {
-    const int hl = it / (NCB * 16), c = (it % (NCB * 16)) * 8;
+  const int RW = a.R + a.P;
+  constexpr int kQPieces = NCB * 16 + PK * 4;
+  for (int it = tid; it < hw * HT * 16 * kQPieces; it += 256) {
+    const int hl = it / kQPieces, c = (it % kQPieces) * 8;
+    const int p = c - NCB * 128;                                 // >= 0: of the rotated part
     u32x4 v = {0u, 0u, 0u, 0u};
-    if (head0 + hl < a.H && c < a.R)
-      v = *(const u32x4*)((const uint16_t*)a.q + ((int64_t)row * a.H + head0 + hl) * a.R + c);
-    *(u32x4*)(qlds + hl * Lds::kStride + c) = v;
+    if (head0 + hl < a.H && (p < 0 ? c < a.R : p < a.P))
+      v = *(const u32x4*)((const uint16_t*)a.q + ((int64_t)row * a.H + head0 + hl) * RW + (p < 0 ? c : a.R + p));
+    *(u32x4*)(qlds + hl * Lds::kQStride + c) = v;
   }
   const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
   const int n = min(a.ctx[row], a.NB * a.BS);
@@ -239,9 +329,12 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
     for (int i = 0; i < NCB * 8; ++i) o[ht][i] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const float sc = a.scale * 1.44269504088896f;
-  const uint16_t* const qrow = qlds + (hwi * HT * 16 + l16) * Lds::kStride + g * 8;
+  const uint16_t* const qrow = qlds + (hwi * HT * 16 + l16) * Lds::kQStride + g * 8;
   const int mask = a.BS - 1;
-  u32x4 v[NCB][8];
+  u32x4 v[NCB][8], kr[2][PK ? PK : 1];
+  int rot_off[PK ? PK : 1];                   // past P: the part's start again, against zeros in q
+#pragma unroll
+  for (int ks = 0; ks < PK; ++ks) rot_off[ks] = (a.R + (ks * 32 + g * 8 < a.P ? ks * 32 + g * 8 : 0)) * 2;
 
   // Page of the visible keys of block b's half (16 keys lie in one page) and the range its rows are
   // clamped to: keys outside the visible range repeat a visible row, with weight zero.
@@ -255,13 +348,22 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
       upto[hf] = max(min(h0 + 15, n - 1), from[hf]);
       if (h0 + 15 < lo) upto[hf] = from[hf] = lo;
       const int page = __builtin_amdgcn_readfirstlane(pg[(from[hf] >> a.bs_shift) - p0]);
-      base[hf] = (const char*)a.cache + (int64_t)page * a.BS * a.R * 2;
+      base[hf] = (const char*)a.cache + (int64_t)page * a.BS * RW * 2;
     }
   };
   auto row_off = [&](int b, int i) {                             // bytes into the page
     const int hf = i >> 2;
     const int key = min(max(b * 32 + step_key(g, i), from[hf]), upto[hf]);
-    return (uint32_t)((key & mask) * a.R * 2);
+    return (uint32_t)((key & mask) * RW * 2);
+  };
+  auto load_rotated = [&](int b) {
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      const int key = min(max(b * 32 + hf * 16 + l16, from[hf]), upto[hf]);
+      const uint32_t ro = (uint32_t)((key & mask) * RW * 2);
+#pragma unroll
+      for (int ks = 0; ks < PK; ++ks) kr[hf][ks] = *(const u32x4*)(base[hf] + (ro + rot_off[ks]));
+    }
   };
 
   const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = a.splits * kw;
@@ -274,6 +376,7 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
 #pragma unroll
       for (int cb = 0; cb < NCB; ++cb) v[cb][i] = *(const u32x4*)(base[i >> 2] + (ro + col_off[cb]));
     }
+    load_rotated(b);
   }
   for (; b <= b1; b += step) {
     const int k0 = b * 32;
@@ -296,8 +399,14 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
         const u32x4 kf = *(const u32x4*)(stage + l16 * Lds::kStride + ks * 32 + g * 8);
 #pragma unroll
         for (int ht = 0; ht < HT; ++ht)
-          part[ht][ks & 1] = mfma_bf16(kf, *(const u32x4*)(qrow + ht * 16 * Lds::kStride + ks * 32), part[ht][ks & 1]);
+          part[ht][ks & 1] = mfma_bf16(kf, *(const u32x4*)(qrow + ht * 16 * Lds::kQStride + ks * 32), part[ht][ks & 1]);
       }
+#pragma unroll
+      for (int ks = 0; ks < PK; ++ks)
+#pragma unroll
+        for (int ht = 0; ht < HT; ++ht)
+          part[ht][ks & 1] = mfma_bf16(kr[hf][ks], *(const u32x4*)(qrow + ht * 16 * Lds::kQStride + NCB * 128 + ks * 32),
+                                       part[ht][ks & 1]);
 #pragma unroll
       for (int ht = 0; ht < HT; ++ht) s[ht][hf] = part[ht][0] + part[ht][1];
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -343,6 +452,7 @@ __global__ __launch_bounds__(256, NCB * HT <= 2 ? 2 : 1) void latent_rows_kernel
     uint32_t ro[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) ro[i] = row_off(next, i);
+    load_rotated(next);
 #pragma unroll
     for (int cb = 0; cb < NCB; ++cb) {
 #pragma unroll
@@ -449,25 +559,26 @@ __global__ __launch_bounds__(64) void latent_rows_combine_kernel(RowsArgs a) {
   }
 }
 
-// One workgroup per (token, head), plain fp32 arithmetic, any R.
+// One workgroup per (token, head), plain fp32 arithmetic, any R and P.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_plain_kernel(RowsArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
-  float* q = (float*)lds_raw;              // R
+  float* q = (float*)lds_raw;              // R + P
   __shared__ float sc[256];
   __shared__ float red[4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int row = blockIdx.x / a.H;
-  const int64_t qat = (int64_t)blockIdx.x * a.R;
+  const int RW = a.R + a.P;
+  const int64_t qat = (int64_t)blockIdx.x * RW, oat = (int64_t)blockIdx.x * a.R;
   const int seq = a.seq ? min(max(a.seq[row], 0), a.B - 1) : row;
   const int n = min(a.ctx[row], a.NB * a.BS);
   const int lo = a.window > 0 ? max(0, n - a.window) : 0;
-  for (int c = tid; c < a.R; c += 256) q[c] = Elem<T>::ld(a.q, qat + c);
+  for (int c = tid; c < RW; c += 256) q[c] = Elem<T>::ld(a.q, qat + c);
   auto key_at = [&](int t) -> int64_t {
     const int p = page_of(a, t);
     int page = a.table[(int64_t)seq * a.NB + p];
     if (page < 0 || page >= a.num_pages) page = 0;
-    return ((int64_t)page * a.BS + (t - p * a.BS)) * a.R;
+    return ((int64_t)page * a.BS + (t - p * a.BS)) * RW;
   };
   constexpr int kCols = 16;                // columns per thread: R <= 4096
   float o[kCols];
@@ -480,7 +591,7 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(RowsArgs a) {
     for (int j = wave; j < cnt; j += 4) {
       const int64_t at = key_at(c0 + j);
       float acc = 0.f;
-      for (int c = lane; c < a.R; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
+      for (int c = lane; c < RW; c += 64) acc = fmaf(q[c], Elem<T>::ld(a.cache, at + c), acc);
       acc = wave_sum(acc);
       if (lane == 0) sc[j] = acc * a.scale;
     }
@@ -516,11 +627,11 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(RowsArgs a) {
 #pragma unroll
   for (int i = 0; i < kCols; ++i) {
     const int c = tid + i * 256;
-    if (c < a.R) Elem<T>::st(a.out, qat + c, o[i] * inv);
+    if (c < a.R) Elem<T>::st(a.out, oat + c, o[i] * inv);
   }
 }
 
-constexpr int kMaxLdsPages = 4096;
+constexpr int kMaxLdsPages = 4096, kMaxRotated = 64;
 
 // Head tiles per wave, and waves of a workgroup on different heads.
 int rows_ht(int H, int R) { return H > 16 && R <= 256 ? 2 : 1; }   // registers hold 2 x 256 columns
@@ -543,18 +654,18 @@ int rows_splits(int n, int H, int R, int window, int NB, int BS) {
   return s < 1 ? 1 : s;
 }
 
-template <int NCB, int HT> int launch_latent_rows(RowsArgs a, hipStream_t st) {
+template <int NCB, int HT, int PK> int launch_latent_rows(RowsArgs a, hipStream_t st) {
   const size_t merge = 4 * sizeof(float) * (size_t)rows_merge_floats(a.R);
-  const size_t work = 4 * RowsLds<NCB>::kStage + (size_t)a.hw * HT * RowsLds<NCB>::kQ;
+  const size_t work = 4 * RowsLds<NCB, PK>::kStage + (size_t)a.hw * HT * RowsLds<NCB, PK>::kQ;
   const size_t smem = (((size_t)a.lds_pages * 4 + 15) & ~(size_t)15) + (merge > work ? merge : work);
   if (smem > 64 * 1024 &&
-      hipFuncSetAttribute((const void*)latent_rows_kernel<NCB, HT>, hipFuncAttributeMaxDynamicSharedMemorySize,
+      hipFuncSetAttribute((const void*)latent_rows_kernel<NCB, HT, PK>, hipFuncAttributeMaxDynamicSharedMemorySize,
                           (int)smem) != hipSuccess) {
     zp_set_error("latent_rows_attention: cannot reserve %zu bytes of LDS", smem);
     return ZP_EHIP;
   }
   const int hgroups = (a.H + 16 * HT * a.hw - 1) / (16 * HT * a.hw);
-  hipLaunchKernelGGL((latent_rows_kernel<NCB, HT>), dim3((unsigned)a.n * hgroups * a.splits), dim3(256), smem, st, a);
+  hipLaunchKernelGGL((latent_rows_kernel<NCB, HT, PK>), dim3((unsigned)a.n * hgroups * a.splits), dim3(256), smem, st, a);
   ZP_LAUNCH_CHECK();
   if (a.splits > 1) {
     hipLaunchKernelGGL(latent_rows_combine_kernel, dim3((unsigned)a.n * a.H), dim3(64), 0, st, a);
@@ -568,24 +679,26 @@ template <int NCB, int HT> int launch_latent_rows(RowsArgs a, hipStream_t st) {
 
 extern "C" int zp_latent_norm_store(const void* in, const float* q_weight, const float* c_weight,
                                     void* q_out, void* c_out, void* cache, const int32_t* slots,
-                                    int32_t n, int32_t q_width, int32_t c_width, int32_t q_norm,
-                                    int32_t c_norm, int64_t num_slots, float eps, int32_t dtype,
-                                    void* stream) {
-  ZP_REQUIRE(n >= 0 && q_width > 0 && c_width > 0 && q_norm > 0 && q_norm <= q_width && c_norm > 0 &&
-                 c_norm <= c_width, "latent_norm_store: bad dims");
+                                    const int32_t* positions, const float* freqs, int32_t n, int32_t q_width,
+                                    int32_t c_width, int32_t p_width, int32_t q_norm, int32_t c_norm,
+                                    int32_t rot, int64_t num_slots, float eps, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && q_width > 0 && c_width >= 0 && q_norm > 0 && q_norm <= q_width && c_norm <= c_width &&
+                 (c_width ? c_norm > 0 && num_slots > 0 : p_width == 0) && p_width >= 0 && rot >= 0 && rot % 2 == 0 &&
+                 rot <= p_width, "latent_norm_store: bad dims");
   ZP_MODEL_DTYPE("latent_norm_store");
-  if (q_width % 8 || c_width % 8 || q_width > 512 * kNormPieces || c_width > 512 * kNormPieces) {
-    zp_set_error("latent_norm_store: ranks %d, %d unsupported (multiples of 8, <= %d)", q_width, c_width,
-                 512 * kNormPieces);
+  if (q_width % 8 || c_width % 8 || p_width % 8 || q_width > 512 * kNormPieces || c_width > 512 * kNormPieces) {
+    zp_set_error("latent_norm_store: ranks %d, %d, rotated part %d unsupported (multiples of 8, <= %d)", q_width, c_width,
+                 p_width, 512 * kNormPieces);
     return ZP_EUNSUPPORTED;
   }
   if (n == 0) return ZP_OK;
-  ZP_REQUIRE(in && q_weight && c_weight && q_out && cache && slots, "latent_norm_store: null pointer");
+  ZP_REQUIRE(in && q_weight && q_out && (!c_width || (c_weight && cache && slots)) && (!rot || (positions && freqs)),
+             "latent_norm_store: null pointer");
   ZP_REQUIRE(aligned16(in) && aligned16(q_weight) && aligned16(c_weight) && aligned16(q_out) &&
                  aligned16(c_out) && aligned16(cache), "latent_norm_store: tensors must be 16-byte aligned");
-  NormStoreArgs a = {in, q_weight, c_weight, q_out, c_out, cache, slots, n, q_width, c_width, q_norm,
-                     c_norm, num_slots, eps};
-  const unsigned grid = (unsigned)((2 * (int64_t)n + 3) / 4);
+  NormStoreArgs a = {in, q_weight, c_weight, q_out, c_out, cache, slots, positions, freqs, n, q_width, c_width, p_width,
+                     q_norm, c_norm, rot / 2, num_slots, eps};
+  const unsigned grid = (unsigned)(((c_width ? 2 : 1) * (int64_t)n + 3) / 4);
   hipStream_t st = (hipStream_t)stream;
   if (dtype == ZP_BF16) hipLaunchKernelGGL((latent_norm_store_kernel<BF16>), dim3(grid), dim3(256), 0, st, a);
   else hipLaunchKernelGGL((latent_norm_store_kernel<F32>), dim3(grid), dim3(256), 0, st, a);
@@ -593,18 +706,47 @@ extern "C" int zp_latent_norm_store(const void* in, const float* q_weight, const
   return ZP_OK;
 }
 
-extern "C" int zp_headwise_linear(const void* in, const void* w, void* out, int32_t n, int32_t H,
-                                  int32_t K, int32_t M, int32_t dtype, void* stream) {
-  ZP_REQUIRE(n >= 0 && H > 0 && K > 0 && M > 0, "headwise_linear: bad dims");
+extern "C" int zp_rotate_heads(void* x, const int32_t* positions, const float* freqs, int32_t n, int32_t H, int32_t head,
+                               int32_t at, int32_t rot, int64_t x_stride, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && head > 0 && at >= 0 && rot >= 0 && rot % 2 == 0 && at + rot <= head &&
+                 x_stride >= (int64_t)H * head, "rotate_heads: bad dims");
+  ZP_MODEL_DTYPE("rotate_heads");
+  if (rot > 2048) {
+    zp_set_error("rotate_heads: %d rotated dimensions (<= 2048)", rot);
+    return ZP_EUNSUPPORTED;
+  }
+  if (n == 0 || rot == 0) return ZP_OK;
+  ZP_REQUIRE(x && positions && freqs, "rotate_heads: null pointer");
+  RotateArgs a = {x, positions, freqs, n, H, head, at, rot / 2, x_stride};
+  const unsigned grid = (unsigned)((n + kRotTokens - 1) / kRotTokens);
+  const size_t smem = sizeof(float2) * kRotTokens * (rot / 2);
+  hipStream_t st = (hipStream_t)stream;
+  const bool wide = rot % 16 == 0 && head % 8 == 0 && at % 8 == 0 && x_stride % 8 == 0 && aligned16(x);
+#define ZP_ROTATE(T)                                                                                          \
+  do {                                                                                                        \
+    if (wide) hipLaunchKernelGGL((rotate_heads_kernel<T, 8>), dim3(grid), dim3(256), smem, st, a);            \
+    else hipLaunchKernelGGL((rotate_heads_kernel<T, 1>), dim3(grid), dim3(256), smem, st, a);                 \
+  } while (0)
+  if (dtype == ZP_BF16) ZP_ROTATE(BF16); else ZP_ROTATE(F32);
+#undef ZP_ROTATE
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_headwise_linear(const void* in, const void* w, void* out, const int32_t* positions,
+                                  const float* freqs, int32_t n, int32_t H, int32_t K, int32_t M, int32_t tail,
+                                  int32_t rot, int32_t dtype, void* stream) {
+  ZP_REQUIRE(n >= 0 && H > 0 && K > 0 && M > 0 && tail >= 0 && rot >= 0 && rot % 2 == 0 && rot <= tail &&
+                 (rot == 0 || (positions && freqs)), "headwise_linear: bad dims");
   ZP_MODEL_DTYPE("headwise_linear");
-  if (K % 32 != 0 || M % 16 != 0 || H > 65535) {
-    zp_set_error("headwise_linear: K %d, M %d unsupported (K multiple of 32, M multiple of 16)", K, M);
+  if (K % 32 != 0 || M % 16 != 0 || tail % 8 != 0 || H > 65535) {
+    zp_set_error("headwise_linear: K %d, M %d, tail %d unsupported (multiples of 32, 16, 8)", K, M, tail);
     return ZP_EUNSUPPORTED;
   }
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(in && w && out && aligned16(in) && aligned16(w) && aligned16(out),
              "headwise_linear: null or unaligned pointer");
-  HeadArgs a = {in, w, out, n, H, K, M};
+  HeadArgs a = {in, w, out, positions, freqs, n, H, K, M, tail, rot / 2};
   // as many tokens per wave (W is read once for them) as still leave two workgroups per CU
   const int64_t columns = (int64_t)((M + 63) / 64) * H;
   int tt = 4;
@@ -635,15 +777,15 @@ extern "C" int64_t zp_latent_rows_workspace(int32_t n, int32_t H, int32_t R, int
 
 extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const int32_t* table,
                                         const int32_t* context_lens, const int32_t* table_rows,
-                                        void* out, int32_t n, int32_t H, int32_t R, int32_t BS,
+                                        void* out, int32_t n, int32_t H, int32_t R, int32_t P, int32_t BS,
                                         int32_t B, int32_t NB, int32_t num_pages, int32_t window,
                                         float scale, int32_t dtype, void* workspace,
                                         int64_t workspace_bytes, void* stream) {
-  ZP_REQUIRE(n >= 0 && H > 0 && R > 0 && BS > 0 && B > 0 && NB > 0 && num_pages > 0 && window >= 0,
+  ZP_REQUIRE(n >= 0 && H > 0 && R > 0 && P >= 0 && BS > 0 && B > 0 && NB > 0 && num_pages > 0 && window >= 0,
              "latent_rows_attention: bad dims");
   ZP_MODEL_DTYPE("latent_rows_attention");
-  if (R % 32 != 0 || R > 4096) {
-    zp_set_error("latent_rows_attention: latent size %d unsupported (multiple of 32, <= 4096)", R);
+  if (R % 32 != 0 || R > 4096 || P % 8 != 0 || P > 4096) {
+    zp_set_error("latent_rows_attention: latent size %d, rotated part %d unsupported (multiples of 32 and 8, <= 4096)", R, P);
     return ZP_EUNSUPPORTED;
   }
   if (n == 0) return ZP_OK;
@@ -653,15 +795,15 @@ extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const 
              "latent_rows_attention: tensors must be 16-byte aligned");
   RowsArgs a = {};
   a.q = q; a.cache = cache; a.table = table; a.ctx = context_lens; a.seq = table_rows; a.out = out;
-  a.part = (float*)workspace; a.n = n; a.H = H; a.R = R; a.BS = BS; a.B = B; a.NB = NB;
+  a.part = (float*)workspace; a.n = n; a.H = H; a.R = R; a.P = P; a.BS = BS; a.B = B; a.NB = NB;
   a.num_pages = num_pages; a.window = window; a.scale = scale; a.bs_shift = -1;
   if ((BS & (BS - 1)) == 0)
     for (a.bs_shift = 0; (1 << a.bs_shift) < BS; ++a.bs_shift) {}
   int64_t pages = NB;
   if (window > 0 && (window - 1) / BS + 2 < pages) pages = (window - 1) / BS + 2;
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == ZP_F32 || R > 512 || pages > kMaxLdsPages || a.bs_shift < 4) {   // bs_shift -1: not a power of two
-    const size_t smem = sizeof(float) * R;
+  if (dtype == ZP_F32 || R > 512 || P > kMaxRotated || pages > kMaxLdsPages || a.bs_shift < 4) {   // bs_shift -1: not a power of two
+    const size_t smem = sizeof(float) * (R + P);
     if (dtype == ZP_BF16)
       hipLaunchKernelGGL((latent_plain_kernel<BF16>), dim3((unsigned)n * H), dim3(256), smem, st, a);
     else
@@ -675,10 +817,12 @@ extern "C" int zp_latent_rows_attention(const void* q, const void* cache, const 
   ZP_REQUIRE(a.splits == 1 || (workspace && workspace_bytes >= zp_latent_rows_workspace(n, H, R, window, NB, BS, dtype)),
              "latent_rows_attention: workspace too small");
   const bool two = rows_ht(H, R) == 2;
+#define ZP_LATENT_ROWS(NCB, HT) (P ? launch_latent_rows<NCB, HT, 2>(a, st) : launch_latent_rows<NCB, HT, 0>(a, st))
   switch ((R + 127) / 128) {
-    case 1: return two ? launch_latent_rows<1, 2>(a, st) : launch_latent_rows<1, 1>(a, st);
-    case 2: return two ? launch_latent_rows<2, 2>(a, st) : launch_latent_rows<2, 1>(a, st);
-    case 3: return launch_latent_rows<3, 1>(a, st);
-    default: return launch_latent_rows<4, 1>(a, st);
+    case 1: return two ? ZP_LATENT_ROWS(1, 2) : ZP_LATENT_ROWS(1, 1);
+    case 2: return two ? ZP_LATENT_ROWS(2, 2) : ZP_LATENT_ROWS(2, 1);
+    case 3: return ZP_LATENT_ROWS(3, 1);
+    default: return ZP_LATENT_ROWS(4, 1);
   }
+#undef ZP_LATENT_ROWS
 }

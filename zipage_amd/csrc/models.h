@@ -2,6 +2,7 @@
 #pragma once
 #include "common.h"
 #include "../../include/zipage_models.h"
+#include <math.h>
 
 #define ZP_MODEL_DTYPE(name)                                       \
   if (dtype != ZP_BF16 && dtype != ZP_F32) {                       \
@@ -47,3 +48,25 @@ template <> struct Vec8<F32> {
     *(zp_f32x4*)((float*)p + i + 4) = zp_f32x4{o[4], o[5], o[6], o[7]};
   }
 };
+
+// tanh; in 16-bit models on the hardware's exponential and reciprocal (absolute error below 2e-7, relative
+// below 2e-5).
+__device__ __forceinline__ float fast_tanh(float x) {
+  const float t = __builtin_amdgcn_exp2f(-2.88539008177793f * fabsf(x));      // exp(-2 |x|)
+  const float big = copysignf((1.f - t) * __builtin_amdgcn_rcpf(1.f + t), x);
+  const float q = x * x;                          // near zero the difference above loses digits
+  return fabsf(x) < 0.0625f ? x * (1.f - q * (1.f / 3.f - q * (2.f / 15.f))) : big;
+}
+template <typename T> __device__ __forceinline__ float tanh_of(float x);
+template <> __device__ __forceinline__ float tanh_of<F32>(float x) { return tanhf(x); }
+template <> __device__ __forceinline__ float tanh_of<BF16>(float x) { return fast_tanh(x); }
+template <typename T> __device__ __forceinline__ float sigmoid_of(float x);
+template <> __device__ __forceinline__ float sigmoid_of<F32>(float x) { return 1.f / (1.f + expf(-x)); }
+template <> __device__ __forceinline__ float sigmoid_of<BF16>(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+
+// Angles of rotary positions are fp32: position times frequency.
+__device__ __forceinline__ float2 rotary_turn(int position, float freq) {
+  float s, c;
+  sincosf((float)position * freq, &s, &c);
+  return make_float2(c, s);
+}

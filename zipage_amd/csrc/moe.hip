@@ -2,7 +2,7 @@
 // tokens, so a step can be captured into a graph.
 //
 //   small_linear     products with few outputs whose result stays in fp32 (router logits)
-//   moe_select       softmax, the best groups of experts, the best experts of those
+//   moe_select       softmax or sigmoids, the best groups of experts, the best experts of those
 //   moe_plan         assignments in the order of their experts, and the list of row tiles
 //   moe_gate_up      both input products of an expert for a row tile, its activation and the weight
 //   moe_down         the output product; each assignment's row goes to the plane of its slot
@@ -98,7 +98,7 @@ struct SelectArgs {
   int32_t* ids;       // (n, top)
   float* weights;     // (n, top)
   int32_t* counts;    // (E + 1,), cleared here
-  int n, E, top, groups, keep, z_st;
+  int n, E, top, groups, keep, score, z_st;
 };
 
 __device__ __forceinline__ int lowest_holder(float best, const float* v, int per) {
@@ -177,7 +177,7 @@ __global__ __launch_bounds__(256) void moe_select_kernel(SelectArgs a) {
       if (e == lane + 64 * j) z[j] = -INFINITY;
     if (lane == 0) {
       a.ids[(int64_t)n * a.top + k] = e;
-      a.weights[(int64_t)n * a.top + k] = expf(b - mx) * inv;
+      a.weights[(int64_t)n * a.top + k] = a.score == ZP_SCORE_SIGMOID ? 1.f / (1.f + expf(-b)) : expf(b - mx) * inv;
     }
   }
 }
@@ -292,18 +292,19 @@ struct ExpertArgs {
   int K, K_shared;        // contraction, routed and shared
   int M, M_shared;        // outputs (gate_up: of the gate alone)
   int64_t x_st, o_st, w_expert;   // w_expert: elements between experts
+  int act;
   float limit, limit_shared;
 };
 
-// g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(1.702 g) (u + 1)
-template <typename T> __device__ __forceinline__ float gated(float gate, float up, float limit);
-template <> __device__ __forceinline__ float gated<F32>(float gate, float up, float limit) {
+// ZP_GATE_CLAMPED: w g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+// ZP_GATE_SILU: g sigmoid(g) u of the weighted products
+template <typename T> __device__ __forceinline__ float gated(int act, float w, float gate, float up, float limit) {
+  if (act == ZP_GATE_SILU) {
+    const float g = w * gate;
+    return g * sigmoid_of<T>(g) * (w * up);
+  }
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
-}
-template <> __device__ __forceinline__ float gated<BF16>(float gate, float up, float limit) {
-  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
-  return g * __builtin_amdgcn_rcpf(1.f + __expf(-1.702f * g)) * (u + 1.f);
+  return w * (g * sigmoid_of<T>(1.702f * g) * (u + 1.f));
 }
 
 // Few rows per expert: the weights are streamed straight into registers.  A workgroup owns 64 rows of W (gate_up:
@@ -377,7 +378,7 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertArgs a) {
       const float wgt = slot < a.top ? a.weights[(int64_t)n * a.top + slot] : 1.f;
       const float lim = shared ? a.limit_shared : a.limit;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] = wgt * gated<T>(first[e], second[e], lim);
+      for (int e = 0; e < 4; ++e) r[e] = gated<T>(a.act, wgt, first[e], second[e], lim);
       Mma<T>::st4(a.out, (int64_t)pos * a.o_st + wt * 8 + g * 4, r);
     } else {
 #pragma unroll
@@ -491,7 +492,7 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(ExpertArgs a) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
-          for (int k = 0; k < 4; ++k) v[u][k] = wgt * gated<BF16>(acc[i + 2 * u][j][k], acc[i + 2 * u + 1][j][k], lim);
+          for (int k = 0; k < 4; ++k) v[u][k] = gated<BF16>(a.act, wgt, acc[i + 2 * u][j][k], acc[i + 2 * u + 1][j][k], lim);
         store8(v[0], v[1], (int64_t)pos * a.o_st, (w0 + wh * 8 + i) / 2, out_tiles, row);
       }
     } else {
@@ -579,17 +580,18 @@ extern "C" int zp_small_linear(const void* x, const void* w, float* out, int32_t
 }
 
 extern "C" int zp_moe_select(const float* logits, int32_t* ids, float* weights, int32_t* counts, int32_t n,
-                             int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t logits_stride,
-                             void* stream) {
+                             int32_t E, int32_t top, int32_t groups, int32_t keep, int32_t score,
+                             int32_t logits_stride, void* stream) {
   ZP_REQUIRE(n >= 0 && E > 0 && top > 0 && groups > 0 && E % groups == 0 && keep > 0 && keep <= groups &&
-                 top <= E / groups * keep && logits_stride >= E, "moe_select: bad dims");
+                 top <= E / groups * keep && logits_stride >= E &&
+                 (score == ZP_SCORE_SOFTMAX || score == ZP_SCORE_SIGMOID), "moe_select: bad dims");
   if (E > kMaxExperts - 1) {
     zp_set_error("moe_select: %d experts (at most %d)", E, kMaxExperts - 1);
     return ZP_EUNSUPPORTED;
   }
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(logits && ids && weights && counts, "moe_select: null pointer");
-  SelectArgs a = {logits, ids, weights, counts, n, E, top, groups, keep, logits_stride};
+  SelectArgs a = {logits, ids, weights, counts, n, E, top, groups, keep, score, logits_stride};
   const dim3 grid((unsigned)((n + 3) / 4));
   const size_t smem = sizeof(float) * 4 * E;
   hipStream_t st = (hipStream_t)stream;
@@ -639,9 +641,9 @@ extern "C" int zp_moe_plan(const int32_t* ids, int32_t* counts, int32_t* sorted,
 static int experts(bool up, const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
                    const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n, int32_t E,
                    int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared,
-                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
-                   float limit_shared, int32_t dtype, void* stream) {
-  ZP_REQUIRE(n >= 0 && E > 0 && top > 0 && max_tiles > 0 && K > 0 && M > 0 && (!shared || (K_shared > 0 && M_shared > 0)),
+                   int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, int32_t act,
+                   float limit, float limit_shared, int32_t dtype, void* stream) {
+  ZP_REQUIRE((act == ZP_GATE_CLAMPED || act == ZP_GATE_SILU) && n >= 0 && E > 0 && top > 0 && max_tiles > 0 && K > 0 && M > 0 && (!shared || (K_shared > 0 && M_shared > 0)),
              "moe experts: bad dims");
   ZP_MODEL_DTYPE("moe experts");
   if (K % 32 || K_shared % 32 || M % 16 || M_shared % 16 || x_stride % 8 || out_stride % 8 ||
@@ -662,7 +664,7 @@ static int experts(bool up, const void* x, const void* w, const void* w_shared, 
     }
   }
   ExpertArgs a = {x, w, w_shared, out, sorted, tiles, ntiles, weights, n, E, top, top + shared, max_tiles, K, K_shared,
-                  M, shared ? M_shared : 0, x_stride, out_stride, (int64_t)M * K * (up ? 2 : 1), limit, limit_shared};
+                  M, shared ? M_shared : 0, x_stride, out_stride, (int64_t)M * K * (up ? 2 : 1), act, limit, limit_shared};
   return up ? launch_experts<true>(a, rows, dtype, (hipStream_t)stream)
             : launch_experts<false>(a, rows, dtype, (hipStream_t)stream);
 }
@@ -670,15 +672,15 @@ static int experts(bool up, const void* x, const void* w, const void* w_shared, 
 extern "C" int zp_moe_gate_up(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
                               const int32_t* tiles, const int32_t* ntiles, const float* weights, int32_t n,
                               int32_t E, int32_t top, int32_t shared, int32_t rows, int32_t max_tiles, int32_t K,
-                              int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, float limit,
-                              float limit_shared, int32_t dtype, void* stream) {
+                              int32_t M, int32_t M_shared, int64_t x_stride, int64_t out_stride, int32_t act,
+                              float limit, float limit_shared, int32_t dtype, void* stream) {
   return experts(true, x, w, w_shared, out, sorted, tiles, ntiles, weights, n, E, top, shared, rows, max_tiles, K, K,
-                 M, M_shared, x_stride, out_stride, limit, limit_shared, dtype, stream);
+                 M, M_shared, x_stride, out_stride, act, limit, limit_shared, dtype, stream);
 }
 extern "C" int zp_moe_down(const void* x, const void* w, const void* w_shared, void* out, const int32_t* sorted,
                            const int32_t* tiles, const int32_t* ntiles, int32_t n, int32_t E, int32_t top,
                            int32_t shared, int32_t rows, int32_t max_tiles, int32_t K, int32_t K_shared, int32_t M,
                            int64_t x_stride, int64_t out_stride, int32_t dtype, void* stream) {
   return experts(false, x, w, w_shared, out, sorted, tiles, ntiles, nullptr, n, E, top, shared, rows, max_tiles, K,
-                 K_shared, M, M, x_stride, out_stride, 0.f, 0.f, dtype, stream);
+                 K_shared, M, M, x_stride, out_stride, ZP_GATE_CLAMPED, 0.f, 0.f, dtype, stream);
 }

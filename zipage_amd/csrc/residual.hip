@@ -1,7 +1,7 @@
 // Row kernels of decoders that keep their residual stream in fp32 whatever the dtype of their
 // matrix products: token + learned-position embedding, residual add (of a branch output as it is or
-// normed), depth average over all earlier layer results, RMS norm, the xIELU activation, and the
-// soft cap of logits.  Each is one pass over its rows (HBM- or
+// normed), depth average over all earlier layer results, RMS norm or tanh norm, the xIELU and squared
+// relu activations, and the soft cap of logits.  Each is one pass over its rows (HBM- or
 // launch-bound): the stream is read once, and what the next matrix product needs leaves the same
 // launch in that product's dtype.
 #include "models.h"
@@ -32,9 +32,10 @@ struct RowArgs {
   float* result;          // receives x + y before the average, or null
   float* x_out;           // receives what goes on, or null
   const float* w;         // (width,) norm weight, or null: no norm
+  const float* b;         // (width,) tanh norm: tanh(alpha x) * (offset + w) + b; null: RMS norm
   void* out;              // (n, width) T: norm(x_out) * (offset + w) * out_scale
   int width, norm_width;  // padded row length, and the length the mean is taken over
-  float eps, offset, out_scale;
+  float eps, offset, out_scale, alpha;
 };
 
 // One workgroup of THREADS per row; the row lives in registers.
@@ -157,6 +158,21 @@ __global__ __launch_bounds__(THREADS) void row_kernel(RowArgs a) {
     }
   }
   if (!a.w) return;
+  if (a.b) {                               // no statistics: nothing to wait for
+#pragma unroll
+    for (int k = 0; k < kMaxPieces; ++k) {
+      const int pc = tid + k * THREADS;
+      if (pc < pieces) {
+        float wv[8], bv[8];
+        Vec8<F32>::ld(a.w, pc * 8, wv);
+        Vec8<F32>::ld(a.b, pc * 8, bv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[k][i] = (tanh_of<T>(a.alpha * v[k][i]) * (a.offset + wv[i]) + bv[i]) * a.out_scale;
+        Vec8<T>::st(a.out, row * a.width + pc * 8, v[k]);
+      }
+    }
+    return;
+  }
   ss = row_sum<kW>(ss, red, tid);
   const float rs = 1.f / sqrtf(ss / (float)a.norm_width + a.eps);
 #pragma unroll
@@ -186,7 +202,21 @@ int launch_rows(const RowArgs& a, int n, int dtype, hipStream_t st) {
   return ZP_OK;
 }
 
-// ------------------------------------------------------------------ xIELU
+// ------------------------------------------------------------------ activations
+template <typename T>
+__global__ __launch_bounds__(256) void relu_square_kernel(const void* in, void* out, int64_t pieces) {
+  const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (id >= pieces) return;
+  float z[8];
+  Vec8<T>::ld(in, id * 8, z);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const float r = fmaxf(z[i], 0.f);
+    z[i] = r * r;
+  }
+  Vec8<T>::st(out, id * 8, z);
+}
+
 // z > 0: ap z^2 + z/2;  z <= 0: an (e^z - 1 - z) + z/2
 template <typename T> __device__ __forceinline__ float expm1_minus(float z);
 template <> __device__ __forceinline__ float expm1_minus<F32>(float z) { return expm1f(z) - z; }
@@ -239,10 +269,10 @@ __global__ __launch_bounds__(256) void softcap_kernel(const void* in, float* out
   }
 
 extern "C" int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* embed,
-                             const void* pos, float* x, const float* norm_weight, void* out,
-                             int32_t n, int32_t width, int32_t norm_width, int64_t vocab,
+                             const void* pos, float* x, const float* norm_weight, const float* norm_bias,
+                             void* out, int32_t n, int32_t width, int32_t norm_width, int64_t vocab,
                              int64_t max_positions, float embed_scale, float eps, float weight_offset,
-                             int32_t dtype, void* stream) {
+                             float norm_alpha, int32_t dtype, void* stream) {
   ZP_REQUIRE(n >= 0 && width > 0 && norm_width > 0 && norm_width <= width && vocab > 0,
              "embed_norm: bad dims");
   ZP_MODEL_DTYPE("embed_norm");
@@ -250,21 +280,21 @@ extern "C" int zp_embed_norm(const int64_t* tokens, const int32_t* positions, co
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(tokens && embed && x && (!pos || (positions && max_positions > 0)) &&
                  (!norm_weight || out), "embed_norm: null pointer");
-  ZP_REQUIRE(aligned16(embed) && aligned16(pos) && aligned16(x) && aligned16(norm_weight) && aligned16(out),
+  ZP_REQUIRE(aligned16(embed) && aligned16(pos) && aligned16(x) && aligned16(norm_weight) && aligned16(norm_bias) && aligned16(out),
              "embed_norm: tensors must be 16-byte aligned");
   RowArgs a = {};
   a.tokens = tokens; a.positions = positions; a.embed = embed; a.pos = pos; a.vocab = vocab;
   a.max_positions = max_positions; a.x_out = x; a.w = norm_weight; a.out = out; a.width = width;
   a.norm_width = norm_width; a.eps = eps; a.offset = weight_offset; a.out_scale = 1.f;
-  a.embed_scale = embed_scale;
+  a.embed_scale = embed_scale; a.b = norm_bias; a.alpha = norm_alpha;
   return launch_rows<true>(a, n, dtype, (hipStream_t)stream);
 }
 
 extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* y_weight,
                                 const float* hist, int64_t hist_plane, const float* mix, int32_t n_hist,
-                                float* result, float* x_out, const float* norm_weight, void* out,
+                                float* result, float* x_out, const float* norm_weight, const float* norm_bias, void* out,
                                 int32_t n, int32_t width, int32_t norm_width, float eps,
-                                float weight_offset, float out_scale, int32_t dtype, void* stream) {
+                                float weight_offset, float norm_alpha, float out_scale, int32_t dtype, void* stream) {
   ZP_REQUIRE(n >= 0 && width > 0 && norm_width > 0 && norm_width <= width && n_hist >= 0 && n_y >= 1,
              "residual_norm: bad dims");
   ZP_MODEL_DTYPE("residual_norm");
@@ -274,13 +304,13 @@ extern "C" int zp_residual_norm(const float* x, const void* y, int32_t n_y, cons
   ZP_REQUIRE(n_hist == 0 || (hist && mix && hist_plane >= (int64_t)n * width),
              "residual_norm: a depth average needs its weights and planes of n rows");
   ZP_REQUIRE(aligned16(x) && aligned16(y) && aligned16(y_weight) && aligned16(hist) && hist_plane % 4 == 0 && aligned16(result) &&
-                 aligned16(x_out) && aligned16(norm_weight) && aligned16(out),
+                 aligned16(x_out) && aligned16(norm_weight) && aligned16(norm_bias) && aligned16(out),
              "residual_norm: tensors must be 16-byte aligned");
   RowArgs a = {};
   a.x = x; a.y = y; a.n_y = n_y; a.y_plane = (int64_t)n * width; a.hist = hist; a.hist_plane = hist_plane; a.mix = mix; a.n_hist = n_hist;
   a.result = result; a.x_out = x_out; a.w = norm_weight; a.out = out; a.width = width;
   a.norm_width = norm_width; a.eps = eps; a.offset = weight_offset; a.out_scale = out_scale;
-  a.yw = y_weight;
+  a.yw = y_weight; a.b = norm_bias; a.alpha = norm_alpha;
   if (y_weight) return launch_rows<false, true>(a, n, dtype, (hipStream_t)stream);
   return launch_rows<false>(a, n, dtype, (hipStream_t)stream);
 }
@@ -298,6 +328,20 @@ extern "C" int zp_xielu(const void* in, void* out, int64_t count, float alpha_p,
     hipLaunchKernelGGL((xielu_kernel<BF16>), dim3(grid), dim3(256), 0, st, in, out, pieces, alpha_p, alpha_n);
   else
     hipLaunchKernelGGL((xielu_kernel<F32>), dim3(grid), dim3(256), 0, st, in, out, pieces, alpha_p, alpha_n);
+  ZP_LAUNCH_CHECK();
+  return ZP_OK;
+}
+
+extern "C" int zp_relu_square(const void* in, void* out, int64_t count, int32_t dtype, void* stream) {
+  ZP_REQUIRE(count >= 0 && count % 8 == 0, "relu_square: element count must be a multiple of 8");
+  ZP_MODEL_DTYPE("relu_square");
+  if (count == 0) return ZP_OK;
+  ZP_REQUIRE(in && out && aligned16(in) && aligned16(out), "relu_square: null or unaligned pointer");
+  const int64_t pieces = count / 8;
+  const unsigned grid = (unsigned)((pieces + 255) / 256);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == ZP_BF16) hipLaunchKernelGGL((relu_square_kernel<BF16>), dim3(grid), dim3(256), 0, st, in, out, pieces);
+  else hipLaunchKernelGGL((relu_square_kernel<F32>), dim3(grid), dim3(256), 0, st, in, out, pieces);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }

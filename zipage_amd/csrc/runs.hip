@@ -16,17 +16,24 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const char* src, const
 
 // ------------------------------------------------------------------ runs of prompt tokens
 struct TilesArgs {
-  const uint16_t* q;      // token rows of q_st elements, head h at h * D
-  const uint16_t* k;      // key rows of kv_st elements, head h at h * D
+  const uint16_t* q;      // token rows of q_st elements, head h at h * maps * (D + P)
+  const uint16_t* k;      // key rows of kv_st elements, head h at h * maps * D
   const uint16_t* v;      // value rows of kv_st elements, head h at h * V
+  const uint16_t* ks;     // rows of s_st elements: the last P of every head's key; null: P = 0
   uint16_t* out;          // token rows of o_st elements, head h at h * V
   const int32_t* tiles;   // (T, 4): first query row, queries, first key row of the run, position
                           // of the first query counted from that key
   const float* sinks;     // (H,) logits that only join the denominator, or null
-  int T, H, HK, D, V;     // HK key / value heads; query head h uses head h / (H / HK)
+  int T, H, HK, D, P, V;  // HK key / value heads; query head h uses head h / (H / HK)
   int window, chunk;      // at most one is set, see first_seen
-  int64_t q_rows, k_rows, q_st, kv_st, o_st;
+  int64_t q_rows, k_rows, q_st, kv_st, s_st, o_st;
   float scale, out_scale;
+  float cap;              // > 0: soft cap of the scores
+  // two maps: rms(o1 - balance * o2) * out_scale * sigmoid(gate), the mean over vdim
+  float balance, eps;
+  int vdim;
+  const uint16_t* gate;   // token rows of g_st elements, head h at h * V; or null
+  int64_t g_st;
 };
 
 constexpr int kTileQ = 128;   // queries per workgroup
@@ -42,27 +49,32 @@ __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
   return chunk > 0 ? pos / chunk * chunk : 0;
 }
 
-template <int DKS, int VCB> struct TileStage {
-  static constexpr int kK = DKS * 32 + 8, kV = VCB * 128 + 8;    // row strides: rows 16 bytes apart in the banks
+template <int DKS, int VCB, int MAPS> struct TileStage {
+  static constexpr int kK = MAPS * DKS * 32 + 8, kV = VCB * 128 + 8;    // row strides: rows 16 bytes apart in the banks
   static constexpr int kElems = kTileK * (kK + kV);
   static constexpr int kBytes = 2 * kElems * 2;
 };
 
-template <int DKS, int VCB, int kQT>
-__global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
+// Column tile t of a wave: 16 queries, map t % MAPS of the head (differential attention has two, over the same
+// values; elsewhere there is one).  SHARED: the last P elements of every head's key are the row of a.ks.
+template <int DKS, int VCB, int kQT, int MAPS, bool SHARED>
+__global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_tiles_kernel(TilesArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
-  typedef TileStage<DKS, VCB> Stage;
+  typedef TileStage<DKS, VCB, MAPS> Stage;
+  constexpr int kT = kQT * MAPS;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
   const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
   const int kb = a.tiles[tile * 4 + 2], rel = a.tiles[tile * 4 + 3];
   // host-made descriptors: rows outside the buffers are not touched
   if (q0 < 0 || kb < 0 || rel < 0 || (int64_t)q0 + nq > a.q_rows || (int64_t)kb + rel + nq > a.k_rows) return;
-  const int nks = a.D / 32;
-  const float sc = a.scale * 1.44269504088896f;
+  const int DT = a.D + (SHARED ? a.P : 0);
+  const float sc = a.cap > 0.f ? a.scale / a.cap : a.scale * 1.44269504088896f;
+  const float capl2 = a.cap * 1.44269504088896f;
   const int hk = h / (a.H / a.HK);
-  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + hk * a.D;
+  const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + hk * MAPS * a.D;
   const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + hk * a.V;
+  const uint16_t* sbase = SHARED ? a.ks + (int64_t)kb * a.s_st : nullptr;
 
   for (int wg0 = 0; wg0 < nq; wg0 += 64 * kQT) {              // uniform in the workgroup
     const int w0 = wg0 + wave * 16 * kQT;
@@ -72,37 +84,41 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
     const int lo = first_seen(rel + w0, a.window, a.chunk);
     const int lo_last = first_seen(rel + w0 + 16 * kQT - 1, a.window, a.chunk);
 
-    u32x4 qf[kQT][DKS];
+    u32x4 qf[kT][DKS];
     int qpos[kQT], qlow[kQT];                                 // keys qlow .. qpos are seen
 #pragma unroll
-    for (int t = 0; t < kQT; ++t) {
-      const int qi = min(w0 + t * 16 + l16, nq - 1);
-      qpos[t] = rel + qi;
-      qlow[t] = first_seen(qpos[t], a.window, a.chunk);
-      const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + h * a.D + g * 8;
+    for (int t = 0; t < kT; ++t) {
+      const int qi = min(w0 + t / MAPS * 16 + l16, nq - 1);
+      qpos[t / MAPS] = rel + qi;
+      qlow[t / MAPS] = first_seen(rel + qi, a.window, a.chunk);
+      const uint16_t* q = a.q + (int64_t)(q0 + qi) * a.q_st + (h * MAPS + t % MAPS) * DT;
 #pragma unroll
       for (int ks = 0; ks < DKS; ++ks) {
-        // D may end inside the last steps: they read the row's start, against zeros in q
-        qf[t][ks] = *(const u32x4*)(q + (ks < nks ? ks * 32 : 0));
-        if (ks >= nks) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
+        // past the head's end: the key columns there hold other elements, against zeros here
+        const int c = ks * 32 + g * 8;
+        qf[t][ks] = *(const u32x4*)(q + (c < DT ? c : 0));
+        if (c >= DT) qf[t][ks] = u32x4{0u, 0u, 0u, 0u};
       }
     }
-    f32x4 o[kQT][VCB * 8];
-    float m[kQT], l[kQT];
+    f32x4 o[kT][VCB * 8];
+    float m[kT], l[kT];
 #pragma unroll
-    for (int t = 0; t < kQT; ++t) {
+    for (int t = 0; t < kT; ++t) {
       m[t] = -INFINITY;
       l[t] = 0.f;
 #pragma unroll
       for (int i = 0; i < VCB * 8; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
-    u32x4 rk[DKS], rv[4 * VCB];                                // this thread's pieces of a tile
+    u32x4 rk[MAPS * DKS], rv[4 * VCB];                         // this thread's pieces of a tile
+    constexpr int kKP = 4 * MAPS * DKS;                        // pieces of a key row, DKS * 4 per map
     auto fetch = [&](int k0) {
 #pragma unroll
-      for (int j = 0; j < DKS; ++j) {
-        const int id = tid + 256 * j, r = id / (4 * DKS), c = (id % (4 * DKS)) * 8;
-        rk[j] = *(const u32x4*)(kbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.D ? c : 0));
+      for (int j = 0; j < MAPS * DKS; ++j) {
+        const int id = tid + 256 * j, r = id / kKP, pc = id % kKP, map = pc / (4 * DKS), c = (pc % (4 * DKS)) * 8;
+        const int64_t row = min(k0 + r, last);
+        if (SHARED && c >= a.D) rk[j] = *(const u32x4*)(sbase + row * a.s_st + (c < DT ? c - a.D : 0));
+        else rk[j] = *(const u32x4*)(kbase + row * a.kv_st + map * a.D + (c < a.D ? c : 0));
       }
 #pragma unroll
       for (int j = 0; j < 4 * VCB; ++j) {
@@ -117,9 +133,9 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
       uint16_t* const ldsk = (uint16_t*)lds_raw + buf * Stage::kElems;
       uint16_t* const ldsv = ldsk + kTileK * Stage::kK;
 #pragma unroll
-      for (int j = 0; j < DKS; ++j) {
+      for (int j = 0; j < MAPS * DKS; ++j) {
         const int id = tid + 256 * j;
-        *(u32x4*)(ldsk + id / (4 * DKS) * Stage::kK + (id % (4 * DKS)) * 8) = rk[j];
+        *(u32x4*)(ldsk + id / kKP * Stage::kK + (id % kKP) * 8) = rk[j];
       }
 #pragma unroll
       for (int j = 0; j < 4 * VCB; ++j) {
@@ -132,31 +148,37 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
       for (int sub = 0; sub < kTileK; sub += 32) {
         const int k0 = t0 + sub;
         if (k0 > hi || k0 + 31 < lo) continue;                 // uniform in the wave
-        f32x4 s[kQT][2];
+        f32x4 s[kT][2];
 #pragma unroll
         for (int tt = 0; tt < 2; ++tt) {
 #pragma unroll
-          for (int t = 0; t < kQT; ++t) s[t][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+          for (int t = 0; t < kT; ++t) s[t][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int ks = 0; ks < DKS; ++ks) {
-            const u32x4 kf = *(const u32x4*)(ldsk + (sub + tt * 16 + l16) * Stage::kK + ks * 32 + g * 8);
+          for (int ks = 0; ks < DKS; ++ks)
 #pragma unroll
-            for (int t = 0; t < kQT; ++t) s[t][tt] = mfma_bf16(kf, qf[t][ks], s[t][tt]);
-          }
+            for (int map = 0; map < MAPS; ++map) {
+              const u32x4 kf = *(const u32x4*)(ldsk + (sub + tt * 16 + l16) * Stage::kK + (map * DKS + ks) * 32 + g * 8);
+#pragma unroll
+              for (int t = map; t < kT; t += MAPS) s[t][tt] = mfma_bf16(kf, qf[t][ks], s[t][tt]);
+            }
         }
         // every query of the wave sees all 32 keys: no masks
         const bool inner = k0 + 31 <= rel + w0 && k0 >= lo_last;
-        u32x4 pf[kQT];
+        u32x4 pf[kT];
 #pragma unroll
-        for (int t = 0; t < kQT; ++t) {
+        for (int t = 0; t < kT; ++t) {
           float p[8], mx = -INFINITY;
 #pragma unroll
           for (int i = 0; i < 8; ++i) p[i] = s[t][i >> 2][i & 3] * sc;
+          if (a.cap > 0.f) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) p[i] = capl2 * fast_tanh(p[i]);
+          }
           if (!inner) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
               const int key = k0 + step_key(g, i);
-              if (key > qpos[t] || key < qlow[t]) p[i] = -INFINITY;
+              if (key > qpos[t / MAPS] || key < qlow[t / MAPS]) p[i] = -INFINITY;
             }
           }
 #pragma unroll
@@ -191,21 +213,43 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
           for (int c = 0; c < 8; ++c) {
             const u32x4 vf = column_of(v, c);
 #pragma unroll
-            for (int t = 0; t < kQT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
+            for (int t = 0; t < kT; ++t) o[t][cb * 8 + c] = mfma_bf16(vf, pf[t], o[t][cb * 8 + c]);
           }
         }
       }
     }
 #pragma unroll
-    for (int t = 0; t < kQT; ++t) {
-      float lt = l[t];
-      lt += lane_xor16(lt);
-      lt += lane_xor32(lt);
-      if (a.sinks) lt += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - m[t]);
-      const float inv = lt > 0.f ? a.out_scale / lt : 0.f;
-      const int qi = w0 + t * 16 + l16;
+    for (int qt = 0; qt < kQT; ++qt) {
+      float inv[MAPS];
+#pragma unroll
+      for (int map = 0; map < MAPS; ++map) {
+        float lt = l[qt * MAPS + map];
+        lt += lane_xor16(lt);
+        lt += lane_xor32(lt);
+        if (MAPS == 1 && a.sinks) lt += __builtin_amdgcn_exp2f(a.sinks[h] * 1.44269504088896f - m[qt]);
+        inv[map] = lt > 0.f ? 1.f / lt : 0.f;
+      }
+      if constexpr (MAPS == 1) {
+        inv[0] *= a.out_scale;
+      } else {                                                 // o1 <- rms(o1 / l1 - balance * o2 / l2) * out_scale
+        const float second = a.balance * inv[1];
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < VCB * 8; ++j)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float r = o[qt * 2][j][i] * inv[0] - o[qt * 2 + 1][j][i] * second;
+            o[qt * 2][j][i] = r;
+            if ((j >> 3) * 128 + (4 * g + i) * 8 < a.V) ss += r * r;
+          }
+        ss += lane_xor16(ss);
+        ss += lane_xor32(ss);
+        inv[0] = a.out_scale / sqrtf(ss / (float)a.vdim + a.eps);
+      }
+      const int qi = w0 + qt * 16 + l16;
       if (qi >= nq) continue;
       uint16_t* out = a.out + (int64_t)(q0 + qi) * a.o_st + h * a.V;
+      const uint16_t* gate = MAPS == 2 && a.gate ? a.gate + (int64_t)(q0 + qi) * a.g_st + h * a.V : nullptr;
 #pragma unroll
       for (int cb = 0; cb < VCB; ++cb)
 #pragma unroll
@@ -214,7 +258,13 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
           if (col < a.V) {
             float r[8];
 #pragma unroll
-            for (int c = 0; c < 8; ++c) r[c] = o[t][cb * 8 + c][i] * inv;
+            for (int c = 0; c < 8; ++c) r[c] = o[qt * MAPS][cb * 8 + c][i] * inv[0];
+            if (MAPS == 2 && gate) {
+              float z[8];
+              Vec8<BF16>::ld(gate, col, z);
+#pragma unroll
+              for (int c = 0; c < 8; ++c) r[c] *= sigmoid_of<BF16>(z[c]);
+            }
             Vec8<BF16>::st(out, col, r);
           }
         }
@@ -222,17 +272,37 @@ __global__ __launch_bounds__(256, 2) void run_tiles_kernel(TilesArgs a) {
   }
 }
 
-template <int DKS, int VCB, int kQT> int launch_run_tiles(const TilesArgs& a, hipStream_t st) {
-  constexpr int smem = TileStage<DKS, VCB>::kBytes;
+template <int DKS, int VCB, int kQT, int MAPS, bool SHARED> int launch_run_tiles(const TilesArgs& a, hipStream_t st) {
+  constexpr int smem = TileStage<DKS, VCB, MAPS>::kBytes;
   if (smem > 64 * 1024 &&
-      hipFuncSetAttribute((const void*)run_tiles_kernel<DKS, VCB, kQT>,
+      hipFuncSetAttribute((const void*)run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED>,
                           hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
     zp_set_error("run_attention: cannot reserve %d bytes of LDS", smem);
     return ZP_EHIP;
   }
-  hipLaunchKernelGGL((run_tiles_kernel<DKS, VCB, kQT>), dim3((unsigned)a.T * a.H), dim3(256), smem, st, a);
+  hipLaunchKernelGGL((run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED>), dim3((unsigned)a.T * a.H), dim3(256), smem, st, a);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
+}
+
+template <bool SHARED> int launch_one_map(const TilesArgs& a, hipStream_t st) {
+  const int dk = (a.D + a.P + 31) / 32;
+  if (a.V <= 128) {
+    if (dk <= 2) return launch_run_tiles<2, 1, 2, 1, SHARED>(a, st);
+    if (dk <= 4) return launch_run_tiles<4, 1, 2, 1, SHARED>(a, st);
+    if (dk <= 6) return launch_run_tiles<6, 1, 2, 1, SHARED>(a, st);
+    return launch_run_tiles<8, 1, 2, 1, SHARED>(a, st);
+  }
+  if (dk <= 4) return launch_run_tiles<4, 2, 1, 1, SHARED>(a, st);
+  return launch_run_tiles<8, 2, 1, 1, SHARED>(a, st);
+}
+int launch_two_maps(const TilesArgs& a, hipStream_t st) {
+  const int dk = (a.D + 31) / 32;
+  if (a.V <= 128) {
+    if (dk <= 2) return launch_run_tiles<2, 1, 1, 2, false>(a, st);
+    return launch_run_tiles<4, 1, 1, 2, false>(a, st);
+  }
+  return launch_run_tiles<4, 2, 1, 2, false>(a, st);
 }
 
 }  // namespace
@@ -250,34 +320,35 @@ extern "C" int zp_gather_rows(const void* src, const int32_t* rows, void* out, i
   return ZP_OK;
 }
 
-extern "C" int zp_run_attention(const void* q, const void* k, const void* v, void* out,
-                                const int32_t* tiles, const float* sinks, int32_t T, int32_t H,
-                                int32_t HK, int32_t D, int32_t V, int32_t window, int32_t chunk,
-                                int64_t q_rows, int64_t k_rows, int64_t q_stride, int64_t kv_stride,
-                                int64_t out_stride, float scale, float out_scale, int32_t dtype,
-                                void* stream) {
-  ZP_REQUIRE(T >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && V > 0 && window >= 0 && chunk >= 0 &&
-                 !(window && chunk), "run_attention: bad dims");
-  if (dtype != ZP_BF16 || D % 32 != 0 || D > 256 || V % 8 != 0 || V > 256) {
-    zp_set_error("run_attention: bfloat16, D %d (multiple of 32, <= 256), V %d (multiple of 8, <= 256)", D, V);
+extern "C" int zp_run_attention(const void* q, const void* k, const void* v, const void* k_shared, void* out,
+                                const int32_t* tiles, const float* sinks, const zp_attention_form* form, int32_t T,
+                                int32_t H, int32_t HK, int32_t D, int32_t P, int32_t V, int32_t window,
+                                int32_t chunk, int64_t q_rows, int64_t k_rows, int64_t q_stride,
+                                int64_t kv_stride, int64_t shared_stride, int64_t out_stride, float scale,
+                                float out_scale, int32_t dtype, void* stream) {
+  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0}, f = form ? *form : plain;
+  const bool two = f.maps == 2;
+  ZP_REQUIRE(T >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && P >= 0 && V > 0 && window >= 0 && chunk >= 0 &&
+                 !(window && chunk) && (f.maps == 1 || two) && f.softcap >= 0.f && (P > 0) == (k_shared != nullptr),
+             "run_attention: bad dims");
+  if (dtype != ZP_BF16 || D % 8 != 0 || P % 8 != 0 || D + P > (two ? 128 : 256) || V % 8 != 0 || V > 256) {
+    zp_set_error("run_attention: bfloat16, D %d + %d (multiples of 8, <= 256, of two maps <= 128), V %d (multiple of 8, <= 256)",
+                 D, P, V);
     return ZP_EUNSUPPORTED;
   }
   if (T == 0) return ZP_OK;
   ZP_REQUIRE(q && k && v && out && tiles, "run_attention: null pointer");
-  ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && q_stride % 8 == 0 &&
-                 kv_stride % 8 == 0 && out_stride % 8 == 0 && q_stride >= (int64_t)H * D &&
-                 out_stride >= (int64_t)H * V && (int64_t)T * H < (1ll << 31),
+  ZP_REQUIRE(!two || (!sinks && !P && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
+             "run_attention: two maps go without sinks and shared keys, with a mean over the values");
+  ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && aligned16(k_shared) && aligned16(f.gate) &&
+                 f.gate_stride % 8 == 0 && q_stride % 8 == 0 && kv_stride % 8 == 0 && shared_stride % 8 == 0 &&
+                 out_stride % 8 == 0 && q_stride >= (int64_t)H * f.maps * (D + P) && out_stride >= (int64_t)H * V &&
+                 (!P || shared_stride >= P) && (int64_t)T * H < (1ll << 31),
              "run_attention: unaligned rows or too many tiles");
-  TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (uint16_t*)out, tiles, sinks, T, H, HK,
-                 D, V, window, chunk, q_rows, k_rows, q_stride, kv_stride, out_stride, scale, out_scale};
+  TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (const uint16_t*)k_shared, (uint16_t*)out,
+                 tiles, sinks, T, H, HK, D, P, V, window, chunk, q_rows, k_rows, q_stride, kv_stride, shared_stride,
+                 out_stride, scale, out_scale, f.softcap, f.balance, f.eps, f.vdim, (const uint16_t*)f.gate, f.gate_stride};
   hipStream_t st = (hipStream_t)stream;
-  const int dk = D / 32;
-  if (V <= 128) {
-    if (dk <= 2) return launch_run_tiles<2, 1, 2>(a, st);
-    if (dk <= 4) return launch_run_tiles<4, 1, 2>(a, st);
-    if (dk <= 6) return launch_run_tiles<6, 1, 2>(a, st);
-    return launch_run_tiles<8, 1, 2>(a, st);
-  }
-  if (dk <= 4) return launch_run_tiles<4, 2, 1>(a, st);
-  return launch_run_tiles<8, 2, 1>(a, st);
+  if (two) return launch_two_maps(a, st);
+  return P ? launch_one_map<true>(a, st) : launch_one_map<false>(a, st);
 }

@@ -18,6 +18,7 @@ from zipage_amd.layers.linear import ResidualLinear, fit, pad_to_multiple
 from zipage_amd.layers.moe import Experts
 from zipage_amd.layers.recurrent import ChannelDelta, MatrixMemory
 from zipage_amd.layers.residual import embed_norm, residual_norm, softcap
+from zipage_amd.layers.rotary import Rotary
 from zipage_amd.sight import Chunk
 
 
@@ -142,8 +143,8 @@ class Parallel:
     the rows that enter the latter."""
 
     def __init__(self, m: ParallelMixer, width: int, eps: float):
-        self.left = GroupedAttention(width, m.heads, m.kv_heads, m.dim, m.vdim, m.scale, Chunk(m.chunk), m.rot_base,
-                                     m.rot_dims, sinks=True, out_scale=m.left_scale)
+        self.left = GroupedAttention(width, m.heads, m.kv_heads, m.dim, m.vdim, m.scale, Chunk(m.chunk),
+                                     Rotary(m.rot_base, m.rot_dims), sinks=True, out_scale=m.left_scale)
         self.right = MatrixMemory(width, m.memory_heads, m.memory_dim, m.memory_vdim, m.gate_cap, eps,
                                   out_scale=m.right_scale)
         self.out_columns = self.left.out_columns + self.right.out_columns

@@ -125,10 +125,7 @@ class Pedivik:
         self.layers = []
         for i, (l, mixer) in enumerate(zip(s.layers, self.mixers)):
             pre = f"l{i}."
-            H, D, V, Q, R = l.heads, l.dim, l.vdim, l.q_rank, l.kv_rank
-            mixer.load({k: get(f"{pre}mix.{k}", *shape) for k, shape in {
-                "dq": (Q, s.width), "dq.norm": (Q,), "uq": (H * D, Q), "dkv": (R, s.width), "dkv.norm": (R,),
-                "uk": (H * D, R), "uv": (H * V, R), "o": (s.width, H * V)}.items()}, self.dtype, self.device)
+            mixer.load({k: get(f"{pre}mix.{k}", *shape) for k, shape in mixer.shapes().items()}, self.dtype, self.device)
             p = dict(norm1=vec(pre + "norm1"), dwa=f32(get(pre + "dwa", i + 2)))
             if l.ff is not None:
                 ffp = -(-l.ff // 8) * 8
@@ -165,8 +162,7 @@ class Pedivik:
     # ------------------------------------------------------------------ cache
     def allocate_caches(self, num_pages: int, page_size: int, num_slots: int):
         """One page pool per layer; a page holds page_size latents of that layer."""
-        self.caches = [torch.zeros(num_pages, page_size, m.kv_rank_p, dtype=self.dtype, device=self.device)
-                       for m in self.mixers]
+        self.caches = [m.allocate(num_pages, page_size, self.dtype, self.device) for m in self.mixers]
 
     # ------------------------------------------------------------------ forward
     @torch.inference_mode()

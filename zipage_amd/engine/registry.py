@@ -9,6 +9,7 @@ from typing import Any, Callable
 from .kapolorn import Kapolorn, KapolornShape
 from .pedivik import Pedivik, PedivikShape
 from .qwen3 import Qwen3, Qwen3Shape
+from .rutevik import Rutevik, RutevikShape
 from .weights import read_folder
 
 
@@ -25,7 +26,10 @@ class Architecture:
 ARCHITECTURES = {a.name: a for a in (
     Architecture("Qwen3ForCausalLM", Qwen3, Qwen3Shape, Qwen3Shape.from_config, ("LIB",), loads_weights=False),
     Architecture("Pedivik", Pedivik, PedivikShape, PedivikShape.from_config, ("MODELS_LIB", "LATENT_LIB")),
-    Architecture("Kapolorn", Kapolorn, KapolornShape, KapolornShape.from_config, ("MODELS_LIB", "HYBRID_LIB")),
+    Architecture("Kapolorn", Kapolorn, KapolornShape, KapolornShape.from_config,
+                 ("MODELS_LIB", "GROUPED_LIB", "RECURRENT_LIB", "MOE_LIB")),
+    Architecture("Rutevik", Rutevik, RutevikShape, RutevikShape.from_config,
+                 ("MODELS_LIB", "LATENT_LIB", "GROUPED_LIB", "MOE_LIB")),
 )}
 
 

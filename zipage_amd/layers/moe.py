@@ -19,9 +19,10 @@ def small_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return out
 
 
-def moe_select(logits: torch.Tensor, experts: int, top: int, groups: int = 1, keep: int = 1):
-    """Softmax over the first `experts` logits of each row (fp32), the `keep` groups with the best single
-    score, the `top` best experts of those: (ids, scores, cleared counters for the plan)."""
+def moe_select(logits: torch.Tensor, experts: int, top: int, groups: int = 1, keep: int = 1,
+               score: int = _lib.SCORE_SOFTMAX):
+    """Softmax over the first `experts` logits of each row (fp32), or their sigmoids, the `keep` groups with the
+    best single score, the `top` best experts of those: (ids, scores, cleared counters for the plan)."""
     N = logits.shape[0]
     assert logits.dtype == torch.float32 and logits.stride(1) == 1
     dev = logits.device
@@ -29,7 +30,8 @@ def moe_select(logits: torch.Tensor, experts: int, top: int, groups: int = 1, ke
     weights = torch.empty((N, top), dtype=torch.float32, device=dev)
     counts = torch.empty(experts + 1, dtype=torch.int32, device=dev)
     _lib.call_models("zp_moe_select", _lib.dev_ptr(logits), _lib.dev_ptr(ids), _lib.dev_ptr(weights),
-                     _lib.dev_ptr(counts), N, experts, top, groups, keep, logits.stride(0), _lib.stream_ptr(logits))
+                     _lib.dev_ptr(counts), N, experts, top, groups, keep, score, logits.stride(0),
+                     _lib.stream_ptr(logits))
     return ids, weights, counts
 
 
@@ -38,7 +40,7 @@ class Plan:
 
     def __init__(self, ids: torch.Tensor, counts: torch.Tensor, experts: int, shared: bool, dtype):
         N, top = ids.shape
-        lib, dev = _lib.load_models("hybrid"), ids.device
+        lib, dev = _lib.load_models("moe"), ids.device
         self.n, self.experts, self.top, self.shared, self.slots = N, experts, top, int(shared), top + int(shared)
         self.rows = lib.zp_moe_tile_rows(N, experts, top, _lib._DTYPES[dtype])
         self.max_tiles = lib.zp_moe_max_tiles(N, experts, top, self.shared, self.rows)
@@ -69,16 +71,20 @@ def gate_up_order(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 
 
 class Experts:
-    """Gated experts (g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(1.702 g) (u + 1), then down)
-    of which every token uses `top`, chosen among its best `keep` of `groups` groups, weighted with their
-    softmax scores as they are; and, if `shared_ff` is given, one more for every token."""
+    """Gated experts of which every token uses `top`, chosen among its best `keep` of `groups` groups, weighted
+    with their scores as they are; and, if `shared_ff` is given, one more for every token.  Scores are a
+    softmax or sigmoids.  `act` "clamped": g = min(gate, limit), u = clamp(up, +-limit), w g sigmoid(1.702 g)
+    (u + 1) with the weight w on the output; "silu": g sigmoid(g) u with the weight on the expert's input."""
 
     def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, groups: int = 1, keep: int = 1,
-                 shared_ff: int | None = None, shared_limit: float = 0.0):
+                 shared_ff: int | None = None, shared_limit: float = 0.0, score: str = "softmax",
+                 act: str = "clamped"):
         if experts % groups or not 0 < keep <= groups or not 0 < top <= experts // groups * keep:
             raise ValueError(f"{top} of {experts} experts in {keep} of {groups} groups")
         self.width, self.experts, self.top, self.ff, self.limit = width, experts, top, ff, limit
         self.groups, self.keep, self.shared_ff, self.shared_limit = groups, keep, shared_ff, shared_limit
+        self.score = {"softmax": _lib.SCORE_SOFTMAX, "sigmoid": _lib.SCORE_SIGMOID}[score]
+        self.act = {"clamped": _lib.GATE_CLAMPED, "silu": _lib.GATE_SILU}[act]
         self.ff_p = pad_to_multiple(ff, 32)
         self.shared_p = pad_to_multiple(shared_ff, 32) if shared_ff else 0
         self.width_p = pad_to_multiple(width, 32)
@@ -120,7 +126,7 @@ class Experts:
 
     # ------------------------------------------------------------------ forward
     def route(self, h: torch.Tensor):
-        return moe_select(small_linear(h, self.router), self.experts, self.top, self.groups, self.keep)
+        return moe_select(small_linear(h, self.router), self.experts, self.top, self.groups, self.keep, self.score)
 
     def gate_up_rows(self, h: torch.Tensor, plan: Plan, weights: torch.Tensor) -> torch.Tensor:
         """Activations by position in plan.sorted, times the assignment's weight."""
@@ -130,7 +136,7 @@ class Experts:
         _lib.call_models("zp_moe_gate_up", _lib.dev_ptr(h), _lib.dev_ptr(self.gate_up), _lib.dev_ptr(self.shared_gate_up),
                          _lib.dev_ptr(act), _lib.dev_ptr(plan.sorted), _lib.dev_ptr(plan.tiles), _lib.dev_ptr(plan.ntiles),
                          _lib.dev_ptr(weights), plan.n, self.experts, self.top, plan.shared, plan.rows, plan.max_tiles,
-                         self.width_p, self.ff_p, self.shared_p, h.stride(0), ff, self.limit, self.shared_limit,
+                         self.width_p, self.ff_p, self.shared_p, h.stride(0), ff, self.act, self.limit, self.shared_limit,
                          _lib.dtype_tag(h), _lib.stream_ptr(h))
         return act
 

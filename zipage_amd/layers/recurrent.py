@@ -95,7 +95,7 @@ class MatrixMemory:
             if not runs:
                 _lib.call_models("zp_mlstm_scan", ctypes.byref(args), tag, stream)
                 continue
-            size = _lib.load_models("hybrid").zp_mlstm_runs_workspace(h.shape[0] - segments.first_row,
+            size = _lib.load_models("recurrent").zp_mlstm_runs_workspace(h.shape[0] - segments.first_row,
                                                                       segments.counts.numel(), H)
             ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
             _lib.call_models("zp_mlstm_runs", ctypes.byref(args), segments.first_row, segments.longest, _lib.dev_ptr(ws),
@@ -181,7 +181,7 @@ class ChannelDelta:
             if not runs:
                 _lib.call_models("zp_delta_scan", ctypes.byref(args), tag, stream)
                 continue
-            size = _lib.load_models("hybrid").zp_delta_runs_workspace(proj.shape[0] - segments.first_row,
+            size = _lib.load_models("recurrent").zp_delta_runs_workspace(proj.shape[0] - segments.first_row,
                                                                       segments.counts.numel(), H, D, self.vdim_p)
             ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
             _lib.call_models("zp_delta_runs", ctypes.byref(args), segments.first_row, segments.longest,

@@ -1,7 +1,8 @@
 """Row steps of decoders with an fp32 residual stream (one HIP launch each).
 
 `x` is the stream (N, width) fp32; what feeds a matrix product has the model's dtype.  Widths are
-padded to a multiple of 8 with zeros, `norm_width` is the length the mean runs over."""
+padded to a multiple of 8 with zeros, `norm_width` is the length the mean runs over.  With `norm_bias` the
+norm is tanh(norm_alpha x) * (weight_offset + norm_weight) + norm_bias, without a mean."""
 import torch
 
 from zipage_amd import _lib
@@ -15,19 +16,21 @@ def _rows(t: torch.Tensor | None, width: int):
 
 def embed_norm(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.Tensor,
                pos: torch.Tensor | None, x: torch.Tensor, norm_weight: torch.Tensor, eps: float,
-               norm_width: int, weight_offset: float = 0.0, embed_scale: float = 1.0) -> torch.Tensor:
+               norm_width: int, weight_offset: float = 0.0, embed_scale: float = 1.0,
+               norm_bias: torch.Tensor | None = None, norm_alpha: float = 0.0) -> torch.Tensor:
     """x = embed[tokens] * embed_scale (+ pos[positions]) into `x`; returns its RMS norm times
     (weight_offset + norm_weight) in the table's dtype.  tokens (N,) int64, positions (N,) int32."""
     N, W = x.shape
     assert tokens.dtype == torch.int64 and positions.dtype == torch.int32
     assert tokens.is_contiguous() and positions.is_contiguous() and tokens.numel() == positions.numel() == N
     assert x.dtype == torch.float32 and norm_weight.dtype == torch.float32
+    assert norm_bias is None or norm_bias.dtype == torch.float32
     assert pos is None or pos.dtype == embed.dtype
     out = torch.empty((N, W), dtype=embed.dtype, device=x.device)
     _lib.call_models("zp_embed_norm", _lib.dev_ptr(tokens), _lib.dev_ptr(positions), _rows(embed, W),
-                     _rows(pos, W), _rows(x, W), _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width,
-                     embed.shape[0], 0 if pos is None else pos.shape[0], float(embed_scale), float(eps), float(weight_offset),
-                     _lib.dtype_tag(embed), _lib.stream_ptr(x))
+                     _rows(pos, W), _rows(x, W), _rows(norm_weight, W), _rows(norm_bias, W), _lib.dev_ptr(out), N, W,
+                     norm_width, embed.shape[0], 0 if pos is None else pos.shape[0], float(embed_scale), float(eps),
+                     float(weight_offset), float(norm_alpha), _lib.dtype_tag(embed), _lib.stream_ptr(x))
     return out
 
 
@@ -35,7 +38,8 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
                   norm_width: int, weight_offset: float = 0.0, out_scale: float = 1.0,
                   x_out: torch.Tensor | None = None, result: torch.Tensor | None = None,
                   history: torch.Tensor | None = None, mix: torch.Tensor | None = None,
-                  y_weight: torch.Tensor | None = None):
+                  y_weight: torch.Tensor | None = None, norm_bias: torch.Tensor | None = None,
+                  norm_alpha: float = 0.0):
     """r = x + y (y also as planes (P, N, width), all of them added; with `y_weight` their sum is
     RMS-normed, times that weight, before it joins x), kept in `result`; with `mix`,
     r <- mix[-1] r + sum_j mix[j] history[j]; kept in `x_out`; returns rmsnorm(r) * (weight_offset + norm_weight) * out_scale in y's dtype (None
@@ -43,7 +47,7 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
     N, W = x.shape
     y = y if y.dim() == 3 else y.unsqueeze(0)
     assert x.dtype == torch.float32 and y.shape[1:] == x.shape
-    assert y_weight is None or y_weight.dtype == torch.float32
+    assert all(t is None or t.dtype == torch.float32 for t in (y_weight, norm_bias))
     n_hist, plane = 0, 0
     if mix is not None:
         assert mix.dtype == torch.float32 and mix.is_contiguous()
@@ -56,8 +60,8 @@ def residual_norm(x: torch.Tensor, y: torch.Tensor, norm_weight: torch.Tensor | 
     _lib.call_models("zp_residual_norm", _rows(x, W), _rows(y, W), y.shape[0], _rows(y_weight, W),
                      _lib.dev_ptr(history if n_hist else None),
                      plane, _lib.dev_ptr(mix), n_hist, _rows(result, W), _rows(x_out, W),
-                     _rows(norm_weight, W), _lib.dev_ptr(out), N, W, norm_width, float(eps),
-                     float(weight_offset), float(out_scale), _lib.dtype_tag(y), _lib.stream_ptr(x))
+                     _rows(norm_weight, W), _rows(norm_bias, W), _lib.dev_ptr(out), N, W, norm_width, float(eps),
+                     float(weight_offset), float(norm_alpha), float(out_scale), _lib.dtype_tag(y), _lib.stream_ptr(x))
     return out
 
 
@@ -67,6 +71,15 @@ def xielu(z: torch.Tensor, alpha_p: float, alpha_n: float) -> torch.Tensor:
     out = torch.empty_like(z)
     _lib.call_models("zp_xielu", _lib.dev_ptr(z), _lib.dev_ptr(out), z.numel(), float(alpha_p),
                      float(alpha_n), _lib.dtype_tag(z), _lib.stream_ptr(z))
+    return out
+
+
+def relu_square(z: torch.Tensor) -> torch.Tensor:
+    """max(z, 0)^2."""
+    assert z.is_contiguous()
+    out = torch.empty_like(z)
+    _lib.call_models("zp_relu_square", _lib.dev_ptr(z), _lib.dev_ptr(out), z.numel(), _lib.dtype_tag(z),
+                     _lib.stream_ptr(z))
     return out
 
 

@@ -5,6 +5,10 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 
+# how far back a token looks that sees everything, for rules that take a number of tokens
+EVERYTHING = 1 << 40
+
+
 @dataclass(frozen=True)
 class Chunk:
     """Blocks of `size` positions, counted from position 0 of the sequence."""
