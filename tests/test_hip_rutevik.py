@@ -230,7 +230,7 @@ def _pair(q1, q2, k1, k2, v, seen, scale, cap, balance, eps, vdim, diff_scale, g
 @pytest.mark.parametrize("H,G,D,V,vdim,BS,cap,gated", [
     (1, 1, 8, 16, 16, 16, 3.0, True), (6, 3, 24, 48, 40, 64, 0.0, True), (34, 2, 72, 144, 144, 16, 20.0, True),
     (16, 1, 64, 128, 128, 48, 6.0, True), (8, 8, 40, 64, 57, 32, 2.0, False), (20, 2, 128, 96, 96, 64, 50.0, True),
-    (4, 4, 136, 48, 48, 256, 9.0, True), (6, 2, 128, 256, 256, 16, 4.0, True)])
+    (4, 4, 136, 48, 48, 256, 9.0, True), (6, 2, 128, 256, 256, 16, 4.0, True), (12, 4, 32, 32, 32, 64, 90.0, True)])
 def test_differential_rows(dev, dtype, H, G, D, V, vdim, BS, cap, gated):
     """Two maps over the same values; each map points at a key of its own; the soft cap bends large scores."""
     from zipage_amd.layers import attention_form, grouped_rows_attention
@@ -351,6 +351,46 @@ def test_differential_runs(dev, H, G, D, V, vdim, cap, gated):
                   torch.as_tensor(runs.tiles).to(dev), scale, out[:, :H * V], out_scale=0.75,
                   form=attention_form(cap, 2, balance, eps, vdim, gate[:, :H * V] if gated else None))
     _close(out[:, :H * V].view(total, H, V), want, BF16, 3.0)
+
+
+@pytest.mark.parametrize("cap", [4.0, 50.0, 90.0])
+@pytest.mark.parametrize("low", [False, True], ids=["spread", "low"])
+def test_soft_cap_of_one_map(dev, cap, low):
+    """Scores all over the cap's range, and all of them deep below zero, where a softmax without a running maximum
+    has only tiny weights; with a sink that is as low."""
+    from zipage_amd.layers import attention_form, grouped_rows_attention, run_attention
+    parts, rows, runs = _run_parts(16)
+    H, G, D, V, scale = 6, 2, 64, 64, 0.125
+    total = sum(p.count for p in parts)
+    k, v, q = _rand("cpu", BF16, rows, G, D, seed=1), _rand("cpu", BF16, rows, G, V, seed=2), _rand("cpu", BF16, total, H, D, seed=3)
+    sinks = torch.linspace(-2.0, 2.0, H)
+    if low:                                      # every key near one direction, every query against it
+        k, q = 1 + 0.1 * k, -1.1 * cap / (scale * D) + 0.2 * q
+        sinks -= 0.8 * cap
+    want, r = torch.empty(total, H, V, dtype=torch.float64), 0
+    for p in parts:
+        base, m = p.seq.block_table[0] * 16, p.start + p.count
+        seen = torch.arange(m)[None] <= torch.arange(p.start, m)[:, None]
+        for h in range(H):
+            sc = O.capped(q[r:r + p.count, h].double() @ k[base:base + m, h // 3].double().T * scale, cap)
+            sc = torch.cat([sc.masked_fill(~seen, float("-inf")), sinks[h].double().expand(p.count, 1)], -1)
+            want[r:r + p.count, h] = torch.softmax(sc, -1)[:, :-1] @ v[base:base + m, h // 3].double()
+        r += p.count
+    kv = torch.cat([k.flatten(1), v.flatten(1)], 1)
+    t = lambda a: torch.as_tensor(a, dtype=torch.int32).to(dev)
+    out = torch.full((total, H * V), float("nan"), dtype=BF16, device=dev)
+    run_attention(q.flatten(1).to(dev), kv[torch.as_tensor(runs.key_slots).long()].to(dev), H, G, D, V, t(runs.tiles), scale, out,
+                  sinks=sinks.to(dev), form=attention_form(cap))
+    _close(out.view(total, H, V), want, BF16, 3.0)
+    # the last token of every part, singly
+    ends = torch.tensor([p.count for p in parts]).cumsum(0) - 1
+    width = max(len(p.seq.block_table) for p in parts)
+    tables = t([p.seq.block_table + [-1] * (width - len(p.seq.block_table)) for p in parts])
+    for dtype in DTYPES:
+        out = torch.full((len(parts), H * V), float("nan"), dtype=dtype, device=dev)
+        grouped_rows_attention(q[ends].flatten(1).to(dev, dtype), kv.view(-1, 16, kv.shape[1]).to(dev, dtype), H, G, D, V, tables,
+                               t([p.start + p.count for p in parts]), scale, out, sinks=sinks.to(dev), form=attention_form(cap))
+        _close(out.view(-1, H, V), want[ends], dtype, 3.0 if dtype == BF16 else 64.0)
 
 
 # ------------------------------------------------------------------ experts

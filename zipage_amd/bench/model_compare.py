@@ -1,15 +1,17 @@
-"""Pedivik or Kapolorn beside Qwen3 at equal size: prefill and decode throughput through the engine
-(random weights), and every kernel between the matrix products against its roofline, beside the kernel
-of the other model that does the like work.
+"""Pedivik or Kapolorn beside Qwen3, Rutevik beside Pedivik and Kapolorn, at equal size: prefill and decode
+throughput through the engine (random weights), and every kernel between the matrix products against its
+roofline, beside the kernel of the other model that does the like work.
 
 Equal size: same width, heads, head dimensions and vocabulary; Pedivik's ungated feed-forward is 1.5
 times as wide as Qwen3's gated one, so both hold the same parameters; a Kapolorn token passes three of 32
-experts and the shared one, each a quarter as wide as Qwen3's feed-forward.  Kernels are timed as replays
-of a graph of many launches over buffers that together exceed the caches.
+experts and the shared one, each a quarter as wide as Qwen3's feed-forward, a Rutevik token four of 32 such
+experts; its differential layers have half the heads, with values of twice the size.  Kernels are timed as
+replays of a graph of many launches over buffers that together exceed the caches.
 """
 from __future__ import annotations
 
 import time
+from dataclasses import replace
 from types import SimpleNamespace
 
 import torch
@@ -43,6 +45,26 @@ def kapolorn_shapes(size: str):
     delta = KapolornLayer(DeltaMixer(H, H // 2, D, D, 4), moe)
     return (KapolornShape(V, W, (par, delta) * (L // 2), (0, 0, 1), 1e-6, 1.0, 15.0),
             Qwen3Shape(L, W, H, HK, D, FF, V, max_position=8192))
+
+
+def rutevik_shapes(size: str):
+    """One differential layer (the first with a dense feed-forward) to three latent ones, of which one reads the
+    cache of the one before it.  Pedivik's window holds everything here, Kapolorn keeps its chunks."""
+    from zipage_amd.engine import KapolornShape, PedivikShape, RutevikShape
+    from zipage_amd.engine.rutevik import DenseShape, DifferentialMixer, LatentMixer, MixtureShape, RutevikLayer
+    from zipage_amd.layers import Rotary
+    W, H, HK, D, FF, L, V, QR, KR, _ = SIZES[size]
+    moe, rot = MixtureShape(32, 4, FF // 4), Rotary(5e5, D // 2)
+    diff = DifferentialMixer(H // 2, HK // 2, D, 2 * D, Rotary(5e5, D, (8.0, 1.0, 4.0, 2048.0)), D ** -0.5, 30.0, 0.4)
+    layers = []
+    for i in range(L):
+        source = i - 1 if i % 4 == 2 else i
+        m = LatentMixer(H, D, D, QR, KR, rot, (D * 3 // 2) ** -0.5, source) if i % 4 else diff
+        layers.append(RutevikLayer(m, moe if i else DenseShape(FF * 3 // 2)))
+    pedivik, kapolorn = shapes(size)[0], kapolorn_shapes(size)[0]
+    everything = lambda layer: replace(layer, window=8192)
+    return {"rutevik": RutevikShape(V, W, tuple(layers), 1e-6, 1.0),
+            "pedivik": replace(pedivik, layers=tuple(map(everything, pedivik.layers))), "kapolorn": kapolorn}
 
 
 def throughput(shape, batch: int, prompt: int, out_tokens: int) -> dict:
@@ -390,19 +412,171 @@ def kapolorn_kernels(size: str, decode_batch: int, prompts: int, prompt: int) ->
     return rows
 
 
-MODELS = {"pedivik": (shapes, kernels), "kapolorn": (kapolorn_shapes, kapolorn_kernels)}
+def rutevik_kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dict]:
+    """The same for Rutevik's kernels; each has the like kernel of Pedivik or Kapolorn behind it."""
+    from zipage_amd.engine.inputs import plan_runs
+    from zipage_amd.engine.sequence import Portion, Sequence
+    from zipage_amd.layers import (Experts, Rotary, attention_form, grouped_rows_attention, latent_rows_attention,
+                                   latent_tiles_attention, relu_square, residual_norm, rotary_store, rotate_heads,
+                                   run_attention, xielu)
+    from zipage_amd.layers.latent import headwise_linear, latent_norm_store
+    from zipage_amd.layers.moe import Plan, moe_select
+    W, H, HK, D, FF, L, V, QR, KR, _ = SIZES[size]
+    P, H2, HK2, V2 = D // 2, H // 2, HK // 2, 2 * D             # rotated part; heads of the differential layers
+    dev, BS = torch.device("cuda:0"), 256
+    rnd = lambda *s, dt=BF16: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    i32 = lambda a: torch.as_tensor(a, dtype=torch.int32, device=dev)
+    rows = []
+
+    def put(name, where, secs, byts, flops=0.0):
+        roof = max(byts / HBM, flops / MFMA)
+        rows.append({"kernel": name, "at": where, "us": round(secs * 1e6, 1),
+                     "bound": "hbm" if byts / HBM >= flops / MFMA else "mfma",
+                     "roofline_us": round(roof * 1e6, 1), "frac": round(roof / secs, 3)})
+
+    gen = torch.Generator(device=dev).manual_seed(0)
+    silu = Experts(W, 32, 4, FF // 4, 0.0, score="sigmoid", act="silu")
+    clamped = Experts(W, 32, 4, FF // 4, 7.0)
+    silu.random(BF16, dev, gen)
+    clamped.router, clamped.gate_up, clamped.down = silu.router, silu.gate_up, silu.down
+    clamped.shared_gate_up = clamped.shared_down = None
+    freqs, turn = rnd(D // 2, dt=torch.float32).abs(), Rotary(5e5, P).frequencies(dev)
+    w32, b32 = torch.ones(W, device=dev), torch.zeros(W, device=dev)
+    per, E = -(-prompt // BS), 32
+    form = lambda gate: attention_form(30.0, 2, 0.5, 1e-6, V2, gate)
+    for phase, N in (("decode", 64), ("decode", decode_batch), ("prefill", prompts * prompt)):
+        at, big = f"{phase}, {N} tokens", N * W
+        pos, slots = torch.arange(N, device=dev, dtype=torch.int32) % prompt, torch.randperm(N, device=dev).int()
+        for planes in (1, 4):
+            k = _sets(big * (10 + 2 * planes))
+            xs, ys = [rnd(N, W, dt=torch.float32) for _ in range(k)], [rnd(planes, N, W) for _ in range(k)]
+            for name, more in (("residual_norm, tanh norm", dict(norm_bias=b32, norm_alpha=0.6)), ("like: residual_norm, RMS norm", {})):
+                put(f"{name}, {planes} planes", at,
+                    timed(lambda i: residual_norm(xs[i], ys[i], w32, 1e-6, W, x_out=xs[i], **more), k), big * (10 + 2 * planes))
+            del xs, ys
+        n = N * FF * 3 // 2
+        zs = [rnd(N, FF * 3 // 2) for _ in range(_sets(n * 4))]
+        put("relu_square", at, timed(lambda i: relu_square(zs[i]), len(zs)), n * 4)
+        put("like: xielu", at, timed(lambda i: xielu(zs[i], 0.8, 1.3), len(zs)), n * 4)
+        del zs
+        # latent rows
+        wq, wc = torch.ones(QR, device=dev), torch.ones(KR, device=dev)
+        for name, p, more in (("latent_norm_store, rotated part", P, dict(positions=pos, freqs=turn)), ("like: latent_norm_store", 0, {})):
+            k = _sets(N * (QR + KR + p) * 4)
+            downs, caches = [rnd(N, QR + KR + p) for _ in range(k)], [rnd(-(-N // BS), BS, KR + p) for _ in range(k)]
+            put(name, at, timed(lambda i: latent_norm_store(downs[i], wq, wc, QR, KR, 1e-6, caches[i], slots, **more), k),
+                N * (QR + KR + p) * 4)
+            del downs, caches
+        k = _sets(N * QR * 4)
+        downs = [rnd(N, QR) for _ in range(k)]
+        put("latent_norm_store, queries alone", at, timed(lambda i: latent_norm_store(downs[i], wq, None, QR, 0, 1e-6, None, None), k), N * QR * 4)
+        del downs
+        # queries, keys and values of the grouped heads
+        width, kvw = (2 * H2 + 2 * HK2) * D + HK2 * V2, 2 * HK2 * D + HK2 * V2
+        bias = rnd(width, dt=torch.float32)
+        k = _sets(N * width * 4)
+        qkvs, caches = [rnd(N, width) for _ in range(k)], [rnd(-(-N // BS), BS, kvw) for _ in range(k)]
+        put("rotary_store, two maps, bias", at, timed(lambda i: rotary_store(
+            qkvs[i], pos, freqs, H2, HK2, D, V2, caches[i], slots, maps=2, bias=bias), k), N * width * 4)
+        put("like: rotary_store", at, timed(lambda i: rotary_store(qkvs[i], pos, freqs, H, HK, D, D, caches[i], slots), k), N * width * 4)
+        del qkvs, caches
+        if phase == "prefill":
+            k = _sets(N * H * (D + P) * 2)
+            qs = [rnd(N, H * (D + P)) for _ in range(k)]
+            put("rotate_heads (the rotated part's bytes)", at, timed(lambda i: rotate_heads(qs[i], pos, turn, H, D), k), N * H * P * 4)
+            del qs
+        else:
+            for name, w_, tail in (("q into the latent space", rnd(H, KR, D), P), ("values out of it", rnd(H, D, KR), 0)):
+                M, K = w_.shape[1:]
+                ws = [w_] + [rnd(H, M, K) for _ in range(_sets(H * M * K * 2) - 1)]
+                for label, t in (((f"headwise_linear, {name}, turned tail", tail),) if tail else ()) + ((f"like: headwise_linear, {name}", 0),):
+                    x = rnd(N, H, K + t)
+                    more = dict(positions=pos, freqs=turn) if t else {}
+                    put(label, at, timed(lambda i: headwise_linear(x, ws[i], **more), len(ws)),
+                        H * M * K * 2 + N * H * (K + M + 2 * t) * 2, 2.0 * N * H * K * M)
+                del ws
+        # experts
+        h, z = [rnd(N, W) for _ in range(2)], rnd(N, E, dt=torch.float32)
+        for name, moe in (("sigmoids, silu, weight on the input", silu), ("softmax, clamped", clamped)):
+            label = "like: " if moe is clamped else ""
+            put(f"{label}moe_select, {name}", at, timed(lambda i: moe_select(z, E, 4, score=moe.score), 2), N * (E * 4 + 32))
+            ids, wts, counts = moe_select(z, E, 4, score=moe.score)
+            plan = Plan(ids, counts, E, False, BF16)
+            act, used, fl = moe.gate_up_rows(h[0], plan, wts), min(E, N * 4), 2.0 * N * W * FF
+            put(f"{label}moe_gate_up, {name}", at, timed(lambda i: moe.gate_up_rows(h[i], plan, wts), 2, 6),
+                used * (FF // 2) * W * 2 + N * W * 2 + N * FF * 2, 2 * fl)
+        put("moe_down (the same for both)", at, timed(lambda i: silu.down_planes(act, plan), 2, 6),
+            used * (FF // 4) * W * 2 + N * FF * 2 + 4 * N * W * 2, fl)
+        del h, act
+    # ---- decode attention
+    for B, ctx_len in ((1, prompt), (64, prompt), (decode_batch, prompt), (8, 4 * prompt)):
+        at, pages = f"decode, {B} sequences, context {ctx_len}", -(-ctx_len // BS)
+        tables, ctx = torch.randperm(B * pages, device=dev).int().view(B, pages), i32([ctx_len] * B)
+        for name, p in (("latent_rows_attention, rotated part", P), ("like: latent_rows_attention", 0)):
+            k = _sets(B * ctx_len * (KR + p) * 2)
+            caches, q = [rnd(B * pages, BS, KR + p) for _ in range(k)], rnd(B, H, KR + p)
+            put(name, at, timed(lambda i: latent_rows_attention(q, caches[i], tables, ctx, D ** -0.5, rank=KR), k),
+                B * ctx_len * (KR + p) * 2 + B * H * (2 * KR + p) * 2, 2.0 * B * H * ctx_len * (2 * KR + p))
+            del caches
+        k = _sets(B * ctx_len * HK * D * 4)
+        caches, q = [rnd(B * pages, BS, 2 * HK * D) for _ in range(k)], rnd(B, H * D)
+        out, gate = torch.empty(B, H * D, device=dev, dtype=BF16), rnd(B, H * D)
+        byts = 2 * B * ctx_len * HK * D * 2 + 2 * B * H * D * 2
+        put("grouped_rows_attention, differential, soft cap, gate", at,
+            timed(lambda i: grouped_rows_attention(q, caches[i], H2, HK2, D, V2, tables, ctx, D ** -0.5, out, form=form(gate)), k),
+            byts + B * H * D * 2, 6.0 * B * H * ctx_len * D)
+        put("like: grouped_rows_attention", at,
+            timed(lambda i: grouped_rows_attention(q, caches[i], H, HK, D, D, tables, ctx, D ** -0.5, out), k), byts,
+            4.0 * B * H * ctx_len * D)
+        del caches
+    # ---- prefill attention
+    N, at, k = prompts * prompt, f"prefill, {prompts} x {prompt} tokens", 2
+    parts = []
+    for _ in range(prompts):
+        s = Sequence([0] * prompt)
+        s.block_table = list(range(per))
+        parts.append(Portion(s, 0, prompt))
+    tiles, pairs = i32(plan_runs(parts, BS, None).tiles), prompt * (prompt + 1) / 2 * prompts
+    out, gate = torch.empty(N, H * D, device=dev, dtype=BF16), rnd(N, H * D)
+    qs, kvs = [rnd(N, H * (D + P)) for _ in range(k)], [rnd(N, 2 * H * D) for _ in range(k)]
+    shared = [rnd(N, KR + P)[:, KR:] for _ in range(k)]
+    put("latent_tiles_attention, shared rotated part", at,
+        timed(lambda i: latent_tiles_attention(qs[i], kvs[i], H, D, D, tiles, D ** -0.5, None, out, shared[i]), k, 6),
+        N * (H * (4 * D + P) + P) * 2, 2.0 * pairs * H * (2 * D + P))
+    qs = [rnd(N, H * D) for _ in range(k)]
+    put("like: latent_tiles_attention", at,
+        timed(lambda i: latent_tiles_attention(qs[i], kvs[i], H, D, D, tiles, D ** -0.5, None, out), k, 6),
+        N * H * D * 4 * 2, 4.0 * pairs * H * D)
+    kvs = [rnd(N, 2 * HK * D) for _ in range(k)]
+    put("run_attention, differential, soft cap, gate", at,
+        timed(lambda i: run_attention(qs[i], kvs[i], H2, HK2, D, V2, tiles, D ** -0.5, out, form=form(gate)), k, 6),
+        N * (3 * H + 2 * HK) * D * 2, 6.0 * pairs * H * D)
+    put("like: run_attention", at,
+        timed(lambda i: run_attention(qs[i], kvs[i], H, HK, D, D, tiles, D ** -0.5, out), k, 6),
+        N * (2 * H + 2 * HK) * D * 2, 4.0 * pairs * H * D)
+    return rows
+
+
+def beside_qwen3(model: str, make):
+    return lambda size: dict(zip((model, "qwen3"), make(size)))
+
+
+MODELS = {"pedivik": (beside_qwen3("pedivik", shapes), kernels),
+          "kapolorn": (beside_qwen3("kapolorn", kapolorn_shapes), kapolorn_kernels),
+          "rutevik": (rutevik_shapes, rutevik_kernels)}
 
 
 def compare(model: str = "pedivik", sizes=("1k", "4k"), out_tokens: int = 64) -> dict:
     """The whole report.  The headline figure is the model's decode rate at the largest size and batch."""
+    import sys
     report = {"sizes": {}}
     make, table = MODELS[model]
     for size in sizes:
-        own, qwen = make(size)
-        entry = {model: {}, "qwen3": {}}
+        entry = {name: {} for name in make(size)}
         for batch, prompt in ((1, 2048), (64, 2048), (256, 2048)):
-            for name, shape in ((model, own), ("qwen3", qwen)):
+            for name, shape in make(size).items():
                 entry[name][f"{batch} x {prompt}"] = throughput(shape, batch, prompt, out_tokens)
+                print(f"{size}: {name}, {batch} x {prompt} tokens", file=sys.stderr, flush=True)
         entry["kernels"] = table(size, 256, 8, 2048)
         report["sizes"][size] = entry
     return report

@@ -224,9 +224,8 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
   f32x4 o[VCB * 8];
 #pragma unroll
   for (int i = 0; i < VCB * 8; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  const float sc = a.cap > 0.f ? a.scale / a.cap : a.scale * 1.44269504088896f;
-  const float capl2 = a.cap * 1.44269504088896f;
+  const SoftCap cap(a.scale, a.cap);
+  float m = cap.bounded ? 0.f : -INFINITY, l = 0.f;
   const int b1 = n > 0 ? (n - 1) >> 5 : -1, step = 4 * a.splits;
   int b = (lo >> 5) + split * 4 + wave;
   if (b <= b1) {
@@ -243,31 +242,36 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
       for (int ks = 0; ks < DKS; ++ks) s[tt] = mfma_bf16(kf[tt][ks], qf[ks], s[tt]);
     }
     load_keys(next);
-    float p[8], mx = -INFINITY;
+    float p[8], sum = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int key = k0 + step_key(g, i);
-      p[i] = s[i >> 2][i & 3] * sc;
-      if (a.cap > 0.f) p[i] = capl2 * fast_tanh(p[i]);
+      p[i] = cap.log2_score(s[i >> 2][i & 3]);
       if (key < lo || key >= n) p[i] = -INFINITY;
-      mx = fmaxf(mx, p[i]);
     }
-    mx = fmaxf(mx, lane_xor16(mx));
-    mx = fmaxf(mx, lane_xor32(mx));
-    const float mn = fmaxf(m, mx);                          // finite: every step holds a visible key
-    const float f = __builtin_amdgcn_exp2f(m - mn);
-    float sum = 0.f;
+    if (!cap.bounded) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+      mx = fmaxf(mx, lane_xor16(mx));
+      mx = fmaxf(mx, lane_xor32(mx));
+      const float mn = fmaxf(m, mx);                        // finite: every step holds a visible key
+      const float f = __builtin_amdgcn_exp2f(m - mn);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) p[i] -= mn;
+      l *= f;
+      m = mn;
+      if (__any(f != 1.f)) {
+#pragma unroll
+        for (int i = 0; i < VCB * 8; ++i) o[i] *= f;
+      }
+    }
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      p[i] = __builtin_amdgcn_exp2f(p[i] - mn);
+      p[i] = __builtin_amdgcn_exp2f(p[i]);
       sum += p[i];
     }
-    l = l * f + sum;
-    m = mn;
-    if (__any(f != 1.f)) {
-#pragma unroll
-      for (int i = 0; i < VCB * 8; ++i) o[i] *= f;
-    }
+    l += sum;
     const u32x4 pf = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]), pack_bf16(p[6], p[7])};
 #pragma unroll
     for (int cb = 0; cb < VCB; ++cb)

@@ -57,6 +57,22 @@ __device__ __forceinline__ float fast_tanh(float x) {
   const float q = x * x;                          // near zero the difference above loses digits
   return fabsf(x) < 0.0625f ? x * (1.f - q * (1.f / 3.f - q * (2.f / 15.f))) : big;
 }
+// Scores of 16-bit attention in powers of two: log2(e) scale x, under a soft cap log2(e) cap tanh(scale x / cap).
+// The cap's tanh is 1 - 2 / (1 + exp(2 z)), whose error is a rounding of the cap, not of the score.  A cap that
+// keeps the powers far inside fp32's range makes a running maximum unnecessary (`bounded`).
+__host__ __device__ inline bool soft_cap_bounded(float cap) { return cap > 0.f && cap * 1.44269504088896f <= 80.f; }
+struct SoftCap {
+  float factor, top;
+  bool on, bounded;
+  __device__ __forceinline__ SoftCap(float scale, float cap)
+      : factor(cap > 0.f ? scale / cap * 2.88539008177793f : scale * 1.44269504088896f), top(cap * 1.44269504088896f),
+        on(cap > 0.f), bounded(soft_cap_bounded(cap)) {}
+  __device__ __forceinline__ float capped(float x) const {
+    return fmaf(-2.f * top, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * factor)), top);
+  }
+  __device__ __forceinline__ float log2_score(float x) const { return on ? capped(x) : x * factor; }
+};
+
 template <typename T> __device__ __forceinline__ float tanh_of(float x);
 template <> __device__ __forceinline__ float tanh_of<F32>(float x) { return tanhf(x); }
 template <> __device__ __forceinline__ float tanh_of<BF16>(float x) { return fast_tanh(x); }

@@ -49,19 +49,26 @@ __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
   return chunk > 0 ? pos / chunk * chunk : 0;
 }
 
+// Two maps: one workgroup of eight waves per CU; else two of four waves, which share its 160 KB.
+constexpr int tile_waves(int maps) { return maps == 2 ? 8 : 4; }
+
 template <int DKS, int VCB, int MAPS> struct TileStage {
   static constexpr int kK = MAPS * DKS * 32 + 8, kV = VCB * 128 + 8;    // row strides: rows 16 bytes apart in the banks
   static constexpr int kElems = kTileK * (kK + kV);
-  static constexpr int kBytes = 2 * kElems * 2;
+  static constexpr int kWaves = tile_waves(MAPS);
+  static constexpr int kBuffers = MAPS == 2 || 8 * kElems <= 160 * 1024 ? 2 : 1;
+  static constexpr int kBytes = kBuffers * kElems * 2;
 };
+
+enum { kNoCap, kCap, kBoundedCap };   // of the scores, see SoftCap
 
 // Column tile t of a wave: 16 queries, map t % MAPS of the head (differential attention has two, over the same
 // values; elsewhere there is one).  SHARED: the last P elements of every head's key are the row of a.ks.
-template <int DKS, int VCB, int kQT, int MAPS, bool SHARED>
-__global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_tiles_kernel(TilesArgs a) {
+template <int DKS, int VCB, int kQT, int MAPS, bool SHARED, int CAP>
+__global__ __launch_bounds__(64 * tile_waves(MAPS), 2) void run_tiles_kernel(TilesArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
   typedef TileStage<DKS, VCB, MAPS> Stage;
-  constexpr int kT = kQT * MAPS;
+  constexpr int kT = kQT * MAPS, kWaves = Stage::kWaves, kThreads = 64 * kWaves, kPass = 16 * kQT * kWaves;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
   const int q0 = a.tiles[tile * 4], nq = min(a.tiles[tile * 4 + 1], kTileQ);
@@ -69,16 +76,15 @@ __global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_t
   // host-made descriptors: rows outside the buffers are not touched
   if (q0 < 0 || kb < 0 || rel < 0 || (int64_t)q0 + nq > a.q_rows || (int64_t)kb + rel + nq > a.k_rows) return;
   const int DT = a.D + (SHARED ? a.P : 0);
-  const float sc = a.cap > 0.f ? a.scale / a.cap : a.scale * 1.44269504088896f;
-  const float capl2 = a.cap * 1.44269504088896f;
+  const SoftCap cap(a.scale, a.cap);
   const int hk = h / (a.H / a.HK);
   const uint16_t* kbase = a.k + (int64_t)kb * a.kv_st + hk * MAPS * a.D;
   const uint16_t* vbase = a.v + (int64_t)kb * a.kv_st + hk * a.V;
   const uint16_t* sbase = SHARED ? a.ks + (int64_t)kb * a.s_st : nullptr;
 
-  for (int wg0 = 0; wg0 < nq; wg0 += 64 * kQT) {              // uniform in the workgroup
+  for (int wg0 = 0; wg0 < nq; wg0 += kPass) {                 // uniform in the workgroup
     const int w0 = wg0 + wave * 16 * kQT;
-    const int last = rel + min(wg0 + 64 * kQT, nq) - 1;       // last key any query of the pass sees
+    const int last = rel + min(wg0 + kPass, nq) - 1;          // last key any query of the pass sees
     const int first = first_seen(rel + wg0, a.window, a.chunk);
     const int hi = w0 < nq ? rel + min(w0 + 16 * kQT, nq) - 1 : -1;      // the same for the wave
     const int lo = first_seen(rel + w0, a.window, a.chunk);
@@ -104,43 +110,52 @@ __global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_t
     float m[kT], l[kT];
 #pragma unroll
     for (int t = 0; t < kT; ++t) {
-      m[t] = -INFINITY;
+      m[t] = CAP == kBoundedCap ? 0.f : -INFINITY;
       l[t] = 0.f;
 #pragma unroll
       for (int i = 0; i < VCB * 8; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
-    u32x4 rk[MAPS * DKS], rv[4 * VCB];                         // this thread's pieces of a tile
-    constexpr int kKP = 4 * MAPS * DKS;                        // pieces of a key row, DKS * 4 per map
-    auto fetch = [&](int k0) {
+    constexpr int kKP = 4 * MAPS * DKS, kVP = 16 * VCB;        // pieces of a key row, DKS * 4 per map, and of a value row
+    constexpr int kKN = kTileK * kKP / kThreads, kVN = kTileK * kVP / kThreads;
+    u32x4 rk[kKN], rv[kVN];                                    // this thread's pieces of a tile
+    auto fetch = [&](int k0) {                                 // offsets from the tile's first row: 32 bits
+      const uint16_t *kt = kbase + k0 * a.kv_st, *vt = vbase + k0 * a.kv_st, *st = SHARED ? sbase + k0 * a.s_st : nullptr;
+      const uint32_t kv_st = (uint32_t)a.kv_st, s_st = (uint32_t)a.s_st;
 #pragma unroll
-      for (int j = 0; j < MAPS * DKS; ++j) {
-        const int id = tid + 256 * j, r = id / kKP, pc = id % kKP, map = pc / (4 * DKS), c = (pc % (4 * DKS)) * 8;
-        const int64_t row = min(k0 + r, last);
-        if (SHARED && c >= a.D) rk[j] = *(const u32x4*)(sbase + row * a.s_st + (c < DT ? c - a.D : 0));
-        else rk[j] = *(const u32x4*)(kbase + row * a.kv_st + map * a.D + (c < a.D ? c : 0));
+      for (int j = 0; j < kKN; ++j) {
+        const int id = tid + kThreads * j, pc = id % kKP, map = pc / (4 * DKS), c = (pc % (4 * DKS)) * 8;
+        const uint32_t r = min(id / kKP, last - k0);
+        if (SHARED) {
+          const bool own = c < a.D;
+          rk[j] = *(const u32x4*)((own ? kt : st) + (own ? r * kv_st + c : r * s_st + (c < DT ? c - a.D : 0)));
+        } else {
+          rk[j] = *(const u32x4*)(kt + (r * kv_st + map * a.D + (c < a.D ? c : 0)));
+        }
       }
 #pragma unroll
-      for (int j = 0; j < 4 * VCB; ++j) {
-        const int id = tid + 256 * j, r = id / (16 * VCB), c = (id % (16 * VCB)) * 8;
-        rv[j] = *(const u32x4*)(vbase + (int64_t)min(k0 + r, last) * a.kv_st + (c < a.V ? c : 0));
+      for (int j = 0; j < kVN; ++j) {
+        const int id = tid + kThreads * j, c = (id % kVP) * 8;
+        const uint32_t r = min(id / kVP, last - k0);
+        rv[j] = *(const u32x4*)(vt + (r * kv_st + (c < a.V ? c : 0)));
       }
     };
     fetch(first);
-    __syncthreads();                                           // a pass before this one still reads its tiles
+    if (Stage::kBuffers == 2) __syncthreads();                 // a pass before this one still reads its tiles
     int buf = 0;
     for (int t0 = first; t0 <= last; t0 += kTileK, buf ^= 1) {
-      uint16_t* const ldsk = (uint16_t*)lds_raw + buf * Stage::kElems;
+      if (Stage::kBuffers == 1) __syncthreads();               // the tile before this one is used up
+      uint16_t* const ldsk = (uint16_t*)lds_raw + (Stage::kBuffers == 2 ? buf * Stage::kElems : 0);
       uint16_t* const ldsv = ldsk + kTileK * Stage::kK;
 #pragma unroll
-      for (int j = 0; j < MAPS * DKS; ++j) {
-        const int id = tid + 256 * j;
+      for (int j = 0; j < kKN; ++j) {
+        const int id = tid + kThreads * j;
         *(u32x4*)(ldsk + id / kKP * Stage::kK + (id % kKP) * 8) = rk[j];
       }
 #pragma unroll
-      for (int j = 0; j < 4 * VCB; ++j) {
-        const int id = tid + 256 * j;
-        *(u32x4*)(ldsv + id / (16 * VCB) * Stage::kV + (id % (16 * VCB)) * 8) = rv[j];
+      for (int j = 0; j < kVN; ++j) {
+        const int id = tid + kThreads * j;
+        *(u32x4*)(ldsv + id / kVP * Stage::kV + (id % kVP) * 8) = rv[j];
       }
       __syncthreads();
       if (t0 + kTileK <= last) fetch(t0 + kTileK);
@@ -167,12 +182,11 @@ __global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_t
         u32x4 pf[kT];
 #pragma unroll
         for (int t = 0; t < kT; ++t) {
-          float p[8], mx = -INFINITY;
+          float p[8], sum = 0.f;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) p[i] = s[t][i >> 2][i & 3] * sc;
-          if (a.cap > 0.f) {
-#pragma unroll
-            for (int i = 0; i < 8; ++i) p[i] = capl2 * fast_tanh(p[i]);
+          for (int i = 0; i < 8; ++i) {
+            const float x = s[t][i >> 2][i & 3];
+            p[i] = CAP == kNoCap ? x * cap.factor : cap.capped(x);
           }
           if (!inner) {
 #pragma unroll
@@ -181,22 +195,25 @@ __global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_t
               if (key > qpos[t / MAPS] || key < qlow[t / MAPS]) p[i] = -INFINITY;
             }
           }
+          float ms = 0.f, f = 1.f;
+          if (CAP != kBoundedCap) {
+            float mx = -INFINITY;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
-          mx = fmaxf(mx, lane_xor16(mx));
-          mx = fmaxf(mx, lane_xor32(mx));
-          const float mn = fmaxf(m[t], mx);
-          const float ms = mn == -INFINITY ? 0.f : mn;          // a query whose window starts later
-          const float f = __builtin_amdgcn_exp2f(m[t] - ms);
-          float sum = 0.f;
+            for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
+            mx = fmaxf(mx, lane_xor16(mx));
+            mx = fmaxf(mx, lane_xor32(mx));
+            const float mn = fmaxf(m[t], mx);
+            ms = mn == -INFINITY ? 0.f : mn;                    // a query whose window starts later
+            f = __builtin_amdgcn_exp2f(m[t] - ms);
+            m[t] = mn;
+          }
 #pragma unroll
           for (int i = 0; i < 8; ++i) {
-            p[i] = __builtin_amdgcn_exp2f(p[i] - ms);
+            p[i] = __builtin_amdgcn_exp2f(CAP == kBoundedCap ? p[i] : p[i] - ms);
             sum += p[i];
           }
-          l[t] = l[t] * f + sum;
-          m[t] = mn;
-          if (__any(f != 1.f)) {
+          l[t] = CAP == kBoundedCap ? l[t] + sum : l[t] * f + sum;
+          if (CAP != kBoundedCap && __any(f != 1.f)) {
 #pragma unroll
             for (int i = 0; i < VCB * 8; ++i) o[t][i] *= f;
           }
@@ -272,37 +289,41 @@ __global__ __launch_bounds__(256, MAPS == 2 && DKS * VCB > 4 ? 1 : 2) void run_t
   }
 }
 
-template <int DKS, int VCB, int kQT, int MAPS, bool SHARED> int launch_run_tiles(const TilesArgs& a, hipStream_t st) {
+template <int DKS, int VCB, int kQT, int MAPS, bool SHARED, int CAP> int launch_run_tiles(const TilesArgs& a, hipStream_t st) {
   constexpr int smem = TileStage<DKS, VCB, MAPS>::kBytes;
   if (smem > 64 * 1024 &&
-      hipFuncSetAttribute((const void*)run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED>,
+      hipFuncSetAttribute((const void*)run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED, CAP>,
                           hipFuncAttributeMaxDynamicSharedMemorySize, smem) != hipSuccess) {
     zp_set_error("run_attention: cannot reserve %d bytes of LDS", smem);
     return ZP_EHIP;
   }
-  hipLaunchKernelGGL((run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED>), dim3((unsigned)a.T * a.H), dim3(256), smem, st, a);
+  hipLaunchKernelGGL((run_tiles_kernel<DKS, VCB, kQT, MAPS, SHARED, CAP>), dim3((unsigned)a.T * a.H),
+                     dim3(64 * TileStage<DKS, VCB, MAPS>::kWaves), smem, st, a);
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }
 
-template <bool SHARED> int launch_one_map(const TilesArgs& a, hipStream_t st) {
+template <bool SHARED, int CAP> int launch_one_map(const TilesArgs& a, hipStream_t st) {
   const int dk = (a.D + a.P + 31) / 32;
   if (a.V <= 128) {
-    if (dk <= 2) return launch_run_tiles<2, 1, 2, 1, SHARED>(a, st);
-    if (dk <= 4) return launch_run_tiles<4, 1, 2, 1, SHARED>(a, st);
-    if (dk <= 6) return launch_run_tiles<6, 1, 2, 1, SHARED>(a, st);
-    return launch_run_tiles<8, 1, 2, 1, SHARED>(a, st);
+    if (dk <= 2) return launch_run_tiles<2, 1, 2, 1, SHARED, CAP>(a, st);
+    if (dk <= 4) return launch_run_tiles<4, 1, 2, 1, SHARED, CAP>(a, st);
+    if (dk <= 6) return launch_run_tiles<6, 1, 2, 1, SHARED, CAP>(a, st);
+    return launch_run_tiles<8, 1, 2, 1, SHARED, CAP>(a, st);
   }
-  if (dk <= 4) return launch_run_tiles<4, 2, 1, 1, SHARED>(a, st);
-  return launch_run_tiles<8, 2, 1, 1, SHARED>(a, st);
+  if (dk <= 4) return launch_run_tiles<4, 2, 1, 1, SHARED, CAP>(a, st);
+  return launch_run_tiles<8, 2, 1, 1, SHARED, CAP>(a, st);
 }
-int launch_two_maps(const TilesArgs& a, hipStream_t st) {
+template <int CAP> int launch_two_maps(const TilesArgs& a, hipStream_t st) {
   const int dk = (a.D + 31) / 32;
   if (a.V <= 128) {
-    if (dk <= 2) return launch_run_tiles<2, 1, 1, 2, false>(a, st);
-    return launch_run_tiles<4, 1, 1, 2, false>(a, st);
+    if (dk <= 2) return launch_run_tiles<2, 1, 1, 2, false, CAP>(a, st);
+    return launch_run_tiles<4, 1, 1, 2, false, CAP>(a, st);
   }
-  return launch_run_tiles<4, 2, 1, 2, false>(a, st);
+  return launch_run_tiles<4, 2, 1, 2, false, CAP>(a, st);
+}
+template <int CAP> int launch_forms(const TilesArgs& a, bool two, hipStream_t st) {
+  return two ? launch_two_maps<CAP>(a, st) : launch_one_map<false, CAP>(a, st);
 }
 
 }  // namespace
@@ -338,17 +359,20 @@ extern "C" int zp_run_attention(const void* q, const void* k, const void* v, con
   }
   if (T == 0) return ZP_OK;
   ZP_REQUIRE(q && k && v && out && tiles, "run_attention: null pointer");
+  ZP_REQUIRE(!P || f.softcap == 0.f, "run_attention: shared keys go without a soft cap");
   ZP_REQUIRE(!two || (!sinks && !P && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
              "run_attention: two maps go without sinks and shared keys, with a mean over the values");
   ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && aligned16(k_shared) && aligned16(f.gate) &&
                  f.gate_stride % 8 == 0 && q_stride % 8 == 0 && kv_stride % 8 == 0 && shared_stride % 8 == 0 &&
                  out_stride % 8 == 0 && q_stride >= (int64_t)H * f.maps * (D + P) && out_stride >= (int64_t)H * V &&
-                 (!P || shared_stride >= P) && (int64_t)T * H < (1ll << 31),
+                 (!P || shared_stride >= P) && (int64_t)T * H < (1ll << 31) &&
+                 kv_stride < (1ll << 26) && shared_stride < (1ll << 26),
              "run_attention: unaligned rows or too many tiles");
   TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (const uint16_t*)k_shared, (uint16_t*)out,
                  tiles, sinks, T, H, HK, D, P, V, window, chunk, q_rows, k_rows, q_stride, kv_stride, shared_stride,
                  out_stride, scale, out_scale, f.softcap, f.balance, f.eps, f.vdim, (const uint16_t*)f.gate, f.gate_stride};
   hipStream_t st = (hipStream_t)stream;
-  if (two) return launch_two_maps(a, st);
-  return P ? launch_one_map<true>(a, st) : launch_one_map<false>(a, st);
+  if (P) return launch_one_map<true, kNoCap>(a, st);
+  if (!(f.softcap > 0.f)) return launch_forms<kNoCap>(a, two, st);
+  return soft_cap_bounded(f.softcap) ? launch_forms<kBoundedCap>(a, two, st) : launch_forms<kCap>(a, two, st);
 }
