@@ -1,9 +1,9 @@
 /* C ABI of the model-side kernels of decoders that need more than the compression library's layer
- * kernels.  Five shared objects, so that a model compiles only what it runs: libzipage_models.so (an
+ * kernels.  Six shared objects, so that a model compiles only what it runs: libzipage_models.so (an
  * fp32 residual stream, attention of prompt runs), libzipage_latent.so (latent attention over pages of
  * latents), libzipage_grouped.so (grouped-query attention, with sinks or of two maps),
- * libzipage_recurrent.so (recurrent mixers) and libzipage_moe.so (mixtures of experts).  Status codes, dtype tags and conventions are those of
- * zipage_hip.h; every entry point here takes ZP_BF16 or ZP_F32 (true 32-bit products), enqueues on
+ * libzipage_recurrent.so (matrix memory, delta rule), libzipage_linear.so (linear attention with decay) and
+ * libzipage_moe.so (mixtures of experts).  Status codes, dtype tags and conventions are those of zipage_hip.h; every entry point here takes ZP_BF16 or ZP_F32 (true 32-bit products), enqueues on
  * `stream`, allocates nothing and may be captured into a HIP graph. */
 #ifndef ZIPAGE_MODELS_H
 #define ZIPAGE_MODELS_H
@@ -15,29 +15,42 @@ extern "C" {
 
 /* ------------------------------------------------------------------ libzipage_models.so */
 
-/* x = embed[tokens] * embed_scale (+ pos[positions] when pos is given), fp32; with norm_weight also
+/* x = embed[tokens] * embed_scale (+ pos[positions] when pos is given), fp32, which goes to `result` when given,
+ * (+ the row `shift`); with norm_weight also
  * out = x / sqrt(mean(x^2) + eps) * (weight_offset + norm_weight) or, with norm_bias,
  * out = tanh(norm_alpha * x) * (weight_offset + norm_weight) + norm_bias.  Rows are `width` long (multiple
  * of 8, zero padded), the mean runs over norm_width.  embed (vocab, width), pos (max_positions,
  * width) and out are of `dtype`; indices are clamped to the tables. */
 int zp_embed_norm(const int64_t* tokens, const int32_t* positions, const void* embed, const void* pos,
-                  float* x, const float* norm_weight, const float* norm_bias, void* out, int32_t n,
-                  int32_t width, int32_t norm_width, int64_t vocab, int64_t max_positions,
-                  float embed_scale, float eps, float weight_offset, float norm_alpha, int32_t dtype,
-                  void* stream);
+                  const float* shift, float* result, float* x, const float* norm_weight,
+                  const float* norm_bias, void* out, int32_t n, int32_t width, int32_t norm_width,
+                  int64_t vocab, int64_t max_positions, float embed_scale, float eps, float weight_offset,
+                  float norm_alpha, int32_t dtype, void* stream);
 
-/* r = x + the sum of y's n_y planes (x (n, width) fp32; y (n_y, n, width) of dtype), where with
- * y_weight the sum is RMS-normed times y_weight before it is added; written to `result` when given; with a depth average
+/* r = x + the branches (x (n, width) fp32; a branch is the sum of `planes` planes (n, width) of dtype, with
+ * `weight` RMS-normed times that weight before it is added; up to three branches, two of them normed); written to
+ * `result` when given; with a depth average
  * r <- mix[n_hist] * r + sum_{j < n_hist} mix[j] * hist[j] (hist: planes of (n, width) fp32,
- * hist_plane elements apart); written to `x_out` when given; with norm_weight also
+ * hist_plane elements apart); plus the row `shift` when given; written to `x_out` when given; with norm_weight also
  * out = rmsnorm(r) * (weight_offset + norm_weight) * out_scale, or with norm_bias
  * out = (tanh(norm_alpha * r) * (weight_offset + norm_weight) + norm_bias) * out_scale.
  * mix NULL: no average. */
-int zp_residual_norm(const float* x, const void* y, int32_t n_y, const float* y_weight,
-                     const float* hist, int64_t hist_plane, const float* mix, int32_t n_hist, float* result, float* x_out,
-                     const float* norm_weight, const float* norm_bias, void* out, int32_t n,
+typedef struct {
+  const void* y;
+  const float* weight;
+  int32_t planes;
+} zp_branch;
+int zp_residual_norm(const float* x, const zp_branch* branches, int32_t n_branches, const float* hist,
+                     int64_t hist_plane, const float* mix, int32_t n_hist, const float* shift, float* result,
+                     float* x_out, const float* norm_weight, const float* norm_bias, void* out, int32_t n,
                      int32_t width, int32_t norm_width, float eps, float weight_offset,
                      float norm_alpha, float out_scale, int32_t dtype, void* stream);
+
+/* Rows z of `in` (in_stride elements apart): a N(z) + b N(z^2) + c N(z^3) + e, powers element by element, N(y) =
+ * y / sqrt(mean(y^2) + eps) with the mean over the first norm_width elements; those behind them are zero. */
+int zp_normed_powers(const void* in, void* out, int32_t n, int32_t width, int32_t norm_width,
+                     int64_t in_stride, int64_t out_stride, float a, float b, float c, float e, float eps,
+                     int32_t dtype, void* stream);
 
 /* z > 0: alpha_p z^2 + z / 2;  z <= 0: alpha_n (exp(z) - 1 - z) + z / 2.  count % 8 == 0. */
 int zp_xielu(const void* in, void* out, int64_t count, float alpha_p, float alpha_n, int32_t dtype,
@@ -59,7 +72,9 @@ int zp_gather_rows(const void* src, const int32_t* rows, void* out, int32_t n, i
  * back; both softmaxes weight the same values, and with their results o1, o2 the output is
  *   rms(o1 - balance * o2) * out_scale * sigmoid(gate),  rms over the first `vdim` values with eps,
  * gate (rows gate_stride elements apart, heads of V back to back, of the call's dtype) or NULL: no gate.
- * Sinks are for one map only. */
+ * Sinks are for one map only.
+ * turns: (rows of q, V / 2) pairs cos, sin of one map whose values turned by angles of their positions; elements 2 i
+ * and 2 i + 1 of every head's output turn back by the query's.  16-byte aligned; NULL: nothing turns. */
 typedef struct {
   float softcap;
   int32_t maps;
@@ -67,6 +82,7 @@ typedef struct {
   int32_t vdim;
   const void* gate;
   int64_t gate_stride;
+  const float* turns;
 } zp_attention_form;
 
 /* Attention of runs of tokens, bfloat16.  tiles (T, 4) int32, one entry per up to 128 queries of one
@@ -124,14 +140,30 @@ int zp_latent_rows_attention(const void* q, const void* cache, const int32_t* ta
 
 /* ------------------------------------------------------------------ libzipage_grouped.so */
 
+/* What else a store of queries, keys and values does; NULL stands for nothing.
+ * norm (H * D + HK * D): weights of RMS norms over the whole of q and the whole of k (means over q_norm and k_norm
+ * elements), before they turn.
+ * tied: the values are the keys as they are in `in`, which has no value columns; VT = HK * D.
+ * value_freqs (V / 2): the values' heads of V turn too, elements 2 i and 2 i + 1 by positions[.] * value_freqs[i];
+ * turns (n, V / 2) receives cos and sin of these angles. */
+typedef struct {
+  const float* norm;
+  int32_t q_norm, k_norm;
+  float eps;
+  int32_t tied;
+  int32_t V;
+  const float* value_freqs;
+  float* turns;
+} zp_store_form;
+
 /* Rows `in` (in_stride elements apart) hold q (H heads of D), k (HK of D) and VT value columns; with `bias`
  * (a row of them) it is added first.  The first `rot` dimensions of q's and k's heads turn by positions[i] *
  * freqs[.], dimension j with j + rot / 2.  q goes to q_out, [k | v] to slot slots[i] of the cache (-1
  * skips) and to kv_out when given. */
 int zp_rotary_store(const void* in, const float* bias, const int32_t* positions, const float* freqs,
-                    void* q_out, void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
-                    int32_t HK, int32_t D, int32_t VT, int32_t rot, int64_t in_stride,
-                    int64_t num_slots, int32_t dtype, void* stream);
+                    const zp_store_form* form, void* q_out, void* kv_out, void* cache, const int32_t* slots,
+                    int32_t n, int32_t H, int32_t HK, int32_t D, int32_t VT, int32_t rot,
+                    int64_t in_stride, int64_t num_slots, int32_t dtype, void* stream);
 
 /* Attention of single tokens over paged rows [k (HK heads of maps * D) | v (HK of V)].  q (n, H, maps * D);
  * token i is the last of the context_lens[i] tokens of its sequence (0: inert, zeros) in row table_rows[i]
@@ -203,6 +235,32 @@ int zp_delta_scan(const zp_delta* args, int32_t dtype, void* stream);
 int64_t zp_delta_runs_workspace(int32_t rows, int32_t segments, int32_t heads, int32_t dk, int32_t dv);
 int zp_delta_runs(const zp_delta* args, int32_t first_row, int32_t longest, void* workspace,
                   int64_t workspace_bytes, int32_t dtype, void* stream);
+
+/* ------------------------------------------------------------------ libzipage_linear.so */
+
+/* Linear attention with decay, S <- g S (rows) + k v^T, o = S^T q, and the normed, silu-gated read-out.  Rows `in`
+ * hold q, k (heads of dk), v, g (heads of dv) from columns q_at, k_at, v_at, g_at.  The first `rot` dimensions of q's
+ * and k's heads turn by position * freqs[.], dimension j with j + rot / 2; q is scaled by q_scale, k by k_scale.
+ * Decays: with `low` (rows of heads of dk), sigmoid(low + decay)^inv_tau with `decay` (heads * dk); without it decay
+ * (heads) itself.  dk 32, 64, 128 or 256, dv a multiple of 32 up to 256, zero padded; the norm's mean runs over vdim,
+ * its weights are (heads * dv).  state: (num_slots, heads, dk, dv) fp32. */
+typedef struct {
+  zp_segments seg;
+  const void *in, *low;
+  const float *decay, *freqs, *norm;
+  float* state;
+  void* out;
+  int64_t in_stride, low_stride, out_stride;
+  int32_t heads, dk, dv, vdim, rot, q_at, k_at, v_at, g_at;
+  float q_scale, k_scale, inv_tau, eps;
+} zp_linear;
+int zp_linear_scan(const zp_linear* args, int32_t dtype, void* stream);
+/* The same for long runs, 16 tokens at a time on the matrix cores (fp32): bfloat16, dk 32, 64 or 128, dv up
+ * to 128, rows given in rising order from first_row on, none longer than `longest`.  `workspace`:
+ * zp_linear_runs_workspace() bytes for the rows from first_row to the end. */
+int64_t zp_linear_runs_workspace(int32_t rows, int32_t segments, int32_t heads, int32_t dk);
+int zp_linear_runs(const zp_linear* args, int32_t first_row, int32_t longest, void* workspace,
+                   int64_t workspace_bytes, int32_t dtype, void* stream);
 
 /* ------------------------------------------------------------------ libzipage_moe.so */
 

@@ -49,7 +49,7 @@ def test_models_library_exports_every_declared_symbol():
     assert lib.zp_latent_rows_attention(None, None, None, None, None, None, 1, 1, 32, 0, 16, 1, 1, 1, -1, 1.0, 0,
                                         None, 0, None) == 1
     lib = _lib.load_models("models")
-    assert lib.zp_embed_norm(None, None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1.0, 1e-6, 0.0, 0.0, 0, None) != 0
+    assert lib.zp_embed_norm(None, None, None, None, None, None, None, None, None, None, 1, 12, 12, 5, 5, 1.0, 1e-6, 0.0, 0.0, 0, None) != 0
     assert lib.zp_run_attention(None, None, None, None, None, None, None, None, 1, 4, 3, 32, 0, 32, 0, 0, 1, 1, 128, 256, 0,
                                 128, 1.0, 1.0, 0, None) == 1
     lib = _lib.load_models("grouped")

@@ -85,6 +85,11 @@ I64_RETURNING = {
 }
 EXPORTS = sorted(list(SIGNATURES) + list(I64_RETURNING) + ["zp_abi_version", "zp_last_error"])
 
+class Branch(C.Structure):
+    """zp_branch of include/zipage_models.h."""
+    _fields_ = [("y", ptr), ("weight", ptr), ("planes", i32)]
+
+
 class Segments(C.Structure):
     """zp_segments of include/zipage_models.h."""
     _fields_ = [(n, ptr) for n in ("rows", "counts", "slots", "starts")] + \
@@ -109,10 +114,25 @@ class DeltaArgs(C.Structure):
         [(n, f32) for n in ("q_scale", "eps", "out_scale")]
 
 
+class LinearArgs(C.Structure):
+    """zp_linear."""
+    _fields_ = [("seg", Segments)] + \
+        [(n, ptr) for n in ("inp", "low", "decay", "freqs", "norm", "state", "out")] + \
+        [(n, i64) for n in ("in_stride", "low_stride", "out_stride")] + \
+        [(n, i32) for n in ("heads", "dk", "dv", "vdim", "rot", "q_at", "k_at", "v_at", "g_at")] + \
+        [(n, f32) for n in ("q_scale", "k_scale", "inv_tau", "eps")]
+
+
 class AttentionForm(C.Structure):
     """zp_attention_form."""
     _fields_ = [("softcap", f32), ("maps", i32), ("balance", f32), ("eps", f32), ("vdim", i32), ("gate", ptr),
-                ("gate_stride", i64)]
+                ("gate_stride", i64), ("turns", ptr)]
+
+
+class StoreForm(C.Structure):
+    """zp_store_form."""
+    _fields_ = [("norm", ptr), ("q_norm", i32), ("k_norm", i32), ("eps", f32), ("tied", i32), ("V", i32),
+                ("value_freqs", ptr), ("turns", ptr)]
 
 
 SCORE_SOFTMAX, SCORE_SIGMOID = 0, 1      # ZP_SCORE_*
@@ -123,9 +143,10 @@ form_ptr = C.POINTER(AttentionForm)
 # return an int64 count instead of a status)
 MODEL_LIBS = {
     "models": ({
-        "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, f32, i32, ptr],
-        "zp_residual_norm": [ptr, ptr, i32, ptr, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, f32, f32,
-                             f32, f32, i32, ptr],
+        "zp_embed_norm": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, f32, i32, ptr],
+        "zp_residual_norm": [ptr, C.POINTER(Branch), i32, ptr, i64, ptr, i32, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32,
+                             f32, f32, f32, f32, i32, ptr],
+        "zp_normed_powers": [ptr, ptr, i32, i32, i32, i64, i64, f32, f32, f32, f32, f32, i32, ptr],
         "zp_xielu": [ptr, ptr, i64, f32, f32, i32, ptr],
         "zp_relu_square": [ptr, ptr, i64, i32, ptr],
         "zp_softcap": [ptr, ptr, i64, f32, i32, ptr],
@@ -142,7 +163,8 @@ MODEL_LIBS = {
                                      i32, ptr, i64, ptr],
     }, {"zp_latent_rows_workspace": [i32, i32, i32, i32, i32, i32, i32]}),
     "grouped": ({
-        "zp_rotary_store": [ptr, ptr, ptr, ptr, ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i64, i64, i32, ptr],
+        "zp_rotary_store": [ptr, ptr, ptr, ptr, C.POINTER(StoreForm), ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i64,
+                            i64, i32, ptr],
         "zp_grouped_rows_attention": [ptr, ptr, ptr, ptr, ptr, ptr, form_ptr, ptr, i32, i32, i32, i32, i32, i32, i32,
                                       i32, i32, i32, i32, i64, f32, f32, i32, ptr, i64, ptr],
     }, {"zp_grouped_rows_workspace": [i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32]}),
@@ -152,6 +174,10 @@ MODEL_LIBS = {
         "zp_delta_scan": [C.POINTER(DeltaArgs), i32, ptr],
         "zp_delta_runs": [C.POINTER(DeltaArgs), i32, i32, ptr, i64, i32, ptr],
     }, {"zp_mlstm_runs_workspace": [i32, i32, i32], "zp_delta_runs_workspace": [i32, i32, i32, i32, i32]}),
+    "linear": ({
+        "zp_linear_scan": [C.POINTER(LinearArgs), i32, ptr],
+        "zp_linear_runs": [C.POINTER(LinearArgs), i32, i32, ptr, i64, i32, ptr],
+    }, {"zp_linear_runs_workspace": [i32, i32, i32, i32]}),
     "moe": ({
         "zp_small_linear": [ptr, ptr, ptr, i32, i32, i32, i64, i32, ptr],
         "zp_moe_select": [ptr, ptr, ptr, ptr, i32, i32, i32, i32, i32, i32, i32, ptr],

@@ -3,7 +3,7 @@
 Run as ``python -m zipage_amd.build``.  Shared objects with a plain C ABI, none linked against
 torch: ``libzipage_hip.so`` (``include/zipage_hip.h``: the compression path and the kernels of the
 models that use it) and, for the other models, ``libzipage_models.so``, ``libzipage_latent.so``,
-``libzipage_grouped.so``, ``libzipage_recurrent.so`` and ``libzipage_moe.so``
+``libzipage_grouped.so``, ``libzipage_recurrent.so``, ``libzipage_linear.so`` and ``libzipage_moe.so``
 (``include/zipage_models.h``), so that a model compiles only what it runs.
 """
 from __future__ import annotations
@@ -20,6 +20,7 @@ MODELS_LIB = os.path.join(HERE, "libzipage_models.so")
 LATENT_LIB = os.path.join(HERE, "libzipage_latent.so")
 GROUPED_LIB = os.path.join(HERE, "libzipage_grouped.so")
 RECURRENT_LIB = os.path.join(HERE, "libzipage_recurrent.so")
+LINEAR_LIB = os.path.join(HERE, "libzipage_linear.so")
 MOE_LIB = os.path.join(HERE, "libzipage_moe.so")
 
 # packed fp32 VALU ops are disabled on purpose (some forms misbehave on this fleet)
@@ -37,6 +38,7 @@ MODEL_SOURCES = {
     LATENT_LIB: ("latent.hip",),
     GROUPED_LIB: ("grouped.hip",),
     RECURRENT_LIB: ("mlstm.hip", "mlstm_runs.hip", "delta.hip", "delta_runs.hip"),
+    LINEAR_LIB: ("linear.hip", "linear_runs.hip"),
     MOE_LIB: ("moe.hip",),
 }
 COMMON_SOURCES = ("runtime.hip",)

@@ -1,6 +1,7 @@
 // Grouped-query attention over paged rows [keys of all heads | values of all heads] per token.
 //
-//   rotary_store    rotary positions on queries and keys; keys and values to their cache slot
+//   rotary_store    rotary positions on queries and keys, and on values where those turn too; norms over
+//                   the whole projections before that; keys and values to their cache slot
 //   grouped_rows    attention of single tokens over the pages; the query heads of a key head share
 //                   one read of its keys and values
 //   grouped_plain   float32 form (true fp32 products), any sizes
@@ -9,7 +10,8 @@
 // block of positions, or everything before it; a sink is a logit per head that joins the softmax's
 // denominator only.  A head may hold two maps over the same values (differential attention): in
 // grouped_rows they are two query columns of a key head of twice the length, each with zeros where the
-// other one's elements are, so that keys and values are still read once.
+// other one's elements are, so that keys and values are still read once.  Values that turned with their
+// position turn back with the query's in the last step of a kernel.
 #include "mfma.h"
 
 namespace {
@@ -26,20 +28,58 @@ struct RotaryArgs {
   const int32_t* slots;     // (n,), -1 skips
   int n, H, HK, D, VT, half; // half = rotated dimensions / 2
   int64_t in_st, num_slots;
+  // what only some designs have
+  const float* norm;        // (H * D + HK * D,) weights of RMS norms over all of q and all of k, or null
+  int q_norm, k_norm;       // lengths of their means
+  float eps;
+  bool tied;                // the values are the keys as projected; rows of `in` end with k
+  int V;                    // of a value head
+  const float* vfreqs;      // (V / 2,): values turn, elements 2 i and 2 i + 1 with frequency i; or null
+  float2* turns;            // (n, V / 2): cos and sin of the values' angles, for the way back
 };
 constexpr int kRotTokens = 4;
 
 // Four tokens per workgroup: their angles once, in LDS, for all heads.  VEC elements per item; an
-// item of the rotated part is the pair (i .. i + VEC, i + half ..).
-template <typename T, int VEC>
+// item of the rotated part is the pair (i .. i + VEC, i + half ..).  FORMS: norms, tied or turning values.
+template <typename T, int VEC, bool FORMS>
 __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
+  __shared__ float rms[2][kRotTokens];
   float2* cs = (float2*)lds_raw;            // [kRotTokens][half]
+  float2* vcs = cs + kRotTokens * a.half;   // [kRotTokens][V / 2]
   const int n0 = blockIdx.x * kRotTokens, tid = threadIdx.x;
   for (int i = tid; i < kRotTokens * a.half; i += 256) {
     const int tok = i / a.half;
     if (n0 + tok < a.n) {
       cs[i] = rotary_turn(a.positions[n0 + tok], a.freqs[i - tok * a.half]);
+    }
+  }
+  if (FORMS && a.vfreqs) {
+    const int vh = a.V / 2;
+    for (int i = tid; i < kRotTokens * vh; i += 256) {
+      const int tok = i / vh;
+      if (n0 + tok < a.n) {
+        vcs[i] = rotary_turn(a.positions[n0 + tok], a.vfreqs[i - tok * vh]);
+        a.turns[(int64_t)n0 * vh + i] = vcs[i];
+      }
+    }
+  }
+  if (FORMS && a.norm) {                    // a wave per token
+    const int64_t row = min(n0 + (tid >> 6), a.n - 1);
+    const int edge = a.H * a.D, end = edge + a.HK * a.D;
+    float qs = 0.f, ks = 0.f;
+    for (int c = (tid & 63) * 8; c < end; c += 512) {
+      float x[8], s = 0.f;
+      Vec8<T>::ld(a.in, row * a.in_st + c, x);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s = fmaf(x[i], x[i], s);
+      if (c < edge) qs += s; else ks += s;
+    }
+    qs = wave_sum(qs);
+    ks = wave_sum(ks);
+    if ((tid & 63) == 0) {
+      rms[0][tid >> 6] = 1.f / sqrtf(qs / (float)a.q_norm + a.eps);
+      rms[1][tid >> 6] = 1.f / sqrtf(ks / (float)a.k_norm + a.eps);
     }
   }
   __syncthreads();
@@ -51,7 +91,7 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
     const int64_t row = n0 + tok;
     if (row >= a.n) break;
     float x[VEC], y[VEC];
-    auto load = [&](int c, float* o) {
+    auto raw = [&](int c, float* o) {
       const int64_t at = row * a.in_st + c;
       if constexpr (VEC == 8) Vec8<T>::ld(a.in, at, o); else o[0] = Elem<T>::ld(a.in, at);
       if (a.bias) {
@@ -59,6 +99,16 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
         if constexpr (VEC == 8) Vec8<F32>::ld(a.bias, c, b); else b[0] = a.bias[c];
 #pragma unroll
         for (int i = 0; i < VEC; ++i) o[i] += b[i];
+      }
+    };
+    auto load = [&](int c, float* o) {         // of q or k
+      raw(c, o);
+      if (FORMS && a.norm) {
+        float w[VEC];
+        if constexpr (VEC == 8) Vec8<F32>::ld(a.norm, c, w); else w[0] = a.norm[c];
+        const float r = rms[c < a.H * a.D ? 0 : 1][tok];
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) o[i] *= r * w[i];
       }
     };
     int64_t slot = a.slots[row];
@@ -80,8 +130,19 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
       }
     };
     if (it >= rotated) {
-      const int c = heads * a.D + (it - rotated) * VEC;
-      load(c, x);
+      const int v = (it - rotated) * VEC, c = heads * a.D + v;
+      const int from = FORMS && a.tied ? a.H * a.D + v : c;
+      raw(from, x);
+      if (FORMS && a.vfreqs) {
+        const float2* r = vcs + tok * (a.V / 2) + v % a.V / 2;
+        if constexpr (VEC == 8) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) turn_pair(x[2 * i], x[2 * i + 1], r[i].x, r[i].y);
+        } else {
+          raw(from ^ 1, y);                    // heads start at even columns
+          x[0] = v & 1 ? x[0] * r->x + y[0] * r->y : x[0] * r->x - y[0] * r->y;
+        }
+      }
       put(c, x);
       continue;
     }
@@ -98,9 +159,7 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
 #pragma unroll
     for (int i = 0; i < VEC; ++i) {
       const float2 r = cs[tok * a.half + p * VEC + i];
-      const float u = x[i], v = y[i];
-      x[i] = u * r.x - v * r.y;
-      y[i] = v * r.x + u * r.y;
+      turn_pair(x[i], y[i], r.x, r.y);
     }
     put(c, x);
     put(c + a.half, y);
@@ -129,6 +188,7 @@ struct RowsArgs {
   int vdim;
   const void* gate;       // token rows of g_st elements, head h at h * V; or null
   int64_t g_st;
+  const float2* turns;    // one map: (n, V / 2) cos and sin, results turn back by them; or null
 };
 
 // A piece of a head's result, normed: scale and gate it, and store it.
@@ -358,8 +418,10 @@ __global__ __launch_bounds__(256, 2) void grouped_rows_kernel(RowsArgs a) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) r[i] += x[i] * f;
     }
-    if (a.splits == 1) Vec8<BF16>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, r);
-    else Vec8<F32>::st(a.part, (((int64_t)row * a.H + h) * a.splits + split) * a.V + c, r);
+    if (a.splits == 1) {
+      if (a.turns) turn_back8(r, a.turns + ((int64_t)row * a.V + c) / 2);
+      Vec8<BF16>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, r);
+    } else Vec8<F32>::st(a.part, (((int64_t)row * a.H + h) * a.splits + split) * a.V + c, r);
   }
 }
 
@@ -384,6 +446,7 @@ __global__ __launch_bounds__(64) void grouped_combine_kernel(RowsArgs a) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) acc[i] += v[i] * f;
     }
+    if (a.turns) turn_back8(acc, a.turns + (item / a.H * a.V + c) / 2);
     Vec8<BF16>::st(a.out, item / a.H * a.o_st + (int64_t)h * a.V + c, acc);
   }
 }
@@ -503,6 +566,11 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(RowsArgs a) {
     const int c = tid + i * 256;
     if (c >= a.V) continue;
     float r = total[i] * scale;
+    if (MAPS == 1 && a.turns) {              // the pair's other element is the neighbouring lane's
+      const float other = __shfl_xor(r, 1);
+      const float2 t = a.turns[((int64_t)row * a.V + c) / 2];
+      r = c & 1 ? r * t.x - other * t.y : r * t.x + other * t.y;
+    }
     if (MAPS == 2 && a.gate) r *= sigmoid_of<T>(Elem<T>::ld(a.gate, row * a.g_st + (int64_t)h * a.V + c));
     Elem<T>::st(a.out, row * a.o_st + (int64_t)h * a.V + c, r);
   }
@@ -554,11 +622,12 @@ template <int MAPS> int dispatch_rows(const RowsArgs& a, hipStream_t st) {
 }  // namespace
 
 extern "C" int zp_rotary_store(const void* in, const float* bias, const int32_t* positions, const float* freqs,
-                               void* q_out, void* kv_out, void* cache, const int32_t* slots, int32_t n, int32_t H,
-                               int32_t HK, int32_t D, int32_t VT, int32_t rot, int64_t in_stride,
-                               int64_t num_slots, int32_t dtype, void* stream) {
+                               const zp_store_form* form, void* q_out, void* kv_out, void* cache, const int32_t* slots,
+                               int32_t n, int32_t H, int32_t HK, int32_t D, int32_t VT, int32_t rot,
+                               int64_t in_stride, int64_t num_slots, int32_t dtype, void* stream) {
+  const zp_store_form plain = {}, f = form ? *form : plain;
   ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && D > 0 && VT > 0 && rot >= 0 && rot % 2 == 0 && rot <= D && num_slots > 0 &&
-                 in_stride >= (int64_t)(H + HK) * D + VT, "rotary_store: bad dims");
+                 in_stride >= (int64_t)(H + HK) * D + (f.tied ? 0 : VT), "rotary_store: bad dims");
   ZP_MODEL_DTYPE("rotary_store");
   if (D % 8 != 0 || VT % 8 != 0 || in_stride % 8 != 0 || rot > 2048) {
     zp_set_error("rotary_store: head size %d, value columns %d (multiples of 8), %d rotated (<= 2048)", D, VT, rot);
@@ -566,18 +635,27 @@ extern "C" int zp_rotary_store(const void* in, const float* bias, const int32_t*
   }
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(in && positions && q_out && cache && slots && (rot == 0 || freqs), "rotary_store: null pointer");
-  ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache) && aligned16(bias),
+  ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache) && aligned16(bias) && aligned16(f.norm),
              "rotary_store: tensors must be 16-byte aligned");
-  RotaryArgs a = {in, bias, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, VT, rot / 2, in_stride, num_slots};
+  ZP_REQUIRE(!f.norm || (!bias && f.q_norm > 0 && f.k_norm > 0), "rotary_store: norms of whole projections go without a bias");
+  ZP_REQUIRE(!f.tied || VT == HK * D, "rotary_store: values that are the keys have their size");
+  ZP_REQUIRE(!f.value_freqs || (f.turns && f.V > 0 && f.V % 8 == 0 && f.V <= 1024 && VT % f.V == 0),
+             "rotary_store: values that turn need their head size and room for the turns");
+  RotaryArgs a = {in, bias, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, VT, rot / 2, in_stride, num_slots,
+                  f.norm, f.q_norm, f.k_norm, f.eps, f.tied != 0, f.V, f.value_freqs, (float2*)f.turns};
   const unsigned grid = (unsigned)((n + kRotTokens - 1) / kRotTokens);
-  const size_t smem = sizeof(float2) * kRotTokens * (rot / 2);
+  const size_t smem = sizeof(float2) * kRotTokens * (rot / 2 + (f.value_freqs ? f.V / 2 : 0));
   hipStream_t st = (hipStream_t)stream;
-#define ZP_ROTARY(T)                                                                                          \
-  do {                                                                                                        \
-    if (rot % 16 == 0) hipLaunchKernelGGL((rotary_store_kernel<T, 8>), dim3(grid), dim3(256), smem, st, a);   \
-    else hipLaunchKernelGGL((rotary_store_kernel<T, 1>), dim3(grid), dim3(256), smem, st, a);                 \
+#define ZP_ROTARY(T, VEC)                                                                                          \
+  do {                                                                                                             \
+    if (form) hipLaunchKernelGGL((rotary_store_kernel<T, VEC, true>), dim3(grid), dim3(256), smem, st, a);         \
+    else hipLaunchKernelGGL((rotary_store_kernel<T, VEC, false>), dim3(grid), dim3(256), smem, st, a);             \
   } while (0)
-  if (dtype == ZP_BF16) ZP_ROTARY(BF16); else ZP_ROTARY(F32);
+  if (dtype == ZP_BF16) {
+    if (rot % 16 == 0) ZP_ROTARY(BF16, 8); else ZP_ROTARY(BF16, 1);
+  } else {
+    if (rot % 16 == 0) ZP_ROTARY(F32, 8); else ZP_ROTARY(F32, 1);
+  }
 #undef ZP_ROTARY
   ZP_LAUNCH_CHECK();
   return ZP_OK;
@@ -604,7 +682,7 @@ extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const
                                          int32_t NB, int32_t num_pages, int32_t window, int32_t chunk,
                                          int64_t out_stride, float scale, float out_scale, int32_t dtype,
                                          void* workspace, int64_t workspace_bytes, void* stream) {
-  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0}, f = form ? *form : plain;
+  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0, nullptr}, f = form ? *form : plain;
   const bool two = f.maps == 2;
   ZP_REQUIRE(n >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && V > 0 && BS > 0 && B > 0 && NB > 0 &&
                  num_pages > 0 && window >= 0 && chunk >= 0 && !(window && chunk) && (f.maps == 1 || two) &&
@@ -617,8 +695,8 @@ extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const
   if (n == 0) return ZP_OK;
   ZP_REQUIRE(q && cache && table && context_lens && out, "grouped_rows_attention: null pointer");
   ZP_REQUIRE(table_rows || n <= B, "grouped_rows_attention: more tokens than table rows");
-  ZP_REQUIRE(!two || (!sinks && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
-             "grouped_rows_attention: two maps go without sinks, with a mean over the values");
+  ZP_REQUIRE(!two || (!sinks && !f.turns && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
+             "grouped_rows_attention: two maps go without sinks and turns, with a mean over the values");
   ZP_REQUIRE(aligned16(q) && aligned16(cache) && aligned16(out) && aligned16(workspace) && aligned16(f.gate) &&
                  f.gate_stride % 8 == 0 && out_stride % 8 == 0 && out_stride >= (int64_t)H * V,
              "grouped_rows_attention: tensors must be 16-byte aligned");
@@ -628,7 +706,7 @@ extern "C" int zp_grouped_rows_attention(const void* q, const void* cache, const
   a.part = (float*)workspace; a.n = n; a.H = H * f.maps; a.HK = HK; a.D = DK; a.V = V; a.BS = BS; a.B = B; a.NB = NB;
   a.num_pages = num_pages; a.window = window; a.chunk = chunk; a.o_st = out_stride; a.scale = scale;
   a.out_scale = out_scale; a.bs_shift = -1; a.cap = f.softcap; a.balance = f.balance; a.eps = f.eps; a.vdim = f.vdim;
-  a.gate = f.gate; a.g_st = f.gate_stride;
+  a.gate = f.gate; a.g_st = f.gate_stride; a.turns = (const float2*)f.turns;
   if ((BS & (BS - 1)) == 0)
     for (a.bs_shift = 0; (1 << a.bs_shift) < BS; ++a.bs_shift) {}
   int64_t pages = NB;

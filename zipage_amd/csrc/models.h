@@ -86,3 +86,17 @@ __device__ __forceinline__ float2 rotary_turn(int position, float freq) {
   sincosf((float)position * freq, &s, &c);
   return make_float2(c, s);
 }
+// A pair turns by an angle.
+__device__ __forceinline__ void turn_pair(float& u, float& v, float c, float s) {
+  const float x = u, y = v;
+  u = x * c - y * s;
+  v = y * c + x * s;
+}
+// Eight elements, adjacent ones a pair, turn back by the angles of four (cos, sin).
+__device__ __forceinline__ void turn_back8(float* r, const float2* t) {
+  const zp_f32x4 a = ((const zp_f32x4*)t)[0], b = ((const zp_f32x4*)t)[1];
+  turn_pair(r[0], r[1], a[0], -a[1]);
+  turn_pair(r[2], r[3], a[2], -a[3]);
+  turn_pair(r[4], r[5], b[0], -b[1]);
+  turn_pair(r[6], r[7], b[2], -b[3]);
+}

@@ -34,6 +34,7 @@ struct TilesArgs {
   int vdim;
   const uint16_t* gate;   // token rows of g_st elements, head h at h * V; or null
   int64_t g_st;
+  const float2* turns;    // one map: (q_rows, V / 2) cos and sin, results turn back by them; or null
 };
 
 constexpr int kTileQ = 128;   // queries per workgroup
@@ -68,6 +69,7 @@ template <int DKS, int VCB, int kQT, int MAPS, bool SHARED, int CAP>
 __global__ __launch_bounds__(64 * tile_waves(MAPS), 2) void run_tiles_kernel(TilesArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
   typedef TileStage<DKS, VCB, MAPS> Stage;
+  constexpr bool kTurns = MAPS == 1 && !SHARED && CAP == kNoCap;
   constexpr int kT = kQT * MAPS, kWaves = Stage::kWaves, kThreads = 64 * kWaves, kPass = 16 * kQT * kWaves;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % a.H, tile = blockIdx.x / a.H;   // one head's tiles share an L2 when H % 8 == 0
@@ -266,6 +268,8 @@ __global__ __launch_bounds__(64 * tile_waves(MAPS), 2) void run_tiles_kernel(Til
       const int qi = w0 + qt * 16 + l16;
       if (qi >= nq) continue;
       uint16_t* out = a.out + (int64_t)(q0 + qi) * a.o_st + h * a.V;
+      const float2* turns = a.turns;
+      asm volatile("" : "+s"(turns));                          // nothing of the way back is computed before the loop
       const uint16_t* gate = MAPS == 2 && a.gate ? a.gate + (int64_t)(q0 + qi) * a.g_st + h * a.V : nullptr;
 #pragma unroll
       for (int cb = 0; cb < VCB; ++cb)
@@ -276,6 +280,7 @@ __global__ __launch_bounds__(64 * tile_waves(MAPS), 2) void run_tiles_kernel(Til
             float r[8];
 #pragma unroll
             for (int c = 0; c < 8; ++c) r[c] = o[qt * MAPS][cb * 8 + c][i] * inv[0];
+            if (kTurns && turns) turn_back8(r, turns + ((int64_t)(q0 + qi) * a.V + col) / 2);
             if (MAPS == 2 && gate) {
               float z[8];
               Vec8<BF16>::ld(gate, col, z);
@@ -347,7 +352,7 @@ extern "C" int zp_run_attention(const void* q, const void* k, const void* v, con
                                 int32_t chunk, int64_t q_rows, int64_t k_rows, int64_t q_stride,
                                 int64_t kv_stride, int64_t shared_stride, int64_t out_stride, float scale,
                                 float out_scale, int32_t dtype, void* stream) {
-  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0}, f = form ? *form : plain;
+  const zp_attention_form plain = {0.f, 1, 0.f, 0.f, 0, nullptr, 0, nullptr}, f = form ? *form : plain;
   const bool two = f.maps == 2;
   ZP_REQUIRE(T >= 0 && H > 0 && HK > 0 && H % HK == 0 && D > 0 && P >= 0 && V > 0 && window >= 0 && chunk >= 0 &&
                  !(window && chunk) && (f.maps == 1 || two) && f.softcap >= 0.f && (P > 0) == (k_shared != nullptr),
@@ -360,8 +365,9 @@ extern "C" int zp_run_attention(const void* q, const void* k, const void* v, con
   if (T == 0) return ZP_OK;
   ZP_REQUIRE(q && k && v && out && tiles, "run_attention: null pointer");
   ZP_REQUIRE(!P || f.softcap == 0.f, "run_attention: shared keys go without a soft cap");
-  ZP_REQUIRE(!two || (!sinks && !P && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
-             "run_attention: two maps go without sinks and shared keys, with a mean over the values");
+  ZP_REQUIRE(!f.turns || (!P && f.softcap == 0.f && aligned16(f.turns)), "run_attention: turns go without shared keys and soft cap");
+  ZP_REQUIRE(!two || (!sinks && !P && !f.turns && f.vdim > 0 && f.vdim <= V && (!f.gate || f.gate_stride >= (int64_t)H * V)),
+             "run_attention: two maps go without sinks, shared keys and turns, with a mean over the values");
   ZP_REQUIRE(aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out) && aligned16(k_shared) && aligned16(f.gate) &&
                  f.gate_stride % 8 == 0 && q_stride % 8 == 0 && kv_stride % 8 == 0 && shared_stride % 8 == 0 &&
                  out_stride % 8 == 0 && q_stride >= (int64_t)H * f.maps * (D + P) && out_stride >= (int64_t)H * V &&
@@ -370,7 +376,8 @@ extern "C" int zp_run_attention(const void* q, const void* k, const void* v, con
              "run_attention: unaligned rows or too many tiles");
   TilesArgs a = {(const uint16_t*)q, (const uint16_t*)k, (const uint16_t*)v, (const uint16_t*)k_shared, (uint16_t*)out,
                  tiles, sinks, T, H, HK, D, P, V, window, chunk, q_rows, k_rows, q_stride, kv_stride, shared_stride,
-                 out_stride, scale, out_scale, f.softcap, f.balance, f.eps, f.vdim, (const uint16_t*)f.gate, f.gate_stride};
+                 out_stride, scale, out_scale, f.softcap, f.balance, f.eps, f.vdim, (const uint16_t*)f.gate, f.gate_stride,
+                 (const float2*)f.turns};
   hipStream_t st = (hipStream_t)stream;
   if (P) return launch_one_map<true, kNoCap>(a, st);
   if (!(f.softcap > 0.f)) return launch_forms<kNoCap>(a, two, st);

@@ -71,8 +71,9 @@ template <> __device__ __forceinline__ void store4<F32>(void* p, int64_t i, cons
 
 constexpr int kScanTokens = 16;   // tokens staged in LDS at a time
 
-// Readout of one token by one wave: o (dv values in LDS, the mean over vdim) normed, weighted, gated.
-template <typename T>
+// Readout of one token by one wave: o (dv values in LDS, the mean over vdim) normed, weighted, gated by a sigmoid
+// or a silu.
+template <typename T, bool SILU = false>
 __device__ __forceinline__ void gated_norm_row(const float* o, float o_scale, int dv, int vdim, float eps,
                                                const float* w, const void* gate, int64_t gate_at, float scale,
                                                void* out, int64_t out_at) {
@@ -84,8 +85,10 @@ __device__ __forceinline__ void gated_norm_row(const float* o, float o_scale, in
   }
   ss = wave_sum(ss);
   const float rs = scale / sqrtf(ss / (float)vdim + eps) * o_scale;
-  for (int c = lane; c < dv; c += 64)
-    Elem<T>::st(out, out_at + c, o[c] * rs * w[c] * sigmoid_f(Elem<T>::ld(gate, gate_at + c)));
+  for (int c = lane; c < dv; c += 64) {
+    const float z = Elem<T>::ld(gate, gate_at + c);
+    Elem<T>::st(out, out_at + c, o[c] * rs * w[c] * (SILU ? z * sigmoid_f(z) : sigmoid_f(z)));
+  }
 }
 
 template <typename T>

@@ -7,6 +7,7 @@ from dataclasses import dataclass
 from typing import Any, Callable
 
 from .kapolorn import Kapolorn, KapolornShape
+from .mefupel import Mefupel, MefupelShape
 from .pedivik import Pedivik, PedivikShape
 from .qwen3 import Qwen3, Qwen3Shape
 from .rutevik import Rutevik, RutevikShape
@@ -30,6 +31,8 @@ ARCHITECTURES = {a.name: a for a in (
                  ("MODELS_LIB", "GROUPED_LIB", "RECURRENT_LIB", "MOE_LIB")),
     Architecture("Rutevik", Rutevik, RutevikShape, RutevikShape.from_config,
                  ("MODELS_LIB", "LATENT_LIB", "GROUPED_LIB", "MOE_LIB")),
+    Architecture("Mefupel", Mefupel, MefupelShape, MefupelShape.from_config,
+                 ("MODELS_LIB", "GROUPED_LIB", "LINEAR_LIB")),
 )}
 
 

@@ -1,5 +1,5 @@
-"""Recurrent mixers: a matrix memory with exponential gates, and a gated delta rule with a decay per key
-channel.  Both keep a float32 matrix per head and sequence slot; a step hands them its portions as
+"""Recurrent mixers: a matrix memory with exponential gates, a gated delta rule with a decay per key channel, and
+linear attention with decay.  All keep a float32 matrix per head and sequence slot; a step hands them its portions as
 segments (`StepContext.segments`, and `.run_segments` where 16 tokens at a time pay)."""
 from __future__ import annotations
 
@@ -12,6 +12,7 @@ from zipage_amd import _lib
 
 from .linear import fit, pad_to_multiple
 from .moe import small_linear
+from .rotary import Rotary
 
 
 def _key_size(n: int) -> int:
@@ -186,3 +187,86 @@ class ChannelDelta:
             ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
             _lib.call_models("zp_delta_runs", ctypes.byref(args), segments.first_row, segments.longest,
                              _lib.dev_ptr(ws), size, tag, stream)
+
+
+class LinearAttention:
+    """Per head S <- g * S (rows) + k v^T, o = S^T q, a norm per head and a silu gate.  Decays: with `tau` one per key
+    channel, sigmoid(a low-rank product + bias)^(1 / tau), whose rank the tensors give; else the numbers `decay`, one
+    per head.  `rotary`: q and k turn with their position.  `weighted`: the norm has weights, shared by the heads."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, eps: float, q_scale: float = 1.0, k_scale: float = 1.0,
+                 tau: float | None = None, decay: tuple[float, ...] | None = None, rotary: Rotary | None = None,
+                 weighted: bool = False):
+        if (tau is None) == (decay is None) or decay is not None and len(decay) != heads:
+            raise ValueError(f"decays come from tau or are one per head: {tau}, {decay} for {heads} heads")
+        if rotary is not None and (rotary.dims % 2 or rotary.dims > dim):
+            raise ValueError(f"{rotary.dims} rotated dimensions of {dim}")
+        self.width, self.heads, self.dim, self.vdim, self.eps = width, heads, dim, vdim, eps
+        self.q_scale, self.k_scale, self.tau, self.decay, self.rotary, self.weighted = q_scale, k_scale, tau, decay, rotary, weighted
+        self.dim_p, self.vdim_p = _key_size(dim), _value_size(vdim)
+        self.low_at = 2 * heads * (self.dim_p + self.vdim_p)
+        self.out_columns = heads * self.vdim_p
+
+    def shapes(self, a_rank: int = 1) -> dict:
+        H, D, V, W = self.heads, self.dim, self.vdim, self.width
+        return {"q": (H * D, W), "k": (H * D, W), "v": (H * V, W), "g": (H * V, W), "o": (W, H * V),
+                **({"norm": (V,)} if self.weighted else {}),
+                **({"a1": (a_rank, W), "a2": (H * D, a_rank), "a2.b": (H * D,)} if self.tau is not None else {})}
+
+    def load(self, w: dict, dtype, device, padded_width: int):
+        """Returns the rows of the common input product and the columns of the output product."""
+        H, D, V, W = self.heads, self.dim, self.vdim, self.width
+        order = list(range(D)) if self.rotary is None else self.rotary.order(D)
+        f32 = lambda t: t.to(device=device, dtype=torch.float32).contiguous()
+        keys = lambda t: fit(t.view(H, D, W)[:, order], H, self.dim_p, padded_width).flatten(0, 1)
+        values = lambda t: fit(t.view(H, V, W), H, self.vdim_p, padded_width).flatten(0, 1)
+        norm = w["norm"] if self.weighted else torch.ones(V)
+        self.norm = f32(fit(norm.to(device), self.vdim_p).repeat(H))
+        self.freqs = None if self.rotary is None or not self.rotary.dims else self.rotary.frequencies(device)
+        into = [keys(w["q"]), keys(w["k"]), values(w["v"]), values(w["g"])]
+        self.low, self.low_rank = None, 0
+        if self.tau is not None:
+            rank = w["a1"].shape[0]
+            self.low_rank = pad_to_multiple(rank, 8)
+            into.append(fit(w["a1"], self.low_rank, padded_width))
+            low = w["a2"].view(H, D, rank)[:, order]
+            self.low = fit(low, H, self.dim_p, self.low_rank).flatten(0, 1).to(device=device, dtype=dtype).contiguous()
+            self.decays = f32(fit(w["a2.b"].view(H, D)[:, order], H, self.dim_p).flatten())
+        else:
+            self.decays = torch.tensor(self.decay, dtype=torch.float32, device=device)
+        out = fit(w["o"].view(W, H, V), padded_width, H, self.vdim_p).flatten(1, 2)
+        self.columns = self.low_at + self.low_rank
+        return torch.cat(into), out
+
+    def allocate(self, num_slots: int, dtype, device) -> torch.Tensor:
+        """Per slot and head: S (dim, vdim)."""
+        return torch.zeros(num_slots, self.heads, self.dim_p, self.vdim_p, dtype=torch.float32, device=device)
+
+    @property
+    def can_run(self) -> bool:
+        """Sizes the blocked kernels cover; others run token by token."""
+        return self.dim_p <= 128 and self.vdim_p <= 128
+
+    def scan(self, proj: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor):
+        """proj: this mixer's columns of the projections, out: of the output rows."""
+        H, D, V = self.heads, self.dim_p, self.vdim_p
+        assert proj.stride(1) == out.stride(1) == 1 and proj.dtype == out.dtype and state.is_contiguous()
+        low = None if self.low is None else F.linear(proj[:, self.low_at:self.low_at + self.low_rank], self.low)
+        tag, stream = _lib.dtype_tag(proj), _lib.stream_ptr(proj)
+        for segments, runs in ((ctx.segments, False), (ctx.run_segments, self.can_run and proj.dtype == torch.bfloat16)):
+            if segments is None:
+                continue
+            args = _lib.LinearArgs(
+                _segments(segments, state.shape[0], proj.shape[0]), _lib.dev_ptr(proj), _lib.dev_ptr(low),
+                _lib.dev_ptr(self.decays), _lib.dev_ptr(self.freqs), _lib.dev_ptr(self.norm), _lib.dev_ptr(state),
+                _lib.dev_ptr(out), proj.stride(0), 0 if low is None else low.stride(0), out.stride(0), H, D, V, self.vdim,
+                0 if self.freqs is None else 2 * self.freqs.numel(), 0, H * D, 2 * H * D, 2 * H * D + H * V, self.q_scale,
+                self.k_scale, 0.0 if self.tau is None else 1.0 / self.tau, self.eps)
+            if not runs:
+                _lib.call_models("zp_linear_scan", ctypes.byref(args), tag, stream)
+                continue
+            size = _lib.load_models("linear").zp_linear_runs_workspace(proj.shape[0] - segments.first_row,
+                                                                    segments.counts.numel(), H, D)
+            ws = torch.empty(size, dtype=torch.uint8, device=proj.device)
+            _lib.call_models("zp_linear_runs", ctypes.byref(args), segments.first_row, segments.longest, _lib.dev_ptr(ws),
+                             size, tag, stream)

@@ -9,14 +9,16 @@ from zipage_amd import _lib
 
 
 def attention_form(softcap: float = 0.0, maps: int = 1, balance: float = 0.0, eps: float = 0.0, vdim: int = 0,
-                   gate: torch.Tensor | None = None):
+                   gate: torch.Tensor | None = None, turns: torch.Tensor | None = None):
     """What an attention does beyond the softmax of scaled products (zp_attention_form), or None.  maps 2: two
-    softmaxes over the same values, o = rms(o1 - balance o2) (mean over `vdim`) times sigmoid(gate)."""
-    if not softcap and maps == 1:
+    softmaxes over the same values, o = rms(o1 - balance o2) (mean over `vdim`) times sigmoid(gate).  turns (N,
+    V / 2, 2) fp32: cos and sin by which adjacent elements of every head's output turn back."""
+    if not softcap and maps == 1 and turns is None:
         return None
     assert gate is None or gate.stride(1) == 1
+    assert turns is None or (turns.dtype == torch.float32 and turns.is_contiguous() and turns.shape[2] == 2)
     return _lib.AttentionForm(float(softcap), maps, float(balance), float(eps), vdim, _lib.dev_ptr(gate) or None,
-                              0 if gate is None else gate.stride(0))
+                              0 if gate is None else gate.stride(0), _lib.dev_ptr(turns) or None)
 
 
 def gather_rows(src: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
