@@ -67,6 +67,11 @@ def test_models_library_exports_every_declared_symbol():
     bad = _lib.DeltaArgs(heads=3, kv_heads=2, dk=32, dv=32, vdim=32, taps=4, out_stride=96,
                          seg=_lib.Segments(n=1, num_slots=1, num_rows=1))
     assert lib.zp_delta_scan(ctypes.byref(bad), 0, None) == 1
+    lib = _lib.load_models("linear")
+    bad = _lib.LinearArgs(heads=2, dk=48, dv=32, vdim=32, in_stride=512, out_stride=64, seg=_lib.Segments(n=1, num_slots=1, num_rows=1))
+    assert lib.zp_linear_scan(ctypes.byref(bad), 0, None) != 0 and b"48" in lib.zp_last_error()
+    bad.dk, bad.rot = 32, 34                                                             # more than a head has
+    assert lib.zp_linear_runs(ctypes.byref(bad), 0, 16, None, 0, 0, None) == 1
 
 
 def test_version_and_error_string():

@@ -54,9 +54,11 @@ def store_form(norm: torch.Tensor | None = None, q_norm: int = 0, k_norm: int = 
     if value_freqs is not None:
         assert value_freqs.dtype == turns.dtype == torch.float32 and value_freqs.is_contiguous() and turns.is_contiguous()
         assert turns.shape[1:] == (value_freqs.numel(), 2)
-    return _lib.StoreForm(_lib.dev_ptr(norm) or None, q_norm, k_norm, float(eps), int(tied),
+    form = _lib.StoreForm(_lib.dev_ptr(norm) or None, q_norm, k_norm, float(eps), int(tied),
                           0 if value_freqs is None else 2 * value_freqs.numel(), _lib.dev_ptr(value_freqs) or None,
                           _lib.dev_ptr(turns) or None)
+    form.held = (norm, value_freqs, turns)    # the form alone has their addresses
+    return form
 
 
 def grouped_rows_attention(q: torch.Tensor, cache: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int,

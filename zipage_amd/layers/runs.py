@@ -17,8 +17,10 @@ def attention_form(softcap: float = 0.0, maps: int = 1, balance: float = 0.0, ep
         return None
     assert gate is None or gate.stride(1) == 1
     assert turns is None or (turns.dtype == torch.float32 and turns.is_contiguous() and turns.shape[2] == 2)
-    return _lib.AttentionForm(float(softcap), maps, float(balance), float(eps), vdim, _lib.dev_ptr(gate) or None,
+    form = _lib.AttentionForm(float(softcap), maps, float(balance), float(eps), vdim, _lib.dev_ptr(gate) or None,
                               0 if gate is None else gate.stride(0), _lib.dev_ptr(turns) or None)
+    form.held = (gate, turns)                 # the form alone has their addresses
+    return form
 
 
 def gather_rows(src: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
