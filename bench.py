@@ -18,7 +18,7 @@ through the decode engine as `end_to_end` (decode tokens/s and the compression s
 
   python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--no-cpu-baseline] [--no-e2e]
   python bench.py --config 5 [--requests R] [--prompt P] [--out-tokens T] [--sync-compress]
-  python bench.py --compare-models [pedivik|kapolorn|rutevik] [--model-sizes 1k,4k]   (the model beside others at equal size)
+  python bench.py --compare-models [pedivik|kapolorn|rutevik|mefupel] [--model-sizes 1k,4k]   (the model beside others at equal size)
 """
 from __future__ import annotations
 
@@ -413,9 +413,9 @@ def main():
     ap.add_argument("--traffic", type=float, default=None,
                     help="HBM bytes per compaction launch measured with rocprofv3 --pmc "
                          "(reported as roofline.traffic)")
-    ap.add_argument("--compare-models", nargs="?", const="pedivik", choices=("pedivik", "kapolorn", "rutevik"),
+    ap.add_argument("--compare-models", nargs="?", const="pedivik", choices=("pedivik", "kapolorn", "rutevik", "mefupel"),
                     help="instead of the compression workload: prefill and decode throughput of "
-                         "Pedivik or Kapolorn beside Qwen3, or of Rutevik beside both, at equal size, and their "
+                         "Pedivik or Kapolorn beside Qwen3, or of Rutevik or Mefupel beside both, at equal size, and their "
                          "kernels against the roofline")
     ap.add_argument("--model-sizes", default="1k,4k", help="sizes of --compare-models")
     args = ap.parse_args()

@@ -1,11 +1,12 @@
-"""Pedivik or Kapolorn beside Qwen3, Rutevik beside Pedivik and Kapolorn, at equal size: prefill and decode
+"""Pedivik or Kapolorn beside Qwen3, Rutevik or Mefupel beside Pedivik and Kapolorn, at equal size: prefill and decode
 throughput through the engine (random weights), and every kernel between the matrix products against its
 roofline, beside the kernel of the other model that does the like work.
 
 Equal size: same width, heads, head dimensions and vocabulary; Pedivik's ungated feed-forward is 1.5
 times as wide as Qwen3's gated one, so both hold the same parameters; a Kapolorn token passes three of 32
 experts and the shared one, each a quarter as wide as Qwen3's feed-forward, a Rutevik token four of 32 such
-experts; its differential layers have half the heads, with values of twice the size.  Kernels are timed as
+experts; its differential layers have half the heads, with values of twice the size.  Mefupel's feed-forwards are
+as wide as Pedivik's.  Kernels are timed as
 replays of a graph of many launches over buffers that together exceed the caches.
 """
 from __future__ import annotations
@@ -557,13 +558,149 @@ def rutevik_kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> 
     return rows
 
 
+def mefupel_shapes(size: str):
+    """Two attention layers with turning values, one of gated linear attention and one of attention over its keys
+    beside retention, in turn, without a loop.  Pedivik and Kapolorn keep their windows and chunks of the same length."""
+    from zipage_amd.engine import MefupelShape
+    from zipage_amd.engine.mefupel import GatedMixer, MefupelLayer, PairMixer, TurningMixer
+    from zipage_amd.layers import Rotary
+    W, H, HK, D, FF, L, V, _, _, win = SIZES[size]
+    turning = TurningMixer(H, HK, D, D, win, Rotary(5e5, D, interleaved=True), D ** -0.5)
+    pair = PairMixer(H, HK, D, win, Rotary(2e4, D // 2), D ** -0.5, H // 2, D, D, Rotary(1e6, D),
+                     tuple(1 - 2.0 ** (-5 - 6 * i / (H // 2)) for i in range(H // 2)))
+    layers = tuple(MefupelLayer((turning, turning, GatedMixer(H, D, D, 16.0), pair)[i % 4], FF * 3 // 2) for i in range(L))
+    return {"mefupel": MefupelShape(V, W, layers, None, 1e-6), "pedivik": shapes(size)[0], "kapolorn": kapolorn_shapes(size)[0]}
+
+
+def mefupel_kernels(size: str, decode_batch: int, prompts: int, prompt: int) -> list[dict]:
+    """The same for Mefupel's kernels; each has the like kernel of Kapolorn, Rutevik or Pedivik behind it."""
+    import torch.nn.functional as F
+    from zipage_amd.engine.inputs import plan_runs
+    from zipage_amd.engine.qwen3 import Segments
+    from zipage_amd.engine.sequence import Portion, Sequence
+    from zipage_amd.layers import (ChannelDelta, LinearAttention, MatrixMemory, Rotary, attention_form, grouped_rows_attention,
+                                   normed_powers, residual_norm, rotary_store, run_attention, small_linear, store_form, xielu)
+    from zipage_amd.sight import Chunk
+    W, H, HK, D, FF, L, V, _, _, win = SIZES[size]
+    dev, BS = torch.device("cuda:0"), 256
+    rnd = lambda *s, dt=BF16: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    i32 = lambda a: torch.as_tensor(a, dtype=torch.int32, device=dev)
+    rows = []
+
+    def put(name, where, secs, byts, flops=0.0, peak=MFMA):
+        roof = max(byts / HBM, flops / peak)
+        bound = "hbm" if byts / HBM >= flops / peak else ("mfma" if peak == MFMA else "fp32")
+        rows.append({"kernel": name, "at": where, "us": round(secs * 1e6, 1), "bound": bound,
+                     "roofline_us": round(roof * 1e6, 1), "frac": round(roof / secs, 3)})
+
+    w32, one, per = torch.ones(W, device=dev), torch.ones(2, device=dev), -(-prompt // BS)
+    for phase, N in (("decode", 64), ("decode", decode_batch), ("prefill", prompts * prompt)):
+        at, big = f"{phase}, {N} tokens", N * W
+        seqs = N if phase == "decode" else prompts
+        # branches joining the stream
+        k = _sets(big * 16)
+        xs, ys = [rnd(N, W, dt=torch.float32) for _ in range(k)], [rnd(3, N, W) for _ in range(k)]
+        held = [rnd(1, N, W, dt=torch.float32) for _ in range(k)]
+        put("residual_norm, two normed branches and a plain one", at,
+            timed(lambda i: residual_norm(xs[i], ys[i][0], w32, 1e-6, W, 1.0, x_out=xs[i], y_weight=w32,
+                                          more=((ys[i][1], w32), (ys[i][2], None))), k), big * 16)
+        put("residual_norm, embedding and vector before a pass", at,
+            timed(lambda i: residual_norm(xs[i], ys[i][0], w32, 1e-6, W, 1.0, x_out=xs[i], history=held[i], mix=one, shift=w32), k),
+            big * 16)
+        put("residual_norm, one plain branch", at,
+            timed(lambda i: residual_norm(xs[i], ys[i][0], w32, 1e-6, W, 1.0, x_out=xs[i]), k), big * 12)
+        put("like: residual_norm of a normed branch", at,
+            timed(lambda i: residual_norm(xs[i], ys[i][0], w32, 1e-6, W, x_out=xs[i], y_weight=w32), k), big * 12)
+        del xs, ys, held
+        n = N * FF * 3 // 2
+        zs, out = [rnd(N, FF * 3 // 2) for _ in range(_sets(n * 4))], rnd(N, FF * 3 // 2)
+        put("normed_powers", at, timed(lambda i: normed_powers(zs[i], (0.7, -0.5, 0.4, 0.3), 1e-6, FF * 3 // 2, out), len(zs)), n * 4)
+        put("like: xielu", at, timed(lambda i: xielu(zs[i], 0.8, 1.3), len(zs)), n * 4)
+        del zs, out
+        # queries, keys and values of the grouped heads
+        pos, slots = torch.arange(N, device=dev, dtype=torch.int32) % prompt, torch.randperm(N, device=dev).int()
+        width, freqs, half = (H + 2 * HK) * D, Rotary(5e5, D).frequencies(dev), Rotary(2e4, D // 2).frequencies(dev)
+        k = _sets(N * width * 4)
+        qkvs, caches = [rnd(N, width) for _ in range(k)], [rnd(-(-N // BS), BS, 2 * HK * D) for _ in range(k)]
+        turns, qk = torch.empty(N, D // 2, 2, device=dev), torch.ones((H + HK) * D, device=dev)
+        turning, keys = store_form(value_freqs=freqs, turns=turns), store_form(qk, H * D, HK * D, 1e-6, tied=True)
+        put("rotary_store, turning values", at,
+            timed(lambda i: rotary_store(qkvs[i], pos, freqs, H, HK, D, D, caches[i], slots, form=turning), k), N * (width + 2 * D) * 4)
+        put("rotary_store, norms, keys as values", at,
+            timed(lambda i: rotary_store(qkvs[i], pos, half, H, HK, D, D, caches[i], slots, form=keys), k),
+            N * (2 * width - HK * D) * 2)
+        put("like: rotary_store", at, timed(lambda i: rotary_store(qkvs[i], pos, freqs, H, HK, D, D, caches[i], slots), k), N * width * 4)
+        del qkvs, caches
+        # recurrences
+        n = N // seqs
+        seg = Segments(i32(range(0, N, n)), i32([n] * seqs), i32(torch.randperm(seqs)), i32([5] * seqs), longest=n,
+                       max_count=int(n == 1))
+        seg = SimpleNamespace(segments=seg if n < 16 else None, run_segments=None if n < 16 else seg)
+        retention = LinearAttention(W, H // 2, D, D, 1e-6, decay=(0.99,) * (H // 2), rotary=Rotary(1e6, D))
+        for name, mixer, ops in ((f"linear attention, a decay per channel, {H} heads", LinearAttention(W, H, D, D, 1e-6, tau=16.0, weighted=True), 5),
+                                 (f"like: delta_scan, {H} heads", ChannelDelta(W, H, H // 2, D, D, 4, 1e-6), 7),
+                                 (f"linear attention, retention, {H // 2} heads", retention, 4),
+                                 (f"like: mlstm_scan, {H // 2} heads", MatrixMemory(W, H // 2, D, D, 15.0, 1e-6), 5)):
+            ranks = (128, 128) if isinstance(mixer, ChannelDelta) else () if isinstance(mixer, MatrixMemory) else (16,)
+            small = {q: torch.randn(*s) * 0.02 for q, s in mixer.shapes(*ranks).items()}
+            mixer.load({q: t.to(BF16) for q, t in small.items()}, BF16, dev, W)
+            h, k = rnd(N, W), 2
+            projs = [rnd(N, mixer.columns) for _ in range(k)]
+            states = [mixer.allocate(seqs + 1, BF16, dev) for _ in range(k)]
+            out = torch.empty(N, mixer.out_columns, device=dev, dtype=BF16)
+            byts = 2 * seqs * mixer.heads * D * D * 4 + N * (mixer.columns + mixer.out_columns) * 2
+            gates = isinstance(mixer, MatrixMemory)
+            secs = timed((lambda i: mixer.scan(h, projs[i], states[i], seg, out)) if gates else
+                         (lambda i: mixer.scan(projs[i], states[i], seg, out)), k, 6)
+            if gates:
+                secs -= timed(lambda i: small_linear(h, mixer.gates), k, 6)
+            elif mixer.low is not None:
+                secs -= timed(lambda i: F.linear(projs[i][:, mixer.low_at:mixer.low_at + mixer.low_rank], mixer.low), k, 6)
+                byts += N * mixer.low.shape[0] * 2
+            put(name, at, max(secs, 1e-9), byts, float(ops) * N * mixer.heads * D * D, FP32)
+            del projs, states, out
+    # ---- decode attention
+    sinks = rnd(H, dt=torch.float32)
+    for B, ctx_len in ((1, prompt), (64, prompt), (decode_batch, prompt)):
+        at, pages = f"decode, {B} sequences, context {ctx_len}", -(-ctx_len // BS)
+        tables, ctx = torch.randperm(B * pages, device=dev).int().view(B, pages), i32([ctx_len] * B)
+        k = _sets(B * win * HK * D * 4)
+        caches, q = [rnd(B * pages, BS, 2 * HK * D) for _ in range(k)], rnd(B, H * D)
+        out, form = torch.empty(B, H * D, device=dev, dtype=BF16), attention_form(turns=rnd(B, D // 2, 2, dt=torch.float32))
+        for name, seen, more in ((f"grouped_rows_attention, window {win}, turning back", min(win, ctx_len), dict(window=win, form=form)),
+                                 (f"grouped_rows_attention, window {win}, sinks", min(win, ctx_len), dict(window=win, sinks=sinks)),
+                                 (f"like: grouped_rows_attention, chunk {win}, sinks", (ctx_len - 1) % win + 1, dict(chunk=win, sinks=sinks))):
+            put(name, at, timed(lambda i: grouped_rows_attention(q, caches[i], H, HK, D, D, tables, ctx, D ** -0.5, out, **more), k),
+                2 * B * seen * HK * D * 2 + 2 * B * H * D * 2, 4.0 * B * H * seen * D)
+        del caches
+    # ---- prefill attention
+    N, at, k = prompts * prompt, f"prefill, {prompts} x {prompt} tokens", 2
+    parts = []
+    for _ in range(prompts):
+        s = Sequence([0] * prompt)
+        s.block_table = list(range(per))
+        parts.append(Portion(s, 0, prompt))
+    qs, kvs, out = [rnd(N, H * D) for _ in range(k)], [rnd(N, 2 * HK * D) for _ in range(k)], torch.empty(N, H * D, device=dev, dtype=BF16)
+    form, chunk = attention_form(turns=rnd(N, D // 2, 2, dt=torch.float32)), Chunk(win)
+    window, blocks = i32(plan_runs(parts, BS, win).tiles), i32(plan_runs(parts, BS, chunk).tiles)
+    pairs = sum(min(i + 1, win) for i in range(prompt)) * prompts
+    for name, tiles, seen, more in ((f"run_attention, window {win}, turning back", window, pairs, dict(window=win, form=form)),
+                                    (f"run_attention, window {win}, sinks", window, pairs, dict(window=win, sinks=sinks)),
+                                    (f"like: run_attention, chunk {win}, sinks", blocks, sum(i % win + 1 for i in range(prompt)) * prompts,
+                                     dict(chunk=win, sinks=sinks))):
+        put(name, at, timed(lambda i: run_attention(qs[i], kvs[i], H, HK, D, D, tiles, D ** -0.5, out, **more), k, 6),
+            N * (2 * H + 2 * HK) * D * 2, 4.0 * seen * H * D)
+    return rows
+
+
 def beside_qwen3(model: str, make):
     return lambda size: dict(zip((model, "qwen3"), make(size)))
 
 
 MODELS = {"pedivik": (beside_qwen3("pedivik", shapes), kernels),
           "kapolorn": (beside_qwen3("kapolorn", kapolorn_shapes), kapolorn_kernels),
-          "rutevik": (rutevik_shapes, rutevik_kernels)}
+          "rutevik": (rutevik_shapes, rutevik_kernels),
+          "mefupel": (mefupel_shapes, mefupel_kernels)}
 
 
 def compare(model: str = "pedivik", sizes=("1k", "4k"), out_tokens: int = 64) -> dict:

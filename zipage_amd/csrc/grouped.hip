@@ -36,105 +36,128 @@ struct RotaryArgs {
   int V;                    // of a value head
   const float* vfreqs;      // (V / 2,): values turn, elements 2 i and 2 i + 1 with frequency i; or null
   float2* turns;            // (n, V / 2): cos and sin of the values' angles, for the way back
+  int staged;               // bytes of q and k that wait in LDS while their norms are taken; 0: they are read twice
 };
-constexpr int kRotTokens = 4;
 
-// Four tokens per workgroup: their angles once, in LDS, for all heads.  VEC elements per item; an
-// item of the rotated part is the pair (i .. i + VEC, i + half ..).  FORMS: norms, tied or turning values.
-template <typename T, int VEC, bool FORMS>
+// Four tokens per workgroup, or one where there are few, each with its own threads; a token's angles once, in LDS, for
+// all heads.  VEC elements per item; an item of the rotated part is the pair (i .. i + VEC, i + half ..).  NORM: norms
+// over q and k, and tied values; TURN: values turn.
+template <typename T, int VEC, int TOKENS, bool NORM, bool TURN>
 __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
   extern __shared__ __align__(16) char lds_raw[];
-  __shared__ float rms[2][kRotTokens];
-  float2* cs = (float2*)lds_raw;            // [kRotTokens][half]
-  float2* vcs = cs + kRotTokens * a.half;   // [kRotTokens][V / 2]
-  const int n0 = blockIdx.x * kRotTokens, tid = threadIdx.x;
-  for (int i = tid; i < kRotTokens * a.half; i += 256) {
-    const int tok = i / a.half;
-    if (n0 + tok < a.n) {
-      cs[i] = rotary_turn(a.positions[n0 + tok], a.freqs[i - tok * a.half]);
-    }
-  }
-  if (FORMS && a.vfreqs) {
-    const int vh = a.V / 2;
-    for (int i = tid; i < kRotTokens * vh; i += 256) {
-      const int tok = i / vh;
-      if (n0 + tok < a.n) {
-        vcs[i] = rotary_turn(a.positions[n0 + tok], a.vfreqs[i - tok * vh]);
-        a.turns[(int64_t)n0 * vh + i] = vcs[i];
-      }
-    }
-  }
-  if (FORMS && a.norm) {                    // a wave per token
-    const int64_t row = min(n0 + (tid >> 6), a.n - 1);
-    const int edge = a.H * a.D, end = edge + a.HK * a.D;
-    float qs = 0.f, ks = 0.f;
-    for (int c = (tid & 63) * 8; c < end; c += 512) {
-      float x[8], s = 0.f;
-      Vec8<T>::ld(a.in, row * a.in_st + c, x);
+  __shared__ float squares[2][4];           // of q and k, by wave
+  constexpr int kPer = 256 / TOKENS;        // threads per token
+  const int tok = TOKENS == 1 ? 0 : __builtin_amdgcn_readfirstlane(threadIdx.x / kPer), tid = threadIdx.x % kPer;
+  const int64_t row = blockIdx.x * TOKENS + tok;
+  const bool live = row < a.n;              // uniform in the wave
+  const int heads = a.H + a.HK, edge = a.H * a.D, end = heads * a.D;
+  float2* const cs = (float2*)lds_raw + tok * a.half;                        // [TOKENS][half]
+  float2* const vcs = (float2*)lds_raw + TOKENS * a.half + tok * (a.V / 2);   // [TOKENS][V / 2]
+  char* const wait = lds_raw + ((TOKENS * (a.half + (TURN ? a.V / 2 : 0)) * 8 + 15) & ~15) + tok * a.staged;   // [TOKENS][staged]
+  if (live) {
+    typename Vec8<T>::Raw x[4];              // pieces of q and k, requested while the angles are computed
+    auto fetch = [&](int c0) {
 #pragma unroll
-      for (int i = 0; i < 8; ++i) s = fmaf(x[i], x[i], s);
-      if (c < edge) qs += s; else ks += s;
-    }
-    qs = wave_sum(qs);
-    ks = wave_sum(ks);
-    if ((tid & 63) == 0) {
-      rms[0][tid >> 6] = 1.f / sqrtf(qs / (float)a.q_norm + a.eps);
-      rms[1][tid >> 6] = 1.f / sqrtf(ks / (float)a.k_norm + a.eps);
+      for (int u = 0; u < 4; ++u) x[u] = Vec8<T>::raw(a.in, row * a.in_st + min(c0 + u * kPer * 8, end - 8));
+    };
+    if (NORM && a.norm) fetch(tid * 8);
+    const int position = a.positions[row];
+    for (int i = tid; i < a.half; i += kPer) cs[i] = rotary_turn(position, a.freqs[i]);
+    if (TURN)
+      for (int i = tid; i < a.V / 2; i += kPer) {
+        vcs[i] = rotary_turn(position, a.vfreqs[i]);
+        a.turns[row * (a.V / 2) + i] = vcs[i];
+      }
+    if (NORM && a.norm) {
+      float qs = 0.f, ks = 0.f;
+      for (int c0 = tid * 8; c0 < end; c0 += 4 * kPer * 8) {
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int c = c0 + u * kPer * 8;
+          float v[8], s = 0.f;
+          Vec8<T>::unpack(x[u], v);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) s = fmaf(v[i], v[i], s);
+          if (c < edge) qs += s; else if (c < end) ks += s;
+          if (a.staged && c < end) Vec8<T>::st(wait, c, v);
+        }
+        if (c0 + 4 * kPer * 8 < end) fetch(c0 + 4 * kPer * 8);
+      }
+      qs = wave_sum(qs);
+      ks = wave_sum(ks);
+      if ((threadIdx.x & 63) == 0) {
+        squares[0][threadIdx.x >> 6] = qs;
+        squares[1][threadIdx.x >> 6] = ks;
+      }
     }
   }
   __syncthreads();
+  if (!live) return;
+  float rq = 1.f, rk = 1.f;
+  if (NORM && a.norm) {
+    float qs = 0.f, ks = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4 / TOKENS; ++w) {
+      qs += squares[0][tok * (4 / TOKENS) + w];
+      ks += squares[1][tok * (4 / TOKENS) + w];
+    }
+    rq = 1.f / sqrtf(qs / (float)a.q_norm + a.eps);
+    rk = 1.f / sqrtf(ks / (float)a.k_norm + a.eps);
+  }
   const int pairs = a.half / VEC, per_head = (a.D - a.half) / VEC;
-  const int heads = a.H + a.HK, rotated = heads * per_head, items = rotated + a.VT / VEC;
+  const int rotated = heads * per_head, items = rotated + a.VT / VEC;
+  const uint32_t inv = 0xffffffffu / per_head + 1;           // of a division; per_head 1 overflows to 0
   const int kvw = a.HK * a.D + a.VT;
-  for (int id = tid; id < kRotTokens * items; id += 256) {
-    const int tok = id / items, it = id - tok * items;
-    const int64_t row = n0 + tok;
-    if (row >= a.n) break;
+  int64_t slot = a.slots[row];
+  if (slot >= a.num_slots) slot = -1;
+  auto raw = [&](int c, float* o) {
+    if (NORM && a.staged && c < end) {
+      if constexpr (VEC == 8) Vec8<T>::ld(wait, c, o); else o[0] = Elem<T>::ld(wait, c);
+      return;
+    }
+    const int64_t at = row * a.in_st + c;
+    if constexpr (VEC == 8) Vec8<T>::ld(a.in, at, o); else o[0] = Elem<T>::ld(a.in, at);
+    if (!NORM && a.bias) {
+      float b[VEC];
+      if constexpr (VEC == 8) Vec8<F32>::ld(a.bias, c, b); else b[0] = a.bias[c];
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) o[i] += b[i];
+    }
+  };
+  auto load = [&](int c, float* o) {         // of q or k
+    raw(c, o);
+    if (NORM && a.norm) {
+      float w[VEC];
+      if constexpr (VEC == 8) Vec8<F32>::ld(a.norm, c, w); else w[0] = a.norm[c];
+      const float r = c < edge ? rq : rk;
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) o[i] *= r * w[i];
+    }
+  };
+  auto put = [&](int c, const float* o) {   // column of the row [q | k | v]
+    const int kc = c - edge;
+    if (kc < 0) {
+      if constexpr (VEC == 8) Vec8<T>::st(a.q_out, row * edge + c, o);
+      else Elem<T>::st(a.q_out, row * edge + c, o[0]);
+      return;
+    }
+    if (a.kv_out) {
+      if constexpr (VEC == 8) Vec8<T>::st(a.kv_out, row * kvw + kc, o);
+      else Elem<T>::st(a.kv_out, row * kvw + kc, o[0]);
+    }
+    if (slot >= 0) {
+      if constexpr (VEC == 8) Vec8<T>::st(a.cache, slot * kvw + kc, o);
+      else Elem<T>::st(a.cache, slot * kvw + kc, o[0]);
+    }
+  };
+  for (int it = tid; it < items; it += kPer) {
     float x[VEC], y[VEC];
-    auto raw = [&](int c, float* o) {
-      const int64_t at = row * a.in_st + c;
-      if constexpr (VEC == 8) Vec8<T>::ld(a.in, at, o); else o[0] = Elem<T>::ld(a.in, at);
-      if (a.bias) {
-        float b[VEC];
-        if constexpr (VEC == 8) Vec8<F32>::ld(a.bias, c, b); else b[0] = a.bias[c];
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) o[i] += b[i];
-      }
-    };
-    auto load = [&](int c, float* o) {         // of q or k
-      raw(c, o);
-      if (FORMS && a.norm) {
-        float w[VEC];
-        if constexpr (VEC == 8) Vec8<F32>::ld(a.norm, c, w); else w[0] = a.norm[c];
-        const float r = rms[c < a.H * a.D ? 0 : 1][tok];
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) o[i] *= r * w[i];
-      }
-    };
-    int64_t slot = a.slots[row];
-    if (slot >= a.num_slots) slot = -1;
-    auto put = [&](int c, const float* o) {   // column of the row [q | k | v]
-      const int kc = c - a.H * a.D;
-      if (kc < 0) {
-        if constexpr (VEC == 8) Vec8<T>::st(a.q_out, row * a.H * a.D + c, o);
-        else Elem<T>::st(a.q_out, row * a.H * a.D + c, o[0]);
-        return;
-      }
-      if (a.kv_out) {
-        if constexpr (VEC == 8) Vec8<T>::st(a.kv_out, row * kvw + kc, o);
-        else Elem<T>::st(a.kv_out, row * kvw + kc, o[0]);
-      }
-      if (slot >= 0) {
-        if constexpr (VEC == 8) Vec8<T>::st(a.cache, slot * kvw + kc, o);
-        else Elem<T>::st(a.cache, slot * kvw + kc, o[0]);
-      }
-    };
     if (it >= rotated) {
-      const int v = (it - rotated) * VEC, c = heads * a.D + v;
-      const int from = FORMS && a.tied ? a.H * a.D + v : c;
+      const int v = (it - rotated) * VEC, c = end + v;
+      const int from = NORM && a.tied ? edge + v : c;
       raw(from, x);
-      if (FORMS && a.vfreqs) {
-        const float2* r = vcs + tok * (a.V / 2) + v % a.V / 2;
+      if (TURN) {
+        const float2* r = vcs + v % a.V / 2;
         if constexpr (VEC == 8) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) turn_pair(x[2 * i], x[2 * i + 1], r[i].x, r[i].y);
@@ -146,7 +169,7 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
       put(c, x);
       continue;
     }
-    const int h = it / per_head, p = it - h * per_head;
+    const int h = per_head == 1 ? it : (int)__umulhi((uint32_t)it, inv), p = it - h * per_head;
     if (p >= pairs) {                          // dimensions behind the rotated ones
       const int c = h * a.D + (p + pairs) * VEC;
       load(c, x);
@@ -158,7 +181,7 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(RotaryArgs a) {
     load(c + a.half, y);
 #pragma unroll
     for (int i = 0; i < VEC; ++i) {
-      const float2 r = cs[tok * a.half + p * VEC + i];
+      const float2 r = cs[p * VEC + i];
       turn_pair(x[i], y[i], r.x, r.y);
     }
     put(c, x);
@@ -638,18 +661,32 @@ extern "C" int zp_rotary_store(const void* in, const float* bias, const int32_t*
   ZP_REQUIRE(aligned16(in) && aligned16(q_out) && aligned16(kv_out) && aligned16(cache) && aligned16(bias) && aligned16(f.norm),
              "rotary_store: tensors must be 16-byte aligned");
   ZP_REQUIRE(!f.norm || (!bias && f.q_norm > 0 && f.k_norm > 0), "rotary_store: norms of whole projections go without a bias");
+  ZP_REQUIRE(!f.tied || !bias, "rotary_store: values that are the keys go without a bias");
   ZP_REQUIRE(!f.tied || VT == HK * D, "rotary_store: values that are the keys have their size");
   ZP_REQUIRE(!f.value_freqs || (f.turns && f.V > 0 && f.V % 8 == 0 && f.V <= 1024 && VT % f.V == 0),
              "rotary_store: values that turn need their head size and room for the turns");
   RotaryArgs a = {in, bias, positions, freqs, q_out, kv_out, cache, slots, n, H, HK, D, VT, rot / 2, in_stride, num_slots,
                   f.norm, f.q_norm, f.k_norm, f.eps, f.tied != 0, f.V, f.value_freqs, (float2*)f.turns};
-  const unsigned grid = (unsigned)((n + kRotTokens - 1) / kRotTokens);
-  const size_t smem = sizeof(float2) * kRotTokens * (rot / 2 + (f.value_freqs ? f.V / 2 : 0));
+  const int tokens = n < 2048 ? 1 : 4;
+  const int64_t row = (int64_t)(H + HK) * D * zp_dtype_bytes(dtype);
+  if (f.norm && row * tokens <= 32 * 1024) a.staged = (int)row;
+  const unsigned grid = (unsigned)((n + tokens - 1) / tokens);
+  const size_t smem = ((sizeof(float2) * tokens * (rot / 2 + (f.value_freqs ? f.V / 2 : 0)) + 15) & ~(size_t)15) + tokens * a.staged;
   hipStream_t st = (hipStream_t)stream;
-#define ZP_ROTARY(T, VEC)                                                                                          \
-  do {                                                                                                             \
-    if (form) hipLaunchKernelGGL((rotary_store_kernel<T, VEC, true>), dim3(grid), dim3(256), smem, st, a);         \
-    else hipLaunchKernelGGL((rotary_store_kernel<T, VEC, false>), dim3(grid), dim3(256), smem, st, a);             \
+  const bool norm = f.norm || f.tied, turn = f.value_freqs != nullptr;
+  ZP_REQUIRE(smem <= 64 * 1024 && (int64_t)(H + HK) * D + VT < (1 << 24), "rotary_store: heads of %d, %d rotated: too long", D, rot);
+#define ZP_ROTARY_FORM(T, VEC, N, NORM, TURN) \
+  hipLaunchKernelGGL((rotary_store_kernel<T, VEC, N, NORM, TURN>), dim3(grid), dim3(256), smem, st, a)
+#define ZP_ROTARY_N(T, VEC, N)                                     \
+  do {                                                             \
+    if (norm && turn) ZP_ROTARY_FORM(T, VEC, N, true, true);       \
+    else if (norm) ZP_ROTARY_FORM(T, VEC, N, true, false);         \
+    else if (turn) ZP_ROTARY_FORM(T, VEC, N, false, true);         \
+    else ZP_ROTARY_FORM(T, VEC, N, false, false);                  \
+  } while (0)
+#define ZP_ROTARY(T, VEC)                                          \
+  do {                                                             \
+    if (tokens == 1) ZP_ROTARY_N(T, VEC, 1); else ZP_ROTARY_N(T, VEC, 4); \
   } while (0)
   if (dtype == ZP_BF16) {
     if (rot % 16 == 0) ZP_ROTARY(BF16, 8); else ZP_ROTARY(BF16, 1);
@@ -657,6 +694,8 @@ extern "C" int zp_rotary_store(const void* in, const float* bias, const int32_t*
     if (rot % 16 == 0) ZP_ROTARY(F32, 8); else ZP_ROTARY(F32, 1);
   }
 #undef ZP_ROTARY
+#undef ZP_ROTARY_N
+#undef ZP_ROTARY_FORM
   ZP_LAUNCH_CHECK();
   return ZP_OK;
 }

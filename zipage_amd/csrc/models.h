@@ -16,10 +16,13 @@ typedef uint32_t zp_u32x4 __attribute__((ext_vector_type(4)));
 typedef float zp_f32x4 __attribute__((ext_vector_type(4)));
 
 // Eight consecutive elements as fp32, 16-byte accesses; `i` is a multiple of 8.
+// Or in two steps, so that nothing waits for the load before its use: raw() and unpack().
 template <typename T> struct Vec8;
 template <> struct Vec8<BF16> {
-  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) {
-    const zp_u32x4 v = *(const zp_u32x4*)((const uint16_t*)p + i);
+  typedef zp_u32x4 Raw;
+  __device__ static __forceinline__ Raw raw(const void* p, int64_t i) { return *(const zp_u32x4*)((const uint16_t*)p + i); }
+  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) { unpack(raw(p, i), o); }
+  __device__ static __forceinline__ void unpack(const Raw& v, float* o) {
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
       o[2 * k] = __uint_as_float(v[k] << 16);
@@ -37,11 +40,14 @@ template <> struct Vec8<BF16> {
   }
 };
 template <> struct Vec8<F32> {
-  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) {
-    const zp_f32x4 a = *(const zp_f32x4*)((const float*)p + i);
-    const zp_f32x4 b = *(const zp_f32x4*)((const float*)p + i + 4);
+  struct Raw { zp_f32x4 a, b; };
+  __device__ static __forceinline__ Raw raw(const void* p, int64_t i) {
+    return Raw{*(const zp_f32x4*)((const float*)p + i), *(const zp_f32x4*)((const float*)p + i + 4)};
+  }
+  __device__ static __forceinline__ void ld(const void* p, int64_t i, float* o) { unpack(raw(p, i), o); }
+  __device__ static __forceinline__ void unpack(const Raw& v, float* o) {
 #pragma unroll
-    for (int k = 0; k < 4; ++k) { o[k] = a[k]; o[k + 4] = b[k]; }
+    for (int k = 0; k < 4; ++k) { o[k] = v.a[k]; o[k + 4] = v.b[k]; }
   }
   __device__ static __forceinline__ void st(void* p, int64_t i, const float* o) {
     *(zp_f32x4*)((float*)p + i) = zp_f32x4{o[0], o[1], o[2], o[3]};
