@@ -61,6 +61,12 @@ CONFIGS = {
         layer(gla(1, 200, 250, 1.0), 16),
         layer(pair((18, 9, 40, 2, 8), (1, 32, 32), 32, (0.97,)), None),
     ], (0, 5, 2), eps=1e-2),
+    # a loop of one pass up to the last layer; one head of each kind
+    "once": config(64, 89, [
+        layer(gla(1, 16, 16, 4.0), 48),
+        layer(attention(3, 1, 16, 32, 9, 16), 24),
+        layer(pair((2, 1, 32, 12, 16), (1, 64, 16), 30, (0.9,)), 40),
+    ], (1, 3, 1)),
     # bfloat16 on the kernels of serving sizes
     "calm": config(128, 113, [
         layer(attention(8, 2, 32, 48, 37, 16), 160),

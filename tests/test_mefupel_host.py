@@ -177,6 +177,8 @@ def test_cases_show_planted_faults(name, monkeypatch):
                     > limit, (i, j)
     assert fault(lambda c: c["norm"].update(eps=cfg["norm"]["eps"] * 100 + 1e-2)) > limit
     if "loop" in cfg:
+        assert fault(change_w=lambda t: t.update({"loop.step": t["loop.step"] * 0})) > limit
+    if cfg.get("loop", {"times": 1})["times"] > 1:
         assert fault(change_w=lambda t: t.update({"loop.step": t["loop.step"].flip(0)})) > limit
         assert fault(change_w=lambda t: t.update({"loop.step": t["loop.step"][:1].expand_as(t["loop.step"])})) > limit
         once = {**cfg, "loop": None}              # the passes written out, without what joins before each
