@@ -463,7 +463,9 @@ def main():
         del src, dst
         torch.cuda.empty_cache()
 
-    run = run_pipeline(args.config, args, args.pipeline_switches, args.batch)
+    # the JSON line is the only one on standard output; a finished leg is told on standard error
+    told = lambda leg, result: print(f"bench: {leg}", file=sys.stderr, flush=True) or result
+    run = told("pipeline", run_pipeline(args.config, args, args.pipeline_switches, args.batch))
     out = {"metric": "sequences compressed/sec", "value": run.pop("value"), "unit": run.pop("unit"),
            "n_gpus": 1, "steps": run.pop("steps"), "warmup": run.pop("warmup"),
            "ms_per_step": run.pop("ms_per_step"), "higher_is_better": True, "scaling": "weak",
@@ -472,11 +474,11 @@ def main():
     headline = args.config == 4 and args.batch is None
     if headline and not args.no_extra_legs:
         # the smaller single-layer workload of BASELINE configs[1], more steps (a step is 0.4 ms)
-        out["configs1_b64"] = run_pipeline(2, args, steps=max(args.steps, 100), warmup=10)
+        out["configs1_b64"] = told("64 sequences", run_pipeline(2, args, steps=max(args.steps, 100), warmup=10))
         if not args.no_e2e:
-            out["end_to_end"] = end_to_end(args.requests, args.prompt, args.out_tokens,
-                                           not args.sync_compress, args.ragged_prompts,
-                                           args.script_switches)
+            out["end_to_end"] = told("end to end", end_to_end(args.requests, args.prompt, args.out_tokens,
+                                                              not args.sync_compress, args.ragged_prompts,
+                                                              args.script_switches))
             if not args.no_e2e_variants:
                 # where overlap can exist: ragged prompts, on the side stream and in line, from this
                 # same process (shorter runs: every sequence still compresses 2-4 times); with
@@ -485,7 +487,7 @@ def main():
                 n = min(args.out_tokens, args.variant_tokens)
                 pairs = ((True, False), (False, True)) if args.all_e2e_variants else ((False, True),)
                 out["end_to_end"]["variants"] = [
-                    end_to_end(args.requests, args.prompt, n, a, ragged, scripts, attention_probe=False)
+                    told("variant", end_to_end(args.requests, args.prompt, n, a, ragged, scripts, attention_probe=False))
                     for scripts, ragged in pairs for a in (True, False)]
     print(json.dumps(out))
 
